@@ -44,6 +44,10 @@ extern "C" {
 #define TLF_KV_BF16 0
 #define TLF_KV_FP8_E4M3 1 /* OCP e4m3fn, per-KV-head fp32 scale */
 
+/* Tensor element types of the entry points that take a `dtype` */
+#define TLF_DT_BF16 0
+#define TLF_DT_F32 1
+
 /* ABI version of the loaded library (== TLF_ABI_VERSION it was built with). */
 int tlf_version(void);
 /* Static, human readable text for a return code of this library. */
@@ -463,6 +467,113 @@ int tlf_probe_copy(const void *src, void *dst, size_t bytes, void *stream);
 int tlf_probe_mfma(void *out, int32_t iters, int32_t mode, void *stream);
 int tlf_probe_mix(const void *big, size_t big_bytes, const void *small_region, size_t small_bytes,
                   int32_t l2_eighths, void *sink, void *stream);
+
+/* ===========================================================================
+ * Mechanisms of hybrid (attention + recurrent) decoders.  No counterpart in the reference.  `dtype` is the
+ * element type of activations, weights and caches (TLF_DT_BF16 or TLF_DT_F32); the residual stream, norms,
+ * rotations, scores, attention weights, decays and recurrent states are fp32 in both.
+ *
+ * A step is a batch of sequences: sequence s owns the rows cu_seqlens_q[s] .. cu_seqlens_q[s + 1] - 1 of the step's
+ * tensors and has seq_starts[s] tokens before them in the caches.
+ *
+ * Grouped RMSNorm around an fp32 residual.  A row of `width` values is split into `groups` equal parts, each
+ * divided by its own sqrt(mean(part^2) + eps); the whole is multiplied by a weight.
+ *
+ *   tlf_group_rmsnorm_add:    x += norm(y + y_bias) * w_post;  h = norm(x) * w_next
+ *   tlf_embed_group_rmsnorm:  x  = table[id];                  h = norm(x) * w_next
+ *
+ * x fp32 [rows, width] contiguous; y, h, table, weights: dtype; y_bias may be NULL; w_next NULL: no h.
+ * width / groups <= 16384.  An id outside [0, vocab) embeds as zeros. */
+int tlf_group_rmsnorm_add(const void *y, int64_t y_stride, const void *y_bias, const void *w_post, float *x,
+                          const void *w_next, void *h, int32_t rows, int32_t width, int32_t groups, float eps,
+                          int32_t dtype, void *stream);
+int tlf_embed_group_rmsnorm(const int64_t *ids, const void *table, int32_t vocab, float *x, const void *w_next,
+                            void *h, int32_t rows, int32_t width, int32_t groups, float eps, int32_t dtype,
+                            void *stream);
+
+/* Dense operations of 32-bit mode (fp32 products and sums; any M, N, K): y = x . w^T, y = silu(x[:, :I]) * x[:, I:],
+ * greedy argmax (first index among ties). */
+int tlf_f32_gemm(const float *x, int64_t x_stride, const float *w, float *y, int32_t M, int32_t N, int32_t K,
+                 void *stream);
+int tlf_f32_silu_and_mul(const float *x, float *y, int32_t rows, int32_t inter, void *stream);
+int tlf_f32_argmax(const float *logits, int64_t row_stride, int64_t *out, int32_t rows, int32_t vocab, void *stream);
+
+/* Attention with unnormalised sigmoid weights over a sliding window and pooled blocks.
+ *
+ * Position i sees the tokens j with 0 <= i - j < window, and for every block b of `pool` tokens with
+ * b * pool + pool - 1 <= i - window one key (the mean of the block's cached keys) and one value (the mean of its
+ * values).  weight = sigmoid(q . k * scale + score_bias[head]);  out = sum(weight * value) * gate[row, head].
+ *
+ * Caches: k_cache / v_cache [num_pages, block_size, Hkv, Dp], pk_cache / pv_cache [num_pages, ceil(block_size / pool),
+ * Hkv, Dp] with the same page numbers: block b is row b - (page * block_size) / pool of the page that holds its last
+ * token (page = index in the sequence).  Dp = head_dim rounded up to a multiple of 32, pads are zeros.
+ * block_size % 64 == 0, head_dim even and <= 256.
+ *
+ * tlf_attn_prep: projection rows [q heads | k heads | one gate value per q head] -> biases (may be NULL) added;
+ *   v row = the key so far; first rot_dims dimensions of q and k rotated pairwise (2 i, 2 i + 1) with
+ *   cos_sin[pos] = cos of the rot_dims / 2 angles, then their sines (a position outside the table is not rotated);
+ *   q and k divided by their root mean square; k / v rows stored at slot_mapping (negative: not stored),
+ *   q_out [n, Hq, Dp], gate [n, Hq] = sigmoid, fp32.
+ * tlf_pool_blocks: pooled rows of the blocks that sequences first_seq .. first_seq + num_seqs - 1 complete in this step
+ *   (max_tokens: the most tokens one of them has in the step).
+ * tlf_pooled_attn_rows: any rows; row_seq[r] is the block-table row (NULL: r).  slot_mapping[r] < 0: a padding row,
+ *   out = 0.  pool_new: also write the pooled row of a block that a row's own token completes (decode).
+ *   max_len bounds the positions.  out rows: Hq * head_dim values.
+ * tlf_pooled_attn_prefill: bf16 matrix-core kernel for the portions of sequences first_seq .. + num_seqs - 1 (all other
+ *   arguments as above; q, gate and out are indexed by the step's rows). */
+int tlf_attn_prep(const void *proj, int64_t proj_stride, const void *q_bias, const void *k_bias,
+                  const int64_t *positions, const float *cos_sin, int32_t max_pos, int32_t rot_dims,
+                  const int32_t *slot_mapping, int64_t num_slots, void *q_out, void *k_cache, void *v_cache,
+                  float *gate, int32_t n, int32_t num_q_heads, int32_t num_kv_heads, int32_t head_dim,
+                  int32_t padded_dim, float eps, int32_t dtype, void *stream);
+int tlf_pool_blocks(const void *k_cache, const void *v_cache, void *pk_cache, void *pv_cache,
+                    const int32_t *block_tables, int64_t bt_stride, const int32_t *cu_seqlens_q,
+                    const int32_t *seq_starts, int32_t first_seq, int32_t num_seqs, int32_t max_tokens,
+                    int32_t num_kv_heads, int32_t head_dim, int32_t block_size, int32_t pool, int32_t window,
+                    int64_t num_pages, int32_t dtype, void *stream);
+size_t tlf_pooled_attn_rows_workspace_bytes(int32_t rows, int32_t num_q_heads, int32_t num_kv_heads, int32_t head_dim,
+                                            int32_t pool, int32_t window, int32_t max_len);
+int tlf_pooled_attn_rows(const void *q, const void *score_bias, const float *gate, const void *k_cache,
+                         const void *v_cache, void *pk_cache, void *pv_cache, const int32_t *block_tables,
+                         int64_t bt_stride, const int64_t *positions, const int32_t *slot_mapping,
+                         const int32_t *row_seq, void *out, int64_t out_stride, int32_t rows, int32_t num_q_heads,
+                         int32_t num_kv_heads, int32_t head_dim, int32_t block_size, int32_t pool, int32_t window,
+                         int32_t max_len, int64_t num_pages, float scale, int32_t pool_new, int32_t dtype,
+                         void *workspace, size_t workspace_bytes, void *stream);
+int tlf_pooled_attn_prefill(const void *q, const void *score_bias, const float *gate, const void *k_cache,
+                            const void *v_cache, const void *pk_cache, const void *pv_cache,
+                            const int32_t *block_tables, int64_t bt_stride, const int32_t *cu_seqlens_q,
+                            const int32_t *seq_starts, int32_t first_seq, int32_t num_seqs, int32_t max_tokens,
+                            void *out, int64_t out_stride, int32_t num_q_heads, int32_t num_kv_heads, int32_t head_dim,
+                            int32_t block_size, int32_t pool, int32_t window, int64_t num_pages, float scale,
+                            void *stream);
+
+/* Gated linear attention with a decay per key channel.  Projection rows are [q | k | v | g | r] (heads * key_dim twice,
+ * heads * value_dim twice, rank values).  Per head, state S [key_dim, value_dim] fp32 at state[slot, head]:
+ *   alpha = sigmoid(a2 . r + a2_bias)^(1 / tau);  S = diag(alpha) S + k v^T;  o = S^T (q * q_scale)
+ *   out = o / sqrt(mean(o^2) + eps) * norm_weight * silu(g)
+ * a2 [heads * key_dim, rank].  key_dim <= 256, value_dim <= 512, rank <= 256.
+ *
+ * tlf_gla_decode: one token per row; position 0 starts from a zero state, a slot outside [0, num_slots) is a padding
+ *   row (out = 0).
+ * tlf_gla_portions: sequences first_seq .. + num_seqs - 1 of the step (state_slots and seq_starts are indexed by the
+ *   step's sequences, a start of 0 begins with a zero state).  Their tokens are cut into chunks of at most 16 that do not
+ *   cross a sequence: chunk c holds the chunk_lens[c] rows from chunk_rows[c] on, counted from the row `proj` and
+ *   `out` point to; sequence first_seq + s owns the chunks cu_chunks[s] .. cu_chunks[s + 1] - 1.  `rows` rows in all. */
+int tlf_gla_decode(const void *proj, int64_t proj_stride, const void *a2, const void *a2_bias,
+                   const void *norm_weight, float *state, const int32_t *state_slots, int32_t num_slots,
+                   const int64_t *positions, void *out, int64_t out_stride, int32_t rows, int32_t heads,
+                   int32_t key_dim, int32_t value_dim, int32_t rank, float tau, float q_scale, float eps,
+                   int32_t dtype, void *stream);
+size_t tlf_gla_portions_workspace_bytes(int32_t rows, int32_t chunks, int32_t heads, int32_t key_dim,
+                                        int32_t value_dim);
+int tlf_gla_portions(const void *proj, int64_t proj_stride, const void *a2, const void *a2_bias,
+                     const void *norm_weight, float *state, const int32_t *state_slots, int32_t num_slots,
+                     const int32_t *seq_starts, const int32_t *chunk_rows, const int32_t *chunk_lens,
+                     const int32_t *cu_chunks, int32_t chunks, int32_t first_seq, int32_t num_seqs, void *out,
+                     int64_t out_stride, int32_t rows, int32_t heads, int32_t key_dim, int32_t value_dim,
+                     int32_t rank, float tau, float q_scale, float eps, int32_t dtype, void *workspace,
+                     size_t workspace_bytes, void *stream);
 
 #ifdef __cplusplus
 }

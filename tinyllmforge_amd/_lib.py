@@ -16,6 +16,8 @@ LIB_PATH = os.path.join(_HERE, "libtlf_hip.so")
 ABI_VERSION = 1
 KV_BF16 = 0
 KV_FP8_E4M3 = 1
+DT_BF16 = 0
+DT_F32 = 1
 
 _P, _I32, _I64, _F, _SZ = c_void_p, c_int32, c_int64, c_float, c_size_t
 
@@ -66,6 +68,25 @@ SIGNATURES = {
     "tlf_varlen_prefill_attn": (c_int32, [_P, _I64, _P, _I64, _P, _I64, _I32, _P, _P, _P, _P, _P, _I64,
                                           _P, _I32, _I32, _I32, _I32, _I32, _I32, _I64, _F, _P]),
     "tlf_embedding": (c_int32, [_P, _P, _P, _I32, _I32, _I32, _P]),
+    "tlf_group_rmsnorm_add": (c_int32, [_P, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _F, _I32, _P]),
+    "tlf_embed_group_rmsnorm": (c_int32, [_P, _P, _I32, _P, _P, _P, _I32, _I32, _I32, _F, _I32, _P]),
+    "tlf_f32_gemm": (c_int32, [_P, _I64, _P, _P, _I32, _I32, _I32, _P]),
+    "tlf_f32_silu_and_mul": (c_int32, [_P, _P, _I32, _I32, _P]),
+    "tlf_f32_argmax": (c_int32, [_P, _I64, _P, _I32, _I32, _P]),
+    "tlf_attn_prep": (c_int32, [_P, _I64, _P, _P, _P, _P, _I32, _I32, _P, _I64, _P, _P, _P, _P,
+                                _I32, _I32, _I32, _I32, _I32, _F, _I32, _P]),
+    "tlf_pool_blocks": (c_int32, [_P, _P, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _I32,
+                                  _I64, _I32, _P]),
+    "tlf_pooled_attn_rows_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32, _I32, _I32, _I32]),
+    "tlf_pooled_attn_rows": (c_int32, [_P, _P, _P, _P, _P, _P, _P, _P, _I64, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32,
+                                       _I32, _I32, _I32, _I32, _I64, _F, _I32, _I32, _P, _SZ, _P]),
+    "tlf_pooled_attn_prefill": (c_int32, [_P, _P, _P, _P, _P, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _P, _I64,
+                                          _I32, _I32, _I32, _I32, _I32, _I32, _I64, _F, _P]),
+    "tlf_gla_decode": (c_int32, [_P, _I64, _P, _P, _P, _P, _P, _I32, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _F, _F,
+                                 _F, _I32, _P]),
+    "tlf_gla_portions_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32, _I32]),
+    "tlf_gla_portions": (c_int32, [_P, _I64, _P, _P, _P, _P, _P, _I32, _P, _P, _P, _P, _I32, _I32, _I32, _P, _I64, _I32,
+                                   _I32, _I32, _I32, _I32, _F, _F, _F, _I32, _P, _SZ, _P]),
     "tlf_probe_read": (c_int32, [_P, _SZ, _P, _P]),
     "tlf_probe_copy": (c_int32, [_P, _P, _SZ, _P]),
     "tlf_probe_mfma": (c_int32, [_P, c_int32, c_int32, _P]),

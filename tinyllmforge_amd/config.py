@@ -18,6 +18,11 @@ import torch
 @dataclass
 class ModelConfig:
     """The architecture fields the reference reads from ``hf_config`` (models/qwen3.py:139-153)."""
+    # what the engine has to know about a design (class attributes, one set per configuration class)
+    portioned = False        # prompts may run in portions, in one batch with single decoded tokens
+    recurrent = False        # some layers carry a per-sequence state besides the KV cache
+    float32 = False          # the design's kernels exist in 32-bit
+    position_quirk = True    # the reference's decode position (len instead of len - 1) applies
     hidden_size: int
     num_hidden_layers: int
     num_attention_heads: int
@@ -51,6 +56,101 @@ class ModelConfig:
         return cls(**{k: v for k, v in dict(src).items() if k in names})
 
 
+@dataclass
+class GitopelConfig:
+    """A Gitopel model: a list of layers, each with its own mixer ('attention' or 'gla') and sizes.
+
+    Keys of ``config.json``: ``vocab``, ``width``, ``norm`` (``groups``, ``eps``) and ``layers``; a layer has ``type``,
+    ``mixer`` and ``mlp`` (``kind``, ``ff``, or null).  ``mixer`` of an attention layer: ``heads``, ``kv_heads``, ``dim``,
+    ``vdim``, ``scale``, ``rot`` (``dims``, ``base``), ``mask`` (``size``, ``pool``); of a gla layer: ``heads``, ``dim``,
+    ``vdim``, ``tau``.  The rank of a gla layer's decay projection is not in the file: it is the row count of its
+    first factor (``mixer["rank"]`` once known, 16 if no checkpoint says otherwise)."""
+    vocab: int
+    width: int
+    norm: dict
+    layers: list
+    torch_dtype: Any = torch.bfloat16
+    max_position_embeddings: int | None = None    # no limit of its own: the engine's max_model_len
+
+    portioned = True
+    recurrent = True
+    float32 = True
+    position_quirk = False
+    tie_word_embeddings = False
+
+    def __post_init__(self):
+        if isinstance(self.torch_dtype, str):
+            self.torch_dtype = getattr(torch, self.torch_dtype.replace("torch.", ""))
+        assert self.width % self.norm["groups"] == 0
+        for layer in self.layers:
+            m = layer["mixer"]
+            if layer["type"] == "attention":
+                assert m["heads"] % m["kv_heads"] == 0
+                assert m["vdim"] == m["dim"], "the values are the keys: one size"
+                assert m["rot"]["dims"] <= m["dim"] and m["mask"]["size"] >= 1 and m["mask"]["pool"] >= 1
+            else:
+                assert layer["type"] == "gla", f"unknown mixer {layer['type']!r}"
+            assert not layer.get("mlp") or layer["mlp"]["kind"] == "dense"
+
+    @property
+    def hidden_size(self) -> int:
+        return self.width
+
+    @property
+    def vocab_size(self) -> int:
+        return self.vocab
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @classmethod
+    def from_dict(cls, src: dict, directory: str | None = None) -> "GitopelConfig":
+        import copy
+        names = {f.name for f in fields(cls)}
+        cfg = cls(**{k: copy.deepcopy(v) for k, v in src.items() if k in names})
+        if directory is not None:
+            shapes = tensor_shapes(directory)
+            for i, layer in enumerate(cfg.layers):
+                if layer["type"] == "gla":
+                    layer["mixer"].setdefault("rank", shapes[f"l{i}.mix.a1"][0])
+        return cfg
+
+
+def tensor_shapes(directory: str) -> dict:
+    """name -> shape of every tensor in ``directory/*.safetensors``, from the files' headers."""
+    from glob import glob
+    out = {}
+    for file in sorted(glob(os.path.join(directory, "*.safetensors"))):
+        with open(file, "rb") as f:
+            header = json.loads(f.read(int.from_bytes(f.read(8), "little")))
+        out.update({k: tuple(v["shape"]) for k, v in header.items() if k != "__metadata__"})
+    return out
+
+
+def architecture_of(src: dict) -> str:
+    """The design a ``config.json`` names: ``architecture``, or the first of ``architectures``; Qwen3 when it names none."""
+    name = src.get("architecture") or (src.get("architectures") or ["Qwen3ForCausalLM"])[0]
+    return name.removesuffix("ForCausalLM")
+
+
+def model_config(src):
+    """Configuration object from a configuration object, a dict of its keys or a checkpoint directory."""
+    if isinstance(src, (ModelConfig, GitopelConfig)):
+        return src
+    directory = None
+    if isinstance(src, str):
+        directory = src
+        with open(os.path.join(src, "config.json")) as f:
+            src = json.load(f)
+    name = architecture_of(src)
+    if name == "Gitopel":
+        return GitopelConfig.from_dict(src, directory)
+    if name == "Qwen3":
+        return ModelConfig.from_any(src)
+    raise ValueError(f"no model of this framework has the architecture {name!r}")
+
+
 # Architectures named by the benchmark configurations (Qwen3 family shapes).
 QWEN3_SHAPES = {
     "qwen3-0.6b": dict(hidden_size=1024, num_hidden_layers=28, num_attention_heads=16, num_key_value_heads=8,
@@ -82,6 +182,8 @@ class Config:
     # 1/16 represents |x| <= 28 (448 / 16); larger K or V entries saturate.
     kv_k_scale: Any = 1.0 / 16
     kv_v_scale: Any = 1.0 / 16
+    dtype: str | None = None                # "bfloat16" or "float32" instead of the model configuration's own
+    num_state_slots: int = -1               # recurrent designs: sequences that can be live at once (-1: max_num_seqs)
     seed: int = 0                           # random-init seed when no weights are given
     decode_position_quirk: bool = True      # reference feeds positions = len(seq) in decode (model_runner.py:219)
     # Decode steps of sequences that can only end by length (ignore_eos) are launched before the token ids of
@@ -98,12 +200,27 @@ class Config:
             self.hf_config = ModelConfig.from_any(QWEN3_SHAPES[self.model.lower()])
         elif isinstance(self.model, str):
             assert os.path.isdir(self.model), f"{self.model} is neither a known shape nor a directory"
-            self.hf_config = ModelConfig.from_any(self.model)
+            self.hf_config = model_config(self.model)
         else:
-            self.hf_config = ModelConfig.from_any(self.model)
-        assert self.kvcache_block_size % 256 == 0
+            self.hf_config = model_config(self.model)
+        hf = self.hf_config
+        if self.dtype is not None:
+            hf.torch_dtype = getattr(torch, self.dtype)
+        if hf.torch_dtype != torch.bfloat16 and not (hf.float32 and hf.torch_dtype == torch.float32):
+            raise ValueError(f"no {hf.torch_dtype} kernels for this model")
+        assert self.kvcache_block_size % (64 if hf.portioned else 256) == 0
         assert self.tensor_parallel_size == 1, "this build runs one GPU, no tensor parallelism"
         assert self.quantization in (None, "w8a16")
         assert self.kv_cache_dtype in ("bf16", "fp8_e4m3")
-        self.max_model_len = min(self.max_model_len, self.hf_config.max_position_embeddings)
-        assert self.max_num_batched_tokens >= self.max_model_len
+        if hf.portioned:
+            assert self.kv_cache_dtype == "bf16", "the caches of this design are held in its own dtype"
+            assert self.quantization is None or hf.torch_dtype == torch.bfloat16
+        if not hf.position_quirk:
+            self.decode_position_quirk = False
+        if hf.max_position_embeddings is None:
+            hf.max_position_embeddings = self.max_model_len
+        if self.num_state_slots < 0:
+            self.num_state_slots = self.max_num_seqs
+        self.max_model_len = min(self.max_model_len, hf.max_position_embeddings)
+        # a design that takes its prompts whole must fit the longest one into a step
+        assert hf.portioned or self.max_num_batched_tokens >= self.max_model_len

@@ -1,0 +1,80 @@
+// Element access for kernels that exist for bf16 (uint16 bits) and fp32 tensors alike: all arithmetic is fp32,
+// only loads and stores differ.
+#pragma once
+#include "common.h"
+
+namespace tlf {
+
+template <typename T>
+struct Elem;
+
+template <>
+struct Elem<unsigned short> {
+  static __device__ __forceinline__ float ld(const unsigned short *p) { return bf16_bits_to_float(*p); }
+  static __device__ __forceinline__ void st(unsigned short *p, float v) { *p = float_to_bf16_bits(v); }
+  static __device__ __forceinline__ float rnd(float v) { return bf16_bits_to_float(float_to_bf16_bits(v)); }
+  static __device__ __forceinline__ void ld8(const unsigned short *p, float (&f)[8]) {
+    unpack8(*reinterpret_cast<const uint4 *>(p), f);
+  }
+  static __device__ __forceinline__ void st8(unsigned short *p, const float (&f)[8]) {
+    *reinterpret_cast<uint4 *>(p) = pack8(f);
+  }
+  struct Raw8 {
+    uint4 a;
+  };
+  static __device__ __forceinline__ void raw8(const unsigned short *p, Raw8 &r) {
+    r.a = *reinterpret_cast<const uint4 *>(p);
+  }
+  static __device__ __forceinline__ void zero8(Raw8 &r) { r.a = make_uint4(0, 0, 0, 0); }
+  static __device__ __forceinline__ void cvt8(const Raw8 &r, float (&f)[8]) { unpack8(r.a, f); }
+};
+
+template <>
+struct Elem<float> {
+  static __device__ __forceinline__ float ld(const float *p) { return *p; }
+  static __device__ __forceinline__ void st(float *p, float v) { *p = v; }
+  static __device__ __forceinline__ float rnd(float v) { return v; }
+  static __device__ __forceinline__ void ld8(const float *p, float (&f)[8]) {
+    const float4 a = reinterpret_cast<const float4 *>(p)[0], b = reinterpret_cast<const float4 *>(p)[1];
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
+    f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+  }
+  static __device__ __forceinline__ void st8(float *p, const float (&f)[8]) {
+    reinterpret_cast<float4 *>(p)[0] = make_float4(f[0], f[1], f[2], f[3]);
+    reinterpret_cast<float4 *>(p)[1] = make_float4(f[4], f[5], f[6], f[7]);
+  }
+  struct Raw8 {
+    float4 a, b;
+  };
+  static __device__ __forceinline__ void raw8(const float *p, Raw8 &r) {
+    r.a = reinterpret_cast<const float4 *>(p)[0];
+    r.b = reinterpret_cast<const float4 *>(p)[1];
+  }
+  static __device__ __forceinline__ void zero8(Raw8 &r) { r.a = r.b = make_float4(0.f, 0.f, 0.f, 0.f); }
+  static __device__ __forceinline__ void cvt8(const Raw8 &r, float (&f)[8]) {
+    f[0] = r.a.x; f[1] = r.a.y; f[2] = r.a.z; f[3] = r.a.w;
+    f[4] = r.b.x; f[5] = r.b.y; f[6] = r.b.z; f[7] = r.b.w;
+  }
+};
+
+__device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
+
+// Sum over aligned groups of N lanes (4, 8, 16, 32 or 64), on the vector ALU (DPP) up to a row of 16 lanes.
+template <int CTRL>
+__device__ __forceinline__ float dpp_move(float v) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xf, 0xf, false));
+}
+template <int N>
+__device__ __forceinline__ float group_sum(float v) {
+  static_assert(N == 4 || N == 8 || N == 16 || N == 32 || N == 64, "lanes per group");
+  v += dpp_move<0xB1>(v);                   // quad_perm [1, 0, 3, 2]
+  v += dpp_move<0x4E>(v);                   // quad_perm [2, 3, 0, 1]
+  if (N >= 8) v += dpp_move<0x141>(v);      // row_half_mirror
+  if (N >= 16) v += dpp_move<0x140>(v);     // row_mirror
+  if (N >= 32) v += __shfl_xor(v, 16, 64);
+  if (N >= 64) v += __shfl_xor(v, 32, 64);
+  return v;
+}
+
+}  // namespace tlf

@@ -1,0 +1,207 @@
+// Grouped RMSNorm around an fp32 residual stream (sandwich norms): a row of `width` values is split into `groups`
+// equal parts and each part is divided by its own root mean square.
+//
+//   mode embed:  x = table[id];                              h = norm(x) * w_next
+//   mode add:    x = x + norm(y + y_bias) * w_post;           h = norm(x) * w_next
+//
+// The norm after a sublayer, the residual add and the norm in front of the next sublayer share their grouping, so a
+// (row, group) pair is one independent unit: the three steps are one pass over memory.  HBM bound: y and x are read
+// once, x and h written once.  The residual is fp32; y, h and the weights are T (bf16 or fp32); arithmetic is fp32.
+#include "elem.h"
+
+namespace tlf {
+
+struct GroupNormArgs {
+  const void *y;        // [rows, width] sublayer output, row stride y_stride (add mode)
+  int64_t y_stride;
+  const void *y_bias;   // [width] or NULL
+  const void *w_post;   // [width]
+  const int64_t *ids;   // embed mode
+  const void *table;    // [vocab, width]
+  int32_t vocab;
+  float *x;             // [rows, width] fp32 residual, updated in place
+  const void *w_next;   // [width] or NULL: no h
+  void *h;              // [rows, width]
+  int64_t units;        // rows * groups
+  int32_t width, groups, cols;
+  float eps;
+};
+
+template <int TPR>
+__device__ __forceinline__ float unit_sum(float v, float *part) {
+  if (TPR <= 64) {
+#pragma unroll
+    for (int o = TPR / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
+    return v;
+  }
+  v = wave_sum(v);
+  __syncthreads();
+  if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = v;
+  __syncthreads();
+  v = 0.f;
+#pragma unroll
+  for (int w = 0; w < TPR / 64; ++w) v += part[w];
+  return v;
+}
+
+template <typename T, int VEC>
+__device__ __forceinline__ void ldv(const T *p, float (&f)[VEC]) {
+  if constexpr (VEC == 8) Elem<T>::ld8(p, f);
+  else f[0] = Elem<T>::ld(p);
+}
+template <typename T, int VEC>
+__device__ __forceinline__ void stv(T *p, const float (&f)[VEC]) {
+  if constexpr (VEC == 8) Elem<T>::st8(p, f);
+  else Elem<T>::st(p, f[0]);
+}
+
+template <typename T, int VEC, int TPR, int MAXC, bool EMBED>
+__global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
+  __shared__ float part[4];
+  const int tid = threadIdx.x, sub = tid % TPR;
+  const int64_t unit = static_cast<int64_t>(blockIdx.x) * (256 / TPR) + tid / TPR;
+  const bool active = unit < a.units;
+  const int64_t safe = active ? unit : 0;
+  const int64_t row = safe / a.groups;
+  const int grp = static_cast<int>(safe - row * a.groups);
+  const int nch = a.cols / VEC;
+  const int col0 = grp * a.cols;
+  float v[MAXC][VEC];
+  float *xr = a.x + row * a.width + col0;
+  const float inv_cols = 1.0f / static_cast<float>(a.cols);
+  if constexpr (EMBED) {
+    const int64_t id = a.ids[row];
+    const bool ok = id >= 0 && id < a.vocab;
+    const T *src = static_cast<const T *>(a.table) + (ok ? id : 0) * a.width + col0;
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int ch = sub + c * TPR;
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) v[c][i] = 0.f;
+      if (ch < nch && ok) ldv<T, VEC>(src + ch * VEC, v[c]);
+    }
+  } else {
+    const T *yr = static_cast<const T *>(a.y) + row * a.y_stride + col0;
+    const T *wp = static_cast<const T *>(a.w_post) + col0;
+    const T *yb = a.y_bias ? static_cast<const T *>(a.y_bias) + col0 : nullptr;
+    float xo[MAXC][VEC], w[MAXC][VEC];
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int at = min(sub + c * TPR, nch - 1) * VEC;
+      ldv<T, VEC>(yr + at, v[c]);
+      ldv<float, VEC>(xr + at, xo[c]);
+      ldv<T, VEC>(wp + at, w[c]);
+    }
+    if (yb) {
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        float b[VEC];
+        ldv<T, VEC>(yb + min(sub + c * TPR, nch - 1) * VEC, b);
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) v[c][i] += b[i];
+      }
+    }
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+      if (sub + c * TPR < nch)
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) ss = fmaf(v[c][i], v[c][i], ss);
+    ss = unit_sum<TPR>(ss, part);
+    const float inv = 1.0f / sqrtf(ss * inv_cols + a.eps);
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) v[c][i] = fmaf(v[c][i] * inv, w[c][i], xo[c][i]);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = sub + c * TPR;
+    if (ch < nch) {
+      if (active) stv<float, VEC>(xr + ch * VEC, v[c]);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) ss = fmaf(v[c][i], v[c][i], ss);
+    }
+  }
+  if (a.w_next == nullptr) return;  // uniform
+  ss = unit_sum<TPR>(ss, part);
+  const float inv = 1.0f / sqrtf(ss * inv_cols + a.eps);
+  const T *wn = static_cast<const T *>(a.w_next) + col0;
+  T *hr = static_cast<T *>(a.h) + row * a.width + col0;
+#pragma unroll
+  for (int c = 0; c < MAXC; ++c) {
+    const int ch = sub + c * TPR;
+    if (active && ch < nch) {
+      float w[VEC];
+      ldv<T, VEC>(wn + ch * VEC, w);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) w[i] = v[c][i] * inv * w[i];
+      stv<T, VEC>(hr + ch * VEC, w);
+    }
+  }
+}
+
+template <typename T, bool EMBED>
+int launch_groupnorm(const GroupNormArgs &a, bool vec8, hipStream_t stream) {
+#define TLF_GN(VEC, TPR, MAXC)                                                                               \
+  TLF_LAUNCH((groupnorm_kernel<T, VEC, TPR, MAXC, EMBED>),                                                   \
+             dim3(static_cast<unsigned>((a.units + (256 / TPR) - 1) / (256 / TPR))), dim3(256), 0, stream, a)
+  if (vec8) {
+    if (a.cols <= 128) TLF_GN(8, 16, 1);
+    else if (a.cols <= 512) TLF_GN(8, 64, 1);
+    else if (a.cols <= 1024) TLF_GN(8, 64, 2);
+    else if (a.cols <= 2048) TLF_GN(8, 256, 1);
+    else if (a.cols <= 4096) TLF_GN(8, 256, 2);
+    else if (a.cols <= 8192) TLF_GN(8, 256, 4);
+    else TLF_GN(8, 256, 8);
+  } else {
+    if (a.cols <= 256) TLF_GN(1, 64, 4);
+    else if (a.cols <= 2048) TLF_GN(1, 256, 8);
+    else TLF_GN(1, 256, 64);
+  }
+#undef TLF_GN
+  return launch_status();
+}
+
+template <bool EMBED>
+int groupnorm_entry(GroupNormArgs &a, int32_t rows, int32_t dtype, hipStream_t stream) {
+  if (rows < 0 || a.width <= 0 || a.groups <= 0 || a.width % a.groups) return TLF_E_SHAPE;
+  if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
+  if (rows == 0) return TLF_OK;
+  if (!a.x || (a.w_next && !a.h)) return TLF_E_NULL;
+  a.cols = a.width / a.groups;
+  if (a.cols > 16384) return TLF_E_SHAPE;
+  a.units = static_cast<int64_t>(rows) * a.groups;
+  bool vec8 = a.cols % 8 == 0 && aligned16(a.x) && aligned16(a.w_next) && aligned16(a.h);
+  if (EMBED)
+    vec8 = vec8 && aligned16(a.table);
+  else
+    vec8 = vec8 && aligned16(a.y) && aligned16(a.y_bias) && aligned16(a.w_post) && a.y_stride % 8 == 0;
+  return dtype == TLF_DT_BF16 ? launch_groupnorm<unsigned short, EMBED>(a, vec8, stream)
+                              : launch_groupnorm<float, EMBED>(a, vec8, stream);
+}
+
+}  // namespace tlf
+
+extern "C" int tlf_group_rmsnorm_add(const void *y, int64_t y_stride, const void *y_bias, const void *w_post, float *x,
+                                     const void *w_next, void *h, int32_t rows, int32_t width, int32_t groups,
+                                     float eps, int32_t dtype, void *stream) {
+  tlf::GroupNormArgs a{};
+  if (rows > 0 && (!y || !w_post)) return TLF_E_NULL;
+  if (y_stride < width) return TLF_E_SHAPE;
+  a.y = y; a.y_stride = y_stride; a.y_bias = y_bias; a.w_post = w_post; a.x = x; a.w_next = w_next; a.h = h;
+  a.width = width; a.groups = groups; a.eps = eps;
+  return tlf::groupnorm_entry<false>(a, rows, dtype, static_cast<hipStream_t>(stream));
+}
+
+extern "C" int tlf_embed_group_rmsnorm(const int64_t *ids, const void *table, int32_t vocab, float *x,
+                                       const void *w_next, void *h, int32_t rows, int32_t width, int32_t groups,
+                                       float eps, int32_t dtype, void *stream) {
+  tlf::GroupNormArgs a{};
+  if (rows > 0 && (!ids || !table)) return TLF_E_NULL;
+  if (vocab <= 0) return TLF_E_SHAPE;
+  a.ids = ids; a.table = table; a.vocab = vocab; a.x = x; a.w_next = w_next; a.h = h;
+  a.width = width; a.groups = groups; a.eps = eps;
+  return tlf::groupnorm_entry<true>(a, rows, dtype, static_cast<hipStream_t>(stream));
+}

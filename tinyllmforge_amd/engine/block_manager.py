@@ -114,6 +114,17 @@ class BlockManager:
         seq.num_cached_tokens = 0
         seq.block_table.clear()
 
+    # -- without prefix caching (designs whose recurrent state a block does not hold): a sequence owns just the blocks
+    #    its tokens need, whatever step they come in
+    def can_grow(self, seq: Sequence) -> bool:
+        return len(self.free_block_ids) >= seq.num_blocks - len(seq.block_table)
+
+    def grow(self, seq: Sequence):
+        while len(seq.block_table) < seq.num_blocks:
+            block_id = self.free_block_ids[0]
+            self._take(block_id)
+            seq.block_table.append(block_id)
+
     # -- decode side
     def can_append(self, seq: Sequence) -> bool:
         return len(self.free_block_ids) >= (len(seq) % self.block_size == 1)

@@ -74,3 +74,35 @@ def decode_inputs(seqs, block_size: int, position_quirk: bool = True) -> dict:
         context_lens=n.astype(np.int32),
         block_tables=block_tables_array(seqs),
     )
+
+
+CHUNK = 16    # tokens per chunk of the recurrent layers' prompt kernels
+
+
+def portion_inputs(seqs, block_size: int) -> dict:
+    """Inputs of a step in which sequence ``s`` brings its tokens ``num_computed .. num_computed + num_scheduled - 1``,
+    sequences with one token first (no counterpart in the reference).  Besides the usual arrays: per sequence the tokens
+    before the step and the state slot, per row its sequence, and the portions of more than one token cut into chunks of
+    at most ``CHUNK`` that do not cross a sequence (rows counted from the first portion's first row)."""
+    n = np.asarray([s.num_scheduled for s in seqs], dtype=np.int64)
+    single = int((n == 1).sum())
+    assert (n[:single] == 1).all() and (n[single:] > 1).all()
+    start = np.asarray([s.num_computed for s in seqs], dtype=np.int64)
+    ids = np.concatenate([np.asarray(s.token_ids[s.num_computed:s.num_computed + s.num_scheduled], dtype=np.int64) for s in seqs])
+    cu = np.concatenate([[0], np.cumsum(n)])
+    row_seq = np.repeat(np.arange(len(seqs)), n)
+    pos = np.arange(cu[-1]) - cu[row_seq] + start[row_seq]
+    tables = block_tables_array(seqs)
+    slots = tables[row_seq, pos // block_size].astype(np.int64) * block_size + pos % block_size
+    chunks = -(-n[single:] // CHUNK)
+    cu_chunks = np.concatenate([[0], np.cumsum(chunks)])
+    chunk_seq = np.repeat(np.arange(len(chunks)), chunks)
+    within = (np.arange(cu_chunks[-1]) - cu_chunks[chunk_seq]) * CHUNK
+    return dict(
+        input_ids=ids, positions=pos.astype(np.int64), slot_mapping=slots.astype(np.int32),
+        cu_seqlens_q=cu.astype(np.int32), block_tables=tables, seq_starts=start.astype(np.int32),
+        state_slots=np.asarray([s.state_slot for s in seqs], dtype=np.int32), row_seq=row_seq.astype(np.int32),
+        chunk_rows=(cu[single:-1][chunk_seq] - single + within).astype(np.int32),
+        chunk_lens=np.minimum(CHUNK, n[single:][chunk_seq] - within).astype(np.int32),
+        cu_chunks=cu_chunks.astype(np.int32), num_single=single, max_portion=int(n.max()),
+    )

@@ -78,6 +78,7 @@ class LLMEngine:
         ahead = self.config.run_ahead and sched.can_run_ahead() and bool(runner.graph_bs) and not runner.enforce_eager
         outputs = [] if ahead else self._drain()
         seqs, is_prefill = sched.schedule()
+        rows = sum(s.num_scheduled for s in seqs)
         if ahead and not is_prefill and runner.graph_ready(seqs):
             while len(self._ahead) >= self.AHEAD:
                 outputs += self._retire()
@@ -96,7 +97,10 @@ class LLMEngine:
             token_ids = runner.call("run", seqs, is_prefill)
             sched.postprocess(seqs, token_ids)
             outputs += [(s.seq_id, s.completion_token_ids) for s in seqs if s.is_finished]
-        num_tokens = sum(len(s) for s in seqs) if is_prefill else -len(seqs)
+        if runner.portioned:      # a step with portions counts as a prefill step, with the rows it ran
+            num_tokens = rows if is_prefill else -rows
+        else:
+            num_tokens = sum(len(s) for s in seqs) if is_prefill else -len(seqs)
         # for the statistics of generate(): cached prompt tokens of a prefill step, context tokens a
         # decode step's attention reads (the token stored in this step included)
         self._step_info = (sum(s.num_cached_tokens for s in seqs) if is_prefill else 0,

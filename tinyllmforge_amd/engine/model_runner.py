@@ -14,8 +14,8 @@ import torch
 from .. import _lib, ops
 from ..config import Config
 from ..layers.sampler import Sampler
-from ..models.qwen3 import Qwen3ForCausalLM
-from ..utils.context import get_context, reset_context, set_context
+from ..models.registry import model_class
+from ..utils.context import get_context, reset_context, set_context, set_portions_context
 from ..utils.loader import load_model, random_init_
 from . import inputs as I
 from .sequence import Sequence
@@ -31,6 +31,7 @@ class ModelRunner:
         self.block_size = config.kvcache_block_size
         Sequence.block_size = self.block_size
         self.enforce_eager = config.enforce_eager
+        self.portioned = hf.portioned          # steps are batches of single tokens and portions (run_portions)
         self.device = torch.device("cuda", torch.cuda.current_device())
         self.kv_dtype = torch.bfloat16 if config.kv_cache_dtype == "bf16" else torch.float8_e4m3fn
 
@@ -38,7 +39,7 @@ class ModelRunner:
         torch.set_default_dtype(hf.torch_dtype)
         try:
             with torch.device(self.device):
-                self.model = Qwen3ForCausalLM(hf)
+                self.model = model_class(hf)(hf)
             # the RoPE table is built on the host (same bits as a CPU restatement), then moved
             self.model.to(self.device)
             if state_dict is not None:
@@ -61,8 +62,11 @@ class ModelRunner:
         self.graph_bs = []
         self._stage = None            # pinned staging buffer of the eager steps' integer inputs (grow-only)
         with torch.inference_mode():
-            self.warmup_model()
-            self.allocate_kv_cache()
+            if self.portioned:
+                self.allocate_portioned()
+            else:
+                self.warmup_model()
+                self.allocate_kv_cache()
             if not self.enforce_eager:
                 self.capture_graphs()
 
@@ -75,6 +79,8 @@ class ModelRunner:
             for module in self.model.modules():
                 if hasattr(module, "k_cache") and hasattr(module, "v_cache"):
                     module.k_cache = module.v_cache = torch.tensor([])
+            if self.portioned:
+                self.bind_caches(0, 0)
         self.kv_cache = None
         self.model = None
         import gc
@@ -95,6 +101,52 @@ class ModelRunner:
         seqs = [Sequence([0] * cfg.max_model_len) for _ in range(num_seqs)]
         self.run(seqs, True)
         torch.cuda.empty_cache()
+
+    def bind_caches(self, pages: int, slots: int):
+        """Every layer's paged cache (``pages`` blocks) and recurrent state (``slots`` sequences); 0 frees them.  The
+        layers own their layouts: they are asked for bytes and told how many."""
+        for m in self.model.modules():
+            if hasattr(m, "bind_pages"):
+                m.bind_pages(pages, self.block_size, self.device)
+            if hasattr(m, "bind_slots"):
+                m.bind_slots(slots, self.device)
+
+    def allocate_portioned(self):
+        """Caches of a design that runs prompts in portions.  Its layers read K/V from the pages only, so the warm-up
+        (the activation peak, the kernels' workspaces) is one largest step over a pool of just its size."""
+        cfg = self.config
+        torch.cuda.empty_cache()
+        torch.cuda.reset_peak_memory_stats()
+        modules = list(self.model.modules())
+        page = sum(m.page_bytes(self.block_size) for m in modules if hasattr(m, "page_bytes"))
+        slot = sum(m.slot_bytes() for m in modules if hasattr(m, "slot_bytes"))
+        lens, left = [], cfg.max_num_batched_tokens
+        while left > 0 and len(lens) < cfg.max_num_seqs:
+            lens.append(min(left, cfg.max_model_len))
+            left -= lens[-1]
+        seqs, at = [], 0
+        for i, n in enumerate(lens):
+            seq = Sequence([0] * n)
+            seq.num_scheduled, seq.state_slot = n, i % cfg.num_state_slots
+            seq.block_table = list(range(at, at + seq.num_blocks))
+            at += seq.num_blocks
+            seqs.append(seq)
+        self.bind_caches(at, cfg.num_state_slots)
+        self.run_portions(seqs)
+        torch.cuda.synchronize()
+        stats = torch.cuda.memory_stats()
+        held = at * page + slot * cfg.num_state_slots
+        weights = stats["allocated_bytes.all.current"] - held
+        activations = stats["allocated_bytes.all.peak"] - held - weights
+        self.bind_caches(0, 0)
+        torch.cuda.empty_cache()
+        if cfg.num_kvcache_blocks <= 0:
+            free, total = torch.cuda.mem_get_info()
+            room = total * cfg.gpu_memory_utilization - (total - free) - activations - slot * cfg.num_state_slots
+            cfg.num_kvcache_blocks = int(room) // page if page else cfg.max_num_seqs * -(-cfg.max_model_len // self.block_size)
+        assert cfg.num_kvcache_blocks > 0, "no memory left for the KV pool"
+        self.kv_cache = None
+        self.bind_caches(cfg.num_kvcache_blocks, cfg.num_state_slots)
 
     def kv_block_bytes(self) -> int:
         hf = self.config.hf_config
@@ -216,6 +268,51 @@ class ModelRunner:
         set_context(False, slot_mapping=d["slot_mapping"], context_lens=d["context_lens"], block_tables=d["block_tables"])
         return d["input_ids"], d["positions"]
 
+    @torch.inference_mode()
+    def hidden_portions(self, seqs, want=None):
+        """One step of a design that runs prompts in portions: every sequence's ``num_scheduled`` tokens as one batch.
+        ``want[i]``: places among sequence i's tokens whose rows the LM head is asked for; by default the last one of
+        each sequence whose known tokens end with this step.  Returns the final hidden states and leaves the
+        wanted rows, in the caller's order, in the context."""
+        if want is None:
+            want = [[s.num_scheduled - 1] if s.num_computed + s.num_scheduled == len(s) else [] for s in seqs]
+        order = sorted(range(len(seqs)), key=lambda i: seqs[i].num_scheduled > 1)     # single tokens first (stable)
+        batch = [seqs[i] for i in order]
+        first = np.zeros(len(seqs), dtype=np.int64)
+        first[order] = np.concatenate([[0], np.cumsum([s.num_scheduled for s in batch])])[:-1]
+        rows = np.asarray([first[i] + p for i, w in enumerate(want) for p in w], dtype=np.int64)
+        if all(s.num_scheduled == 1 for s in seqs) and self.graph_ready(seqs) and self.graphs:
+            hidden = self.run_decode_graph(batch)
+            get_context().logit_rows = None if len(rows) == len(seqs) and (rows == np.arange(len(rows))).all() \
+                else torch.from_numpy(rows).to(self.device)
+            return hidden
+        arrays = I.portion_inputs(batch, self.block_size)
+        arrays["logit_rows"] = rows
+        done = [s for s, w in zip(seqs, want) if w]
+        arrays["temperatures"] = self._temperatures_of(done) if done else None
+        d = self._upload(arrays)
+        self._temperatures = d.pop("temperatures")
+        ids, positions = d.pop("input_ids"), d.pop("positions")
+        set_portions_context(max_len=self.config.max_model_len, **d)
+        return self.model(ids, positions)
+
+    @torch.inference_mode()
+    def run_portions(self, seqs):
+        """Token ids of a step, None for a sequence whose known tokens go on after it."""
+        ends = [s.num_computed + s.num_scheduled == len(s) for s in seqs]
+        hidden = self.hidden_portions(seqs)
+        out = iter(self.sample(hidden, self._temperatures) if any(ends) else ())
+        reset_context()
+        return [next(out) if e else None for e in ends]
+
+    @torch.inference_mode()
+    def logits_portions(self, seqs, want):
+        """Logits of a step at the wanted places (in the order of ``seqs`` and of ``want``), None if there are none."""
+        hidden = self.hidden_portions(seqs, want)
+        logits = self.model.compute_logits(hidden) if any(len(w) for w in want) else None
+        reset_context()
+        return logits
+
     def prepare_sample(self, seqs):
         """Temperatures of the step on the device (model_runner.py:230-236), None when all are 0: what the
         step's ``prepare_prefill`` / ``prepare_decode`` / graph upload already carried over."""
@@ -289,6 +386,7 @@ class ModelRunner:
         h["positions"][:bs] = d["positions"]
         h["slot_mapping"][:bs] = d["slot_mapping"]
         h["context_lens"][:bs] = d["context_lens"]
+        h["state_slots"][:bs] = [s.state_slot for s in seqs]
         w = d["block_tables"].shape[1]
         h["block_tables"][:bs, :w] = d["block_tables"]
         if feed is not None:
@@ -298,6 +396,7 @@ class ModelRunner:
             h["positions"][bs:gbs] = 0
             h["slot_mapping"][bs:gbs] = -1
             h["context_lens"][bs:gbs] = 0
+            h["state_slots"][bs:gbs] = -1
         t = self._temperatures_of(seqs)
         self._temperatures = None
         if t is not None:
@@ -342,6 +441,8 @@ class ModelRunner:
         return self.sampler(self.model.compute_logits(hidden), temperatures, self._all_greedy).tolist()
 
     def run(self, seqs, is_prefill):
+        if self.portioned:
+            return self.run_portions(seqs)
         use_graph = not is_prefill and self.graph_ready(seqs)
         if use_graph:
             hidden = self.run_decode_graph(seqs)
@@ -372,7 +473,7 @@ class ModelRunner:
         for name, dt, shape in (("input_ids", torch.int64, (max_bs,)), ("positions", torch.int64, (max_bs,)),
                                 ("feed_index", torch.int64, (max_bs,)),
                                 ("slot_mapping", torch.int32, (max_bs,)), ("context_lens", torch.int32, (max_bs,)),
-                                ("temperatures", torch.float32, (max_bs,)),
+                                ("state_slots", torch.int32, (max_bs,)), ("temperatures", torch.float32, (max_bs,)),
                                 ("block_tables", torch.int32, (max_bs, max_blocks))):
             nbytes = int(np.prod(shape)) * torch.empty(0, dtype=dt).element_size()
             layout[name] = (off, nbytes, dt, shape)
@@ -388,6 +489,7 @@ class ModelRunner:
             host_np = pack.numpy()
             views = {name: host_np[o:o + nbytes].view(np_dt[dt]).reshape(shape) for name, (o, nbytes, dt, shape) in layout.items()}
             views["slot_mapping"][:] = -1
+            views["state_slots"][:] = -1
             self.graph_ring.append(dict(pack=pack, views=views, copied=None,
                                         tokens=torch.zeros(max_bs, dtype=torch.int64, pin_memory=True)))
         self.graph_ring_at = 0
@@ -403,8 +505,12 @@ class ModelRunner:
         self.graph_kernels = {}      # batch bucket -> kernels in its graph
         for bs in reversed(self.graph_bs):
             graph = torch.cuda.CUDAGraph()
-            set_context(False, slot_mapping=gv["slot_mapping"][:bs], context_lens=gv["context_lens"][:bs],
-                        block_tables=gv["block_tables"][:bs, :])
+            if self.portioned:
+                set_portions_context(slot_mapping=gv["slot_mapping"][:bs], block_tables=gv["block_tables"][:bs, :],
+                                     state_slots=gv["state_slots"][:bs], num_single=bs, max_len=cfg.max_model_len)
+            else:
+                set_context(False, slot_mapping=gv["slot_mapping"][:bs], context_lens=gv["context_lens"][:bs],
+                            block_tables=gv["block_tables"][:bs, :])
             self.plan_decode()
             gv["outputs"][:bs] = self.model(gv["input_ids"][:bs], gv["positions"][:bs])    # warm-up
             launched = lib.tlf_kernel_launches()

@@ -33,6 +33,11 @@ class Sequence:
         # tokens at the tail whose values are not on the host yet (a decode step that runs ahead of the
         # read-back of the step before it appends a stand-in and patches the value in later)
         self.num_unknown = 0
+        # designs that run prompts in portions: tokens the caches and the recurrent state hold, tokens of the
+        # step being run, and the slot of that state
+        self.num_computed = 0
+        self.num_scheduled = 0
+        self.state_slot = -1
         self.block_table: list[int] = []
         self.temperature = sp.temperature
         self.max_tokens = sp.max_tokens

@@ -4,6 +4,7 @@ from torch import nn
 
 from .. import ops
 from ..utils.context import get_context
+from .linear import StackedLinear
 
 
 class VocabParallelEmbedding(nn.Module):
@@ -28,18 +29,37 @@ class ParallelLMHead(VocabParallelEmbedding):
         super().__init__(num_embeddings, embedding_dim)
         assert not bias
 
-    def forward(self, x: torch.Tensor):
+    @staticmethod
+    def _wanted_rows(x: torch.Tensor):
         ctx = get_context()
+        if ctx.logit_rows is not None:                       # the step says which rows
+            return x[ctx.logit_rows].contiguous()
         if ctx.is_prefill:                                   # only the last token of each sequence
             last = (ctx.cu_seqlens_q[1:] - 1).long()
             x = x[last].contiguous()
-        return ops.bf16_linear(x, self.weight.data)
+        return x
+
+    def forward(self, x: torch.Tensor):
+        return ops.bf16_linear(self._wanted_rows(x), self.weight.data)
 
     def forward_greedy(self, x: torch.Tensor):
         """``argmax(self(x), -1)``: the greedy branch of the sampler (sampler.py:13-14,21) applied to this
         layer's logits, in one call that never stores them."""
-        ctx = get_context()
-        if ctx.is_prefill:
-            last = (ctx.cu_seqlens_q[1:] - 1).long()
-            x = x[last].contiguous()
-        return ops.bf16_linear_argmax(x, self.weight.data)
+        return ops.bf16_linear_argmax(self._wanted_rows(x), self.weight.data)
+
+
+class PaddedLMHead(StackedLinear):
+    """LM head of any vocabulary and width, bf16 or 32-bit."""
+
+    def __init__(self, num_embeddings: int, embedding_dim: int):
+        super().__init__(embedding_dim, {"head": num_embeddings})
+        self.num_embeddings = num_embeddings
+
+    def forward(self, x: torch.Tensor):
+        return super().forward(ParallelLMHead._wanted_rows(x))[:, :self.num_embeddings]
+
+    def forward_greedy(self, x: torch.Tensor):
+        x = ParallelLMHead._wanted_rows(x)
+        if self.weight.dtype == torch.bfloat16 and self.weight.shape == (self.num_embeddings, x.shape[-1]):
+            return ops.bf16_linear_argmax(x, self.weight.data)
+        return ops.argmax(super().forward(x)[:, :self.num_embeddings].contiguous())

@@ -95,7 +95,7 @@ class LinearBase(nn.Module):
         if self.is_quantized:
             y = ops.w8a16_linear(x, self.pack_().qpacked, self.qscale)
         else:
-            y = ops.bf16_linear(x, self.weight.data)
+            y = ops.linear(x, self.weight.data)
         if self.bias is not None:
             y = y + self.bias
         return y
@@ -191,6 +191,78 @@ class MergedColumnParallelLinear(ColumnParallelLinear):
         size = self.output_sizes[loaded_shard_id] // self.tp_size
         dst = param.data.narrow(self.tp_dim, offset, size)
         dst.copy_(loaded_weight.chunk(self.tp_size, self.tp_dim)[self.tp_rank])
+
+
+def _round_up(n: int, m: int) -> int:
+    return -(-n // m) * m
+
+
+def pad_2d(t: torch.Tensor, rows: int, cols: int) -> torch.Tensor:
+    return torch.nn.functional.pad(t, (0, cols - t.shape[1], 0, rows - t.shape[0]))
+
+
+def pad_columns(x: torch.Tensor, cols: int) -> torch.Tensor:
+    """``x`` as it is, or with zero columns up to ``cols`` (sizes that are no multiple of the GEMM kernels' K step)."""
+    return x if x.shape[-1] == cols else torch.nn.functional.pad(x, (0, cols - x.shape[-1]))
+
+
+class StackedLinear(LinearBase):
+    """Projections of one input stacked along the output dim in the order of ``parts`` (name -> rows), of any size: the
+    weight is held with its rows padded to 16 and its columns to 64, pads are zero.  ``forward`` returns the padded
+    row; ``offset(name)`` says where a part begins in it."""
+
+    def __init__(self, input_size: int, parts: dict[str, int]):
+        super().__init__(input_size, sum(parts.values()), 0)
+        self.parts = dict(parts)
+        self._make_params(_round_up(self.output_size, 16), _round_up(input_size, 64), bias=False)
+        self.weight.data.zero_()
+
+    def offset(self, name: str) -> int:
+        at = 0
+        for part, rows in self.parts.items():
+            if part == name:
+                return at
+            at += rows
+        raise KeyError(name)
+
+    def weight_loader(self, param: nn.Parameter, loaded_weight: torch.Tensor, loaded_shard_id: str | None = None):
+        name = loaded_shard_id if loaded_shard_id is not None else next(iter(self.parts))
+        assert tuple(loaded_weight.shape) == (self.parts[name], self.input_size), (name, tuple(loaded_weight.shape))
+        at = self.offset(name)
+        param.data[at:at + self.parts[name], :self.input_size].copy_(loaded_weight)
+
+    def zero_pads_(self):
+        """After a random fill: the pads are zeros again."""
+        if self.weight.numel():
+            self.weight.data[self.output_size:].zero_()
+            self.weight.data[:, self.input_size:].zero_()
+
+    def forward(self, x: torch.Tensor) -> torch.Tensor:
+        return super().forward(pad_columns(x, _round_up(self.input_size, 64)))
+
+
+class GatedUpLinear(MergedColumnParallelLinear):
+    """gate and up projections of any size: the intermediate dim is padded to a multiple of 64 and the input to one of
+    64, with zeros (a padded channel is silu(0) * 0), so the result is the input of a ``StackedLinear`` as it is."""
+
+    def __init__(self, input_size: int, inter_size: int):
+        self.inter_size, self.true_input_size = inter_size, input_size
+        super().__init__(_round_up(input_size, 64), [_round_up(inter_size, 64)] * 2)
+        self.weight.data.zero_()
+
+    def weight_loader(self, param: nn.Parameter, loaded_weight: torch.Tensor, loaded_shard_id: int):
+        assert tuple(loaded_weight.shape) == (self.inter_size, self.true_input_size), tuple(loaded_weight.shape)
+        super().weight_loader(param, pad_2d(loaded_weight, self.output_sizes[0], self.input_size), loaded_shard_id)
+
+    def zero_pads_(self):
+        if self.weight.numel():
+            for first in (0, self.output_sizes[0]):
+                self.weight.data[first + self.inter_size:first + self.output_sizes[0]].zero_()
+            self.weight.data[:, self.true_input_size:].zero_()
+
+    def forward_silu_mul(self, x: torch.Tensor) -> torch.Tensor:
+        """``[N, padded inter_size]``."""
+        return super().forward_silu_mul(pad_columns(x, self.input_size))
 
 
 class QKVParallelLinear(ColumnParallelLinear):

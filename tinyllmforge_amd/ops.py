@@ -10,7 +10,7 @@ from __future__ import annotations
 import torch
 
 from . import _lib
-from ._lib import KV_BF16, KV_FP8_E4M3, check
+from ._lib import DT_BF16, DT_F32, KV_BF16, KV_FP8_E4M3, check
 
 BF16 = torch.bfloat16
 
@@ -155,6 +155,14 @@ def qknorm_rope_store(qkv, q_weight, k_weight, eps, positions, cos_sin, num_q_he
 # ------------------------------------------------------------------ a8
 def silu_and_mul(x):
     lib = _lib.load()
+    if x.dtype == torch.float32:
+        _need(x, torch.float32, "x")
+        assert x.is_contiguous() and x.shape[-1] % 2 == 0
+        inter = x.shape[-1] // 2
+        y = torch.empty(*x.shape[:-1], inter, dtype=x.dtype, device=x.device)
+        check(lib.tlf_f32_silu_and_mul(x.data_ptr(), y.data_ptr(), x.numel() // (2 * inter), inter, _stream()),
+              "tlf_f32_silu_and_mul")
+        return y
     _need(x, BF16, "x")
     assert x.is_contiguous() and x.shape[-1] % 2 == 0
     inter = x.shape[-1] // 2
@@ -167,6 +175,12 @@ def silu_and_mul(x):
 # ------------------------------------------------------------------ a9
 def argmax(logits):
     lib = _lib.load()
+    if logits.dtype == torch.float32:
+        _need(logits, torch.float32, "logits")
+        assert logits.dim() == 2 and logits.stride(1) == 1
+        out = torch.empty(logits.shape[0], dtype=torch.int64, device=logits.device)
+        check(lib.tlf_f32_argmax(logits.data_ptr(), logits.stride(0), out.data_ptr(), *logits.shape, _stream()), "tlf_f32_argmax")
+        return out
     _need(logits, BF16, "logits")
     assert logits.dim() == 2 and logits.stride(1) == 1
     rows, vocab = logits.shape
@@ -183,6 +197,8 @@ def sample(logits, temperatures, seed: int, offset: int):
     ``softmax(logits / T)`` by the exponential-race formula of the reference, noise from Philox4x32-10
     at (``seed``, ``offset``).  int64 ``[rows]``."""
     lib = _lib.load()
+    if logits.dtype == torch.float32 and logits.is_cuda:
+        logits = logits.to(BF16)        # the draw's noise is far coarser than the rounding
     _need(logits, BF16, "logits"); _need(temperatures, torch.float32, "temperatures")
     assert logits.dim() == 2 and logits.stride(1) == 1 and temperatures.is_contiguous()
     rows, vocab = logits.shape
@@ -308,6 +324,24 @@ def bf16_linear_silu_mul(x, w_interleaved):
     check(lib.tlf_bf16_gemm_silu_mul(x2.data_ptr(), x2.stride(0), w_interleaved.data_ptr(), y.data_ptr(), M, N, K,
                                      _stream()), "tlf_bf16_gemm_silu_mul")
     return y.view(*x.shape[:-1], N // 2)
+
+
+def linear(x, w):
+    """``x . w^T`` in the weight's dtype (bf16 or 32-bit)."""
+    return f32_linear(x, w) if w.dtype == torch.float32 else bf16_linear(x, w)
+
+
+def f32_linear(x, w):
+    lib = _lib.load()
+    _need(x, torch.float32, "x"); _need(w, torch.float32, "w")
+    assert x.stride(-1) == 1 and w.is_contiguous()
+    x2 = x.reshape(-1, x.shape[-1])
+    M, K = x2.shape
+    N = w.shape[0]
+    assert w.shape[1] == K
+    y = torch.empty(M, N, dtype=torch.float32, device=x.device)
+    check(lib.tlf_f32_gemm(x2.data_ptr(), x2.stride(0), w.data_ptr(), y.data_ptr(), M, N, K, _stream()), "tlf_f32_gemm")
+    return y.view(*x.shape[:-1], N)
 
 
 def bf16_linear(x, w):
@@ -493,4 +527,164 @@ def varlen_prefill_attention(q, k, v, cu_seqlens_q, cu_seqlens_k, max_seqlen_q, 
         v_scale.data_ptr() if v_scale is not None else None,
         cu_seqlens_q.data_ptr(), cu_seqlens_k.data_ptr(), btp, bts, out.data_ptr(), nseq,
         int(max_seqlen_q), Hq, Hkv, Dh, bs, nblk, float(scale), _stream()), "tlf_varlen_prefill_attn")
+    return out
+
+
+# ------------------------------------------------------------------ hybrid decoders
+def _dt(t: torch.Tensor) -> int:
+    if t.dtype == BF16:
+        return DT_BF16
+    if t.dtype == torch.float32:
+        return DT_F32
+    raise _lib.TlfError(f"unsupported dtype {t.dtype}")
+
+
+def _opt(t):
+    return t.data_ptr() if t is not None else None
+
+
+def group_rms_norm_add(y, y_bias, w_post, x, w_next, groups, eps):
+    """In place ``x += norm(y + y_bias) * w_post`` (``x`` fp32 ``[N, W]``), then ``norm(x) * w_next`` in y's dtype."""
+    lib = _lib.load()
+    _need(y, w_post.dtype, "y"); _need(x, torch.float32, "x"); _need(w_next, y.dtype, "w_next")
+    rows, width = x.shape
+    assert y.shape[0] == rows and y.shape[1] >= width and y.stride(1) == 1 and x.is_contiguous()
+    assert w_post.numel() == width and w_next.numel() == width and (y_bias is None or y_bias.numel() == width)
+    h = torch.empty(rows, width, dtype=y.dtype, device=x.device)
+    check(lib.tlf_group_rmsnorm_add(y.data_ptr(), y.stride(0), _opt(y_bias), w_post.data_ptr(), x.data_ptr(),
+                                    w_next.data_ptr(), h.data_ptr(), rows, width, groups, float(eps), _dt(y), _stream()),
+          "tlf_group_rmsnorm_add")
+    return h
+
+
+def embed_group_rms_norm(ids, table, w_next, groups, eps):
+    """``x = table[ids]`` in fp32 and ``norm(x) * w_next`` in the table's dtype."""
+    lib = _lib.load()
+    _need(ids, torch.int64, "ids"); _need(table, w_next.dtype, "table")
+    assert ids.is_contiguous() and table.is_contiguous()
+    rows, (vocab, width) = ids.numel(), table.shape
+    x = torch.empty(rows, width, dtype=torch.float32, device=table.device)
+    h = torch.empty(rows, width, dtype=table.dtype, device=table.device)
+    check(lib.tlf_embed_group_rmsnorm(ids.data_ptr(), table.data_ptr(), vocab, x.data_ptr(), w_next.data_ptr(),
+                                      h.data_ptr(), rows, width, groups, float(eps), _dt(table), _stream()),
+          "tlf_embed_group_rmsnorm")
+    return x, h
+
+
+def attn_prep(proj, q_bias, k_bias, positions, cos_sin, rot_dims, slot_mapping, k_cache, v_cache, num_q_heads, head_dim, eps):
+    """Biases, V store, interleaved RoPE, unit RMS, K store.  Returns ``(q [N, Hq, Dp], gate fp32 [N, Hq])``."""
+    lib = _lib.load()
+    _need(proj, k_cache.dtype, "proj"); _need(positions, torch.int64, "positions"); _need(slot_mapping, torch.int32, "slot_mapping")
+    n = proj.shape[0]
+    pages, bs, hkv, dp = k_cache.shape
+    assert proj.stride(1) == 1 and positions.numel() == n and slot_mapping.numel() == n
+    assert k_cache.is_contiguous() and v_cache.is_contiguous() and (rot_dims == 0 or cos_sin.shape[1] == rot_dims)
+    q = torch.empty(n, num_q_heads, dp, dtype=proj.dtype, device=proj.device)
+    gate = torch.empty(n, num_q_heads, dtype=torch.float32, device=proj.device)
+    check(lib.tlf_attn_prep(proj.data_ptr(), proj.stride(0), _opt(q_bias), _opt(k_bias), positions.data_ptr(),
+                            _opt(cos_sin), cos_sin.shape[0] if cos_sin is not None else 0, rot_dims,
+                            slot_mapping.data_ptr(), pages * bs, q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
+                            gate.data_ptr(), n, num_q_heads, hkv, head_dim, dp, float(eps), _dt(proj), _stream()),
+          "tlf_attn_prep")
+    return q, gate
+
+
+HAVE_POOLED_PREFILL = False
+
+
+class PooledKV:
+    """The paged caches of one windowed layer with pooled blocks, and the layer's constants."""
+    __slots__ = ("k", "v", "pk", "pv", "head_dim", "pool", "window")
+
+    def __init__(self, pages, block_size, kv_heads, head_dim, pool, window, dtype, device):
+        dp = (head_dim + 31) // 32 * 32
+        rows = -(-block_size // pool)
+        self.k, self.v = torch.zeros(2, pages, block_size, kv_heads, dp, dtype=dtype, device=device)
+        self.pk, self.pv = torch.zeros(2, pages, rows, kv_heads, dp, dtype=dtype, device=device)
+        self.head_dim, self.pool, self.window = head_dim, pool, window
+
+    @staticmethod
+    def page_bytes(block_size, kv_heads, head_dim, pool, itemsize):
+        return 2 * (block_size + -(-block_size // pool)) * kv_heads * ((head_dim + 31) // 32 * 32) * itemsize
+
+
+def pool_blocks(kv: PooledKV, block_tables, cu_seqlens_q, seq_starts, first_seq, num_seqs, max_tokens):
+    lib = _lib.load()
+    pages, bs, hkv, _ = kv.k.shape
+    assert block_tables.shape[0] >= first_seq + num_seqs and block_tables.stride(1) == 1
+    check(lib.tlf_pool_blocks(kv.k.data_ptr(), kv.v.data_ptr(), kv.pk.data_ptr(), kv.pv.data_ptr(), block_tables.data_ptr(),
+                              block_tables.stride(0), cu_seqlens_q.data_ptr(), seq_starts.data_ptr(), first_seq, num_seqs,
+                              max_tokens, hkv, kv.head_dim, bs, kv.pool, kv.window, pages, _dt(kv.k), _stream()),
+          "tlf_pool_blocks")
+
+
+def pooled_attention_rows(q, score_bias, gate, kv: PooledKV, block_tables, positions, slot_mapping, scale, max_len,
+                          out, row_seq=None, pool_new=False):
+    """Rows of ``out`` ``[N, Hq * D]`` from ``q [N, Hq, Dp]``; see ``tlf_pooled_attn_rows``."""
+    lib = _lib.load()
+    _need(q, kv.k.dtype, "q"); _need(score_bias, q.dtype, "score_bias"); _need(gate, torch.float32, "gate")
+    _need(block_tables, torch.int32, "block_tables"); _need(positions, torch.int64, "positions")
+    n, hq, dp = q.shape
+    pages, bs, hkv, _ = kv.k.shape
+    assert q.is_contiguous() and gate.is_contiguous() and gate.numel() == n * hq and out.stride(1) == 1
+    assert out.shape[0] == n and positions.numel() == n and slot_mapping.numel() == n and dp == kv.k.shape[3]
+    assert row_seq is not None or block_tables.shape[0] >= n
+    nbytes = lib.tlf_pooled_attn_rows_workspace_bytes(n, hq, hkv, kv.head_dim, kv.pool, kv.window, max_len)
+    ws = _workspace(nbytes, q.device, "pooled_rows")
+    check(lib.tlf_pooled_attn_rows(
+        q.data_ptr(), score_bias.data_ptr(), gate.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), kv.pk.data_ptr(),
+        kv.pv.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), positions.data_ptr(), slot_mapping.data_ptr(),
+        _opt(row_seq), out.data_ptr(), out.stride(0), n, hq, hkv, kv.head_dim, bs, kv.pool, kv.window, max_len, pages,
+        float(scale), int(pool_new), _dt(q), ws.data_ptr(), ws.numel(), _stream()), "tlf_pooled_attn_rows")
+    return out
+
+
+def pooled_attention_prefill(q, score_bias, gate, kv: PooledKV, block_tables, cu_seqlens_q, seq_starts, first_seq,
+                             num_seqs, max_tokens, scale, out):
+    """Portions of sequences ``first_seq ..`` on the matrix cores (bf16); rows indexed as in the step."""
+    lib = _lib.load()
+    _need(q, BF16, "q"); _need(score_bias, BF16, "score_bias"); _need(gate, torch.float32, "gate")
+    n, hq, dp = q.shape
+    pages, bs, hkv, _ = kv.k.shape
+    assert q.is_contiguous() and gate.is_contiguous() and out.stride(1) == 1 and out.shape[0] == n
+    check(lib.tlf_pooled_attn_prefill(
+        q.data_ptr(), score_bias.data_ptr(), gate.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), kv.pk.data_ptr(),
+        kv.pv.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), cu_seqlens_q.data_ptr(), seq_starts.data_ptr(),
+        first_seq, num_seqs, max_tokens, out.data_ptr(), out.stride(0), hq, hkv, kv.head_dim, bs, kv.pool, kv.window,
+        pages, float(scale), _stream()), "tlf_pooled_attn_prefill")
+    return out
+
+
+def gla_decode(proj, a2, a2_bias, norm_weight, state, state_slots, positions, tau, eps, out):
+    """One token per row of ``proj``; ``state`` fp32 ``[slots, H, dk, dv]`` updated in place."""
+    lib = _lib.load()
+    _need(proj, a2.dtype, "proj"); _need(state, torch.float32, "state"); _need(state_slots, torch.int32, "state_slots")
+    slots, heads, dk, dv = state.shape
+    rows = proj.shape[0]
+    assert proj.stride(1) == 1 and out.stride(1) == 1 and out.shape[0] == rows and state.is_contiguous()
+    assert a2.is_contiguous() and a2.shape[0] == heads * dk and state_slots.numel() >= rows and positions.numel() == rows
+    check(lib.tlf_gla_decode(proj.data_ptr(), proj.stride(0), a2.data_ptr(), a2_bias.data_ptr(), norm_weight.data_ptr(),
+                             state.data_ptr(), state_slots.data_ptr(), slots, positions.data_ptr(), out.data_ptr(),
+                             out.stride(0), rows, heads, dk, dv, a2.shape[1], float(tau), dk ** -0.5, float(eps),
+                             _dt(proj), _stream()), "tlf_gla_decode")
+    return out
+
+
+def gla_portions(proj, a2, a2_bias, norm_weight, state, state_slots, seq_starts, chunk_rows, chunk_lens, cu_chunks,
+                 first_seq, num_seqs, tau, eps, out):
+    """Portions of sequences ``first_seq ..``; ``proj`` / ``out`` begin at the first portion's row."""
+    lib = _lib.load()
+    _need(proj, a2.dtype, "proj"); _need(state, torch.float32, "state"); _need(state_slots, torch.int32, "state_slots")
+    slots, heads, dk, dv = state.shape
+    rows, chunks = proj.shape[0], chunk_rows.numel()
+    assert proj.stride(1) == 1 and out.stride(1) == 1 and out.shape[0] == rows and state.is_contiguous()
+    assert a2.is_contiguous() and a2.shape[0] == heads * dk and cu_chunks.numel() == num_seqs + 1
+    assert state_slots.numel() >= first_seq + num_seqs and chunk_lens.numel() == chunks
+    ws = _workspace(lib.tlf_gla_portions_workspace_bytes(rows, chunks, heads, dk, dv), proj.device, "gla")
+    check(lib.tlf_gla_portions(
+        proj.data_ptr(), proj.stride(0), a2.data_ptr(), a2_bias.data_ptr(), norm_weight.data_ptr(), state.data_ptr(),
+        state_slots.data_ptr(), slots, seq_starts.data_ptr(), chunk_rows.data_ptr(), chunk_lens.data_ptr(),
+        cu_chunks.data_ptr(), chunks, first_seq, num_seqs, out.data_ptr(), out.stride(0), rows, heads, dk, dv,
+        a2.shape[1], float(tau), dk ** -0.5, float(eps), _dt(proj), ws.data_ptr(), ws.numel(), _stream()),
+        "tlf_gla_portions")
     return out

@@ -27,6 +27,17 @@ def load_model(model: nn.Module, path: str):
 
 
 def load_tensor(model: nn.Module, packed: dict, name: str, tensor: torch.Tensor):
+    route = getattr(model, "route_tensor", None)
+    if route is not None:                      # a design with tensor names of its own
+        target, shard_id = route(name)
+        param = model.get_parameter(target)
+        if shard_id is not None:
+            param.weight_loader(param, tensor, shard_id)
+        else:
+            assert param.shape == tensor.shape, (name, tuple(tensor.shape), tuple(param.shape))
+            param.data.copy_(tensor)
+        model.loaded_tensors.add(name)
+        return
     kind = name.rsplit(".", 1)[-1]
     if kind in ("qweight", "qscale"):          # a checkpoint written by quantize_checkpoint
         module_name, shard_id = name.rsplit(".", 1)[0], None
@@ -51,6 +62,10 @@ def load_tensor(model: nn.Module, packed: dict, name: str, tensor: torch.Tensor)
 
 
 def finish_load(model: nn.Module):
+    if hasattr(model, "expected_tensors"):
+        missing = model.expected_tensors() - model.loaded_tensors
+        if missing:
+            raise ValueError(f"checkpoint lacks {sorted(missing)[:8]}")
     for m in model.modules():
         if getattr(m, "pending_quantized", False):
             m.finish_quantized_load()
@@ -111,7 +126,7 @@ def random_init_(model: nn.Module, seed: int = 0, std: float = 0.02, device_fill
     for name, p in model.named_parameters():
         if tied and name == "lm_head.weight":
             continue                                   # shares the embedding's storage
-        if name.endswith("norm.weight") or name.endswith("layernorm.weight"):
+        if name.endswith("norm.weight") or name.rsplit(".", 2)[-2].startswith("norm"):
             p.data.fill_(1.0)
             continue
         if device_fill:
