@@ -34,6 +34,7 @@ FLAGS = [
 EXTRA_FLAGS = {
     "prefill_attn.hip": ["-fno-honor-nans"],
     "decode_attn.hip": ["-fno-honor-nans"],
+    "pooled_prefill.hip": ["-fno-honor-nans"],
 }
 
 

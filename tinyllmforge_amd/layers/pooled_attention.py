@@ -51,7 +51,7 @@ class PooledWindowAttention(nn.Module):
         if single < n:
             portions = ctx.cu_seqlens_q.numel() - 1 - single
             ops.pool_blocks(kv, ctx.block_tables, ctx.cu_seqlens_q, ctx.seq_starts, single, portions, ctx.max_portion)
-            if proj.dtype == torch.bfloat16 and ops.HAVE_POOLED_PREFILL:
+            if proj.dtype == torch.bfloat16:
                 ops.pooled_attention_prefill(q, bias, gate, kv, ctx.block_tables, ctx.cu_seqlens_q, ctx.seq_starts,
                                              single, portions, ctx.max_portion, self.scale, out)
             else:

@@ -589,9 +589,6 @@ def attn_prep(proj, q_bias, k_bias, positions, cos_sin, rot_dims, slot_mapping, 
     return q, gate
 
 
-HAVE_POOLED_PREFILL = False
-
-
 class PooledKV:
     """The paged caches of one windowed layer with pooled blocks, and the layer's constants."""
     __slots__ = ("k", "v", "pk", "pv", "head_dim", "pool", "window")
