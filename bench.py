@@ -53,7 +53,7 @@ def parse():
                     help="engine steps that steps/ms_per_step describe (0 = all); value is always the whole job")
     ap.add_argument("--warmup", type=int, default=1, help="warm-up generate() calls before the timed run")
     ap.add_argument("--workload", default="e2e",
-                    choices=["e2e", "decode_attn", "gemm", "prefill_attn", "elementwise", "clock", "c5", "all"])
+                    choices=["e2e", "decode_attn", "gemm", "prefill_attn", "elementwise", "clock", "c5", "gitopel", "all"])
     ap.add_argument("--attn-steps", type=int, default=200, help="timed launches of the decode-attention microbench")
     ap.add_argument("--num-seqs", type=int, default=256)
     ap.add_argument("--no-cpu-baseline", action="store_true")
@@ -612,6 +612,182 @@ def bench_c5(args):
     return res
 
 
+# ----------------------------------------------------------------------------- Gitopel beside Qwen3 at equal size
+MFMA_F32_PEAK_TFLOPS = 157.3
+# width, query heads, KV heads, head dim, intermediate size; gla heads, key dim, value dim
+GITOPEL_SIZES = {"1024-wide": (1024, 16, 8, 128, 3072, 8, 64, 128), "4096-wide": (4096, 32, 8, 128, 12288, 16, 128, 256)}
+
+
+def gitopel_shape(size, layers=8, vocab=32768, window=1024, pool=16):
+    w, hq, hkv, d, ff, gh, gk, gv = GITOPEL_SIZES[size]
+    attention = dict(type="attention", mlp=dict(kind="dense", ff=ff),
+                     mixer=dict(heads=hq, kv_heads=hkv, dim=d, vdim=d, scale=d ** -0.5, rot=dict(base=10000.0, dims=d),
+                                mask=dict(size=window, pool=pool)))
+    gla = dict(type="gla", mlp=dict(kind="dense", ff=ff), mixer=dict(heads=gh, dim=gk, vdim=gv, tau=16.0))
+    return dict(architecture="Gitopel", vocab=vocab, width=w, norm=dict(groups=4, eps=1e-6),
+                layers=[attention, gla] * (layers // 2))
+
+
+def qwen3_shape(size, layers=8, vocab=32768):
+    w, hq, hkv, d, ff, *_ = GITOPEL_SIZES[size]
+    return dict(hidden_size=w, num_hidden_layers=layers, num_attention_heads=hq, num_key_value_heads=hkv, head_dim=d,
+                intermediate_size=ff, vocab_size=vocab)
+
+
+def bench_gitopel_kernels():
+    """Kernels of the Gitopel layers beside the like kernel of Qwen3 at the same sizes: algorithmic bytes or flops over
+    the graph-timed launch, as a fraction of the HBM or matrix peak."""
+    import torch
+    from tinyllmforge_amd import ops as P
+    from tinyllmforge_amd.layers.rotary_embedding import build_cos_sin_cache
+    from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
+    torch.manual_seed(0)
+    BF, F32, dev = torch.bfloat16, torch.float32, "cuda"
+    rows = []
+
+    def add(name, size, fn, amount, bound, copies=1, launches=10):
+        """``fn(i)`` runs on copy ``i`` of its data; ``amount``: bytes or flops of one call."""
+        def cycle():
+            for i in range(copies):
+                fn(i)
+        sec = time_graph(cycle, launches=max(1, launches // copies), replays=10) * 1e-3 / copies
+        peak = {"hbm": HBM_PEAK_GBPS * 1e9, "mfma bf16": MFMA_BF16_PEAK_TFLOPS * 1e12, "mfma f32": MFMA_F32_PEAK_TFLOPS * 1e12}[bound]
+        rows.append(dict(kernel=name, size=size, us=round(sec * 1e6, 2), bound=bound,
+                         rate=round(amount / sec / (1e9 if bound == "hbm" else 1e12), 1), frac=round(amount / sec / peak, 4)))
+        torch.cuda.empty_cache()
+
+    g = torch.Generator().manual_seed(0)
+    for size, (w, hq, hkv, d, ff, gh, gk, gv) in GITOPEL_SIZES.items():
+        # -- decode attention: 64 sequences, contexts U[512, 4096], pages of 256
+        B, bs = 64, 256
+        ctx = torch.randint(512, 4097, (B,), generator=g)
+        case = make_decode_case(batch=B, hq=hq, hkv=hkv, dh=d)
+        plan = P.paged_decode_plan(case["ctx"], case["bt"], bs)
+        add("paged decode attention (Qwen3)", size,
+            lambda i: P.paged_decode_attention(case["q"], case["k_cache"], case["v_cache"], case["ctx"], case["bt"], d ** -0.5, plan=plan),
+            case["algo_bytes"], "hbm")
+        maxlen = 4096
+        for window, pool in ((4096, 16), (1024, 16)):
+            kv = P.PooledKV(2048, bs, hkv, d, pool, window, BF, dev)
+            for t in (kv.k, kv.v, kv.pk, kv.pv):
+                t.normal_()
+            pos = (case["ctx"].long() - 1)
+            seen = sum(min(int(c), window) + max(0, (int(c) - window) // pool) for c in case["ctx"].cpu())
+            q = torch.randn(B, hq, d, device=dev).to(BF)
+            gate, bias = torch.rand(B, hq, device=dev), torch.full((hq,), -5.0, device=dev, dtype=BF)
+            out = torch.empty(B, hq * d, device=dev, dtype=BF)
+            slots = torch.zeros(B, dtype=torch.int32, device=dev)
+            add(f"pooled-window decode attention, window {window}", size,
+                lambda i: P.pooled_attention_rows(q, bias, gate, kv, case["bt"], pos, slots, d ** -0.5, maxlen, out, pool_new=True),
+                seen * hkv * d * 4 + B * hq * d * 4, "hbm")
+            del kv
+        del case, plan
+        # -- prompt attention: 8 x 2048 tokens
+        S, L = 8, 2048
+        N = S * L
+        q = torch.randn(N, hq, d, device=dev).to(BF)
+        k, v = torch.randn(N, hkv, d, device=dev).to(BF), torch.randn(N, hkv, d, device=dev).to(BF)
+        cu = torch.arange(0, N + 1, L, dtype=torch.int32, device=dev)
+        add("prompt attention (Qwen3)", size, lambda i: P.varlen_prefill_attention(q, k, v, cu, cu, L, d ** -0.5),
+            4.0 * hq * d * S * L * L / 2, "mfma bf16")
+        gate, out = torch.rand(N, hq, device=dev), torch.empty(N, hq * d, device=dev, dtype=BF)
+        bt = torch.arange(N // bs, dtype=torch.int32, device=dev).view(S, -1)
+        starts = torch.zeros(S, dtype=torch.int32, device=dev)
+        for window, pool in ((2048, 16), (1024, 16), (512, 16)):
+            kv = P.PooledKV(N // bs, bs, hkv, d, pool, window, BF, dev)
+            for t in (kv.k, kv.v, kv.pk, kv.pv):
+                t.normal_()
+            seen = sum(min(i + 1, window) + max(0, (i - window + 1) // pool) for i in range(L)) * S
+            add(f"pooled-window prompt attention, window {window}", size,
+                lambda i: P.pooled_attention_prefill(q, bias, gate, kv, bt, cu, starts, 0, S, L, d ** -0.5, out),
+                4.0 * hq * d * seen, "mfma bf16")
+        add("pooled rows of a prompt", size, lambda i: P.pool_blocks(kv, bt, cu, starts, 0, S, L),
+            N * hkv * d * 4 * (1 + 1 / pool), "hbm")
+        # -- what stands between the projections and attention
+        tab, tab2 = build_cos_sin_cache(d, 4096, 1e6).to(dev), interleaved_cos_sin(d, 4096, 1e4).to(dev)
+        wd = torch.ones(d, dtype=BF, device=dev)
+        slots = torch.arange(N, dtype=torch.int32, device=dev)
+        pos = torch.arange(L, device=dev).repeat(S)
+        for n, copies in ((N, 3), (B, 1)):
+            qkv = torch.randn(copies, n, (hq + 2 * hkv) * d, device=dev).to(BF)
+            add(f"q/k norm + RoPE + store (Qwen3), {n} tokens", size,
+                lambda i: P.qknorm_rope_store(qkv[i], wd, wd, 1e-6, pos[:n], tab, hq, hkv, d, kv.k, kv.v, slots[:n]),
+                n * ((hq + 2 * hkv) * d * 4 + d * 4), "hbm", copies)
+            proj = torch.randn(copies, n, -(-((hq + hkv) * d + hq) // 16) * 16, device=dev).to(BF)
+            qb, kb = torch.zeros(hq * d, device=dev, dtype=BF), torch.zeros(hkv * d, device=dev, dtype=BF)
+            add(f"attention preparation, {n} tokens", size,
+                lambda i: P.attn_prep(proj[i], qb, kb, pos[:n], tab2, d, slots[:n], kv.k, kv.v, hq, d, 1e-6),
+                n * ((hq + hkv) * d * 2 + (hq + 2 * hkv) * d * 2 + hq * 6 + d * 4), "hbm", copies)
+            # -- norms
+            y = torch.randn(copies, n, w, device=dev).to(BF)
+            r = torch.randn(copies, n, w, device=dev).to(BF)
+            x = torch.randn(copies, n, w, device=dev)
+            ww = torch.ones(w, device=dev, dtype=BF)
+            add(f"add + RMSNorm (Qwen3), {n} tokens", size, lambda i: P.add_rms_norm(y[i], r[i], ww, 1e-6), n * w * 8, "hbm", copies)
+            add(f"norm + add + norm in groups, {n} tokens", size, lambda i: P.group_rms_norm_add(y[i], None, ww, x[i], ww, 4, 1e-6),
+                n * w * 12, "hbm", copies)
+            del qkv, proj, y, r, x
+        del q, k, v, kv, out
+        # -- gated linear attention
+        rank = 16
+        ld = 2 * gh * (gk + gv) + rank
+        a2, a2b = (torch.randn(gh * gk, rank, device=dev) * 0.1).to(BF), torch.zeros(gh * gk, device=dev, dtype=BF)
+        nw = torch.ones(gv, device=dev, dtype=BF)
+        for b in (64, 256):
+            state = torch.zeros(b, gh, gk, gv, device=dev)
+            proj, out = torch.randn(b, ld, device=dev).to(BF), torch.empty(b, gh * gv, device=dev, dtype=BF)
+            sl, ps = torch.arange(b, dtype=torch.int32, device=dev), torch.full((b,), 5, device=dev)
+            add(f"gated linear attention, {b} decoded tokens", size,
+                lambda i: P.gla_decode(proj, a2, a2b, nw, state, sl, ps, 16.0, 1e-6, out), b * gh * gk * gv * 8, "hbm")
+            del state
+        for s, l in ((8, 2048), (1, 8192)):
+            n = s * l
+            state = torch.zeros(s, gh, gk, gv, device=dev)
+            proj, out = torch.randn(n, ld, device=dev).to(BF), torch.empty(n, gh * gv, device=dev, dtype=BF)
+            chunk_rows = torch.arange(0, n, 16, dtype=torch.int32, device=dev)
+            chunk_lens = torch.full_like(chunk_rows, 16)
+            cuc = torch.arange(0, n // 16 + 1, l // 16, dtype=torch.int32, device=dev)
+            sl, st = torch.arange(s, dtype=torch.int32, device=dev), torch.zeros(s, dtype=torch.int32, device=dev)
+            add(f"gated linear attention, prompts {s} x {l}", size,
+                lambda i: P.gla_portions(proj, a2, a2b, nw, state, sl, st, chunk_rows, chunk_lens, cuc, 0, s, 16.0, 1e-6, out),
+                n * gh * (4.0 * gk * gv + 2 * 16 * (gk + gv)), "mfma f32")
+            del state, proj, out
+    return rows
+
+
+def bench_gitopel_throughput(size, batch=64, prompt=1024, out_tokens=128):
+    """Prompt and decode tokens/s of both models through ``LLM.generate`` (bf16, random weights, hipGraph decode)."""
+    import gc
+    import random
+    import torch
+    from tinyllmforge_amd import LLM, SamplingParams
+    rng = random.Random(0)
+    res = {}
+    for name, shape in (("gitopel", gitopel_shape(size)), ("qwen3", qwen3_shape(size))):
+        llm = LLM(shape, max_model_len=2048, max_num_batched_tokens=16384, max_num_seqs=batch, gpu_memory_utilization=0.5, seed=0)
+        vocab = llm.config.hf_config.vocab_size
+
+        def run(n):
+            prompts = [[rng.randrange(vocab) for _ in range(prompt)] for _ in range(batch)]
+            sp = SamplingParams(temperature=0.0, ignore_eos=True, max_tokens=n)
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            llm.generate(prompts, sp)
+            torch.cuda.synchronize()
+            return time.perf_counter() - t0
+        run(2)
+        t1 = min(run(1) for _ in range(2))
+        t2 = min(run(1 + out_tokens) for _ in range(2))
+        res[name] = dict(prefill_tok_s=round(batch * prompt / t1), decode_tok_s=round(batch * out_tokens / (t2 - t1)),
+                         decode_ms_per_step=round(1e3 * (t2 - t1) / out_tokens, 3),
+                         kernels_per_decode_step=llm.model_runner.graph_kernels[batch])
+        llm.exit()
+        del llm
+        gc.collect()
+        torch.cuda.empty_cache()
+    return dict(size=size, batch=batch, prompt_tokens=prompt, output_tokens=out_tokens, layers=8, **res)
+
+
 # ----------------------------------------------------------------------------- config 4 (end to end)
 def e2e_workload(num_seqs=256):
     """The reference's bench.py recipe (pure-python ``random``: platform independent)."""
@@ -752,6 +928,19 @@ def main():
         print("bench.py needs a GPU (the HIP path has no CPU fallback)", file=sys.stderr)
         sys.exit(1)
     torch.cuda.set_device(0)
+    if args.workload == "gitopel":   # its own line: the Gitopel model beside Qwen3 at equal size
+        rows = bench_gitopel_kernels()
+        through = [bench_gitopel_throughput(size) for size in GITOPEL_SIZES]
+        big = through[-1]
+        print(json.dumps({
+            "metric": "output tok/s (Gitopel, 8 layers of 4096, 64 sequences, decode)", "value": big["gitopel"]["decode_tok_s"],
+            "unit": "tok/s", "n_gpus": 1, "steps": big["output_tokens"], "warmup": 1,
+            "ms_per_step": big["gitopel"]["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak",
+            "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+            "config": {"workload": "Gitopel layers (alternating attention and gla, window 1024, pool 16) and Qwen3 layers of "
+                                   "equal size, random weights, bf16"},
+            "extra": {"throughput": through, "kernels": rows}}))
+        return
     extra = {}
     attn = bench_decode_attn(args, fp8=args.fp8, hq=args.hq) if args.workload == "decode_attn" else bench_decode_attn(args)
     roofline = attn["roofline"]

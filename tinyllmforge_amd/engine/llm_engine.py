@@ -78,7 +78,7 @@ class LLMEngine:
         ahead = self.config.run_ahead and sched.can_run_ahead() and bool(runner.graph_bs) and not runner.enforce_eager
         outputs = [] if ahead else self._drain()
         seqs, is_prefill = sched.schedule()
-        rows = sum(s.num_scheduled for s in seqs)
+        num_rows = sum(s.num_scheduled for s in seqs)
         if ahead and not is_prefill and runner.graph_ready(seqs):
             while len(self._ahead) >= self.AHEAD:
                 outputs += self._retire()
@@ -98,7 +98,7 @@ class LLMEngine:
             sched.postprocess(seqs, token_ids)
             outputs += [(s.seq_id, s.completion_token_ids) for s in seqs if s.is_finished]
         if runner.portioned:      # a step with portions counts as a prefill step, with the rows it ran
-            num_tokens = rows if is_prefill else -rows
+            num_tokens = num_rows if is_prefill else -num_rows
         else:
             num_tokens = sum(len(s) for s in seqs) if is_prefill else -len(seqs)
         # for the statistics of generate(): cached prompt tokens of a prefill step, context tokens a

@@ -126,7 +126,7 @@ def random_init_(model: nn.Module, seed: int = 0, std: float = 0.02, device_fill
     for name, p in model.named_parameters():
         if tied and name == "lm_head.weight":
             continue                                   # shares the embedding's storage
-        if name.endswith("norm.weight") or name.rsplit(".", 2)[-2].startswith("norm"):
+        if name.endswith("norm.weight") or name.split(".")[-2:-1] and name.split(".")[-2].startswith("norm"):
             p.data.fill_(1.0)
             continue
         if device_fill:
