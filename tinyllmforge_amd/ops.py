@@ -198,7 +198,9 @@ def sample(logits, temperatures, seed: int, offset: int):
     at (``seed``, ``offset``).  int64 ``[rows]``."""
     lib = _lib.load()
     if logits.dtype == torch.float32 and logits.is_cuda:
-        logits = logits.to(BF16)        # the draw's noise is far coarser than the rounding
+        # the draw's noise is far coarser than the rounding; rows stay 16-byte aligned
+        rows = torch.empty(logits.shape[0], (logits.shape[1] + 7) // 8 * 8, dtype=BF16, device=logits.device)
+        logits = rows[:, :logits.shape[1]].copy_(logits)
     _need(logits, BF16, "logits"); _need(temperatures, torch.float32, "temperatures")
     assert logits.dim() == 2 and logits.stride(1) == 1 and temperatures.is_contiguous()
     rows, vocab = logits.shape
