@@ -476,6 +476,13 @@ int tlf_probe_mix(const void *big, size_t big_bytes, const void *small_region, s
  * A step is a batch of sequences: sequence s owns the rows cu_seqlens_q[s] .. cu_seqlens_q[s + 1] - 1 of the step's
  * tensors and has seq_starts[s] tokens before them in the caches.
  *
+ * Deferred projections.  tlf_gemm_deferred is tlf_w8a16_gemm (scale given) or tlf_bf16_gemm (scale NULL) without the
+ * last step of a plan that splits K across workgroups: *splits (host memory, set before the call returns; it depends on
+ * M, N and K only) says how many partial sums [splits, M, N] fp32 stand at the head of the workspace, 1: y is complete.
+ * The entry points with the arguments (partials, splits, scale) read such a projection: with splits > 1 its value is
+ * bf16(sum * scale), what the reduce kernel would store, and the row stride is N (bf16 only, partials 16-byte aligned,
+ * the row pointer is not read); with splits <= 1 they read the rows.
+ *
  * Grouped RMSNorm around an fp32 residual.  A row of `width` values is split into `groups` equal parts, each
  * divided by its own sqrt(mean(part^2) + eps); the whole is multiplied by a weight.
  *
@@ -484,8 +491,10 @@ int tlf_probe_mix(const void *big, size_t big_bytes, const void *small_region, s
  *
  * x fp32 [rows, width] contiguous; y, h, table, weights: dtype; y_bias may be NULL; w_next NULL: no h.
  * width / groups <= 16384.  An id outside [0, vocab) embeds as zeros. */
-int tlf_group_rmsnorm_add(const void *y, int64_t y_stride, const void *y_bias, const void *w_post, float *x,
-                          const void *w_next, void *h, int32_t rows, int32_t width, int32_t groups, float eps,
+int tlf_gemm_deferred(const void *x, int64_t x_stride, const void *w, const float *scale, void *y, int32_t M, int32_t N,
+                      int32_t K, void *workspace, size_t workspace_bytes, int32_t *splits, void *stream);
+int tlf_group_rmsnorm_add(const void *y, int64_t y_stride, const float *partials, int32_t splits, const float *scale,
+                          const void *y_bias, const void *w_post, float *x, const void *w_next, void *h, int32_t rows, int32_t width, int32_t groups, float eps,
                           int32_t dtype, void *stream);
 int tlf_embed_group_rmsnorm(const int64_t *ids, const void *table, int32_t vocab, float *x, const void *w_next,
                             void *h, int32_t rows, int32_t width, int32_t groups, float eps, int32_t dtype,
@@ -513,7 +522,7 @@ int tlf_f32_argmax(const float *logits, int64_t row_stride, int64_t *out, int32_
  *   v row = the key so far; first rot_dims dimensions of q and k rotated pairwise (2 i, 2 i + 1) with
  *   cos_sin[pos] = cos of the rot_dims / 2 angles, then their sines (a position outside the table is not rotated);
  *   q and k divided by their root mean square; k / v rows stored at slot_mapping (negative: not stored),
- *   q_out [n, Hq, Dp], gate [n, Hq] = sigmoid, fp32.
+ *   q_out [n, Hq, Dp], gate [n, Hq] = sigmoid, fp32.  Partial sums: head_dim and rot_dims multiples of 8 only.
  * tlf_pool_blocks: pooled rows of the blocks that sequences first_seq .. first_seq + num_seqs - 1 complete in this step
  *   (max_tokens: the most tokens one of them has in the step).
  * tlf_pooled_attn_rows: any rows; row_seq[r] is the block-table row (NULL: r).  slot_mapping[r] < 0: a padding row,
@@ -521,7 +530,8 @@ int tlf_f32_argmax(const float *logits, int64_t row_stride, int64_t *out, int32_
  *   max_len bounds the positions.  out rows: Hq * head_dim values.
  * tlf_pooled_attn_prefill: bf16 matrix-core kernel for the portions of sequences first_seq .. + num_seqs - 1 (all other
  *   arguments as above; q, gate and out are indexed by the step's rows). */
-int tlf_attn_prep(const void *proj, int64_t proj_stride, const void *q_bias, const void *k_bias,
+int tlf_attn_prep(const void *proj, int64_t proj_stride, const float *partials, int32_t splits, const float *scale,
+                  const void *q_bias, const void *k_bias,
                   const int64_t *positions, const float *cos_sin, int32_t max_pos, int32_t rot_dims,
                   const int32_t *slot_mapping, int64_t num_slots, void *q_out, void *k_cache, void *v_cache,
                   float *gate, int32_t n, int32_t num_q_heads, int32_t num_kv_heads, int32_t head_dim,
@@ -557,16 +567,17 @@ int tlf_pooled_attn_prefill(const void *q, const void *score_bias, const float *
  * tlf_gla_decode: one token per row; position 0 starts from a zero state, a slot outside [0, num_slots) is a padding
  *   row (out = 0).
  * tlf_gla_portions: sequences first_seq .. + num_seqs - 1 of the step (state_slots and seq_starts are indexed by the
- *   step's sequences, a start of 0 begins with a zero state).  Their tokens are cut into chunks of at most 16 that do not
- *   cross a sequence: chunk c holds the chunk_lens[c] rows from chunk_rows[c] on, counted from the row `proj` and
+ *   step's sequences, a start of 0 begins with a zero state).  Their tokens are cut into chunks of 16 that do not cross a
+ *   sequence (a sequence's last chunk may be shorter) and follow each other: chunk c holds the chunk_lens[c] rows from chunk_rows[c] on, counted from the row `proj` and
  *   `out` point to; sequence first_seq + s owns the chunks cu_chunks[s] .. cu_chunks[s + 1] - 1.  `rows` rows in all. */
-int tlf_gla_decode(const void *proj, int64_t proj_stride, const void *a2, const void *a2_bias,
+int tlf_gla_decode(const void *proj, int64_t proj_stride, const float *partials, int32_t splits,
+                   const float *scale, const void *a2, const void *a2_bias,
                    const void *norm_weight, float *state, const int32_t *state_slots, int32_t num_slots,
                    const int64_t *positions, void *out, int64_t out_stride, int32_t rows, int32_t heads,
                    int32_t key_dim, int32_t value_dim, int32_t rank, float tau, float q_scale, float eps,
                    int32_t dtype, void *stream);
-size_t tlf_gla_portions_workspace_bytes(int32_t rows, int32_t chunks, int32_t heads, int32_t key_dim,
-                                        int32_t value_dim);
+size_t tlf_gla_portions_workspace_bytes(int32_t rows, int32_t chunks, int32_t num_seqs, int32_t heads,
+                                        int32_t key_dim, int32_t value_dim);
 int tlf_gla_portions(const void *proj, int64_t proj_stride, const void *a2, const void *a2_bias,
                      const void *norm_weight, float *state, const int32_t *state_slots, int32_t num_slots,
                      const int32_t *seq_starts, const int32_t *chunk_rows, const int32_t *chunk_lens,

@@ -281,19 +281,19 @@ def test_scheduler_waits_for_a_state_slot():
 def test_entry_points_reject_bad_arguments_on_the_host():
     from tinyllmforge_amd import _lib
     lib, a = _lib.load(), 4096
-    norm = lambda **k: lib.tlf_group_rmsnorm_add(*[{**dict(y=a, s=64, b=None, w=a, x=a, n=a, h=a, rows=2, width=64, groups=4, eps=1e-6, dt=0, st=None), **k}[n]
-                                                   for n in ("y", "s", "b", "w", "x", "n", "h", "rows", "width", "groups", "eps", "dt", "st")])
-    assert norm(y=None) == -1 and norm(groups=3) == -2 and norm(s=32) == -2 and norm(dt=7) == -5 and norm(rows=0) == 0
+    norm = lambda **k: lib.tlf_group_rmsnorm_add(*[{**dict(y=a, s=64, p=None, sp=1, sc=None, b=None, w=a, x=a, n=a, h=a, rows=2, width=64, groups=4, eps=1e-6, dt=0, st=None), **k}[n]
+                                                   for n in ("y", "s", "p", "sp", "sc", "b", "w", "x", "n", "h", "rows", "width", "groups", "eps", "dt", "st")])
+    assert norm(y=None) == -1 and norm(sp=3) == -1 and norm(p=a + 4, sp=3) == -3 and norm(p=a, sp=3, dt=1) == -5 and norm(groups=3) == -2 and norm(s=32) == -2 and norm(dt=7) == -5 and norm(rows=0) == 0
     assert lib.tlf_embed_group_rmsnorm(a, a, 0, a, a, a, 1, 64, 1, 1e-6, 0, None) == -2
-    assert lib.tlf_attn_prep(a, 100, None, None, a, a, 10, 32, a, 64, a, a, a, a, 1, 1, 1, 33, 64, 1e-6, 0, None) == -2   # odd dim
-    assert lib.tlf_attn_prep(a, 60, None, None, a, a, 10, 32, a, 64, a, a, a, a, 1, 1, 1, 32, 32, 1e-6, 0, None) == -2    # row too short
-    assert lib.tlf_attn_prep(a, 80, None, None, a, a, 10, 32, a, 64, a, a, a, None, 1, 1, 1, 32, 32, 1e-6, 0, None) == -1
+    assert lib.tlf_attn_prep(a, 100, None, 1, None, None, None, a, a, 10, 32, a, 64, a, a, a, a, 1, 1, 1, 33, 64, 1e-6, 0, None) == -2   # odd dim
+    assert lib.tlf_attn_prep(a, 60, None, 1, None, None, None, a, a, 10, 32, a, 64, a, a, a, a, 1, 1, 1, 32, 32, 1e-6, 0, None) == -2    # row too short
+    assert lib.tlf_attn_prep(a, 80, None, 1, None, None, None, a, a, 10, 32, a, 64, a, a, a, None, 1, 1, 1, 32, 32, 1e-6, 0, None) == -1
     rows = lambda bs=64, pool=4, win=8, ws=a, wsb=1 << 30, dim=32, n=2: lib.tlf_pooled_attn_rows(
         a, a, a, a, a, a, a, a, 4, a, a, None, a, 64, n, 2, 1, dim, bs, pool, win, 100, 10, 0.1, 1, 0, ws, wsb, None)
     assert rows(bs=100) == -2 and rows(pool=0) == -2 and rows(win=0) == -2 and rows(n=0) == 0 and rows(dim=64) == -2
     assert lib.tlf_pooled_attn_prefill(a, a, a, a, a, a, a, a, 4, a, None, 0, 1, 8, a, 64, 2, 1, 32, 64, 4, 8, 10, 0.1, None) == -1
     assert lib.tlf_pool_blocks(a, a, a, a, a, 4, a, a, 0, 0, 8, 1, 32, 64, 4, 8, 10, 0, None) == 0
-    gla = lambda dk=16, dv=16, r=4, ld=132, tau=2.0: lib.tlf_gla_decode(a, ld, a, a, a, a, a, 4, a, a, 64, 2, 2, dk, dv, r, tau, 1.0, 1e-6, 0, None)
+    gla = lambda dk=16, dv=16, r=4, ld=132, tau=2.0: lib.tlf_gla_decode(a, ld, None, 1, None, a, a, a, a, a, 4, a, a, 64, 2, 2, dk, dv, r, tau, 1.0, 1e-6, 0, None)
     assert gla(dk=300, ld=4000) == -2 and gla(ld=131) == -2 and gla(tau=0.0) == -2 and gla(dv=1000, ld=8000) == -2
     assert lib.tlf_gla_portions(a, 132, a, a, a, a, a, 4, a, a, a, a, 1, 0, 1, a, 64, 8, 2, 16, 16, 4, 2.0, 1.0, 1e-6, 0, None, 0, None) == -4
     assert lib.tlf_f32_gemm(a, 8, a, a, 2, 4, 16, None) == -2 and lib.tlf_f32_argmax(a, 4, a, 1, 8, None) == -2

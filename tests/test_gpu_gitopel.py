@@ -274,6 +274,87 @@ def test_gated_linear_attention(dtype, H, dk, dv, rank, decay):
         assert (state[1] == 5.0).all()
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("lens,start", [([1200], 0), ([700, 515], 0), ([900], 5)])
+def test_gated_linear_attention_in_segments(dtype, lens, start):
+    """Prompts long enough for the kernels to cut a sequence into segments, from zero and from a state."""
+    from tinyllmforge_amd import ops as P
+    dt, g, eps, tau = DTYPES[dtype], torch.Generator().manual_seed(7), 1e-5, 16.0
+    H, dk, dv, rank = 2, 48, 40, 4
+    proj = [torch.randn(n, 2 * H * (dk + dv) + rank, generator=g).to(dt) for n in lens]
+    a2, a2b, nw = torch.randn(H * dk, rank, generator=g).to(dt), 3 + torch.randn(H * dk, generator=g).to(dt), torch.randn(dv, generator=g).to(dt)
+    first = [torch.randn(H, dk, dv, generator=g) for _ in lens]
+    state = torch.stack([torch.full((H, dk, dv), 5.0)] + first).cuda()
+    rows = torch.cat(proj).cuda()
+    out = torch.empty(rows.shape[0], H * dv, dtype=dt, device="cuda")
+    crow, clen, cu, at = [], [], [0], 0
+    for n in lens:
+        crow += list(range(at, at + n, 16))
+        clen += [min(16, n - c) for c in range(0, n, 16)]
+        cu.append(len(crow))
+        at += n
+    t = lambda x: torch.tensor(x, dtype=torch.int32, device="cuda")
+    P.gla_portions(rows, a2.cuda(), a2b.cuda(), nw.cuda(), state, t([i + 1 for i in range(len(lens))]), t([start] * len(lens)),
+                   t(crow), t(clen), t(cu), 0, len(lens), tau, eps, out)
+    at = 0
+    for i, n in enumerate(lens):
+        p = proj[i].double()
+        q, k, v, gt, r = p.split([H * dk, H * dk, H * dv, H * dv, rank], dim=1)
+        la = -torch.nn.functional.softplus(-(r @ a2.double().T + a2b.double())).view(-1, H, dk) / tau
+        o, s = O.gla_recurrence(q.view(-1, H, dk) * dk ** -0.5, k.view(-1, H, dk), v.view(-1, H, dv), la,
+                                first[i].double() if start else None)
+        want = (O.unit_rms(o, eps) * nw.double()).reshape(-1, H * dv) * O.silu(gt)
+        assert rel(out[at:at + n], want) < (4e-3 if dtype == "bf16" else 2e-5)
+        assert rel(state[i + 1], s) < 2e-5
+        at += n
+    assert (state[0] == 5.0).all()
+
+
+@pytest.mark.parametrize("quantized", [False, True])
+def test_consumers_add_up_split_projections(quantized):
+    """A projection left as partial sums gives the bits of the finished one, in every kernel that may read it."""
+    from tinyllmforge_amd import ops as P
+    from tinyllmforge_amd.layers.linear import quantize_per_channel
+    from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
+    g, n, K = torch.Generator().manual_seed(2), 40, 4096
+    bf = lambda *s: torch.randn(*s, generator=g).to(torch.bfloat16).cuda()
+
+    def both(N):
+        x, w = bf(n, K), bf(N, K) * K ** -0.5
+        if quantized:
+            q, scale = quantize_per_channel(w)
+            packed = P.pack_w8(q)
+            return P.w8a16_linear(x, packed, scale), P.linear_deferred(x, packed, scale)
+        return P.bf16_linear(x, w), P.linear_deferred(x, w)
+
+    y, d = both(1024)
+    assert d.splits > 1, "this size is meant to split K"
+    x, wp, wn, b = torch.randn(n, 1024, generator=g).cuda(), bf(1024), bf(1024), bf(1024)
+    x2 = x.clone()
+    h2 = P.group_rms_norm_add(d, b, wp, x2, wn, 4, 1e-6)
+    h1 = P.group_rms_norm_add(y, b, wp, x, wn, 4, 1e-6)
+    assert torch.equal(h1, h2) and torch.equal(x, x2)
+    H, G, D = 8, 2, 96
+    y, d = both(-(-((H + G) * D + H) // 16) * 16)
+    assert d.splits > 1
+    tab, pos, slots = interleaved_cos_sin(64, 100, 1e4).cuda(), torch.arange(n).cuda(), torch.arange(n, dtype=torch.int32).cuda()
+    kv = [P.PooledKV(1, 64, G, D, 8, 8, torch.bfloat16, "cuda") for _ in range(2)]
+    args = lambda c: (None, None, pos, tab, 64, slots, c.k, c.v, H, D, 1e-6)
+    q2, g2 = P.attn_prep(d, *args(kv[1]))
+    q1, g1 = P.attn_prep(y, *args(kv[0]))
+    assert torch.equal(q1, q2) and torch.equal(g1, g2) and torch.equal(kv[0].k, kv[1].k) and torch.equal(kv[0].v, kv[1].v)
+    H, dk, dv, r = 2, 48, 72, 16
+    y, d = both(2 * H * (dk + dv) + r)
+    assert d.splits > 1
+    st = torch.randn(n, H, dk, dv, generator=g).cuda()
+    st2 = st.clone()
+    a2, a2b, nw, sl = bf(H * dk, r), bf(H * dk), bf(dv), torch.arange(n, dtype=torch.int32).cuda()
+    outs = [torch.empty(n, H * dv, dtype=torch.bfloat16, device="cuda") for _ in range(2)]
+    P.gla_decode(d, a2, a2b, nw, st2, sl, pos, 8.0, 1e-6, outs[1])
+    P.gla_decode(y, a2, a2b, nw, st, sl, pos, 8.0, 1e-6, outs[0])
+    assert torch.equal(outs[0], outs[1]) and torch.equal(st, st2)
+
+
 # ---------------------------------------------------------------------------------------------- the model
 def engine(cfg, dtype, seed=0, blocks=12, seqs=4, max_len=256, **kw):
     from tinyllmforge_amd.engine.llm_engine import LLMEngine

@@ -68,12 +68,13 @@ SIGNATURES = {
     "tlf_varlen_prefill_attn": (c_int32, [_P, _I64, _P, _I64, _P, _I64, _I32, _P, _P, _P, _P, _P, _I64,
                                           _P, _I32, _I32, _I32, _I32, _I32, _I32, _I64, _F, _P]),
     "tlf_embedding": (c_int32, [_P, _P, _P, _I32, _I32, _I32, _P]),
-    "tlf_group_rmsnorm_add": (c_int32, [_P, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _F, _I32, _P]),
+    "tlf_gemm_deferred": (c_int32, [_P, _I64, _P, _P, _P, _I32, _I32, _I32, _P, _SZ, _P, _P]),
+    "tlf_group_rmsnorm_add": (c_int32, [_P, _I64, _P, _I32, _P, _P, _P, _P, _P, _P, _I32, _I32, _I32, _F, _I32, _P]),
     "tlf_embed_group_rmsnorm": (c_int32, [_P, _P, _I32, _P, _P, _P, _I32, _I32, _I32, _F, _I32, _P]),
     "tlf_f32_gemm": (c_int32, [_P, _I64, _P, _P, _I32, _I32, _I32, _P]),
     "tlf_f32_silu_and_mul": (c_int32, [_P, _P, _I32, _I32, _P]),
     "tlf_f32_argmax": (c_int32, [_P, _I64, _P, _I32, _I32, _P]),
-    "tlf_attn_prep": (c_int32, [_P, _I64, _P, _P, _P, _P, _I32, _I32, _P, _I64, _P, _P, _P, _P,
+    "tlf_attn_prep": (c_int32, [_P, _I64, _P, _I32, _P, _P, _P, _P, _P, _I32, _I32, _P, _I64, _P, _P, _P, _P,
                                 _I32, _I32, _I32, _I32, _I32, _F, _I32, _P]),
     "tlf_pool_blocks": (c_int32, [_P, _P, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _I32,
                                   _I64, _I32, _P]),
@@ -82,9 +83,9 @@ SIGNATURES = {
                                        _I32, _I32, _I32, _I32, _I64, _F, _I32, _I32, _P, _SZ, _P]),
     "tlf_pooled_attn_prefill": (c_int32, [_P, _P, _P, _P, _P, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _P, _I64,
                                           _I32, _I32, _I32, _I32, _I32, _I32, _I64, _F, _P]),
-    "tlf_gla_decode": (c_int32, [_P, _I64, _P, _P, _P, _P, _P, _I32, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _F, _F,
+    "tlf_gla_decode": (c_int32, [_P, _I64, _P, _I32, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _F, _F,
                                  _F, _I32, _P]),
-    "tlf_gla_portions_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32, _I32]),
+    "tlf_gla_portions_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32, _I32, _I32]),
     "tlf_gla_portions": (c_int32, [_P, _I64, _P, _P, _P, _P, _P, _I32, _P, _P, _P, _P, _I32, _I32, _I32, _P, _I64, _I32,
                                    _I32, _I32, _I32, _I32, _F, _F, _F, _I32, _P, _SZ, _P]),
     "tlf_probe_read": (c_int32, [_P, _SZ, _P, _P]),

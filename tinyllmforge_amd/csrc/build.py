@@ -77,11 +77,13 @@ def build(force: bool = True, verbose: bool = True) -> str:
             print(out)
         if rc:
             raise RuntimeError("hipcc failed")
-    link = ["hipcc", "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", OUT]
+    part = OUT + ".part"           # the library appears whole or not at all
+    link = ["hipcc", "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", part]
     r = subprocess.run(link, capture_output=True, text=True)
     if r.returncode:
         print(r.stdout + r.stderr)
         raise RuntimeError("link failed")
+    os.replace(part, OUT)
     if verbose:
         print("[build] ->", OUT, flush=True)
     return OUT

@@ -57,6 +57,41 @@ struct Elem<float> {
   }
 };
 
+// A bf16 projection [rows, n] that exists as fp32 partial sums [splits, rows, n] (times a scale per column where the
+// weight is int8): the value is their sum, rounded to bf16 as the projection's own kernel would.
+struct Partials {
+  const float *p;
+  const float *scale;
+  int64_t plane;      // rows * n
+  int32_t n, splits;
+  __device__ __forceinline__ float ld(int64_t row, int col) const {
+    const float *s = p + row * n + col;
+    float v = 0.f;
+#pragma unroll 4
+    for (int k = 0; k < splits; ++k) v += s[k * plane];
+    return Elem<unsigned short>::rnd(scale ? v * scale[col] : v);
+  }
+  __device__ __forceinline__ void ld8(int64_t row, int col, float (&f)[8]) const {
+    const float *s = p + row * n + col;
+    float4 a = make_float4(0.f, 0.f, 0.f, 0.f), b = a;
+#pragma unroll 4
+    for (int k = 0; k < splits; ++k) {
+      const float4 x = reinterpret_cast<const float4 *>(s + k * plane)[0], y = reinterpret_cast<const float4 *>(s + k * plane)[1];
+      a.x += x.x; a.y += x.y; a.z += x.z; a.w += x.w;
+      b.x += y.x; b.y += y.y; b.z += y.z; b.w += y.w;
+    }
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w; f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[e] = Elem<unsigned short>::rnd(scale ? f[e] * scale[col + e] : f[e]);
+  }
+};
+inline int partials_check(const void *partials, const float *scale, int32_t splits, int32_t dtype) {
+  if (splits < 0 || splits > 64) return TLF_E_SHAPE;
+  if (splits > 1 && dtype != TLF_DT_BF16) return TLF_E_UNSUPPORTED;
+  if (splits > 1 && !partials) return TLF_E_NULL;
+  return splits > 1 && (!aligned16(partials) || !aligned16(scale)) ? TLF_E_ALIGN : TLF_OK;
+}
+
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
 

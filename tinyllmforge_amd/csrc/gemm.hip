@@ -1382,7 +1382,8 @@ template <bool W8>
 int launch_gemm(const void *x, int64_t x_stride, const void *w, const float *scale, void *y,
                 int32_t M, int32_t N, int32_t K, void *workspace, size_t workspace_bytes,
                 hipStream_t stream, int32_t *plan_out = nullptr, int32_t act = 0,
-                const NormTail *tail = nullptr, const QkRopeStoreArgs *qk = nullptr) {
+                const NormTail *tail = nullptr, const QkRopeStoreArgs *qk = nullptr, int32_t *deferred = nullptr) {
+  if (deferred) *deferred = 1;
   const bool dry = plan_out != nullptr;
   GemmParams p;
   p.x = static_cast<const unsigned char *>(x);
@@ -1534,6 +1535,10 @@ int launch_gemm(const void *x, int64_t x_stride, const void *w, const float *sca
   if (act == 2)  // y is the int64 token-id vector here
     return launch_argmax_final(p.amax, p.amax_parts, static_cast<int64_t *>(y), M, stream);
   if (g.splits > 1) {
+    if (deferred) {  // the partial sums stay in the workspace: whoever reads the result adds them up
+      *deferred = g.splits;
+      return rc;
+    }
     if (tail) {  // the caller checked that this plan splits K and that the row fits the kernel
 #define TLF_TAIL(TPR_, MAXC_)                                                                 \
   TLF_LAUNCH((splitk_reduce_add_rmsnorm_kernel<TPR_, MAXC_, W8>),                     \
@@ -1690,6 +1695,20 @@ extern "C" int tlf_bf16_gemm(const void *x, int64_t x_stride, const void *w, voi
   if (rc != TLF_OK) return rc;
   return launch_gemm<false>(x, x_stride, w, nullptr, y, M, N, K, workspace, workspace_bytes,
                             static_cast<hipStream_t>(stream));
+}
+
+extern "C" int tlf_gemm_deferred(const void *x, int64_t x_stride, const void *w, const float *scale, void *y, int32_t M,
+                                 int32_t N, int32_t K, void *workspace, size_t workspace_bytes, int32_t *splits,
+                                 void *stream) {
+  if (!splits) return TLF_E_NULL;
+  *splits = 1;
+  if (M == 0) return TLF_OK;
+  const int rc = check_gemm_args(x, x_stride, w, y, M, N, K);
+  if (rc != TLF_OK) return rc;
+  if (reinterpret_cast<uintptr_t>(scale) & 15u) return TLF_E_ALIGN;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  return scale ? launch_gemm<true>(x, x_stride, w, scale, y, M, N, K, workspace, workspace_bytes, s, nullptr, 0, nullptr, nullptr, splits)
+               : launch_gemm<false>(x, x_stride, w, nullptr, y, M, N, K, workspace, workspace_bytes, s, nullptr, 0, nullptr, nullptr, splits);
 }
 
 extern "C" int tlf_gemm_plan(int32_t M, int32_t N, int32_t K, int32_t w8, int32_t *plan8) {

@@ -13,6 +13,7 @@ namespace tlf {
 
 struct GroupNormArgs {
   const void *y;        // [rows, width] sublayer output, row stride y_stride (add mode)
+  Partials part;        // or its partial sums
   int64_t y_stride;
   const void *y_bias;   // [width] or NULL
   const void *w_post;   // [width]
@@ -55,7 +56,8 @@ __device__ __forceinline__ void stv(T *p, const float (&f)[VEC]) {
   else Elem<T>::st(p, f[0]);
 }
 
-template <typename T, int VEC, int TPR, int MAXC, bool EMBED>
+// MODE 0: embed, 1: add, 2: add with y as partial sums
+template <typename T, int VEC, int TPR, int MAXC, int MODE>
 __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
   __shared__ float part[4];
   const int tid = threadIdx.x, sub = tid % TPR;
@@ -69,7 +71,7 @@ __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
   float v[MAXC][VEC];
   float *xr = a.x + row * a.width + col0;
   const float inv_cols = 1.0f / static_cast<float>(a.cols);
-  if constexpr (EMBED) {
+  if constexpr (MODE == 0) {
     const int64_t id = a.ids[row];
     const bool ok = id >= 0 && id < a.vocab;
     const T *src = static_cast<const T *>(a.table) + (ok ? id : 0) * a.width + col0;
@@ -81,7 +83,7 @@ __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
       if (ch < nch && ok) ldv<T, VEC>(src + ch * VEC, v[c]);
     }
   } else {
-    const T *yr = static_cast<const T *>(a.y) + row * a.y_stride + col0;
+    const T *yr = MODE == 1 ? static_cast<const T *>(a.y) + row * a.y_stride + col0 : nullptr;
     const T *wp = static_cast<const T *>(a.w_post) + col0;
     const T *yb = a.y_bias ? static_cast<const T *>(a.y_bias) + col0 : nullptr;
     float xo[MAXC][VEC], w[MAXC][VEC];
@@ -89,7 +91,9 @@ __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
 #pragma unroll
     for (int c = 0; c < MAXC; ++c) {
       const int at = min(sub + c * TPR, nch - 1) * VEC;
-      ldv<T, VEC>(yr + at, v[c]);
+      if constexpr (MODE == 1) ldv<T, VEC>(yr + at, v[c]);
+      else if constexpr (VEC == 8) a.part.ld8(row, col0 + at, v[c]);
+      else v[c][0] = a.part.ld(row, col0 + at);
       ldv<float, VEC>(xr + at, xo[c]);
       ldv<T, VEC>(wp + at, w[c]);
     }
@@ -142,10 +146,10 @@ __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
   }
 }
 
-template <typename T, bool EMBED>
+template <typename T, int MODE>
 int launch_groupnorm(const GroupNormArgs &a, bool vec8, hipStream_t stream) {
 #define TLF_GN(VEC, TPR, MAXC)                                                                               \
-  TLF_LAUNCH((groupnorm_kernel<T, VEC, TPR, MAXC, EMBED>),                                                   \
+  TLF_LAUNCH((groupnorm_kernel<T, VEC, TPR, MAXC, MODE>),                                                   \
              dim3(static_cast<unsigned>((a.units + (256 / TPR) - 1) / (256 / TPR))), dim3(256), 0, stream, a)
   if (vec8) {
     if (a.cols <= 128) TLF_GN(8, 16, 1);
@@ -178,18 +182,23 @@ int groupnorm_entry(GroupNormArgs &a, int32_t rows, int32_t dtype, hipStream_t s
     vec8 = vec8 && aligned16(a.table);
   else
     vec8 = vec8 && aligned16(a.y) && aligned16(a.y_bias) && aligned16(a.w_post) && a.y_stride % 8 == 0;
-  return dtype == TLF_DT_BF16 ? launch_groupnorm<unsigned short, EMBED>(a, vec8, stream)
-                              : launch_groupnorm<float, EMBED>(a, vec8, stream);
+  constexpr int kMode = EMBED ? 0 : 1;
+  if (!EMBED && a.part.splits > 1) return launch_groupnorm<unsigned short, 2>(a, vec8, stream);
+  return dtype == TLF_DT_BF16 ? launch_groupnorm<unsigned short, kMode>(a, vec8, stream)
+                              : launch_groupnorm<float, kMode>(a, vec8, stream);
 }
 
 }  // namespace tlf
 
-extern "C" int tlf_group_rmsnorm_add(const void *y, int64_t y_stride, const void *y_bias, const void *w_post, float *x,
+extern "C" int tlf_group_rmsnorm_add(const void *y, int64_t y_stride, const float *partials, int32_t splits,
+                                     const float *scale, const void *y_bias, const void *w_post, float *x,
                                      const void *w_next, void *h, int32_t rows, int32_t width, int32_t groups,
                                      float eps, int32_t dtype, void *stream) {
   tlf::GroupNormArgs a{};
-  if (rows > 0 && (!y || !w_post)) return TLF_E_NULL;
+  if (int rc = tlf::partials_check(partials, scale, splits, dtype)) return rc;
+  if (rows > 0 && ((!y && splits <= 1) || !w_post)) return TLF_E_NULL;
   if (y_stride < width) return TLF_E_SHAPE;
+  a.part = tlf::Partials{partials, scale, rows * y_stride, static_cast<int32_t>(y_stride), splits};
   a.y = y; a.y_stride = y_stride; a.y_bias = y_bias; a.w_post = w_post; a.x = x; a.w_next = w_next; a.h = h;
   a.width = width; a.groups = groups; a.eps = eps;
   return tlf::groupnorm_entry<false>(a, rows, dtype, static_cast<hipStream_t>(stream));

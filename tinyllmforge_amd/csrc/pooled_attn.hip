@@ -25,6 +25,7 @@ int pooled_cache_check(const PooledCache &c, int32_t dtype) {
 // ---------------------------------------------------------------------------------------------------------------
 struct AttnPrepArgs {
   const void *proj;        // [n, ld]: q heads, k heads, one gate value per q head
+  Partials part;           // or its partial sums
   int64_t ld;
   const void *q_bias, *k_bias;
   const int64_t *positions;
@@ -40,7 +41,7 @@ struct AttnPrepArgs {
   int32_t vec;             // rows may be read 8 elements at a time
 };
 
-// 16 lanes per (token, head); head H + G is the token's gate row.
+// 16 lanes per (token, head), any size; head H + G is the token's gate row.
 template <typename T, int MAXC>
 __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnPrepArgs a) {
   const int heads = a.H + a.G + 1;
@@ -73,21 +74,9 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnPrepArgs a) {
 #pragma unroll
     for (int e = 0; e < 8; ++e) x[c][e] = 0.f;
     if (ch < nch) {
-      if (a.vec) {
-        if (ch * 8 < a.D) {
-          Elem<T>::ld8(src + ch * 8, x[c]);
-          if (bias) {
-            float b[8];
-            Elem<T>::ld8(bias + ch * 8, b);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) x[c][e] += b[e];
-          }
-        }
-      } else {
-#pragma unroll
-        for (int e = 0; e < 8; ++e)
-          if (ch * 8 + e < a.D) x[c][e] = Elem<T>::ld(src + ch * 8 + e) + (bias ? Elem<T>::ld(bias + ch * 8 + e) : 0.f);
-      }
+      for (int e = 0; e < 8; ++e)
+        if (ch * 8 + e < a.D) x[c][e] = Elem<T>::ld(src + ch * 8 + e) + (bias ? Elem<T>::ld(bias + ch * 8 + e) : 0.f);
       if (!is_q && store)
         Elem<T>::st8(static_cast<T *>(a.v_cache) + (slot * a.G + (head - a.H)) * a.Dp + ch * 8, x[c]);
 #pragma unroll
@@ -118,6 +107,126 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnPrepArgs a) {
         Elem<T>::st8(static_cast<T *>(a.k_cache) + (slot * a.G + (head - a.H)) * a.Dp + ch * 8, x[c]);
     }
   }
+}
+
+// The same for rows that can be read 8 elements at a time (head_dim and rot_dims multiples of 8): a team keeps one head
+// and takes TOK consecutive tokens, with the loads of all of them in flight before the first is touched.
+template <typename T, int MAXC, int TOK, bool PART>
+__global__ __launch_bounds__(256) void attn_prep_vec_kernel(const AttnPrepArgs a) {
+  const int head = blockIdx.y * 16 + threadIdx.x / 16, j = threadIdx.x % 16;
+  const int64_t tok0 = static_cast<int64_t>(blockIdx.x) * TOK;
+  if (head > a.H + a.G) return;                      // whole 16-lane groups leave together
+  const T *base = static_cast<const T *>(a.proj);
+  if (head == a.H + a.G) {
+    for (int k = 0; k < TOK; ++k) {
+      if (tok0 + k >= a.n) return;
+      const T *gr = base + (tok0 + k) * a.ld + static_cast<int64_t>(head) * a.D;
+      for (int h = j; h < a.H; h += 16)
+        a.gate[(tok0 + k) * a.H + h] = sigmoid_f32(PART ? a.part.ld(tok0 + k, head * a.D + h) : Elem<T>::ld(gr + h));
+    }
+    return;
+  }
+  const bool is_q = head < a.H;
+  const T *bias = is_q ? static_cast<const T *>(a.q_bias) : static_cast<const T *>(a.k_bias);
+  if (bias) bias += static_cast<int64_t>(is_q ? head : head - a.H) * a.D;
+  const int half = a.rot_dims / 2, nch = a.Dp / 8;
+  typename Elem<T>::Raw8 raw[TOK][MAXC];
+  int64_t pos[TOK], slot[TOK];
+#pragma unroll
+  for (int k = 0; k < TOK; ++k) {
+    const int64_t tok = min(tok0 + k, static_cast<int64_t>(a.n) - 1);
+    const T *src = base + tok * a.ld + static_cast<int64_t>(head) * a.D;
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+      if (!PART) Elem<T>::raw8(src + min((j + c * 16) * 8, a.D - 8), raw[k][c]);
+    pos[k] = a.positions[tok];
+    slot[k] = a.slots[tok];
+  }
+  float4 co[TOK][MAXC], si[TOK][MAXC];
+#pragma unroll
+  for (int k = 0; k < TOK; ++k) {
+    const bool ok = pos[k] >= 0 && pos[k] < a.max_pos;
+    const float *cs = a.cos_sin + (ok ? pos[k] : 0) * a.rot_dims;
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int i = (j + c * 16) * 4;
+      co[k][c] = make_float4(1.f, 1.f, 1.f, 1.f);
+      si[k][c] = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (ok && i < half) {
+        co[k][c] = *reinterpret_cast<const float4 *>(cs + i);
+        si[k][c] = *reinterpret_cast<const float4 *>(cs + half + i);
+      }
+    }
+  }
+#pragma unroll
+  for (int k = 0; k < TOK; ++k) {
+    if (tok0 + k >= a.n) return;
+    const int64_t tok = tok0 + k;
+    const bool store = !is_q && slot[k] >= 0 && slot[k] < a.num_slots;
+    const int64_t crow = (slot[k] * a.G + (head - a.H)) * a.Dp;
+    float x[MAXC][8], ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int ch = j + c * 16;
+      if constexpr (PART) a.part.ld8(tok, head * a.D + min(ch * 8, a.D - 8), x[c]);
+      else Elem<T>::cvt8(raw[k][c], x[c]);
+      if (ch * 8 >= a.D) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[c][e] = 0.f;
+      } else if (bias) {
+        float b[8];
+        Elem<T>::ld8(bias + ch * 8, b);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[c][e] += b[e];
+      }
+      if (store && ch < nch) Elem<T>::st8(static_cast<T *>(a.v_cache) + crow + ch * 8, x[c]);
+      const float cv[4] = {co[k][c].x, co[k][c].y, co[k][c].z, co[k][c].w}, sv[4] = {si[k][c].x, si[k][c].y, si[k][c].z, si[k][c].w};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float u = x[c][2 * e], v = x[c][2 * e + 1];
+        x[c][2 * e] = __fmul_rn(u, cv[e]) - __fmul_rn(v, sv[e]);
+        x[c][2 * e + 1] = __fmul_rn(v, cv[e]) + __fmul_rn(u, sv[e]);
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss = fmaf(x[c][e], x[c][e], ss);
+    }
+    ss = group_sum<16>(ss);
+    const float inv = 1.0f / sqrtf(ss / static_cast<float>(a.D) + a.eps);
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int ch = j + c * 16;
+      if (ch < nch) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[c][e] *= inv;
+        if (is_q) Elem<T>::st8(static_cast<T *>(a.q_out) + (tok * a.H + head) * a.Dp + ch * 8, x[c]);
+        else if (store) Elem<T>::st8(static_cast<T *>(a.k_cache) + crow + ch * 8, x[c]);
+      }
+    }
+  }
+}
+
+template <typename T>
+int launch_attn_prep(const AttnPrepArgs &a, hipStream_t s) {
+  const int heads = a.H + a.G + 1;
+  if (a.vec) {
+    const bool part = a.part.splits > 1;
+    const int tok = !part && a.n > 1024 ? 4 : 1;
+    const dim3 grid((a.n + tok - 1) / tok, (heads + 15) / 16);
+#define TLF_PREP(MAXC)                                                                         \
+  do {                                                                                         \
+    if (part) TLF_LAUNCH((attn_prep_vec_kernel<unsigned short, MAXC, 1, true>), grid, dim3(256), 0, s, a); \
+    else if (tok == 4) TLF_LAUNCH((attn_prep_vec_kernel<T, MAXC, 4, false>), grid, dim3(256), 0, s, a);    \
+    else TLF_LAUNCH((attn_prep_vec_kernel<T, MAXC, 1, false>), grid, dim3(256), 0, s, a);      \
+  } while (0)
+    if (a.Dp <= 128) TLF_PREP(1);
+    else TLF_PREP(2);
+#undef TLF_PREP
+    return launch_status();
+  }
+  const dim3 grid(static_cast<unsigned>((static_cast<int64_t>(a.n) * heads + 15) / 16));
+  if (a.Dp <= 128) TLF_LAUNCH((attn_prep_kernel<T, 1>), grid, dim3(256), 0, s, a);
+  else TLF_LAUNCH((attn_prep_kernel<T, 2>), grid, dim3(256), 0, s, a);
+  return launch_status();
 }
 
 // ---------------------------------------------------------------------------------------------------------------
@@ -298,7 +407,8 @@ int rows_heads_per_pass(int group) { return group <= 1 ? 1 : group <= 2 ? 2 : gr
 
 }  // namespace tlf
 
-extern "C" int tlf_attn_prep(const void *proj, int64_t proj_stride, const void *q_bias, const void *k_bias,
+extern "C" int tlf_attn_prep(const void *proj, int64_t proj_stride, const float *partials, int32_t splits,
+                             const float *scale, const void *q_bias, const void *k_bias,
                              const int64_t *positions, const float *cos_sin, int32_t max_pos, int32_t rot_dims,
                              const int32_t *slot_mapping, int64_t num_slots, void *q_out, void *k_cache, void *v_cache,
                              float *gate, int32_t n, int32_t num_q_heads, int32_t num_kv_heads, int32_t head_dim,
@@ -309,22 +419,16 @@ extern "C" int tlf_attn_prep(const void *proj, int64_t proj_stride, const void *
   if (proj_stride < static_cast<int64_t>(num_q_heads + num_kv_heads) * head_dim + num_q_heads) return TLF_E_SHAPE;
   if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
   if (n == 0) return TLF_OK;
-  if (!proj || !positions || (rot_dims && !cos_sin) || !slot_mapping || !q_out || !k_cache || !v_cache || !gate) return TLF_E_NULL;
+  if (int rc = partials_check(partials, scale, splits, dtype)) return rc;
+  if ((!proj && splits <= 1) || !positions || (rot_dims && !cos_sin) || !slot_mapping || !q_out || !k_cache || !v_cache || !gate) return TLF_E_NULL;
   if (!aligned16(q_out) || !aligned16(k_cache) || !aligned16(v_cache)) return TLF_E_ALIGN;
-  AttnPrepArgs a{proj, proj_stride, q_bias, k_bias, positions, cos_sin, max_pos, rot_dims, slot_mapping, num_slots,
+  AttnPrepArgs a{proj, Partials{partials, scale, n * proj_stride, static_cast<int32_t>(proj_stride), splits}, proj_stride, q_bias, k_bias, positions, cos_sin, max_pos, rot_dims, slot_mapping, num_slots,
                  q_out, k_cache, v_cache, gate, n, num_q_heads, num_kv_heads, head_dim, padded_dim, eps, 0};
-  a.vec = head_dim % 8 == 0 && proj_stride % 8 == 0 && aligned16(proj) && aligned16(q_bias) && aligned16(k_bias);
-  const int64_t items = static_cast<int64_t>(n) * (num_q_heads + num_kv_heads + 1);
-  const dim3 grid(static_cast<unsigned>((items + 15) / 16));
+  a.vec = head_dim % 8 == 0 && rot_dims % 8 == 0 && proj_stride % 8 == 0 && aligned16(proj) && aligned16(q_bias) &&
+          aligned16(k_bias) && aligned16(cos_sin) && (num_q_heads + num_kv_heads + 16) / 16 <= 65535;
+  if (splits > 1 && !a.vec) return TLF_E_UNSUPPORTED;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  if (dtype == TLF_DT_BF16) {
-    if (padded_dim <= 128) TLF_LAUNCH((attn_prep_kernel<unsigned short, 1>), grid, dim3(256), 0, s, a);
-    else TLF_LAUNCH((attn_prep_kernel<unsigned short, 2>), grid, dim3(256), 0, s, a);
-  } else {
-    if (padded_dim <= 128) TLF_LAUNCH((attn_prep_kernel<float, 1>), grid, dim3(256), 0, s, a);
-    else TLF_LAUNCH((attn_prep_kernel<float, 2>), grid, dim3(256), 0, s, a);
-  }
-  return launch_status();
+  return dtype == TLF_DT_BF16 ? launch_attn_prep<unsigned short>(a, s) : launch_attn_prep<float>(a, s);
 }
 
 extern "C" int tlf_pool_blocks(const void *k_cache, const void *v_cache, void *pk_cache, void *pv_cache,

@@ -22,6 +22,7 @@ class Replay:
         sched, runner = self.engine.scheduler, self.engine.model_runner
         limit = self.engine.config.max_model_len
         seqs = []
+        entries = [e for e in entries if e["tokens"]]
         for e in entries:
             tokens = e["tokens"]
             seq = self.live.get(e["id"])

@@ -33,7 +33,7 @@ class GatedLinearAttention(nn.Module):
         single = ctx.num_single
         weights = (self.decay_weight.data, self.decay_bias.data, self.norm.weight.data)
         if single:
-            ops.gla_decode(proj[:single], *weights, self.state, ctx.state_slots, positions[:single], self.tau, self.eps,
+            ops.gla_decode(proj if single == n else proj[:single], *weights, self.state, ctx.state_slots, positions[:single], self.tau, self.eps,
                            out[:single])
         if single < n:
             ops.gla_portions(proj[single:], *weights, self.state, ctx.state_slots, ctx.seq_starts, ctx.chunk_rows,

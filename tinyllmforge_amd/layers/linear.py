@@ -240,6 +240,15 @@ class StackedLinear(LinearBase):
     def forward(self, x: torch.Tensor) -> torch.Tensor:
         return super().forward(pad_columns(x, _round_up(self.input_size, 64)))
 
+    def forward_deferred(self, x: torch.Tensor):
+        """The same for a consumer that adds up partial sums itself (``ops.Deferred``); plain rows in 32-bit."""
+        if self.weight.dtype == torch.float32:
+            return self.forward(x)
+        x = pad_columns(x, _round_up(self.input_size, 64))
+        if self.is_quantized:
+            return ops.linear_deferred(x, self.pack_().qpacked, self.qscale)
+        return ops.linear_deferred(x, self.weight.data)
+
 
 class GatedUpLinear(MergedColumnParallelLinear):
     """gate and up projections of any size: the intermediate dim is padded to a multiple of 64 and the input to one of

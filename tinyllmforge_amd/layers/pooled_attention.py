@@ -25,6 +25,7 @@ class PooledWindowAttention(nn.Module):
         self.dtype = dtype
         self.register_buffer("cos_sin", rope, persistent=False)
         self.score_bias = nn.Parameter(torch.zeros(num_heads))
+        self.takes_partials = head_dim % 8 == 0 and rot_dims % 8 == 0    # the preparation may add up split projections
         self.kv = None                      # ops.PooledKV, bound by the model runner
 
     # -- what the model runner asks a layer with a paged cache

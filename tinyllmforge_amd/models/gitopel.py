@@ -15,6 +15,7 @@ from ..layers.gla import GatedLinearAttention
 from ..layers.grouped_norm import GroupedRMSNorm
 from ..layers.linear import GatedUpLinear, StackedLinear
 from ..layers.pooled_attention import PooledWindowAttention, interleaved_cos_sin
+from ..utils.context import get_context
 
 DEFAULT_RANK = 16     # rows of a gla layer's first decay factor when no checkpoint fixes them
 
@@ -33,8 +34,9 @@ class GitopelAttention(nn.Module):
 
     def forward(self, h, positions):
         """The output projection without its bias (the norm that follows adds it), and that bias."""
-        o = self.attn(self.qkg(h), self.q_bias.data, self.k_bias.data, positions)
-        return self.o(o), self.o_bias.data
+        project = self.qkg.forward_deferred if self.attn.takes_partials else self.qkg
+        o = self.attn(project(h), self.q_bias.data, self.k_bias.data, positions)
+        return self.o.forward_deferred(o), self.o_bias.data
 
     routes = {"q": ("qkg.weight", "q"), "k": ("qkg.weight", "k"), "g": ("qkg.weight", "g"), "o": ("o.weight", "o"),
               "q.b": ("q_bias", None), "k.b": ("k_bias", None), "o.b": ("o_bias", None), "pb": ("attn.score_bias", None)}
@@ -49,7 +51,9 @@ class GitopelGLA(nn.Module):
         self.o = StackedLinear(heads * dv, {"o": width})
 
     def forward(self, h, positions):
-        return self.o(self.gla(self.qkvgr(h), positions)), None
+        single = get_context().num_single == h.shape[0]      # the prompt kernels read rows, the decode kernel partial sums
+        proj = self.qkvgr.forward_deferred(h) if single else self.qkvgr(h)
+        return self.o.forward_deferred(self.gla(proj, positions)), None
 
     routes = {**{p: ("qkvgr.weight", p) for p in ("q", "k", "v", "g", "a1")}, "o": ("o.weight", "o"),
               "a2": ("gla.decay_weight", None), "a2.b": ("gla.decay_bias", None), "norm": ("gla.norm.weight", None)}
@@ -62,7 +66,7 @@ class GitopelMLP(nn.Module):
         self.down = StackedLinear(ff, {"down": width})
 
     def forward(self, h):
-        return self.down(self.gate_up.forward_silu_mul(h))
+        return self.down.forward_deferred(self.gate_up.forward_silu_mul(h))
 
     routes = {"gate": ("gate_up.weight", 0), "up": ("gate_up.weight", 1), "down": ("down.weight", "down")}
 

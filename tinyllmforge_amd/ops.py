@@ -545,15 +545,60 @@ def _opt(t):
     return t.data_ptr() if t is not None else None
 
 
+class Deferred:
+    """A bf16 projection ``[M, N]`` that may still be partial sums in the GEMM workspace (``splits > 1``): the very next
+    kernels that read it add them up.  ``rows()`` is the plain tensor."""
+    __slots__ = ("y", "partials", "splits", "scale", "shape", "dtype", "device")
+
+    def __init__(self, y, partials, splits, scale):
+        self.y, self.partials, self.splits, self.scale = y, partials, splits, scale
+        self.shape, self.dtype, self.device = y.shape, y.dtype, y.device
+
+    def rows(self):
+        assert self.splits == 1
+        return self.y
+
+
+def linear_deferred(x, w, scale=None) -> Deferred:
+    """``linear`` (``w`` bf16) or ``w8a16_linear`` (``w`` packed int8, ``scale``) without the kernel that adds partial sums."""
+    import ctypes
+    lib = _lib.load()
+    if scale is not None:
+        w = _packed(w)
+        _need(scale, torch.float32, "scale")
+    else:
+        _need(w, BF16, "w")
+        assert w.is_contiguous()
+    _need(x, BF16, "x")
+    assert x.dim() == 2 and x.stride(1) == 1
+    (M, K), N = x.shape, w.shape[0]
+    assert w.shape[1] == K
+    y = torch.empty(M, N, dtype=BF16, device=x.device)
+    ws = _workspace(lib.tlf_w8a16_gemm_workspace_bytes(M, N, K), x.device, "gemm")
+    splits = ctypes.c_int32(1)
+    check(lib.tlf_gemm_deferred(x.data_ptr(), x.stride(0), w.data_ptr(), _opt(scale), y.data_ptr(), M, N, K, ws.data_ptr(),
+                                ws.numel(), ctypes.addressof(splits), _stream()), "tlf_gemm_deferred")
+    return Deferred(y, ws, splits.value, scale)
+
+
+def _source(y):
+    """(row tensor, row stride, partials, splits, scale) of a tensor or a ``Deferred``."""
+    if isinstance(y, Deferred):
+        return y.y.data_ptr(), y.y.stride(0), y.partials.data_ptr(), y.splits, _opt(y.scale)
+    assert y.stride(1) == 1
+    return y.data_ptr(), y.stride(0), None, 1, None
+
+
 def group_rms_norm_add(y, y_bias, w_post, x, w_next, groups, eps):
     """In place ``x += norm(y + y_bias) * w_post`` (``x`` fp32 ``[N, W]``), then ``norm(x) * w_next`` in y's dtype."""
     lib = _lib.load()
-    _need(y, w_post.dtype, "y"); _need(x, torch.float32, "x"); _need(w_next, y.dtype, "w_next")
+    assert y.dtype == w_post.dtype
+    _need(x, torch.float32, "x"); _need(w_next, y.dtype, "w_next")
     rows, width = x.shape
-    assert y.shape[0] == rows and y.shape[1] >= width and y.stride(1) == 1 and x.is_contiguous()
+    assert y.shape[0] == rows and y.shape[1] >= width and x.is_contiguous()
     assert w_post.numel() == width and w_next.numel() == width and (y_bias is None or y_bias.numel() == width)
     h = torch.empty(rows, width, dtype=y.dtype, device=x.device)
-    check(lib.tlf_group_rmsnorm_add(y.data_ptr(), y.stride(0), _opt(y_bias), w_post.data_ptr(), x.data_ptr(),
+    check(lib.tlf_group_rmsnorm_add(*_source(y), _opt(y_bias), w_post.data_ptr(), x.data_ptr(),
                                     w_next.data_ptr(), h.data_ptr(), rows, width, groups, float(eps), _dt(y), _stream()),
           "tlf_group_rmsnorm_add")
     return h
@@ -576,14 +621,15 @@ def embed_group_rms_norm(ids, table, w_next, groups, eps):
 def attn_prep(proj, q_bias, k_bias, positions, cos_sin, rot_dims, slot_mapping, k_cache, v_cache, num_q_heads, head_dim, eps):
     """Biases, V store, interleaved RoPE, unit RMS, K store.  Returns ``(q [N, Hq, Dp], gate fp32 [N, Hq])``."""
     lib = _lib.load()
-    _need(proj, k_cache.dtype, "proj"); _need(positions, torch.int64, "positions"); _need(slot_mapping, torch.int32, "slot_mapping")
+    assert proj.dtype == k_cache.dtype
+    _need(positions, torch.int64, "positions"); _need(slot_mapping, torch.int32, "slot_mapping")
     n = proj.shape[0]
     pages, bs, hkv, dp = k_cache.shape
-    assert proj.stride(1) == 1 and positions.numel() == n and slot_mapping.numel() == n
+    assert positions.numel() == n and slot_mapping.numel() == n
     assert k_cache.is_contiguous() and v_cache.is_contiguous() and (rot_dims == 0 or cos_sin.shape[1] == rot_dims)
     q = torch.empty(n, num_q_heads, dp, dtype=proj.dtype, device=proj.device)
     gate = torch.empty(n, num_q_heads, dtype=torch.float32, device=proj.device)
-    check(lib.tlf_attn_prep(proj.data_ptr(), proj.stride(0), _opt(q_bias), _opt(k_bias), positions.data_ptr(),
+    check(lib.tlf_attn_prep(*_source(proj), _opt(q_bias), _opt(k_bias), positions.data_ptr(),
                             _opt(cos_sin), cos_sin.shape[0] if cos_sin is not None else 0, rot_dims,
                             slot_mapping.data_ptr(), pages * bs, q.data_ptr(), k_cache.data_ptr(), v_cache.data_ptr(),
                             gate.data_ptr(), n, num_q_heads, hkv, head_dim, dp, float(eps), _dt(proj), _stream()),
@@ -657,12 +703,13 @@ def pooled_attention_prefill(q, score_bias, gate, kv: PooledKV, block_tables, cu
 def gla_decode(proj, a2, a2_bias, norm_weight, state, state_slots, positions, tau, eps, out):
     """One token per row of ``proj``; ``state`` fp32 ``[slots, H, dk, dv]`` updated in place."""
     lib = _lib.load()
-    _need(proj, a2.dtype, "proj"); _need(state, torch.float32, "state"); _need(state_slots, torch.int32, "state_slots")
+    assert proj.dtype == a2.dtype
+    _need(state, torch.float32, "state"); _need(state_slots, torch.int32, "state_slots")
     slots, heads, dk, dv = state.shape
     rows = proj.shape[0]
-    assert proj.stride(1) == 1 and out.stride(1) == 1 and out.shape[0] == rows and state.is_contiguous()
+    assert out.stride(1) == 1 and out.shape[0] == rows and state.is_contiguous()
     assert a2.is_contiguous() and a2.shape[0] == heads * dk and state_slots.numel() >= rows and positions.numel() == rows
-    check(lib.tlf_gla_decode(proj.data_ptr(), proj.stride(0), a2.data_ptr(), a2_bias.data_ptr(), norm_weight.data_ptr(),
+    check(lib.tlf_gla_decode(*_source(proj), a2.data_ptr(), a2_bias.data_ptr(), norm_weight.data_ptr(),
                              state.data_ptr(), state_slots.data_ptr(), slots, positions.data_ptr(), out.data_ptr(),
                              out.stride(0), rows, heads, dk, dv, a2.shape[1], float(tau), dk ** -0.5, float(eps),
                              _dt(proj), _stream()), "tlf_gla_decode")
@@ -679,7 +726,7 @@ def gla_portions(proj, a2, a2_bias, norm_weight, state, state_slots, seq_starts,
     assert proj.stride(1) == 1 and out.stride(1) == 1 and out.shape[0] == rows and state.is_contiguous()
     assert a2.is_contiguous() and a2.shape[0] == heads * dk and cu_chunks.numel() == num_seqs + 1
     assert state_slots.numel() >= first_seq + num_seqs and chunk_lens.numel() == chunks
-    ws = _workspace(lib.tlf_gla_portions_workspace_bytes(rows, chunks, heads, dk, dv), proj.device, "gla")
+    ws = _workspace(lib.tlf_gla_portions_workspace_bytes(rows, chunks, num_seqs, heads, dk, dv), proj.device, "gla")
     check(lib.tlf_gla_portions(
         proj.data_ptr(), proj.stride(0), a2.data_ptr(), a2_bias.data_ptr(), norm_weight.data_ptr(), state.data_ptr(),
         state_slots.data_ptr(), slots, seq_starts.data_ptr(), chunk_rows.data_ptr(), chunk_lens.data_ptr(),
