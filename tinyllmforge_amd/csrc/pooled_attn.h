@@ -17,7 +17,13 @@ struct PooledCache {
   int32_t bs, pool, C, size;
   int32_t G, D, Dp;     // KV heads, head dimension, padded head dimension (a multiple of 32; pads hold zeros)
   int64_t pages;
+  int32_t bs_shift;     // log2 of bs, -1 if it is no power of two
 };
+inline void pooled_cache_finish(PooledCache &c) {
+  c.C = (c.bs + c.pool - 1) / c.pool;
+  c.bs_shift = (c.bs & (c.bs - 1)) == 0 ? __builtin_ctz(c.bs) : -1;
+}
+__device__ __forceinline__ int page_of(const PooledCache &c, int j) { return c.bs_shift >= 0 ? j >> c.bs_shift : j / c.bs; }
 
 // Blocks visible to position i.
 __device__ __forceinline__ int pooled_visible(int i, int size, int pool) {
@@ -26,13 +32,13 @@ __device__ __forceinline__ int pooled_visible(int i, int size, int pool) {
 }
 // Cache row (units of G * Dp elements) of token j and of block b; an unmapped page reads row 0 (never visible).
 __device__ __forceinline__ int64_t token_row(const PooledCache &c, const int32_t *bt, int j) {
-  const int pg = j / c.bs;
+  const int pg = page_of(c, j);
   const int64_t page = bt[pg];
   const bool ok = page >= 0 && page < c.pages;
   return ok ? page * c.bs + (j - pg * c.bs) : 0;
 }
 __device__ __forceinline__ int64_t block_row(const PooledCache &c, const int32_t *bt, int b) {
-  const int pg = (b * c.pool + c.pool - 1) / c.bs;
+  const int pg = page_of(c, b * c.pool + c.pool - 1);
   const int64_t page = bt[pg];
   const bool ok = page >= 0 && page < c.pages;
   return ok ? page * c.C + (b - (pg * c.bs) / c.pool) : 0;

@@ -440,10 +440,10 @@ extern "C" int tlf_pool_blocks(const void *k_cache, const void *v_cache, void *p
   if (num_seqs <= 0 || max_tokens <= 0) return num_seqs < 0 || max_tokens < 0 ? TLF_E_SHAPE : TLF_OK;
   if (num_seqs > 65535 || first_seq < 0) return TLF_E_SHAPE;
   PooledCache c{k_cache, v_cache, pk_cache, pv_cache, block_tables, bt_stride, block_size, pool, 0, window,
-                num_kv_heads, head_dim, (head_dim + 31) / 32 * 32, num_pages};
+                num_kv_heads, head_dim, (head_dim + 31) / 32 * 32, num_pages, -1};
   if (int rc = pooled_cache_check(c, dtype)) return rc;
   if (!cu_seqlens_q || !seq_starts) return TLF_E_NULL;
-  c.C = (block_size + pool - 1) / pool;
+  pooled_cache_finish(c);
   const int64_t items = static_cast<int64_t>(c.G) * 2 * (c.Dp / 8) * (max_tokens / pool + 1);
   const dim3 grid(static_cast<unsigned>((items + 255) / 256), num_seqs);
   hipStream_t s = static_cast<hipStream_t>(stream);
@@ -476,11 +476,11 @@ extern "C" int tlf_pooled_attn_rows(const void *q, const void *score_bias, const
   if (out_stride < static_cast<int64_t>(num_q_heads) * head_dim || max_len <= 0) return TLF_E_SHAPE;
   if (rows == 0) return TLF_OK;
   PooledCache c{k_cache, v_cache, pk_cache, pv_cache, block_tables, bt_stride, block_size, pool, 0, window,
-                num_kv_heads, head_dim, (head_dim + 31) / 32 * 32, num_pages};
+                num_kv_heads, head_dim, (head_dim + 31) / 32 * 32, num_pages, -1};
   if (int rc = pooled_cache_check(c, dtype)) return rc;
   if (!q || !score_bias || !gate || !positions || !slot_mapping || !out) return TLF_E_NULL;
   if (!aligned16(q)) return TLF_E_ALIGN;
-  c.C = (block_size + pool - 1) / pool;
+  pooled_cache_finish(c);
   RowsArgs a{c, q, score_bias, gate, positions, slot_mapping, row_seq, out, out_stride, static_cast<float *>(workspace),
              rows, num_q_heads, num_q_heads / num_kv_heads, 1, 1, pool_new, scale * kLog2e};
   const int gh = rows_heads_per_pass(a.group);

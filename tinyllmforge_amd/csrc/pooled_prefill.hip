@@ -236,11 +236,11 @@ extern "C" int tlf_pooled_attn_prefill(const void *q, const void *score_bias, co
   if (out_stride < static_cast<int64_t>(num_q_heads) * head_dim) return TLF_E_SHAPE;
   if (num_seqs == 0 || max_tokens == 0) return TLF_OK;
   PooledCache c{k_cache, v_cache, pk_cache, pv_cache, block_tables, bt_stride, block_size, pool, 0, window,
-                num_kv_heads, head_dim, (head_dim + 31) / 32 * 32, num_pages};
+                num_kv_heads, head_dim, (head_dim + 31) / 32 * 32, num_pages, -1};
   if (int rc = pooled_cache_check(c, TLF_DT_BF16)) return rc;
   if (!q || !score_bias || !gate || !cu_seqlens_q || !seq_starts || !out) return TLF_E_NULL;
   if (!aligned16(q)) return TLF_E_ALIGN;
-  c.C = (block_size + pool - 1) / pool;
+  pooled_cache_finish(c);
   const int dc = c.Dp / 32, ct = dc <= 4 ? 2 : 1, units = 64 * ct;
   PooledPrefillArgs a{c, static_cast<const unsigned short *>(q), static_cast<const unsigned short *>(score_bias), gate,
                       cu_seqlens_q, seq_starts, static_cast<unsigned short *>(out), out_stride, num_q_heads,
