@@ -516,7 +516,7 @@ int tlf_f32_argmax(const float *logits, int64_t row_stride, int64_t *out, int32_
  * Caches: k_cache / v_cache [num_pages, block_size, Hkv, Dp], pk_cache / pv_cache [num_pages, ceil(block_size / pool),
  * Hkv, Dp] with the same page numbers: block b is row b - (page * block_size) / pool of the page that holds its last
  * token (page = index in the sequence).  Dp = head_dim rounded up to a multiple of 32, pads are zeros.
- * block_size % 64 == 0, head_dim even and <= 256.
+ * block_size % 64 == 0, head_dim <= 256, rot_dims even.
  *
  * tlf_attn_prep: projection rows [q heads | k heads | one gate value per q head] -> biases (may be NULL) added;
  *   v row = the key so far; first rot_dims dimensions of q and k rotated pairwise (2 i, 2 i + 1) with

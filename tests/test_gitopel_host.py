@@ -285,7 +285,7 @@ def test_entry_points_reject_bad_arguments_on_the_host():
                                                    for n in ("y", "s", "p", "sp", "sc", "b", "w", "x", "n", "h", "rows", "width", "groups", "eps", "dt", "st")])
     assert norm(y=None) == -1 and norm(sp=3) == -1 and norm(p=a + 4, sp=3) == -3 and norm(p=a, sp=3, dt=1) == -5 and norm(groups=3) == -2 and norm(s=32) == -2 and norm(dt=7) == -5 and norm(rows=0) == 0
     assert lib.tlf_embed_group_rmsnorm(a, a, 0, a, a, a, 1, 64, 1, 1e-6, 0, None) == -2
-    assert lib.tlf_attn_prep(a, 100, None, 1, None, None, None, a, a, 10, 32, a, 64, a, a, a, a, 1, 1, 1, 33, 64, 1e-6, 0, None) == -2   # odd dim
+    assert lib.tlf_attn_prep(a, 100, None, 1, None, None, None, a, a, 10, 32, a, 64, a, a, a, a, 1, 1, 1, 300, 320, 1e-6, 0, None) == -2  # head too wide
     assert lib.tlf_attn_prep(a, 60, None, 1, None, None, None, a, a, 10, 32, a, 64, a, a, a, a, 1, 1, 1, 32, 32, 1e-6, 0, None) == -2    # row too short
     assert lib.tlf_attn_prep(a, 80, None, 1, None, None, None, a, a, 10, 32, a, 64, a, a, a, None, 1, 1, 1, 32, 32, 1e-6, 0, None) == -1
     rows = lambda bs=64, pool=4, win=8, ws=a, wsb=1 << 30, dim=32, n=2: lib.tlf_pooled_attn_rows(

@@ -60,7 +60,7 @@ def test_f32_dense_operations(M, N, K):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("H,G,D,rot", [(6, 2, 40, 24), (8, 8, 128, 128), (3, 1, 32, 0), (2, 1, 256, 64), (4, 2, 18, 18)])
+@pytest.mark.parametrize("H,G,D,rot", [(6, 2, 40, 24), (8, 8, 128, 128), (3, 1, 32, 0), (2, 1, 256, 64), (4, 2, 18, 18), (3, 3, 33, 20)])
 def test_attention_preparation(dtype, H, G, D, rot):
     from tinyllmforge_amd import ops as P
     from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
@@ -149,7 +149,7 @@ class Pages:
         return res
 
 
-ATTN = [(4, 2, 40, 37, 5), (8, 2, 64, 72, 16), (1, 1, 32, 1, 1), (6, 6, 96, 64, 64), (20, 1, 128, 130, 100), (3, 1, 256, 9, 3), (2, 2, 160, 200, 7)]
+ATTN = [(4, 2, 40, 37, 5), (8, 2, 64, 80, 16), (1, 1, 32, 1, 1), (6, 6, 96, 64, 64), (20, 1, 128, 130, 100), (3, 1, 256, 9, 3), (2, 2, 160, 200, 7), (4, 2, 27, 30, 6)]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)

@@ -414,7 +414,7 @@ extern "C" int tlf_attn_prep(const void *proj, int64_t proj_stride, const float 
                              float *gate, int32_t n, int32_t num_q_heads, int32_t num_kv_heads, int32_t head_dim,
                              int32_t padded_dim, float eps, int32_t dtype, void *stream) {
   using namespace tlf;
-  if (n < 0 || num_q_heads <= 0 || num_kv_heads <= 0 || head_dim <= 0 || head_dim % 2 || head_dim > 256) return TLF_E_SHAPE;
+  if (n < 0 || num_q_heads <= 0 || num_kv_heads <= 0 || head_dim <= 0 || head_dim > 256) return TLF_E_SHAPE;
   if (padded_dim != (head_dim + 31) / 32 * 32 || rot_dims < 0 || rot_dims % 2 || rot_dims > head_dim) return TLF_E_SHAPE;
   if (proj_stride < static_cast<int64_t>(num_q_heads + num_kv_heads) * head_dim + num_q_heads) return TLF_E_SHAPE;
   if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
