@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the per-token hot path on one MI355X.
 
-    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload e2e|decode_attn|gemm|all]
+    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload e2e|decode_attn|gemm|gitopel|...|all]
 
 Prints ONE JSON line.
 
