@@ -487,7 +487,7 @@ int tlf_probe_mix(const void *big, size_t big_bytes, const void *small_region, s
  * divided by its own sqrt(mean(part^2) + eps); the whole is multiplied by a weight.
  *
  *   tlf_group_rmsnorm_add:    x += norm(y + y_bias) * w_post;  h = norm(x) * w_next
- *   tlf_embed_group_rmsnorm:  x  = table[id];                  h = norm(x) * w_next
+ *   tlf_embed_group_rmsnorm:  x  = table[id];                  h = norm(x) * (w_next + w_offset)
  *
  * x fp32 [rows, width] contiguous; y, h, table, weights: dtype; y_bias may be NULL; w_next NULL: no h.
  * width / groups <= 16384.  An id outside [0, vocab) embeds as zeros. */
@@ -497,8 +497,8 @@ int tlf_group_rmsnorm_add(const void *y, int64_t y_stride, const float *partials
                           const void *y_bias, const void *w_post, float *x, const void *w_next, void *h, int32_t rows, int32_t width, int32_t groups, float eps,
                           int32_t dtype, void *stream);
 int tlf_embed_group_rmsnorm(const int64_t *ids, const void *table, int32_t vocab, float *x, const void *w_next,
-                            void *h, int32_t rows, int32_t width, int32_t groups, float eps, int32_t dtype,
-                            void *stream);
+                            float w_offset, void *h, int32_t rows, int32_t width, int32_t groups, float eps,
+                            int32_t dtype, void *stream);
 
 /* Dense operations of 32-bit mode (fp32 products and sums; any M, N, K): y = x . w^T, y = silu(x[:, :I]) * x[:, I:],
  * greedy argmax (first index among ties). */
@@ -585,6 +585,95 @@ int tlf_gla_portions(const void *proj, int64_t proj_stride, const void *a2, cons
                      int64_t out_stride, int32_t rows, int32_t heads, int32_t key_dim, int32_t value_dim,
                      int32_t rank, float tau, float q_scale, float eps, int32_t dtype, void *workspace,
                      size_t workspace_bytes, void *stream);
+
+/* Residual add with a multiplier and the next RMSNorm, for layers whose sublayers share one norm:
+ *   x += mult * (y + sum_k extra[extra_rows[row * top + k]], k < top);   h = x / rms(x) * (w_next + w_offset)
+ * (w_offset 1: a weight stored around zero; w_next NULL: no h.  y may be partial sums as above.) */
+int tlf_residual_rmsnorm(const void *y, int64_t y_stride, const float *partials, int32_t splits, const float *scale,
+                         const void *extra, int64_t extra_stride, const int32_t *extra_rows, int32_t top, float mult,
+                         float *x, const void *w_next, float w_offset, void *h, int32_t rows, int32_t width, float
+                         eps, int32_t dtype, void *stream);
+
+/* Latent attention: per token one cache row [latent: Ra | rotated key: Ta | 0] of Lp values for all heads, Ra and Ta being
+ * rank and rot_dim rounded up to 8 and Lp their sum rounded up to 64; head h's key is [Uk_h c | rotated part], its value
+ * Uv_h c.  Softmax over the `window` keys up to a position.  Query rows: [own part: Da | rotated: Ta | 0] of Dq values, Da =
+ * dim rounded up to 8, Dq the sum rounded up to 32.  rank <= 1536, dim, rot_dim, vdim <= 1024, Lp <= 2048.
+ *
+ * tlf_latent_prep: projection rows [q: heads * (dim + rot_dim), own part first in a head | ... | latent at latent_col: rank |
+ *   rot_dim] -> q_out [n, heads, Dq] with the rotated part turned pairwise (2 i, 2 i + 1) by cos_sin[pos] (cos of the pairs,
+ *   then sin), latent / rms * norm_weight and the turned key into the cache row slot_mapping[token] (negative: not stored).
+ * tlf_head_gemm: y[row, head] = W[head] x[row, head], W [heads, N, K]; N a multiple of 16, K of 32.  In rows below n_main
+ *   only the first k_main columns hold weights (n_main 0: all).
+ * tlf_latent_rows: absorbed attention, any rows in either dtype: q [rows, heads, Lp] = [Uk_h^T q_own | q_rot | 0]; writes
+ *   part [rows, heads, Rp] (Rp = Ra rounded up to 32), the unnormalised mix of latents, and ml [rows, heads, 2], maximum
+ *   (of score * log2 e) and denominator.  row_seq[r]: block-table row (NULL: r).
+ * tlf_latent_attn: the same on the matrix cores, bf16, Lp <= 576 (tlf_latent_attn_supported), keys cut into `splits` parts
+ *   (tlf_latent_attn_splits proposes a number): part [splits, rows, heads, Rp], ml [splits, rows, heads, 2].  With
+ *   cu_seqlens_q NULL sequence s is the single row s at positions[s] (slot_mapping[s] < 0: a padding row, no keys), otherwise
+ *   rows cu_seqlens_q[s] - first_row .. of q and part, sequences first_seq .. + num_seqs - 1, after seq_starts[s] cached tokens.
+ * tlf_latent_values: out[row, head] = Uv_h (sum of the splits / denominator); uv [heads, vdim rounded up to 16, Rp]; rows
+ *   without keys give 0.
+ * tlf_latent_gather: for the expanded form: cache rows of the keys that sequence first_seq + s sees in this step (from
+ *   position max(0, start - window + 1) on) as rows kv_offsets[s] .. kv_offsets[s + 1] - 1 of `out`; max_rows bounds them.
+ * tlf_latent_prefill: portions from expanded keys and values (rows [heads * Da | heads * Va], Va = vdim rounded up to 8) and
+ *   the gathered rows; bf16, Dq <= 256, vdim <= 128 (tlf_latent_prefill_supported). */
+int tlf_latent_prep(const void *proj, int64_t proj_stride, const float *partials, int32_t splits, const float *scale,
+                    int32_t latent_col, const void *norm_weight, const int64_t *positions, const float *cos_sin,
+                    int32_t max_pos, const int32_t *slot_mapping, int64_t num_slots, void *q_out, void *cache,
+                    int32_t n, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, float eps,
+                    int32_t dtype, void *stream);
+int tlf_head_gemm(const void *x, const void *w, void *y, int32_t rows, int32_t heads, int32_t N, int32_t K, int32_t
+                  n_main, int32_t k_main, int32_t dtype, void *stream);
+int tlf_latent_rows(const void *q, const void *cache, const int32_t *block_tables, int64_t bt_stride, const int64_t
+                    *positions, const int32_t *slot_mapping, const int32_t *row_seq, float *part, float *ml, int32_t
+                    rows, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, int32_t
+                    block_size, int32_t window, int64_t num_pages, float scale, int32_t dtype, void *stream);
+int tlf_latent_attn_splits(int32_t num_seqs, int32_t max_tokens, int32_t heads, int32_t window, int32_t max_len);
+int tlf_latent_attn_supported(int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim);
+int tlf_latent_attn(const void *q, const void *cache, const int32_t *block_tables, int64_t bt_stride, const int64_t
+                    *positions, const int32_t *slot_mapping, const int32_t *cu_seqlens_q, const int32_t *seq_starts,
+                    int32_t first_seq, int32_t first_row, int32_t num_seqs, int32_t max_tokens, float *part, float *ml, int32_t splits,
+                    int32_t rows, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, int32_t
+                    block_size, int32_t window, int64_t num_pages, float scale, void *stream);
+int tlf_latent_values(const float *part, const float *ml, int32_t splits, const void *uv, void *out, int64_t
+                      out_stride, int32_t rows, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t
+                      vdim, int32_t dtype, void *stream);
+int tlf_latent_gather(const void *cache, const int32_t *block_tables, int64_t bt_stride, const int32_t *cu_seqlens_q,
+                      const int32_t *seq_starts, const int32_t *kv_offsets, int32_t first_seq, int32_t num_seqs,
+                      int32_t max_rows, void *out, int32_t row_size, int32_t block_size, int32_t window, int64_t
+                      num_pages, void *stream);
+int tlf_latent_prefill_supported(int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim);
+int tlf_latent_prefill(const void *q, const void *expanded, int64_t expanded_stride, const void *latents, const
+                       int32_t *cu_seqlens_q, const int32_t *seq_starts, const int32_t *kv_offsets, int32_t
+                       first_seq, int32_t num_seqs, int32_t max_tokens, void *out, int64_t out_stride, int32_t heads,
+                       int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, int32_t window, float scale, void
+                       *stream);
+
+/* Mixture of experts.  Rows (token, k) are put in expert order; nothing on the host depends on the routing.
+ *
+ * tlf_moe_route: z = router h (router [experts rounded up to 16, K], K a multiple of 64; fp32 sums), ids[token, k] the `top`
+ *   largest (ties: the smaller index) and weights[token, k] = sigmoid(z).  experts <= 512.
+ * tlf_moe_group: row_of[token * top + k] = the entry's row in expert order, src[row] its token, row_weight[row] its weight;
+ *   tiles (int32 x 4: expert, first row, rows, 0) cut the rows into at most tile_rows of one expert each, *num_tiles <=
+ *   max_tiles of them; max_tiles >= n * top / tile_rows + min(experts, n * top).
+ * tlf_moe_gemm: y[row] = W[expert] x[x_rows ? x_rows[row] : row]; w [experts, N, K].  clipped_glu: channels are interleaved
+ *   as for the SiLU-and-mul products (8 gate, then the 8 matching up); with f = row_scale[row] (NULL: 1), g = min(f gate,
+ *   limit), u = clamp(f up, +-limit): y [rows, N / 2] = g sigmoid(1.702 g) (u + 1).  bf16: tile_rows 32 or 128, K a multiple
+ *   of 64; fp32: tile_rows 64.  x_count bounds the x rows.
+ * tlf_xielu: with a = softplus(pq[0]), b = 1/2 + softplus(pq[1]), out = a z^2 + z / 2 for z > 0, b (e^z - 1 - z) + z / 2
+ *   otherwise, z = columns col .. col + cols - 1 of x (or of partial sums); columns cols .. padded_cols - 1 become 0. */
+int tlf_moe_route(const void *h, int64_t h_stride, const void *router, int32_t *ids, float *weights, int32_t n,
+                  int32_t experts, int32_t K, int32_t top, int32_t dtype, void *stream);
+int tlf_moe_group(const int32_t *ids, const float *weights, int32_t *row_of, int32_t *src, float *row_weight, int32_t
+                  *tiles, int32_t *num_tiles, int32_t max_tiles, int32_t n, int32_t top, int32_t experts, int32_t
+                  tile_rows, void *stream);
+int tlf_moe_gemm(const void *x, int64_t x_stride, int32_t x_count, const void *w, void *y, const int32_t *tiles,
+                 const int32_t *num_tiles, int32_t max_tiles, int32_t tile_rows, const int32_t *x_rows, const float
+                 *row_scale, int32_t rows, int32_t N, int32_t K, int32_t clipped_glu, float limit, int32_t dtype,
+                 void *stream);
+int tlf_xielu(const void *x, int64_t x_stride, const float *partials, int32_t splits, const float *scale, int32_t
+              col, const void *pq, void *out, int64_t out_stride, int32_t rows, int32_t cols, int32_t padded_cols,
+              int32_t dtype, void *stream);
 
 #ifdef __cplusplus
 }

@@ -284,7 +284,7 @@ def test_entry_points_reject_bad_arguments_on_the_host():
     norm = lambda **k: lib.tlf_group_rmsnorm_add(*[{**dict(y=a, s=64, p=None, sp=1, sc=None, b=None, w=a, x=a, n=a, h=a, rows=2, width=64, groups=4, eps=1e-6, dt=0, st=None), **k}[n]
                                                    for n in ("y", "s", "p", "sp", "sc", "b", "w", "x", "n", "h", "rows", "width", "groups", "eps", "dt", "st")])
     assert norm(y=None) == -1 and norm(sp=3) == -1 and norm(p=a + 4, sp=3) == -3 and norm(p=a, sp=3, dt=1) == -5 and norm(groups=3) == -2 and norm(s=32) == -2 and norm(dt=7) == -5 and norm(rows=0) == 0
-    assert lib.tlf_embed_group_rmsnorm(a, a, 0, a, a, a, 1, 64, 1, 1e-6, 0, None) == -2
+    assert lib.tlf_embed_group_rmsnorm(a, a, 0, a, a, 0.0, a, 1, 64, 1, 1e-6, 0, None) == -2
     assert lib.tlf_attn_prep(a, 100, None, 1, None, None, None, a, a, 10, 32, a, 64, a, a, a, a, 1, 1, 1, 300, 320, 1e-6, 0, None) == -2  # head too wide
     assert lib.tlf_attn_prep(a, 60, None, 1, None, None, None, a, a, 10, 32, a, 64, a, a, a, a, 1, 1, 1, 32, 32, 1e-6, 0, None) == -2    # row too short
     assert lib.tlf_attn_prep(a, 80, None, 1, None, None, None, a, a, 10, 32, a, 64, a, a, a, None, 1, 1, 1, 32, 32, 1e-6, 0, None) == -1

@@ -70,7 +70,7 @@ SIGNATURES = {
     "tlf_embedding": (c_int32, [_P, _P, _P, _I32, _I32, _I32, _P]),
     "tlf_gemm_deferred": (c_int32, [_P, _I64, _P, _P, _P, _I32, _I32, _I32, _P, _SZ, _P, _P]),
     "tlf_group_rmsnorm_add": (c_int32, [_P, _I64, _P, _I32, _P, _P, _P, _P, _P, _P, _I32, _I32, _I32, _F, _I32, _P]),
-    "tlf_embed_group_rmsnorm": (c_int32, [_P, _P, _I32, _P, _P, _P, _I32, _I32, _I32, _F, _I32, _P]),
+    "tlf_embed_group_rmsnorm": (c_int32, [_P, _P, _I32, _P, _P, _F, _P, _I32, _I32, _I32, _F, _I32, _P]),
     "tlf_f32_gemm": (c_int32, [_P, _I64, _P, _P, _I32, _I32, _I32, _P]),
     "tlf_f32_silu_and_mul": (c_int32, [_P, _P, _I32, _I32, _P]),
     "tlf_f32_argmax": (c_int32, [_P, _I64, _P, _I32, _I32, _P]),
@@ -88,6 +88,27 @@ SIGNATURES = {
     "tlf_gla_portions_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32, _I32, _I32]),
     "tlf_gla_portions": (c_int32, [_P, _I64, _P, _P, _P, _P, _P, _I32, _P, _P, _P, _P, _I32, _I32, _I32, _P, _I64, _I32,
                                    _I32, _I32, _I32, _I32, _F, _F, _F, _I32, _P, _SZ, _P]),
+    "tlf_residual_rmsnorm": (c_int32, [_P, _I64, _P, _I32, _P, _P, _I64, _P, _I32, _F, _P, _P, _F, _P, _I32, _I32,
+                                       _F, _I32, _P]),
+    "tlf_latent_prep": (c_int32, [_P, _I64, _P, _I32, _P, _I32, _P, _P, _P, _I32, _P, _I64, _P, _P, _I32, _I32, _I32,
+                                  _I32, _I32, _I32, _F, _I32, _P]),
+    "tlf_head_gemm": (c_int32, [_P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _P]),
+    "tlf_latent_rows": (c_int32, [_P, _P, _P, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I32,
+                                  _I32, _I64, _F, _I32, _P]),
+    "tlf_latent_values": (c_int32, [_P, _P, _I32, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _P]),
+    "tlf_latent_gather": (c_int32, [_P, _P, _I64, _P, _P, _P, _I32, _I32, _I32, _P, _I32, _I32, _I32, _I64, _P]),
+    "tlf_latent_attn_splits": (c_int32, [_I32, _I32, _I32, _I32, _I32]),
+    "tlf_latent_attn_supported": (c_int32, [_I32, _I32, _I32, _I32, _I32]),
+    "tlf_latent_attn": (c_int32, [_P, _P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _P, _P, _I32, _I32, _I32, _I32,
+                                  _I32, _I32, _I32, _I32, _I32, _I64, _F, _P]),
+    "tlf_latent_prefill_supported": (c_int32, [_I32, _I32, _I32, _I32, _I32]),
+    "tlf_latent_prefill": (c_int32, [_P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P, _I64, _I32, _I32, _I32,
+                                     _I32, _I32, _I32, _F, _P]),
+    "tlf_moe_route": (c_int32, [_P, _I64, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P]),
+    "tlf_moe_group": (c_int32, [_P, _P, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P]),
+    "tlf_moe_gemm": (c_int32, [_P, _I64, _I32, _P, _P, _P, _P, _I32, _I32, _P, _P, _I32, _I32, _I32, _I32, _F, _I32,
+                               _P]),
+    "tlf_xielu": (c_int32, [_P, _I64, _P, _I32, _P, _I32, _P, _P, _I64, _I32, _I32, _I32, _I32, _P]),
     "tlf_probe_read": (c_int32, [_P, _SZ, _P, _P]),
     "tlf_probe_copy": (c_int32, [_P, _P, _SZ, _P]),
     "tlf_probe_mfma": (c_int32, [_P, c_int32, c_int32, _P]),

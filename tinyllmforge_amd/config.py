@@ -23,6 +23,8 @@ class ModelConfig:
     recurrent = False        # some layers carry a per-sequence state besides the KV cache
     float32 = False          # the design's kernels exist in 32-bit
     position_quirk = True    # the reference's decode position (len instead of len - 1) applies
+    long_portion = None      # portions of at least this many tokens run a form of attention of their own
+    windows = ()             # the distinct attention windows of that form
     hidden_size: int
     num_hidden_layers: int
     num_attention_heads: int
@@ -57,14 +59,8 @@ class ModelConfig:
 
 
 @dataclass
-class GitopelConfig:
-    """A Gitopel model: a list of layers, each with its own mixer ('attention' or 'gla') and sizes.
-
-    Keys of ``config.json``: ``vocab``, ``width``, ``norm`` (``groups``, ``eps``) and ``layers``; a layer has ``type``,
-    ``mixer`` and ``mlp`` (``kind``, ``ff``, or null).  ``mixer`` of an attention layer: ``heads``, ``kv_heads``, ``dim``,
-    ``vdim``, ``scale``, ``rot`` (``dims``, ``base``), ``mask`` (``size``, ``pool``); of a gla layer: ``heads``, ``dim``,
-    ``vdim``, ``tau``.  The rank of a gla layer's decay projection is not in the file: it is the row count of its
-    first factor (``mixer["rank"]`` once known, 16 if no checkpoint says otherwise)."""
+class LayeredConfig:
+    """A design whose ``config.json`` lists its layers one by one, each with its own mixer, sizes and feed-forward."""
     vocab: int
     width: int
     norm: dict
@@ -73,24 +69,20 @@ class GitopelConfig:
     max_position_embeddings: int | None = None    # no limit of its own: the engine's max_model_len
 
     portioned = True
-    recurrent = True
+    recurrent = False
     float32 = True
     position_quirk = False
     tie_word_embeddings = False
+    long_portion = None
+    windows = ()
 
     def __post_init__(self):
         if isinstance(self.torch_dtype, str):
             self.torch_dtype = getattr(torch, self.torch_dtype.replace("torch.", ""))
-        assert self.width % self.norm["groups"] == 0
-        for layer in self.layers:
-            m = layer["mixer"]
-            if layer["type"] == "attention":
-                assert m["heads"] % m["kv_heads"] == 0
-                assert m["vdim"] == m["dim"], "the values are the keys: one size"
-                assert m["rot"]["dims"] <= m["dim"] and m["mask"]["size"] >= 1 and m["mask"]["pool"] >= 1
-            else:
-                assert layer["type"] == "gla", f"unknown mixer {layer['type']!r}"
-            assert not layer.get("mlp") or layer["mlp"]["kind"] == "dense"
+        self.check_layers()
+
+    def check_layers(self):
+        raise NotImplementedError
 
     @property
     def hidden_size(self) -> int:
@@ -105,16 +97,69 @@ class GitopelConfig:
         return len(self.layers)
 
     @classmethod
-    def from_dict(cls, src: dict, directory: str | None = None) -> "GitopelConfig":
+    def from_dict(cls, src: dict, directory: str | None = None):
         import copy
         names = {f.name for f in fields(cls)}
-        cfg = cls(**{k: copy.deepcopy(v) for k, v in src.items() if k in names})
+        return cls(**{k: copy.deepcopy(v) for k, v in src.items() if k in names})
+
+
+@dataclass
+class GitopelConfig(LayeredConfig):
+    """A Gitopel model: a list of layers, each with its own mixer ('attention' or 'gla') and sizes.
+
+    Keys of ``config.json``: ``vocab``, ``width``, ``norm`` (``groups``, ``eps``) and ``layers``; a layer has ``type``,
+    ``mixer`` and ``mlp`` (``kind``, ``ff``, or null).  ``mixer`` of an attention layer: ``heads``, ``kv_heads``, ``dim``,
+    ``vdim``, ``scale``, ``rot`` (``dims``, ``base``), ``mask`` (``size``, ``pool``); of a gla layer: ``heads``, ``dim``,
+    ``vdim``, ``tau``.  The rank of a gla layer's decay projection is not in the file: it is the row count of its
+    first factor (``mixer["rank"]`` once known, 16 if no checkpoint says otherwise)."""
+    recurrent = True
+
+    def check_layers(self):
+        assert self.width % self.norm["groups"] == 0
+        for layer in self.layers:
+            m = layer["mixer"]
+            if layer["type"] == "attention":
+                assert m["heads"] % m["kv_heads"] == 0
+                assert m["vdim"] == m["dim"], "the values are the keys: one size"
+                assert m["rot"]["dims"] <= m["dim"] and m["mask"]["size"] >= 1 and m["mask"]["pool"] >= 1
+            else:
+                assert layer["type"] == "gla", f"unknown mixer {layer['type']!r}"
+            assert not layer.get("mlp") or layer["mlp"]["kind"] == "dense"
+
+    @classmethod
+    def from_dict(cls, src: dict, directory: str | None = None) -> "GitopelConfig":
+        cfg = super().from_dict(src)
         if directory is not None:
             shapes = tensor_shapes(directory)
             for i, layer in enumerate(cfg.layers):
                 if layer["type"] == "gla":
                     layer["mixer"].setdefault("rank", shapes[f"l{i}.mix.a1"][0])
         return cfg
+
+
+@dataclass
+class GigopelConfig(LayeredConfig):
+    """A Gigopel model: parallel layers of windowed latent attention beside a dense or a mixture-of-experts feed-forward.
+
+    Keys of ``config.json``: ``vocab``, ``width``, ``residual_mult``, ``norm`` (``eps``) and ``layers``; a layer has
+    ``type`` ('latent_attention'), ``mixer`` (``heads``, ``dim``, ``rot_dim``, ``vdim``, ``kv_rank``, ``scale``, ``rot``:
+    ``dims``, ``base``, ``mask``: ``size``) and ``mlp``: null, ``kind`` 'dense' with ``ff``, or ``kind`` 'moe' with
+    ``expert`` (``ff``, ``limit``) and ``router`` (``experts``, ``top``)."""
+    residual_mult: float = 1.0
+
+    # from about this many tokens on it costs less to expand the keys and values of every head than to attend in the
+    # latent space (2 rank + rot_dim instead of dim + rot_dim + vdim products per head, query and key)
+    long_portion = 128
+
+    def check_layers(self):
+        for layer in self.layers:
+            assert layer["type"] == "latent_attention", f"unknown mixer {layer['type']!r}"
+            m, mlp = layer["mixer"], layer.get("mlp")
+            assert m["rot"]["dims"] == m["rot_dim"] and m["rot_dim"] % 2 == 0 and m["mask"]["size"] >= 1
+            assert not mlp or mlp["kind"] in ("dense", "moe")
+            if mlp and mlp["kind"] == "moe":
+                assert 1 <= mlp["router"]["top"] <= mlp["router"]["experts"]
+        self.windows = tuple(sorted({layer["mixer"]["mask"]["size"] for layer in self.layers}))
 
 
 def tensor_shapes(directory: str) -> dict:
@@ -128,6 +173,9 @@ def tensor_shapes(directory: str) -> dict:
     return out
 
 
+LAYERED_DESIGNS = {"Gitopel": GitopelConfig, "Gigopel": GigopelConfig}
+
+
 def architecture_of(src: dict) -> str:
     """The design a ``config.json`` names: ``architecture``, or the first of ``architectures``; Qwen3 when it names none."""
     name = src.get("architecture") or (src.get("architectures") or ["Qwen3ForCausalLM"])[0]
@@ -136,7 +184,7 @@ def architecture_of(src: dict) -> str:
 
 def model_config(src):
     """Configuration object from a configuration object, a dict of its keys or a checkpoint directory."""
-    if isinstance(src, (ModelConfig, GitopelConfig)):
+    if isinstance(src, (ModelConfig, LayeredConfig)):
         return src
     directory = None
     if isinstance(src, str):
@@ -144,8 +192,8 @@ def model_config(src):
         with open(os.path.join(src, "config.json")) as f:
             src = json.load(f)
     name = architecture_of(src)
-    if name == "Gitopel":
-        return GitopelConfig.from_dict(src, directory)
+    if name in LAYERED_DESIGNS:
+        return LAYERED_DESIGNS[name].from_dict(src, directory)
     if name == "Qwen3":
         return ModelConfig.from_any(src)
     raise ValueError(f"no model of this framework has the architecture {name!r}")

@@ -168,9 +168,12 @@ namespace tlf {
 // pipeline over its own 1/KG of the K range in its own LDS stages and the sets' accumulators are
 // summed through LDS at the end.  A latency-bound problem (few tiles, long K) then takes 1/KG of
 // the steps without partial sums in global memory.
-template <int BN, int BM, int WAVES_N, int WAVES_M, bool W8, int NS, int OCC, int KG>
+// GROUPED: the rows of y are grouped by expert and every expert has a weight of its own; a tile row comes from a list
+// the device made (which expert, which rows), and an x row may come through an index.
+template <int BN, int BM, int WAVES_N, int WAVES_M, bool W8, int NS, int OCC, int KG, bool GROUPED = false>
 __global__ __launch_bounds__(WAVES_N * WAVES_M * KG * 64) __attribute__((amdgpu_waves_per_eu(OCC, 8)))
-void gemm_dlds_kernel(const GemmParams p) {
+void gemm_dlds_kernel(const GemmParams params) {
+  std::conditional_t<GROUPED, GemmParams, const GemmParams &> p = params;
   static_assert(NS >= 2 && NS <= 8, "2 to 8 stages");
   constexpr int NW = WAVES_N * WAVES_M;       // waves of one set
   static_assert(NW == 2 || NW == 4 || NW == 8, "2, 4 or 8 waves");  // 8: two waves share each SIMD (not faster in the sweeps)
@@ -225,7 +228,15 @@ void gemm_dlds_kernel(const GemmParams p) {
   const int mt = p.xcd_rows ? owned : across;
   const int nt = p.xcd_rows ? across : owned;
   if (nt >= p.n_tiles || mt >= p.m_tiles) return;
-  const int n0 = nt * BN, m0 = mt * BM;
+  const int n0 = nt * BN;
+  int m0 = mt * BM;
+  if constexpr (GROUPED) {
+    if (mt >= *p.g.num_tiles) return;
+    const int4 tile = p.g.tiles[mt];  // expert, first row, rows
+    m0 = tile.y;
+    p.M = tile.y + tile.z;
+    p.w += tile.x * p.g.w_bytes;
+  }
   const int split = blockIdx.y;
   const int tid = threadIdx.x;
   const int lane = tid & 63;
@@ -242,7 +253,8 @@ void gemm_dlds_kernel(const GemmParams p) {
 
   // copy side: byte offset of this lane's piece for each pass, relative to the tile's first row
   // (rows past the end are clamped to the last row; their results are never stored)
-  const unsigned char *xbase = p.x + m0 * p.ldx_bytes + static_cast<int64_t>(k_begin) * 2;
+  const bool indexed = GROUPED && p.g.x_rows != nullptr;
+  const unsigned char *xbase = p.x + (indexed ? 0 : m0 * p.ldx_bytes) + static_cast<int64_t>(k_begin) * 2;
   // int8 weights are in tile order: the tile's first 32-row group and the K term (1 KiB chunks of 32) make the
   // 64-bit base, woff counts row groups from there (a weight may exceed 2 GiB; a tile never does)
   const unsigned char *wbase = W8 ? p.w + (static_cast<int64_t>(n0 >> 5) * (p.K / 32) + k_begin / 32) * 1024
@@ -253,7 +265,8 @@ void gemm_dlds_kernel(const GemmParams p) {
     const int piece = (lane & 7) ^ ((rl >> 1) & 7);
 #pragma unroll
     for (int q = 0; q < XP; ++q) {
-      const int row = min(m0 + q * (NW * 8) + rl, p.M - 1) - m0;
+      const int at = min(m0 + q * (NW * 8) + rl, p.M - 1);
+      const int row = indexed ? p.g.x_rows[at] : at - m0;
       xoff[q] = static_cast<unsigned int>(row * p.ldx_bytes + piece * 16);
     }
     if constexpr (W8) {
@@ -356,6 +369,12 @@ void gemm_dlds_kernel(const GemmParams p) {
         for (int j = 0; j < TM; ++j)
 #pragma unroll
           for (int v = 0; v < 16; ++v) acc[i][j][v] += src[((i * TM + j) * 16 + v) * (NW * 64)];
+    }
+  }
+  if constexpr (GROUPED) {
+    if (p.act == 3) {
+      gemm_epilogue_clipped_glu<TN, TM, WN, WM>(p, acc, m0, n0, wn, wm, r, kg);
+      return;
     }
   }
   gemm_epilogue<TN, TM, WN, WM, W8>(p, acc, m0, n0, wn, wm, r, kg, split);
@@ -1560,6 +1579,40 @@ int launch_gemm(const void *x, int64_t x_stride, const void *w, const float *sca
     rc = launch_status();
   }
   return rc;
+}
+
+// Grouped product (bf16): rows in expert order, tiles of `bm` rows of one expert each.  Few rows per expert: narrow tiles
+// and wave sets that split K, because the weights stream from HBM; many: the 128 x 128 tile.
+int launch_grouped(GemmParams p, int bm, hipStream_t stream) {
+  if (p.N % 16 || p.K % kBK || p.m_tiles <= 0) return TLF_E_SHAPE;
+  const int ktiles = p.K / kBK;
+  const int kg = bm == 32 ? (ktiles % 4 == 0 ? 4 : ktiles % 2 == 0 ? 2 : 1) : 1;
+  const int bn = bm == 32 ? 64 : 128;
+  p.splits = 1;
+  p.k_per_split = p.K;
+  p.n_tiles = (p.N + bn - 1) / bn;
+  p.xcd_rows = 0;
+  const int each = p.n_tiles / 8;
+  p.group_n = p.m_tiles >= 8 && each > 0 ? (each % 4 == 0 ? 4 : each % 3 == 0 ? 3 : each % 2 == 0 ? 2 : 1) : 1;
+  p.map_full = each * 8;
+  p.map_rem = p.n_tiles - p.map_full;
+  p.map_main = each * 8 * p.m_tiles;
+  const int64_t wgs = p.map_main + static_cast<int64_t>(p.map_rem) * p.m_tiles;
+  if (p.map_rem == 0) p.map_rem = 1;
+  if (wgs > (1 << 30)) return TLF_E_SHAPE;
+  const dim3 grid(static_cast<unsigned>(wgs));
+#define TLF_GROUPED(BN_, BM_, WN_, WM_, NS_, OCC_, KG_)                                                             \
+  TLF_LAUNCH((gemm_dlds_kernel<BN_, BM_, WN_, WM_, false, NS_, OCC_, KG_, true>), grid, dim3(WN_ * WM_ * KG_ * 64), \
+             0, stream, p)
+  if (bm == 32) {
+    if (kg == 4) TLF_GROUPED(64, 32, 2, 1, 2, 4, 4);
+    else if (kg == 2) TLF_GROUPED(64, 32, 2, 1, 3, 4, 2);
+    else TLF_GROUPED(64, 32, 2, 1, 4, 4, 1);
+  } else {
+    TLF_GROUPED(128, 128, 2, 2, 3, 2, 1);
+  }
+#undef TLF_GROUPED
+  return launch_status();
 }
 
 inline size_t align256(size_t n) { return (n + 255) & ~static_cast<size_t>(255); }

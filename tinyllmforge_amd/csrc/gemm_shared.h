@@ -18,6 +18,16 @@ __device__ __forceinline__ uint2 cvt4_i8_bf16(unsigned int w) {
   return make_uint2(pack_bf16x2(f0, f1), pack_bf16x2(f2, f3));
 }
 
+// Rows grouped by expert (device memory, made by tlf_moe_group)
+struct GroupedRows {
+  const int4 *tiles;          // per tile row: expert, first row, rows
+  const int32_t *num_tiles;
+  const int32_t *x_rows;      // x row of every row, NULL: the rows themselves
+  const float *row_scale;     // factor of every row of the product (clipped-GLU epilogue)
+  int64_t w_bytes;            // from one expert's weight to the next
+  float limit;
+};
+
 struct GemmParams {
   const unsigned char *x;
   int64_t ldx_bytes;
@@ -36,9 +46,17 @@ struct GemmParams {
   int32_t map_rem;  // the rest of them (1 ... 7; 1 when there is none): their tiles follow, dealt out one by one
   int32_t act;      // 1: SiLU-and-mul epilogue over interleaved gate/up channels, y is [M, N/2]
                     // 2: greedy-sample epilogue, nothing but argmax keys [M, amax_parts] is stored
+                    // 3: clipped-GLU epilogue over interleaved gate/up channels, y is [M, N/2]
   unsigned long long *amax;
   int32_t amax_parts;  // key columns per token: one per (N-tile, wave along N)
+  GroupedRows g;
 };
+
+// Clipped GLU with a factor on the products: g = min(f gate, limit), u = clamp(f up, +-limit), g sigmoid(1.702 g) (u + 1).
+__device__ __forceinline__ float clipped_glu(float gate, float up, float factor, float limit) {
+  const float g = fminf(gate * factor, limit), u = fminf(fmaxf(up * factor, -limit), limit);
+  return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
+}
 
 // Epilogue of the tiled kernel (BN output channels x BM tokens per workgroup, waves laid out as
 // WAVES_N x WAVES_M): scale (W8), round once to bf16, 8-byte stores; or fp32 partials when K is
@@ -193,6 +211,36 @@ __device__ __forceinline__ void gemm_epilogue_sc(const GemmParams &p, floatx16 (
           *reinterpret_cast<uint4 *>(p.y + static_cast<int64_t>(m) * p.N + n) =
               make_uint4(st[2 * h].x, st[2 * h].y, st[2 * h + 1].x, st[2 * h + 1].y);
       }
+    }
+  }
+}
+
+// Clipped GLU over interleaved gate/up channels (8 gate rows, then the 8 matching up rows), factor per row.
+template <int TN, int TM, int WN, int WM>
+__device__ __forceinline__ void gemm_epilogue_clipped_glu(const GemmParams &p, floatx16 (&acc)[TN][TM], int m0, int n0,
+                                                          int wn, int wm, int r, int kg) {
+#pragma unroll
+  for (int j = 0; j < TM; ++j) {
+    const int m = m0 + wm * WM + j * 32 + r;
+    const bool m_ok = m < p.M;
+    const float factor = m_ok && p.g.row_scale ? p.g.row_scale[m] : 1.0f;
+#pragma unroll
+    for (int i = 0; i < TN; ++i) {
+      uint2 st[2];
+#pragma unroll
+      for (int q = 0; q < 4; q += 2) {
+        float o[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] = clipped_glu(acc[i][j][q * 4 + e], acc[i][j][(q + 1) * 4 + e], factor, p.g.limit);
+        st[q / 2] = make_uint2(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]));
+      }
+      // lanes r and r + 32 hold 4 channels each of two groups of 8: one exchange makes 8 consecutive channels per lane
+      auto rx = __builtin_amdgcn_permlane32_swap(st[0].x, st[1].x, false, false);
+      auto ry = __builtin_amdgcn_permlane32_swap(st[0].y, st[1].y, false, false);
+      const int nfirst = n0 + wn * WN + i * 32;
+      if (m_ok && nfirst + kg * 16 < p.N)
+        *reinterpret_cast<uint4 *>(p.y + static_cast<int64_t>(m) * (p.N / 2) + nfirst / 2 + kg * 8) =
+            make_uint4(rx[0], ry[0], rx[1], ry[1]);
     }
   }
 }

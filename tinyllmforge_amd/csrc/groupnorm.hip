@@ -3,7 +3,9 @@
 //
 //   mode embed:  x = table[id];                              h = norm(x) * w_next
 //   mode add:    x = x + norm(y + y_bias) * w_post;           h = norm(x) * w_next
+//   mode plain:  x = x + mult * (y + sum of extra rows);      h = norm(x) * (w_next + w_offset)
 //
+// (w_offset 1: a weight stored around zero.  The extra rows are a mixture of experts' results, found through an index.)
 // The norm after a sublayer, the residual add and the norm in front of the next sublayer share their grouping, so a
 // (row, group) pair is one independent unit: the three steps are one pass over memory.  HBM bound: y and x are read
 // once, x and h written once.  The residual is fp32; y, h and the weights are T (bf16 or fp32); arithmetic is fp32.
@@ -23,6 +25,11 @@ struct GroupNormArgs {
   float *x;             // [rows, width] fp32 residual, updated in place
   const void *w_next;   // [width] or NULL: no h
   void *h;              // [rows, width]
+  const void *extra;    // [*, extra_stride] or NULL: rows extra_rows[row * top + k], k < top (plain mode)
+  const int32_t *extra_rows;
+  int64_t extra_stride;
+  int32_t top;
+  float mult, w_offset;
   int64_t units;        // rows * groups
   int32_t width, groups, cols;
   float eps;
@@ -56,7 +63,7 @@ __device__ __forceinline__ void stv(T *p, const float (&f)[VEC]) {
   else Elem<T>::st(p, f[0]);
 }
 
-// MODE 0: embed, 1: add, 2: add with y as partial sums
+// MODE 0: embed, 1: add, 2: add with y as partial sums, 3: plain, 4: plain with y as partial sums
 template <typename T, int VEC, int TPR, int MAXC, int MODE>
 __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
   __shared__ float part[4];
@@ -82,6 +89,31 @@ __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
       for (int i = 0; i < VEC; ++i) v[c][i] = 0.f;
       if (ch < nch && ok) ldv<T, VEC>(src + ch * VEC, v[c]);
     }
+  } else if constexpr (MODE >= 3) {
+    const T *yr = MODE == 3 ? static_cast<const T *>(a.y) + row * a.y_stride + col0 : nullptr;
+    float xo[MAXC][VEC];
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c) {
+      const int at = min(sub + c * TPR, nch - 1) * VEC;
+      if constexpr (MODE == 3) ldv<T, VEC>(yr + at, v[c]);
+      else if constexpr (VEC == 8) a.part.ld8(row, col0 + at, v[c]);
+      else v[c][0] = a.part.ld(row, col0 + at);
+      ldv<float, VEC>(xr + at, xo[c]);
+    }
+    for (int k = 0; k < a.top; ++k) {
+      const T *er = static_cast<const T *>(a.extra) + a.extra_rows[row * a.top + k] * a.extra_stride + col0;
+#pragma unroll
+      for (int c = 0; c < MAXC; ++c) {
+        float f[VEC];
+        ldv<T, VEC>(er + min(sub + c * TPR, nch - 1) * VEC, f);
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) v[c][i] += f[i];
+      }
+    }
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) v[c][i] = fmaf(v[c][i], a.mult, xo[c][i]);
   } else {
     const T *yr = MODE == 1 ? static_cast<const T *>(a.y) + row * a.y_stride + col0 : nullptr;
     const T *wp = static_cast<const T *>(a.w_post) + col0;
@@ -140,7 +172,7 @@ __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
       float w[VEC];
       ldv<T, VEC>(wn + ch * VEC, w);
 #pragma unroll
-      for (int i = 0; i < VEC; ++i) w[i] = v[c][i] * inv * w[i];
+      for (int i = 0; i < VEC; ++i) w[i] = v[c][i] * inv * (w[i] + a.w_offset);
       stv<T, VEC>(hr + ch * VEC, w);
     }
   }
@@ -168,7 +200,8 @@ int launch_groupnorm(const GroupNormArgs &a, bool vec8, hipStream_t stream) {
   return launch_status();
 }
 
-template <bool EMBED>
+// kMode 0: embed, 1: add, 3: plain
+template <int kMode>
 int groupnorm_entry(GroupNormArgs &a, int32_t rows, int32_t dtype, hipStream_t stream) {
   if (rows < 0 || a.width <= 0 || a.groups <= 0 || a.width % a.groups) return TLF_E_SHAPE;
   if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
@@ -178,12 +211,13 @@ int groupnorm_entry(GroupNormArgs &a, int32_t rows, int32_t dtype, hipStream_t s
   if (a.cols > 16384) return TLF_E_SHAPE;
   a.units = static_cast<int64_t>(rows) * a.groups;
   bool vec8 = a.cols % 8 == 0 && aligned16(a.x) && aligned16(a.w_next) && aligned16(a.h);
-  if (EMBED)
+  if (kMode == 0)
     vec8 = vec8 && aligned16(a.table);
   else
     vec8 = vec8 && aligned16(a.y) && aligned16(a.y_bias) && aligned16(a.w_post) && a.y_stride % 8 == 0;
-  constexpr int kMode = EMBED ? 0 : 1;
-  if (!EMBED && a.part.splits > 1) return launch_groupnorm<unsigned short, 2>(a, vec8, stream);
+  if (kMode == 3) vec8 = vec8 && aligned16(a.extra) && a.extra_stride % 8 == 0;
+  if constexpr (kMode != 0)
+    if (a.part.splits > 1) return launch_groupnorm<unsigned short, kMode + 1>(a, vec8, stream);
   return dtype == TLF_DT_BF16 ? launch_groupnorm<unsigned short, kMode>(a, vec8, stream)
                               : launch_groupnorm<float, kMode>(a, vec8, stream);
 }
@@ -201,16 +235,32 @@ extern "C" int tlf_group_rmsnorm_add(const void *y, int64_t y_stride, const floa
   a.part = tlf::Partials{partials, scale, rows * y_stride, static_cast<int32_t>(y_stride), splits};
   a.y = y; a.y_stride = y_stride; a.y_bias = y_bias; a.w_post = w_post; a.x = x; a.w_next = w_next; a.h = h;
   a.width = width; a.groups = groups; a.eps = eps;
-  return tlf::groupnorm_entry<false>(a, rows, dtype, static_cast<hipStream_t>(stream));
+  return tlf::groupnorm_entry<1>(a, rows, dtype, static_cast<hipStream_t>(stream));
 }
 
 extern "C" int tlf_embed_group_rmsnorm(const int64_t *ids, const void *table, int32_t vocab, float *x,
-                                       const void *w_next, void *h, int32_t rows, int32_t width, int32_t groups,
-                                       float eps, int32_t dtype, void *stream) {
+                                       const void *w_next, float w_offset, void *h, int32_t rows, int32_t width,
+                                       int32_t groups, float eps, int32_t dtype, void *stream) {
   tlf::GroupNormArgs a{};
   if (rows > 0 && (!ids || !table)) return TLF_E_NULL;
   if (vocab <= 0) return TLF_E_SHAPE;
+  a.w_offset = w_offset;
   a.ids = ids; a.table = table; a.vocab = vocab; a.x = x; a.w_next = w_next; a.h = h;
   a.width = width; a.groups = groups; a.eps = eps;
-  return tlf::groupnorm_entry<true>(a, rows, dtype, static_cast<hipStream_t>(stream));
+  return tlf::groupnorm_entry<0>(a, rows, dtype, static_cast<hipStream_t>(stream));
+}
+
+extern "C" int tlf_residual_rmsnorm(const void *y, int64_t y_stride, const float *partials, int32_t splits,
+                                    const float *scale, const void *extra, int64_t extra_stride, const int32_t *extra_rows,
+                                    int32_t top, float mult, float *x, const void *w_next, float w_offset, void *h,
+                                    int32_t rows, int32_t width, float eps, int32_t dtype, void *stream) {
+  tlf::GroupNormArgs a{};
+  if (int rc = tlf::partials_check(partials, scale, splits, dtype)) return rc;
+  if (rows > 0 && ((!y && splits <= 1) || (top > 0 && (!extra || !extra_rows)))) return TLF_E_NULL;
+  if (y_stride < width || top < 0 || (top > 0 && extra_stride < width)) return TLF_E_SHAPE;
+  a.part = tlf::Partials{partials, scale, rows * y_stride, static_cast<int32_t>(y_stride), splits};
+  a.y = y; a.y_stride = y_stride; a.x = x; a.w_next = w_next; a.h = h;
+  a.extra = extra; a.extra_stride = extra_stride; a.extra_rows = extra_rows; a.top = top; a.mult = mult; a.w_offset = w_offset;
+  a.width = width; a.groups = 1; a.eps = eps;
+  return tlf::groupnorm_entry<3>(a, rows, dtype, static_cast<hipStream_t>(stream));
 }

@@ -79,14 +79,23 @@ def decode_inputs(seqs, block_size: int, position_quirk: bool = True) -> dict:
 CHUNK = 16    # tokens per chunk of the recurrent layers' prompt kernels
 
 
-def portion_inputs(seqs, block_size: int) -> dict:
+def portion_kind(tokens: int, long_portion: int | None) -> int:
+    """Order of a step's sequences: single tokens, short portions, long portions (all portions without ``long_portion``)."""
+    return 0 if tokens == 1 else 1 if long_portion is not None and tokens < long_portion else 2
+
+
+def portion_inputs(seqs, block_size: int, long_portion: int | None = None, windows=()) -> dict:
     """Inputs of a step in which sequence ``s`` brings its tokens ``num_computed .. num_computed + num_scheduled - 1``,
     sequences with one token first (no counterpart in the reference).  Besides the usual arrays: per sequence the tokens
     before the step and the state slot, per row its sequence, and the portions of more than one token cut into chunks of
-    at most ``CHUNK`` that do not cross a sequence (rows counted from the first portion's first row)."""
+    at most ``CHUNK`` that do not cross a sequence (rows counted from the first portion's first row).  A design with
+    ``long_portion`` gets its portions of at least that many tokens last and, per attention window, the dense rows their
+    keys take (from the first key the portion's first token sees to its last token)."""
     n = np.asarray([s.num_scheduled for s in seqs], dtype=np.int64)
     single = int((n == 1).sum())
-    assert (n[:single] == 1).all() and (n[single:] > 1).all()
+    kinds = [portion_kind(int(x), long_portion) for x in n]
+    assert kinds == sorted(kinds)
+    short = kinds.count(1)
     start = np.asarray([s.num_computed for s in seqs], dtype=np.int64)
     ids = np.concatenate([np.asarray(s.token_ids[s.num_computed:s.num_computed + s.num_scheduled], dtype=np.int64) for s in seqs])
     cu = np.concatenate([[0], np.cumsum(n)])
@@ -94,6 +103,9 @@ def portion_inputs(seqs, block_size: int) -> dict:
     pos = np.arange(cu[-1]) - cu[row_seq] + start[row_seq]
     tables = block_tables_array(seqs)
     slots = tables[row_seq, pos // block_size].astype(np.int64) * block_size + pos % block_size
+    far = slice(single + short, None)
+    keys = np.stack([np.minimum(start[far], w - 1) + n[far] for w in windows]) if windows else np.zeros((0, len(n[far])), np.int64)
+    kv_offsets = np.concatenate([np.zeros((len(keys), 1), np.int64), np.cumsum(keys, axis=1)], axis=1)
     chunks = -(-n[single:] // CHUNK)
     cu_chunks = np.concatenate([[0], np.cumsum(chunks)])
     chunk_seq = np.repeat(np.arange(len(chunks)), chunks)
@@ -105,4 +117,7 @@ def portion_inputs(seqs, block_size: int) -> dict:
         chunk_rows=(cu[single:-1][chunk_seq] - single + within).astype(np.int32),
         chunk_lens=np.minimum(CHUNK, n[single:][chunk_seq] - within).astype(np.int32),
         cu_chunks=cu_chunks.astype(np.int32), num_single=single, max_portion=int(n.max()),
+        num_short=short, num_short_rows=int(cu[single + short]), max_short=int(n[single:single + short].max(initial=0)),
+        kv_offsets=kv_offsets.astype(np.int32), kv_rows=tuple(kv_offsets[:, -1].tolist()),
+        max_kv_rows=tuple(keys.max(axis=1, initial=0).tolist()),
     )

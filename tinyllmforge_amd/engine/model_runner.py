@@ -276,7 +276,8 @@ class ModelRunner:
         wanted rows, in the caller's order, in the context."""
         if want is None:
             want = [[s.num_scheduled - 1] if s.num_computed + s.num_scheduled == len(s) else [] for s in seqs]
-        order = sorted(range(len(seqs)), key=lambda i: seqs[i].num_scheduled > 1)     # single tokens first (stable)
+        hf = self.config.hf_config                      # single tokens first, long portions last (stable)
+        order = sorted(range(len(seqs)), key=lambda i: I.portion_kind(seqs[i].num_scheduled, hf.long_portion))
         batch = [seqs[i] for i in order]
         first = np.zeros(len(seqs), dtype=np.int64)
         first[order] = np.concatenate([[0], np.cumsum([s.num_scheduled for s in batch])])[:-1]
@@ -286,7 +287,7 @@ class ModelRunner:
             get_context().logit_rows = None if len(rows) == len(seqs) and (rows == np.arange(len(rows))).all() \
                 else torch.from_numpy(rows).to(self.device)
             return hidden
-        arrays = I.portion_inputs(batch, self.block_size)
+        arrays = I.portion_inputs(batch, self.block_size, hf.long_portion, hf.windows)
         arrays["logit_rows"] = rows
         done = [s for s, w in zip(seqs, want) if w]
         arrays["temperatures"] = self._temperatures_of(done) if done else None
@@ -507,7 +508,8 @@ class ModelRunner:
             graph = torch.cuda.CUDAGraph()
             if self.portioned:
                 set_portions_context(slot_mapping=gv["slot_mapping"][:bs], block_tables=gv["block_tables"][:bs, :],
-                                     state_slots=gv["state_slots"][:bs], num_single=bs, max_len=cfg.max_model_len)
+                                     state_slots=gv["state_slots"][:bs], num_single=bs, num_short_rows=bs,
+                                     max_len=cfg.max_model_len)
             else:
                 set_context(False, slot_mapping=gv["slot_mapping"][:bs], context_lens=gv["context_lens"][:bs],
                             block_tables=gv["block_tables"][:bs, :])

@@ -63,3 +63,13 @@ class PaddedLMHead(StackedLinear):
         if self.weight.dtype == torch.bfloat16 and self.weight.shape == (self.num_embeddings, x.shape[-1]):
             return ops.bf16_linear_argmax(x, self.weight.data)
         return ops.argmax(super().forward(x)[:, :self.num_embeddings].contiguous())
+
+
+class TiedLMHead(PaddedLMHead):
+    """LM head on the embedding table: shares its memory where the sizes need no padding."""
+
+    def tie_(self, table: torch.Tensor):
+        if table.shape == self.weight.shape:
+            self.weight.data = table
+        else:
+            self.weight.data[:table.shape[0], :table.shape[1]].copy_(table)

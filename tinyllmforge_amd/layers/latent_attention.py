@@ -1,0 +1,98 @@
+"""Windowed softmax attention over latents, on a paged cache of one row per token for all heads.
+
+A token caches its normed latent and a rotated key part.  Decoded tokens, short portions and 32-bit mode attend in the
+latent space: the queries are taken there once (``absorb``) and the mixed latents back to values once (``values``).  Long
+portions expand the keys and values of every head with one product (``expand``) and attend on those."""
+import torch
+from torch import nn
+
+from .. import ops
+from ..utils.context import get_context
+
+
+class LatentAttention(nn.Module):
+    def __init__(self, num_heads: int, dim: int, rot_dim: int, rank: int, value_dim: int, scale: float, window: int,
+                 window_index: int, rope, eps: float, dtype: torch.dtype):
+        super().__init__()
+        self.shape = ops.LatentShape(num_heads, dim, rot_dim, rank, value_dim)
+        self.scale, self.window, self.window_index, self.eps, self.dtype = scale, window, window_index, eps, dtype
+        self.register_buffer("cos_sin", rope, persistent=False)
+        self.norm = nn.Module()
+        self.norm.weight = nn.Parameter(torch.ones(rank))
+        self.uk = nn.Parameter(torch.zeros(num_heads * dim, rank))
+        self.uv = nn.Parameter(torch.zeros(num_heads * value_dim, rank))
+        self.absorb = self.values = self.expand = None      # made from uk and uv by pack_
+        self.cache = None                                   # [pages, block, Lp], bound by the model runner
+
+    # -- what the model runner asks a layer with a paged cache
+    def page_bytes(self, block_size: int) -> int:
+        return block_size * self.shape.lp * torch.empty(0, dtype=self.dtype).element_size()
+
+    def bind_pages(self, pages: int, block_size: int, device):
+        self.cache = torch.zeros(pages, block_size, self.shape.lp, dtype=self.dtype, device=device) if pages else None
+
+    def pack_(self):
+        """Once after loading: the three forms of the latent's projections."""
+        s, new = self.shape, self.uk.new_zeros
+        uk, uv = self.uk.data.view(s.heads, s.dim, s.rank), self.uv.data.view(s.heads, s.vdim, s.rank)
+        # [q_own | q_rot] -> [Uk^T q_own | q_rot]: the rotated part passes through an identity
+        self.absorb = new(s.heads, s.lp, s.dq)
+        self.absorb[:, :s.rank, :s.dim] = uk.transpose(1, 2)
+        for i in range(s.rot):
+            self.absorb[:, s.ra + i, s.da + i] = 1
+        self.values = new(s.heads, -(-s.vdim // 16) * 16, s.rp)
+        self.values[:, :s.vdim, :s.rank] = uv
+        self.tiles = self.dtype == torch.bfloat16 and ops.latent_attn_supported(s)
+        if self.dtype == torch.bfloat16 and ops.latent_prefill_supported(s):
+            rows = s.heads * (s.da + s.va)
+            self.expand = new(-(-rows // 16) * 16, -(-s.ra // 64) * 64)
+            self.expand[:s.heads * s.da].view(s.heads, s.da, -1)[:, :s.dim, :s.rank] = uk
+            self.expand[s.heads * s.da:rows].view(s.heads, s.va, -1)[:, :s.vdim, :s.rank] = uv
+
+    def prepare(self, proj, latent_col: int, positions: torch.Tensor) -> torch.Tensor:
+        """Projection rows ``[q | ... | latent | rotated key]`` -> rotated queries; the new cache rows are stored."""
+        return ops.latent_prep(proj, latent_col, self.norm.weight.data, positions, self.cos_sin, get_context().slot_mapping,
+                               self.cache, self.shape, self.eps)
+
+    def forward(self, q: torch.Tensor, positions: torch.Tensor, out: torch.Tensor):
+        """Queries from ``prepare`` -> ``out[:, :heads * value_dim]``."""
+        ctx, n = get_context(), q.shape[0]
+        latent_rows = ctx.num_short_rows if self.expand is not None else n
+        if latent_rows:
+            self._latent(q[:latent_rows], positions[:latent_rows], out[:latent_rows])
+        if latent_rows < n:
+            self._expanded(q, out)
+
+    def _latent(self, q, positions, out):
+        ctx, s, n = get_context(), self.shape, q.shape[0]
+        q = ops.head_gemm(q, self.absorb, s.ra, -(-s.da // 32) * 32)
+        if not self.tiles:
+            part, ml = ops.latent_rows(q, self.cache, ctx.block_tables, positions, ctx.slot_mapping[:n],
+                                       ctx.row_seq[:n] if ctx.row_seq is not None else None, self.window, self.scale, s)
+            ops.latent_values(part, ml, self.values, out, s)
+            return
+        single = ctx.num_single
+        portions = (ctx.num_short if self.expand is not None else ctx.cu_seqlens_q.numel() - 1 - single) if single < n else 0
+        most = ctx.max_short if self.expand is not None else ctx.max_portion
+        for first, rows, seqs, tokens, where in (
+                (0, single, single, 1, dict(positions=positions, slot_mapping=ctx.slot_mapping)),
+                (single, n - single, portions, most, dict(cu_seqlens_q=ctx.cu_seqlens_q, seq_starts=ctx.seq_starts,
+                                                          first_seq=single, first_row=single))):
+            if not rows:
+                continue
+            splits = ops.latent_attention_splits(seqs, tokens, s.heads, self.window, ctx.max_len)
+            part, ml = ops.latent_partials(rows, splits, s, q.device)
+            ops.latent_attention(q[first:first + rows], self.cache, ctx.block_tables, self.window, self.scale, s, part, ml,
+                                 num_seqs=seqs, max_tokens=tokens, **where)
+            ops.latent_values(part, ml, self.values, out[first:first + rows], s)
+
+    def _expanded(self, q, out):
+        ctx, w = get_context(), self.window_index
+        first = ctx.num_single + ctx.num_short
+        seqs = ctx.cu_seqlens_q.numel() - 1 - first
+        offsets = ctx.kv_offsets[w]
+        latents = ops.latent_gather(self.cache, ctx.block_tables, ctx.cu_seqlens_q, ctx.seq_starts, offsets, ctx.kv_rows[w],
+                                    first, seqs, ctx.max_kv_rows[w], self.window)
+        expanded = ops.linear(latents[:, :self.expand.shape[1]], self.expand)
+        ops.latent_prefill(q, expanded, latents, ctx.cu_seqlens_q, ctx.seq_starts, offsets, first, seqs, ctx.max_portion,
+                           self.window, self.scale, self.shape, out)

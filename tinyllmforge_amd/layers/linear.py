@@ -250,6 +250,52 @@ class StackedLinear(LinearBase):
         return ops.linear_deferred(x, self.weight.data)
 
 
+class JoinedLinear(LinearBase):
+    """One projection of several inputs laid side by side in a row, in the order of ``parts`` (name -> columns): the sum of
+    the parts' own projections as one product.  Every part begins at a multiple of 64 columns, pads are zero; the caller
+    fills ``input_rows``."""
+
+    def __init__(self, parts: dict[str, int], output_size: int):
+        self.parts = dict(parts)
+        self.columns = sum(_round_up(n, 64) for n in parts.values())
+        super().__init__(self.columns, output_size, 1)
+        self._make_params(_round_up(output_size, 16), self.columns, bias=False)
+        self.weight.data.zero_()
+
+    def offset(self, name: str) -> int:
+        at = 0
+        for part, n in self.parts.items():
+            if part == name:
+                return at
+            at += _round_up(n, 64)
+        raise KeyError(name)
+
+    def weight_loader(self, param: nn.Parameter, loaded_weight: torch.Tensor, loaded_shard_id: str):
+        assert tuple(loaded_weight.shape) == (self.output_size, self.parts[loaded_shard_id]), (loaded_shard_id, tuple(loaded_weight.shape))
+        at = self.offset(loaded_shard_id)
+        param.data[:self.output_size, at:at + loaded_weight.shape[1]].copy_(loaded_weight)
+
+    def zero_pads_(self):
+        if self.weight.numel():
+            self.weight.data[self.output_size:].zero_()
+            for name, n in self.parts.items():
+                at = self.offset(name)
+                self.weight.data[:, at + n:at + _round_up(n, 64)].zero_()
+
+    def input_rows(self, rows: int, dtype, device) -> torch.Tensor:
+        """An input to fill part by part (pads are zeros already)."""
+        pads = self.columns != sum(self.parts.values())
+        return (torch.zeros if pads else torch.empty)(rows, self.columns, dtype=dtype, device=device)
+
+    def forward_deferred(self, x: torch.Tensor):
+        """``StackedLinear.forward_deferred`` of rows from ``input_rows``."""
+        if self.weight.dtype == torch.float32:
+            return self.forward(x)
+        if self.is_quantized:
+            return ops.linear_deferred(x, self.pack_().qpacked, self.qscale)
+        return ops.linear_deferred(x, self.weight.data)
+
+
 class GatedUpLinear(MergedColumnParallelLinear):
     """gate and up projections of any size: the intermediate dim is padded to a multiple of 64 and the input to one of
     64, with zeros (a padded channel is silu(0) * 0), so the result is the input of a ``StackedLinear`` as it is."""

@@ -1,0 +1,76 @@
+"""Gigopel: a decoder of parallel layers, windowed latent attention beside a dense xIELU feed-forward or a mixture of experts.
+
+Both sublayers read one norm's output and are added to the fp32 residual together, times a constant.  So a layer is one
+product in (queries, latent, rotated key and a dense feed-forward's channels stacked), one product out (attention heads and
+those channels side by side), and one kernel that adds and applies the norm of the next layer."""
+from torch import nn
+
+from ..config import GigopelConfig
+from ..layers.activation import XIELU
+from ..layers.embed_head import TiedLMHead
+from ..layers.latent_attention import LatentAttention
+from ..layers.linear import JoinedLinear, StackedLinear
+from ..layers.moe import ClippedGLUExperts
+from ..layers.residual_norm import ResidualRMSNorm
+from .layered import LayeredForCausalLM
+
+
+class GigopelLayer(nn.Module):
+    def __init__(self, cfg: GigopelConfig, layer: dict, rope):
+        super().__init__()
+        m, mlp, eps = layer["mixer"], layer.get("mlp"), cfg.norm["eps"]
+        self.mult = cfg.residual_mult
+        self.norm1 = ResidualRMSNorm(cfg.width, eps, offset=1.0)
+        self.attn = LatentAttention(m["heads"], m["dim"], m["rot_dim"], m["kv_rank"], m["vdim"], m["scale"], m["mask"]["size"],
+                                    cfg.windows.index(m["mask"]["size"]), rope, eps, cfg.torch_dtype)
+        stacked = {"q": m["heads"] * (m["dim"] + m["rot_dim"]), "dkv": m["kv_rank"] + m["rot_dim"]}
+        joined = {"o": m["heads"] * m["vdim"]}
+        self.act = self.experts = None
+        if mlp and mlp["kind"] == "dense":
+            stacked["up"], joined["down"] = mlp["ff"], mlp["ff"]
+            self.act = XIELU()
+        elif mlp:
+            self.experts = ClippedGLUExperts(cfg.width, mlp["router"]["experts"], mlp["router"]["top"], mlp["expert"]["ff"],
+                                             mlp["expert"]["limit"])
+        self.inp = StackedLinear(cfg.width, stacked)
+        self.out = JoinedLinear(joined, cfg.width)
+
+    def forward(self, positions, h, x, following: ResidualRMSNorm):
+        proj = self.inp.forward_deferred(h)         # read by the next two kernels, before any other product
+        rows = self.out.input_rows(h.shape[0], h.dtype, h.device)
+        q = self.attn.prepare(proj, self.inp.offset("dkv"), positions)
+        if self.act is not None:
+            self.act(proj, self.inp.offset("up"), self.inp.parts["up"], rows[:, self.out.offset("down"):])
+        extra = self.experts(h) if self.experts is not None else (None, None)
+        self.attn(q, positions, rows)
+        return following.after_adding(self.out.forward_deferred(rows), x, self.mult, *extra)
+
+    def routes(self) -> dict:
+        out = {"norm1": ("norm1.weight", None), "mix.q": ("inp.weight", "q"), "mix.dkv": ("inp.weight", "dkv"),
+               "mix.dkv.norm": ("attn.norm.weight", None), "mix.uk": ("attn.uk", None), "mix.uv": ("attn.uv", None),
+               "mix.o": ("out.weight", "o")}
+        if self.act is not None:
+            out |= {"mlp.up": ("inp.weight", "up"), "mlp.down": ("out.weight", "down"), "mlp.act": ("act.pq", None)}
+        if self.experts is not None:
+            out["mlp.router"] = ("experts.router", "router")
+            for e in range(self.experts.experts):
+                for kind, target in (("gate", "gate_up"), ("up", "gate_up"), ("down", "down")):
+                    out[f"mlp.e{e}.{kind}"] = ("experts." + target, (e, kind))
+        return out
+
+
+class GigopelForCausalLM(LayeredForCausalLM):
+    def __init__(self, config: GigopelConfig):
+        super().__init__(config)
+        self.layers = nn.ModuleList([GigopelLayer(config, layer, self.rope_table(layer["mixer"]["rot"])) for layer in config.layers])
+        self.norm = ResidualRMSNorm(config.width, config.norm["eps"], offset=1.0)
+        self.head = TiedLMHead(config.vocab, config.width)
+
+    def pack_linears_(self):
+        super().pack_linears_()
+        for layer in self.layers:
+            layer.attn.pack_()
+            if layer.experts is not None:
+                layer.experts.zero_pads_()
+        self.head.tie_(self.embed.data)
+        return self

@@ -3,19 +3,17 @@ each with an optional gated MLP, between grouped RMSNorms on both sides of every
 
 The residual stream is fp32.  Every sublayer ends in one kernel that applies its closing norm, adds to the residual and
 applies the opening norm of whatever follows; all projections of a sublayer's input are one matrix product."""
-import re
-
 import torch
 from torch import nn
 
-from .. import ops
 from ..config import GitopelConfig
 from ..layers.embed_head import PaddedLMHead
 from ..layers.gla import GatedLinearAttention
 from ..layers.grouped_norm import GroupedRMSNorm
 from ..layers.linear import GatedUpLinear, StackedLinear
-from ..layers.pooled_attention import PooledWindowAttention, interleaved_cos_sin
+from ..layers.pooled_attention import PooledWindowAttention
 from ..utils.context import get_context
+from .layered import LayeredForCausalLM, prefixed
 
 DEFAULT_RANK = 16     # rows of a gla layer's first decay factor when no checkpoint fixes them
 
@@ -93,85 +91,18 @@ class GitopelLayer(nn.Module):
             h = self.norm2b.add_then(self.mlp(h), None, x, following)
         return h
 
+    def routes(self) -> dict:
+        norms = ["norm1", "norm1b"] + (["norm2", "norm2b"] if self.mlp is not None else [])
+        out = {n: (n + ".weight", None) for n in norms} | prefixed("mix.", self.mix.routes)
+        return out | prefixed("mlp.", self.mlp.routes) if self.mlp is not None else out
 
-class GitopelForCausalLM(nn.Module):
+
+class GitopelForCausalLM(LayeredForCausalLM):
+    fixed_tensors = LayeredForCausalLM.fixed_tensors | {"head": ("head.weight", "head")}
+
     def __init__(self, config: GitopelConfig):
-        super().__init__()
-        self.config = config
-        self.embed = nn.Parameter(torch.empty(config.vocab, config.width))
-        tables = {}                          # layers with the same rotation share a table
-
-        def rope(layer):
-            if layer["type"] != "attention":
-                return None
-            key = (layer["mixer"]["rot"]["dims"], layer["mixer"]["rot"]["base"])
-            if key not in tables:
-                tables[key] = interleaved_cos_sin(key[0], config.max_position_embeddings, key[1]).to(self.embed.device)
-            return tables[key]
-
+        super().__init__(config)
+        rope = lambda layer: self.rope_table(layer["mixer"]["rot"]) if layer["type"] == "attention" else None
         self.layers = nn.ModuleList([GitopelLayer(config, layer, rope(layer)) for layer in config.layers])
         self.norm = GroupedRMSNorm(config.width, config.norm["groups"], config.norm["eps"])
         self.head = PaddedLMHead(config.vocab, config.width)
-        self.loaded_tensors: set[str] = set()
-
-    def forward(self, input_ids: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
-        norms = [layer.norm1 for layer in self.layers] + [self.norm]
-        x, h = norms[0].after_embedding(input_ids, self.embed.data)
-        for layer, following in zip(self.layers, norms[1:]):
-            h = layer(positions, h, x, following)
-        return h
-
-    def compute_logits(self, hidden_states: torch.Tensor) -> torch.Tensor:
-        return self.head(hidden_states)
-
-    def compute_greedy_ids(self, hidden_states: torch.Tensor) -> torch.Tensor:
-        return self.head.forward_greedy(hidden_states)
-
-    # -- checkpoint names
-    def route_tensor(self, name: str):
-        """Checkpoint tensor -> (parameter, part of it or None)."""
-        fixed = {"embed": ("embed", None), "final.norm": ("norm.weight", None), "head": ("head.weight", "head")}
-        if name in fixed:
-            return fixed[name]
-        m = re.fullmatch(r"l(\d+)\.(.+)", name)
-        if m is None or int(m[1]) >= len(self.layers):
-            raise KeyError(f"unknown tensor {name!r}")
-        prefix, rest, layer = f"layers.{m[1]}.", m[2], self.layers[int(m[1])]
-        if re.fullmatch(r"norm[12]b?", rest):
-            return prefix + rest + ".weight", None
-        group, _, short = rest.partition(".")
-        module = {"mix": layer.mix, "mlp": layer.mlp}[group]
-        target, part = module.routes[short]
-        return f"{prefix}{group}.{target}", part
-
-    def expected_tensors(self) -> set[str]:
-        out = {"embed", "final.norm", "head"}
-        for i, layer in enumerate(self.layers):
-            names = ["norm1", "norm1b"] + ["mix." + k for k in layer.mix.routes]
-            if layer.mlp is not None:
-                names += ["norm2", "norm2b"] + ["mlp." + k for k in layer.mlp.routes]
-            out |= {f"l{i}.{n}" for n in names}
-        return out
-
-    # -- what the engine does with the weights after loading
-    def _linears(self):
-        for layer in self.layers:
-            yield from (m for m in layer.modules() if isinstance(m, (StackedLinear, GatedUpLinear)))
-
-    def quantize_linears_(self):
-        """Weight-only int8 for the projections of every layer (embedding and head stay as they are)."""
-        for lin in self._linears():
-            lin.zero_pads_()
-            lin.quantize_()
-        return self
-
-    def pack_linears_(self):
-        """Once after loading, on the GPU: pads back to zero, then the row and tile orders the fused kernels read."""
-        for lin in [*self._linears(), self.head]:
-            if not getattr(lin, "interleaved", False):
-                lin.zero_pads_()
-            if lin.is_quantized:
-                lin.pack_()
-            elif isinstance(lin, GatedUpLinear) and lin.weight.dtype == torch.bfloat16:
-                lin.interleave_()
-        return self

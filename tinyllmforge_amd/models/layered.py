@@ -1,0 +1,85 @@
+"""What designs with a list of unlike layers share: rotation tables, the forward loop, checkpoint names, packing.
+
+A layer is a module with ``norm1`` (the norm in front of it), ``forward(positions, h, x, following)`` that updates the fp32
+residual ``x`` in place and returns it normed by ``following``, and ``routes()``: checkpoint names below ``l<i>.`` ->
+(parameter below the layer, part of it or None)."""
+import re
+
+import torch
+from torch import nn
+
+from ..layers.linear import GatedUpLinear, JoinedLinear, StackedLinear
+from ..layers.pooled_attention import interleaved_cos_sin
+
+
+def prefixed(prefix: str, routes: dict) -> dict:
+    return {prefix + name: (prefix + target, part) for name, (target, part) in routes.items()}
+
+
+class LayeredForCausalLM(nn.Module):
+    fixed_tensors = {"embed": ("embed", None), "final.norm": ("norm.weight", None)}
+
+    def __init__(self, config):
+        super().__init__()
+        self.config = config
+        self.embed = nn.Parameter(torch.empty(config.vocab, config.width))
+        self.loaded_tensors: set[str] = set()
+        self._rope_tables = {}
+
+    def rope_table(self, rot: dict):
+        """Layers with the same rotation share a table."""
+        key = (rot["dims"], rot["base"])
+        if key not in self._rope_tables:
+            self._rope_tables[key] = interleaved_cos_sin(key[0], self.config.max_position_embeddings, key[1]).to(self.embed.device)
+        return self._rope_tables[key]
+
+    def forward(self, input_ids: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
+        norms = [layer.norm1 for layer in self.layers] + [self.norm]
+        x, h = norms[0].after_embedding(input_ids, self.embed.data)
+        for layer, following in zip(self.layers, norms[1:]):
+            h = layer(positions, h, x, following)
+        return h
+
+    def compute_logits(self, hidden_states: torch.Tensor) -> torch.Tensor:
+        return self.head(hidden_states)
+
+    def compute_greedy_ids(self, hidden_states: torch.Tensor) -> torch.Tensor:
+        return self.head.forward_greedy(hidden_states)
+
+    # -- checkpoint names
+    def route_tensor(self, name: str):
+        """Checkpoint tensor -> (parameter, part of it or None)."""
+        if name in self.fixed_tensors:
+            return self.fixed_tensors[name]
+        m = re.fullmatch(r"l(\d+)\.(.+)", name)
+        routes = self.layers[int(m[1])].routes() if m and int(m[1]) < len(self.layers) else {}
+        if not m or m[2] not in routes:
+            raise KeyError(f"unknown tensor {name!r}")
+        target, part = routes[m[2]]
+        return f"layers.{m[1]}.{target}", part
+
+    def expected_tensors(self) -> set[str]:
+        return set(self.fixed_tensors) | {f"l{i}.{n}" for i, layer in enumerate(self.layers) for n in layer.routes()}
+
+    # -- what the engine does with the weights after loading
+    def _linears(self):
+        for layer in self.layers:
+            yield from (m for m in layer.modules() if isinstance(m, (StackedLinear, JoinedLinear, GatedUpLinear)))
+
+    def quantize_linears_(self):
+        """Weight-only int8 for the projections of every layer (embedding, head and experts stay as they are)."""
+        for lin in self._linears():
+            lin.zero_pads_()
+            lin.quantize_()
+        return self
+
+    def pack_linears_(self):
+        """Once after loading, on the GPU: pads back to zero, then the row and tile orders the fused kernels read."""
+        for lin in [*self._linears(), self.head]:
+            if not getattr(lin, "interleaved", False):
+                lin.zero_pads_()
+            if lin.is_quantized:
+                lin.pack_()
+            elif isinstance(lin, GatedUpLinear) and lin.weight.dtype == torch.bfloat16:
+                lin.interleave_()
+        return self

@@ -604,8 +604,8 @@ def group_rms_norm_add(y, y_bias, w_post, x, w_next, groups, eps):
     return h
 
 
-def embed_group_rms_norm(ids, table, w_next, groups, eps):
-    """``x = table[ids]`` in fp32 and ``norm(x) * w_next`` in the table's dtype."""
+def embed_group_rms_norm(ids, table, w_next, groups, eps, w_offset=0.0):
+    """``x = table[ids]`` in fp32 and ``norm(x) * (w_next + w_offset)`` in the table's dtype."""
     lib = _lib.load()
     _need(ids, torch.int64, "ids"); _need(table, w_next.dtype, "table")
     assert ids.is_contiguous() and table.is_contiguous()
@@ -613,7 +613,7 @@ def embed_group_rms_norm(ids, table, w_next, groups, eps):
     x = torch.empty(rows, width, dtype=torch.float32, device=table.device)
     h = torch.empty(rows, width, dtype=table.dtype, device=table.device)
     check(lib.tlf_embed_group_rmsnorm(ids.data_ptr(), table.data_ptr(), vocab, x.data_ptr(), w_next.data_ptr(),
-                                      h.data_ptr(), rows, width, groups, float(eps), _dt(table), _stream()),
+                                      float(w_offset), h.data_ptr(), rows, width, groups, float(eps), _dt(table), _stream()),
           "tlf_embed_group_rmsnorm")
     return x, h
 
@@ -733,4 +733,211 @@ def gla_portions(proj, a2, a2_bias, norm_weight, state, state_slots, seq_starts,
         cu_chunks.data_ptr(), chunks, first_seq, num_seqs, out.data_ptr(), out.stride(0), rows, heads, dk, dv,
         a2.shape[1], float(tau), dk ** -0.5, float(eps), _dt(proj), ws.data_ptr(), ws.numel(), _stream()),
         "tlf_gla_portions")
+    return out
+
+
+def residual_rms_norm(y, x, mult, w_next, w_offset, eps, extra=None, extra_rows=None):
+    """In place ``x += mult * (y + sum of the rows extra[extra_rows])`` (``x`` fp32 ``[N, W]``, ``extra_rows`` int32
+    ``[N, top]``), then ``x / rms(x) * (w_next + w_offset)`` in y's dtype."""
+    lib = _lib.load()
+    _need(x, torch.float32, "x"); _need(w_next, y.dtype, "w_next")
+    rows, width = x.shape
+    assert y.shape[0] == rows and y.shape[1] >= width and x.is_contiguous() and w_next.numel() == width
+    top, stride = 0, 0
+    if extra is not None:
+        _need(extra, y.dtype, "extra"); _need(extra_rows, torch.int32, "extra_rows")
+        assert extra.stride(1) == 1 and extra_rows.is_contiguous() and extra_rows.shape[0] == rows
+        top, stride = extra_rows.shape[1], extra.stride(0)
+    h = torch.empty(rows, width, dtype=y.dtype, device=x.device)
+    check(lib.tlf_residual_rmsnorm(*_source(y), _opt(extra), stride, _opt(extra_rows), top, float(mult), x.data_ptr(),
+                                   w_next.data_ptr(), float(w_offset), h.data_ptr(), rows, width, float(eps), _dt(y),
+                                   _stream()), "tlf_residual_rmsnorm")
+    return h
+
+
+class LatentShape:
+    """Sizes of a latent-attention layer and of the padded rows its kernels read (``include/tlf_hip.h``)."""
+    __slots__ = ("heads", "dim", "rot", "rank", "vdim", "da", "ta", "ra", "va", "dq", "lp", "rp")
+
+    def __init__(self, heads, dim, rot, rank, vdim):
+        up = lambda v, m: -(-v // m) * m
+        self.heads, self.dim, self.rot, self.rank, self.vdim = heads, dim, rot, rank, vdim
+        self.da, self.ta, self.ra, self.va = up(dim, 8), up(rot, 8), up(rank, 8), up(vdim, 8)
+        self.dq, self.lp, self.rp = up(self.da + self.ta, 32), up(self.ra + self.ta, 64), up(self.ra, 32)
+
+    @property
+    def sizes(self):
+        return self.heads, self.dim, self.rot, self.rank, self.vdim
+
+
+def latent_prep(proj, latent_col, norm_weight, positions, cos_sin, slot_mapping, cache, shape: LatentShape, eps):
+    """Rotated queries ``[N, H, Dq]``; the normed latent and the rotated key part go to ``cache [pages, bs, Lp]``."""
+    lib = _lib.load()
+    assert proj.dtype == cache.dtype == norm_weight.dtype and cache.is_contiguous() and cache.shape[2] == shape.lp
+    _need(positions, torch.int64, "positions"); _need(slot_mapping, torch.int32, "slot_mapping")
+    n = proj.shape[0]
+    assert positions.numel() == n and slot_mapping.numel() == n and norm_weight.numel() == shape.rank
+    assert cos_sin is None or cos_sin.shape[1] == shape.rot
+    q = torch.empty(n, shape.heads, shape.dq, dtype=proj.dtype, device=proj.device)
+    check(lib.tlf_latent_prep(*_source(proj), latent_col, norm_weight.data_ptr(), positions.data_ptr(), _opt(cos_sin),
+                              cos_sin.shape[0] if cos_sin is not None else 0, slot_mapping.data_ptr(),
+                              cache.shape[0] * cache.shape[1], q.data_ptr(), cache.data_ptr(), n, *shape.sizes, float(eps),
+                              _dt(proj), _stream()), "tlf_latent_prep")
+    return q
+
+
+def head_gemm(x, w, n_main=0, k_main=0):
+    """``y[row, head] = w[head] @ x[row, head]``: ``x [N, H, K]``, ``w [H, Nout, K]`` -> ``[N, H, Nout]``."""
+    lib = _lib.load()
+    _need(x, w.dtype, "x")
+    rows, heads, K = x.shape
+    assert x.is_contiguous() and w.is_contiguous() and w.shape[0] == heads and w.shape[2] == K
+    y = torch.empty(rows, heads, w.shape[1], dtype=x.dtype, device=x.device)
+    check(lib.tlf_head_gemm(x.data_ptr(), w.data_ptr(), y.data_ptr(), rows, heads, w.shape[1], K, n_main, k_main, _dt(x),
+                            _stream()), "tlf_head_gemm")
+    return y
+
+
+def latent_attn_supported(shape: LatentShape) -> bool:
+    return bool(_lib.load().tlf_latent_attn_supported(*shape.sizes))
+
+
+def latent_prefill_supported(shape: LatentShape) -> bool:
+    return bool(_lib.load().tlf_latent_prefill_supported(*shape.sizes))
+
+
+def latent_partials(rows, splits, shape: LatentShape, device):
+    return (torch.empty(splits, rows, shape.heads, shape.rp, dtype=torch.float32, device=device),
+            torch.empty(splits, rows, shape.heads, 2, dtype=torch.float32, device=device))
+
+
+def latent_rows(q, cache, block_tables, positions, slot_mapping, row_seq, window, scale, shape: LatentShape):
+    """Absorbed attention of any rows; ``q [N, H, Lp]``.  Returns ``(part, ml)`` of one split."""
+    lib = _lib.load()
+    _need(q, cache.dtype, "q"); _need(block_tables, torch.int32, "block_tables"); _need(positions, torch.int64, "positions")
+    rows = q.shape[0]
+    assert q.is_contiguous() and q.shape[1:] == (shape.heads, shape.lp) and block_tables.stride(1) == 1
+    assert positions.numel() == rows and slot_mapping.numel() == rows and (row_seq is not None or block_tables.shape[0] >= rows)
+    part, ml = latent_partials(rows, 1, shape, q.device)
+    step = 32768                                     # rows per launch (grid limit)
+    for lo in range(0, rows, step):
+        n = min(step, rows - lo)
+        assert row_seq is not None or lo == 0
+        check(lib.tlf_latent_rows(q[lo:].data_ptr(), cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0),
+                                  positions[lo:].data_ptr(), slot_mapping[lo:].data_ptr(),
+                                  row_seq[lo:].data_ptr() if row_seq is not None else None, part[0, lo:].data_ptr(),
+                                  ml[0, lo:].data_ptr(), n, *shape.sizes, cache.shape[1], window, cache.shape[0],
+                                  float(scale), _dt(q), _stream()), "tlf_latent_rows")
+    return part, ml
+
+
+def latent_attention(q, cache, block_tables, window, scale, shape: LatentShape, part, ml, positions=None, slot_mapping=None,
+                     cu_seqlens_q=None, seq_starts=None, first_seq=0, first_row=0, num_seqs=0, max_tokens=1):
+    """Absorbed attention on the matrix cores: ``num_seqs`` single rows (``positions``, ``slot_mapping``) or portions."""
+    lib = _lib.load()
+    _need(q, BF16, "q"); _need(block_tables, torch.int32, "block_tables")
+    assert q.is_contiguous() and q.shape[1:] == (shape.heads, shape.lp) and block_tables.stride(1) == 1
+    assert block_tables.shape[0] >= first_seq + num_seqs and cache.is_contiguous() and cache.dtype == BF16
+    check(lib.tlf_latent_attn(q.data_ptr(), cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), _opt(positions),
+                              _opt(slot_mapping), _opt(cu_seqlens_q), _opt(seq_starts), first_seq, first_row, num_seqs, max_tokens,
+                              part.data_ptr(), ml.data_ptr(), part.shape[0], part.shape[1], *shape.sizes, cache.shape[1],
+                              window, cache.shape[0], float(scale), _stream()), "tlf_latent_attn")
+
+
+def latent_attention_splits(num_seqs, max_tokens, heads, window, max_len) -> int:
+    return _lib.load().tlf_latent_attn_splits(num_seqs, max_tokens, heads, window, max_len)
+
+
+def latent_values(part, ml, uv, out, shape: LatentShape):
+    """``out [N, >= H * vdim]`` from the splits' mixed latents; ``uv [H, vdim rounded up to 16, Rp]``."""
+    lib = _lib.load()
+    splits, rows = part.shape[:2]
+    assert out.shape[0] == rows and out.stride(1) == 1 and out.dtype == uv.dtype and part.is_contiguous() and uv.is_contiguous()
+    check(lib.tlf_latent_values(part.data_ptr(), ml.data_ptr(), splits, uv.data_ptr(), out.data_ptr(), out.stride(0), rows,
+                                *shape.sizes, _dt(uv), _stream()), "tlf_latent_values")
+
+
+def latent_gather(cache, block_tables, cu_seqlens_q, seq_starts, kv_offsets, kv_rows, first_seq, num_seqs, max_rows, window):
+    """Cache rows of the keys that the portions see, dense: ``[kv_rows, Lp]``."""
+    lib = _lib.load()
+    _need(kv_offsets, torch.int32, "kv_offsets")
+    assert cache.dtype == BF16 and kv_offsets.is_contiguous() and kv_offsets.numel() == num_seqs + 1
+    out = torch.empty(kv_rows, cache.shape[2], dtype=cache.dtype, device=cache.device)
+    check(lib.tlf_latent_gather(cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), cu_seqlens_q.data_ptr(),
+                                seq_starts.data_ptr(), kv_offsets.data_ptr(), first_seq, num_seqs, max_rows, out.data_ptr(),
+                                cache.shape[2], cache.shape[1], window, cache.shape[0], _stream()), "tlf_latent_gather")
+    return out
+
+
+def latent_prefill(q, expanded, latents, cu_seqlens_q, seq_starts, kv_offsets, first_seq, num_seqs, max_tokens, window, scale,
+                   shape: LatentShape, out):
+    """Portions from expanded keys and values; ``q`` and ``out`` are indexed by the step's rows."""
+    lib = _lib.load()
+    _need(q, BF16, "q"); _need(expanded, BF16, "expanded"); _need(latents, BF16, "latents")
+    assert q.is_contiguous() and q.shape[1:] == (shape.heads, shape.dq) and out.stride(1) == 1
+    assert expanded.stride(1) == 1 and latents.is_contiguous() and latents.shape[1] == shape.lp
+    check(lib.tlf_latent_prefill(q.data_ptr(), expanded.data_ptr(), expanded.stride(0), latents.data_ptr(),
+                                 cu_seqlens_q.data_ptr(), seq_starts.data_ptr(), kv_offsets.data_ptr(), first_seq, num_seqs,
+                                 max_tokens, out.data_ptr(), out.stride(0), *shape.sizes, window, float(scale), _stream()),
+          "tlf_latent_prefill")
+    return out
+
+
+# ------------------------------------------------------------------ mixture of experts
+def moe_route(h, router, experts, top):
+    """The ``top`` experts of every row by router logit and their sigmoids: int32 and fp32 ``[N, top]``."""
+    lib = _lib.load()
+    _need(h, router.dtype, "h")
+    n, K = h.shape
+    assert h.stride(1) == 1 and router.is_contiguous() and router.shape[1] == K and router.shape[0] >= experts
+    ids = torch.empty(n, top, dtype=torch.int32, device=h.device)
+    weights = torch.empty(n, top, dtype=torch.float32, device=h.device)
+    check(lib.tlf_moe_route(h.data_ptr(), h.stride(0), router.data_ptr(), ids.data_ptr(), weights.data_ptr(), n, experts, K, top,
+                            _dt(h), _stream()), "tlf_moe_route")
+    return ids, weights
+
+
+class ExpertRows:
+    """Rows (token, k) in expert order: ``row_of [N, top]``, ``src`` / ``weight`` per row, tiles of ``tile_rows`` rows."""
+    __slots__ = ("row_of", "src", "weight", "tiles", "num_tiles", "tile_rows")
+
+
+def moe_group(ids, weights, experts, tile_rows) -> ExpertRows:
+    lib = _lib.load()
+    _need(ids, torch.int32, "ids"); _need(weights, torch.float32, "weights")
+    assert ids.is_contiguous() and weights.is_contiguous() and ids.shape == weights.shape
+    n, top = ids.shape
+    r = ExpertRows()
+    i32 = lambda *s: torch.empty(*s, dtype=torch.int32, device=ids.device)
+    r.row_of, r.src, r.weight = i32(n, top), i32(n * top), torch.empty(n * top, dtype=torch.float32, device=ids.device)
+    r.tiles, r.num_tiles, r.tile_rows = i32(n * top // tile_rows + min(experts, n * top), 4), i32(1), tile_rows
+    check(lib.tlf_moe_group(ids.data_ptr(), weights.data_ptr(), r.row_of.data_ptr(), r.src.data_ptr(), r.weight.data_ptr(),
+                            r.tiles.data_ptr(), r.num_tiles.data_ptr(), r.tiles.shape[0], n, top, experts, tile_rows,
+                            _stream()), "tlf_moe_group")
+    return r
+
+
+def moe_gemm(x, w, rows: ExpertRows, gather: bool, clipped_glu: bool = False, limit: float = 0.0):
+    """One product per expert, ``w [E, Nout, K]``.  ``gather``: x rows are tokens (otherwise rows in expert order);
+    ``clipped_glu``: interleaved gate / up channels, activated, the row's weight on both products."""
+    lib = _lib.load()
+    _need(x, w.dtype, "x")
+    assert x.stride(1) == 1 and w.is_contiguous() and w.shape[2] == x.shape[1]
+    n, N = rows.src.numel(), w.shape[1]
+    assert gather or x.shape[0] == n
+    y = torch.empty(n, N // 2 if clipped_glu else N, dtype=x.dtype, device=x.device)
+    check(lib.tlf_moe_gemm(x.data_ptr(), x.stride(0), x.shape[0], w.data_ptr(), y.data_ptr(), rows.tiles.data_ptr(),
+                           rows.num_tiles.data_ptr(), rows.tiles.shape[0], rows.tile_rows,
+                           rows.src.data_ptr() if gather else None, rows.weight.data_ptr() if clipped_glu else None, n, N,
+                           w.shape[2], int(clipped_glu), float(limit), _dt(x), _stream()), "tlf_moe_gemm")
+    return y
+
+
+def xielu(x, col, cols, pq, out):
+    """``out[:, :cols] = xielu(x[:, col:col + cols])``, zeros in the rest of ``out``'s columns."""
+    lib = _lib.load()
+    _need(pq, out.dtype, "pq")
+    assert pq.numel() == 2 and out.stride(1) == 1 and x.shape[0] == out.shape[0]
+    check(lib.tlf_xielu(*_source(x), col, pq.data_ptr(), out.data_ptr(), out.stride(0), out.shape[0], cols, out.shape[1],
+                        _dt(out), _stream()), "tlf_xielu")
     return out

@@ -127,7 +127,7 @@ def random_init_(model: nn.Module, seed: int = 0, std: float = 0.02, device_fill
         if tied and name == "lm_head.weight":
             continue                                   # shares the embedding's storage
         if name.endswith("norm.weight") or name.split(".")[-2:-1] and name.split(".")[-2].startswith("norm"):
-            p.data.fill_(1.0)
+            p.data.fill_(getattr(p, "identity", 1.0))       # what makes the norm a plain division
             continue
         if device_fill:
             p.data.normal_(0.0, std)
