@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the per-token hot path on one MI355X.
 
-    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload e2e|decode_attn|gemm|gitopel|...|all]
+    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload e2e|decode_attn|gemm|gitopel|gigopel|...|all]
 
 Prints ONE JSON line.
 
@@ -53,7 +53,7 @@ def parse():
                     help="engine steps that steps/ms_per_step describe (0 = all); value is always the whole job")
     ap.add_argument("--warmup", type=int, default=1, help="warm-up generate() calls before the timed run")
     ap.add_argument("--workload", default="e2e",
-                    choices=["e2e", "decode_attn", "gemm", "prefill_attn", "elementwise", "clock", "c5", "gitopel", "all"])
+                    choices=["e2e", "decode_attn", "gemm", "prefill_attn", "elementwise", "clock", "c5", "gitopel", "gigopel", "all"])
     ap.add_argument("--attn-steps", type=int, default=200, help="timed launches of the decode-attention microbench")
     ap.add_argument("--num-seqs", type=int, default=256)
     ap.add_argument("--no-cpu-baseline", action="store_true")
@@ -756,14 +756,18 @@ def bench_gitopel_kernels():
 
 
 def bench_gitopel_throughput(size, batch=64, prompt=1024, out_tokens=128):
-    """Prompt and decode tokens/s of both models through ``LLM.generate`` (bf16, random weights, hipGraph decode)."""
+    return throughput({"gitopel": gitopel_shape(size), "qwen3": qwen3_shape(size)}, size, batch, prompt, out_tokens)
+
+
+def throughput(shapes, size, batch=64, prompt=1024, out_tokens=128):
+    """Prompt and decode tokens/s of each model through ``LLM.generate`` (bf16, random weights, hipGraph decode)."""
     import gc
     import random
     import torch
     from tinyllmforge_amd import LLM, SamplingParams
     rng = random.Random(0)
     res = {}
-    for name, shape in (("gitopel", gitopel_shape(size)), ("qwen3", qwen3_shape(size))):
+    for name, shape in shapes.items():
         llm = LLM(shape, max_model_len=2048, max_num_batched_tokens=16384, max_num_seqs=batch, gpu_memory_utilization=0.5, seed=0)
         vocab = llm.config.hf_config.vocab_size
 
@@ -786,6 +790,171 @@ def bench_gitopel_throughput(size, batch=64, prompt=1024, out_tokens=128):
         gc.collect()
         torch.cuda.empty_cache()
     return dict(size=size, batch=batch, prompt_tokens=prompt, output_tokens=out_tokens, layers=8, **res)
+
+
+# ----------------------------------------------------------------------------- Gigopel beside Qwen3 at equal size
+# width, heads, dim, rotated dim, value dim, latent; dense ff; experts, top, expert ff (top * expert ff = dense ff)
+GIGOPEL_SIZES = {"1024-wide": (1024, 16, 64, 32, 64, 256, 3072, 32, 4, 768),
+                 "4096-wide": (4096, 32, 128, 64, 128, 512, 12288, 64, 8, 1536)}
+
+
+def gigopel_shape(size, layers=8, vocab=32768, window=1024, moe=True):
+    """The first layer dense, the others mixtures of experts (``moe=False``: all dense)."""
+    w, h, d, t, v, r, ff, ne, top, eff = GIGOPEL_SIZES[size]
+    mixer = dict(heads=h, dim=d, rot_dim=t, vdim=v, kv_rank=r, scale=(d + t) ** -0.5, rot=dict(base=10000.0, dims=t),
+                 mask=dict(size=window))
+    dense = dict(type="latent_attention", mixer=mixer, mlp=dict(kind="dense", ff=ff))
+    sparse = dict(type="latent_attention", mixer=mixer, mlp=dict(kind="moe", expert=dict(ff=eff, limit=7.0),
+                                                                 router=dict(experts=ne, top=top)))
+    return dict(architecture="Gigopel", vocab=vocab, width=w, norm=dict(eps=1e-6), residual_mult=0.5,
+                layers=[dense] + [sparse if moe else dense] * (layers - 1))
+
+
+def bench_gigopel_kernels(sizes=None):
+    """Kernels of the Gigopel layers beside the like kernel of Qwen3 at the same width: algorithmic bytes or flops over the
+    graph-timed launch, as a fraction of the HBM or matrix peak."""
+    import torch
+    from tinyllmforge_amd import ops as P
+    from tinyllmforge_amd.layers.latent_attention import LatentAttention
+    from tinyllmforge_amd.layers.moe import ClippedGLUExperts
+    from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
+    torch.manual_seed(0)
+    BF, dev = torch.bfloat16, "cuda"
+    rows = []
+
+    def add(name, size, fn, amount, bound, copies=1, launches=10):
+        def cycle():
+            for i in range(copies):
+                fn(i)
+        sec = time_graph(cycle, launches=max(1, launches // copies), replays=10) * 1e-3 / copies
+        peak = {"hbm": HBM_PEAK_GBPS * 1e9, "mfma bf16": MFMA_BF16_PEAK_TFLOPS * 1e12}[bound]
+        rows.append(dict(kernel=name, size=size, us=round(sec * 1e6, 2), bound=bound,
+                         rate=round(amount / sec / (1e9 if bound == "hbm" else 1e12), 1), frac=round(amount / sec / peak, 4)))
+        print(rows[-1], file=sys.stderr, flush=True)
+        torch.cuda.empty_cache()
+
+    bf = lambda *s: torch.randn(*s, device=dev).to(BF)
+    for size in sizes or GIGOPEL_SIZES:
+        w, h, d, t, v, r, ff, ne, top, eff = GIGOPEL_SIZES[size]
+        hq, hkv, qd = GITOPEL_SIZES[size][1:4]
+        torch.set_default_dtype(BF)
+        with torch.device(dev):
+            layer = LatentAttention(h, d, t, r, v, (d + t) ** -0.5, 1024, 0, None, 1e-6, BF)
+        torch.set_default_dtype(torch.float32)
+        layer.uk.data.normal_(0, r ** -0.5)
+        layer.uv.data.normal_(0, r ** -0.5)
+        layer.pack_()
+        s = layer.shape
+        # -- decode: 64 sequences, contexts U[512, 4096], pages of 256
+        B, bs = 64, 256
+        case = make_decode_case(batch=B, hq=hq, hkv=hkv, dh=qd)
+        plan = P.paged_decode_plan(case["ctx"], case["bt"], bs)
+        add("paged decode attention (Qwen3)", size,
+            lambda i: P.paged_decode_attention(case["q"], case["k_cache"], case["v_cache"], case["ctx"], case["bt"], qd ** -0.5, plan=plan),
+            case["algo_bytes"], "hbm")
+        del case["k_cache"], case["v_cache"]
+        cache = bf(2048, bs, s.lp)
+        pos, slots = case["ctx"].long() - 1, torch.zeros(B, dtype=torch.int32, device=dev)
+        q = bf(B, h, s.lp)
+        for window in (4096, 1024):
+            seen = sum(min(int(c), window) for c in case["ctx"].cpu())
+            batch = P.LatentBatch(B, positions=pos, slot_mapping=slots)
+            plan = P.latent_plan(batch, h, s.lp, window)
+            add(f"latent decode attention, window {window}", size,
+                lambda i: P.latent_attention(q, cache, case["bt"], window, layer.scale, s, batch, plan),
+                seen * (r + t) * 2 + B * h * (r + t) * 2 + B * h * r * 4, "hbm")
+        qd_rows = bf(B, h, s.dq)
+        add("queries into the latent space, 64 tokens", size, lambda i: P.head_gemm(qd_rows, layer.absorb, s.ra, -(-s.da // 32) * 32),
+            h * d * r * 2 + B * h * (d + t + r + t) * 2, "hbm")
+        part, ml = P.latent_attention(q, cache, case["bt"], window, layer.scale, s, batch, plan)
+        out = torch.zeros(B, h * v, device=dev, dtype=BF)
+        add("pieces joined + values, 64 tokens", size, lambda i: P.latent_values(part, ml, layer.values, out, s, batch, plan),
+            h * v * r * 2 + B * h * r * 4 + B * h * v * 2, "hbm")
+        add("work split of the step, 64 sequences", size, lambda i: P.latent_plan(batch, h, s.lp, window), B * 16, "hbm")
+        del case, plan, part, cache
+        # -- prompts: 8 x 2048 tokens
+        S, L = 8, 2048
+        N = S * L
+        qq, kk, vv = bf(N, hq, qd), bf(N, hkv, qd), bf(N, hkv, qd)
+        cu = torch.arange(0, N + 1, L, dtype=torch.int32, device=dev)
+        add("prompt attention (Qwen3)", size, lambda i: P.varlen_prefill_attention(qq, kk, vv, cu, cu, L, qd ** -0.5),
+            4.0 * hq * qd * S * L * L / 2, "mfma bf16")
+        del qq, kk, vv
+        cache = bf(N // bs, bs, s.lp)
+        bt = torch.arange(N // bs, dtype=torch.int32, device=dev).view(S, -1)
+        starts = torch.zeros(S, dtype=torch.int32, device=dev)
+        q, out = bf(N, h, s.dq), torch.empty(N, h * v, device=dev, dtype=BF)
+        add("keys of a prompt gathered", size, lambda i: P.latent_gather(cache, bt, cu, starts, cu, N, 0, S, L, 2048), N * s.lp * 4, "hbm")
+        latents = P.latent_gather(cache, bt, cu, starts, cu, N, 0, S, L, 2048)
+        expanded = P.linear(latents[:, :layer.expand.shape[1]], layer.expand)
+        add("keys and values of a prompt expanded (bf16 linear)", size, lambda i: P.linear(latents[:, :layer.expand.shape[1]], layer.expand),
+            2.0 * N * h * (d + v) * r, "mfma bf16")
+        for window in (2048, 1024, 512):
+            seen = sum(min(i + 1, window) for i in range(L)) * S
+            add(f"latent prompt attention, window {window}", size,
+                lambda i: P.latent_prefill(q, expanded, latents, cu, starts, cu, 0, S, L, window, layer.scale, s, out),
+                2.0 * h * (d + t + v) * seen, "mfma bf16")
+        del q, out, expanded, latents
+        # -- between the products
+        tab = interleaved_cos_sin(t, 4096, 1e4).to(dev)
+        slots = torch.arange(N, dtype=torch.int32, device=dev)
+        pos = torch.arange(L, device=dev).repeat(S)
+        ld = -(-(h * (d + t) + r + t) // 16) * 16
+        nw = torch.ones(r, device=dev, dtype=BF)
+        pq = torch.zeros(2, device=dev, dtype=BF)
+        wd, tabq = torch.ones(qd, dtype=BF, device=dev), interleaved_cos_sin(qd, 4096, 1e6).to(dev)
+        for n, copies in ((N, 3), (B, 1)):
+            qkv = bf(copies, n, (hq + 2 * hkv) * qd)
+            kc, vc = bf(2, N // bs, bs, hkv, qd)
+            add(f"q/k norm + RoPE + store (Qwen3), {n} tokens", size,
+                lambda i: P.qknorm_rope_store(qkv[i], wd, wd, 1e-6, pos[:n], tabq, hq, hkv, qd, kc, vc, slots[:n]),
+                n * ((hq + 2 * hkv) * qd * 4 + qd * 4), "hbm", copies)
+            proj = bf(copies, n, ld)
+            add(f"latent preparation, {n} tokens", size,
+                lambda i: P.latent_prep(proj[i], h * (d + t), nw, pos[:n], tab, slots[:n], cache, s, 1e-6),
+                n * ((h * (d + t) + r + t) * 4 + t * 4), "hbm", copies)
+            y, x, e = bf(copies, n, w), torch.randn(copies, n, w, device=dev), bf(copies, n * top, w)
+            rr, ww = bf(copies, n, w), torch.ones(w, device=dev, dtype=BF)
+            idx = torch.randperm(n * top, device=dev).to(torch.int32).view(n, top)
+            add(f"add + RMSNorm (Qwen3), {n} tokens", size, lambda i: P.add_rms_norm(y[i], rr[i], ww, 1e-6), n * w * 8, "hbm", copies)
+            add(f"add + norm, {n} tokens", size, lambda i: P.residual_rms_norm(y[i], x[i], 0.5, ww, 1.0, 1e-6), n * w * 12, "hbm", copies)
+            add(f"add {top} expert rows + norm, {n} tokens", size,
+                lambda i: P.residual_rms_norm(y[i], x[i], 0.5, ww, 1.0, 1e-6, e[i], idx), n * w * (12 + 2 * top), "hbm", copies)
+            z = bf(copies, n, ff)
+            a = torch.empty(n, ff, device=dev, dtype=BF)
+            zz = bf(copies, n, 2 * ff)
+            add(f"SiLU and mul (Qwen3), {n} tokens", size, lambda i: P.silu_and_mul(zz[i]), n * ff * 6, "hbm", copies)
+            add(f"xIELU, {n} tokens", size, lambda i: P.xielu(z[i], 0, ff, pq, a), n * ff * 4, "hbm", copies)
+            del qkv, kc, vc, proj, y, x, e, rr, z, zz, a
+        del cache
+        # -- experts
+        torch.set_default_dtype(BF)
+        with torch.device(dev):
+            moe = ClippedGLUExperts(w, ne, top, eff, 7.0)
+        torch.set_default_dtype(torch.float32)
+        for p_ in moe.parameters():
+            p_.data.normal_(0, 0.02)
+        gu, dn = bf(2 * ff, w), bf(w, ff)
+        for n in (B, 512, N):
+            x = bf(n, w)
+            ids, wt = P.moe_route(x, moe.router.data, ne, top)
+            add(f"router, {n} tokens", size, lambda i: P.moe_route(x, moe.router.data, ne, top), ne * w * 2 + n * w * 2, "hbm")
+            tile = moe.tile_rows(n)
+            add(f"rows by expert, {n} tokens", size, lambda i: P.moe_group(ids, wt, ne, tile), n * top * 24, "hbm")
+            g = P.moe_group(ids, wt, ne, tile)
+            active = len(set(ids.flatten().tolist()))
+            a = P.moe_gemm(x, moe.gate_up.data, g, True, True, 7.0)
+            ad = bf(n, ff)
+            big = n == N
+            amount = lambda parts: (2.0 * n * top * parts * eff * w, "mfma bf16") if big else (active * parts * eff * w * 2, "hbm")
+            like = lambda parts: (2.0 * n * parts * ff * w, "mfma bf16") if big else (parts * ff * w * 2, "hbm")
+            add(f"gate_up + SiLU-and-mul (Qwen3), {n} tokens", size, lambda i: P.bf16_linear_silu_mul(x, gu), *like(2))
+            add(f"experts' gate_up + clipped GLU, {n} tokens", size, lambda i: P.moe_gemm(x, moe.gate_up.data, g, True, True, 7.0), *amount(2))
+            add(f"down (Qwen3), {n} tokens", size, lambda i: P.bf16_linear(ad, dn), *like(1))
+            add(f"experts' down, {n} tokens", size, lambda i: P.moe_gemm(a, moe.down.data, g, False), *amount(1))
+            del x, a, ad, g
+        del moe, gu, dn
+    return rows
 
 
 # ----------------------------------------------------------------------------- config 4 (end to end)
@@ -939,6 +1108,20 @@ def main():
             "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
             "config": {"workload": "Gitopel layers (alternating attention and gla, window 1024, pool 16) and Qwen3 layers of "
                                    "equal size, random weights, bf16"},
+            "extra": {"throughput": through, "kernels": rows}}))
+        return
+    if args.workload == "gigopel":   # likewise
+        rows = bench_gigopel_kernels()
+        through = [throughput({"gigopel": gigopel_shape(size), "gigopel dense": gigopel_shape(size, moe=False),
+                               "qwen3": qwen3_shape(size)}, size) for size in GIGOPEL_SIZES]
+        big = through[-1]
+        print(json.dumps({
+            "metric": "output tok/s (Gigopel, 8 layers of 4096, 64 sequences, decode)", "value": big["gigopel"]["decode_tok_s"],
+            "unit": "tok/s", "n_gpus": 1, "steps": big["output_tokens"], "warmup": 1,
+            "ms_per_step": big["gigopel"]["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak",
+            "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+            "config": {"workload": "Gigopel layers (latent attention, window 1024; one dense layer, seven of experts) and Qwen3 "
+                                   "layers of equal width and active feed-forward, random weights, bf16"},
             "extra": {"throughput": through, "kernels": rows}}))
         return
     extra = {}

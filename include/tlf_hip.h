@@ -607,12 +607,15 @@ int tlf_residual_rmsnorm(const void *y, int64_t y_stride, const float *partials,
  * tlf_latent_rows: absorbed attention, any rows in either dtype: q [rows, heads, Lp] = [Uk_h^T q_own | q_rot | 0]; writes
  *   part [rows, heads, Rp] (Rp = Ra rounded up to 32), the unnormalised mix of latents, and ml [rows, heads, 2], maximum
  *   (of score * log2 e) and denominator.  row_seq[r]: block-table row (NULL: r).
- * tlf_latent_attn: the same on the matrix cores, bf16, Lp <= 576 (tlf_latent_attn_supported), keys cut into `splits` parts
- *   (tlf_latent_attn_splits proposes a number): part [splits, rows, heads, Rp], ml [splits, rows, heads, 2].  With
- *   cu_seqlens_q NULL sequence s is the single row s at positions[s] (slot_mapping[s] < 0: a padding row, no keys), otherwise
- *   rows cu_seqlens_q[s] - first_row .. of q and part, sequences first_seq .. + num_seqs - 1, after seq_starts[s] cached tokens.
- * tlf_latent_values: out[row, head] = Uv_h (sum of the splits / denominator); uv [heads, vdim rounded up to 16, Rp]; rows
- *   without keys give 0.
+ * tlf_latent_attn: the same on the matrix cores, bf16, Lp <= 576 (tlf_latent_attn_supported).  With cu_seqlens_q NULL
+ *   sequence s is the single row s at positions[s] (slot_mapping[s] < 0: a padding row, no keys; max_tokens 1), otherwise
+ *   rows cu_seqlens_q[s] - first_row .. of q, sequences first_seq .. + num_seqs - 1 of at most max_tokens rows, after
+ *   seq_starts[s] cached tokens.  The work is cut into pieces by a plan (tlf_latent_attn_plan, once per step and window:
+ *   the same arguments, row_size = Lp; it depends on no layer), written to part [pieces, units, Rp] and ml [pieces, units,
+ *   2].  tlf_latent_attn_layout gives (host memory) layout[3] = int32 values of a plan, pieces, units.
+ * tlf_latent_values: out[row, head] = Uv_h (sum of the pieces / denominator); uv [heads, vdim rounded up to 16, Rp]; plan
+ *   NULL: part as from tlf_latent_rows, otherwise the plan and its arguments (with cu_seqlens_q, row_seq[r] is the sequence
+ *   of row r of `out`).  Rows without keys give 0.
  * tlf_latent_gather: for the expanded form: cache rows of the keys that sequence first_seq + s sees in this step (from
  *   position max(0, start - window + 1) on) as rows kv_offsets[s] .. kv_offsets[s + 1] - 1 of `out`; max_rows bounds them.
  * tlf_latent_prefill: portions from expanded keys and values (rows [heads * Da | heads * Va], Va = vdim rounded up to 8) and
@@ -628,16 +631,20 @@ int tlf_latent_rows(const void *q, const void *cache, const int32_t *block_table
                     *positions, const int32_t *slot_mapping, const int32_t *row_seq, float *part, float *ml, int32_t
                     rows, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, int32_t
                     block_size, int32_t window, int64_t num_pages, float scale, int32_t dtype, void *stream);
-int tlf_latent_attn_splits(int32_t num_seqs, int32_t max_tokens, int32_t heads, int32_t window, int32_t max_len);
-int tlf_latent_attn_supported(int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim);
+int tlf_latent_attn_layout(int32_t num_seqs, int32_t max_tokens, int32_t heads, int32_t row_size, int32_t *layout);
+int tlf_latent_attn_plan(const int64_t *positions, const int32_t *slot_mapping, const int32_t *cu_seqlens_q, const
+                         int32_t *seq_starts, int32_t first_seq, int32_t first_row, int32_t num_seqs, int32_t
+                         max_tokens, int32_t heads, int32_t row_size, int32_t window, int32_t *plan, void *stream);
 int tlf_latent_attn(const void *q, const void *cache, const int32_t *block_tables, int64_t bt_stride, const int64_t
                     *positions, const int32_t *slot_mapping, const int32_t *cu_seqlens_q, const int32_t *seq_starts,
-                    int32_t first_seq, int32_t first_row, int32_t num_seqs, int32_t max_tokens, float *part, float *ml, int32_t splits,
-                    int32_t rows, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, int32_t
-                    block_size, int32_t window, int64_t num_pages, float scale, void *stream);
-int tlf_latent_values(const float *part, const float *ml, int32_t splits, const void *uv, void *out, int64_t
-                      out_stride, int32_t rows, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t
-                      vdim, int32_t dtype, void *stream);
+                    int32_t first_seq, int32_t first_row, int32_t num_seqs, int32_t max_tokens, const int32_t *plan,
+                    float *part, float *ml, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim,
+                    int32_t block_size, int32_t window, int64_t num_pages, float scale, void *stream);
+int tlf_latent_values(const float *part, const float *ml, const int32_t *plan, const int32_t *cu_seqlens_q, const
+                      int32_t *row_seq, int32_t first_seq, int32_t first_row, int32_t num_seqs, int32_t max_tokens,
+                      const void *uv, void *out, int64_t out_stride, int32_t rows, int32_t heads, int32_t dim,
+                      int32_t rot_dim, int32_t rank, int32_t vdim, int32_t dtype, void *stream);
+int tlf_latent_attn_supported(int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim);
 int tlf_latent_gather(const void *cache, const int32_t *block_tables, int64_t bt_stride, const int32_t *cu_seqlens_q,
                       const int32_t *seq_starts, const int32_t *kv_offsets, int32_t first_seq, int32_t num_seqs,
                       int32_t max_rows, void *out, int32_t row_size, int32_t block_size, int32_t window, int64_t

@@ -95,12 +95,14 @@ SIGNATURES = {
     "tlf_head_gemm": (c_int32, [_P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _P]),
     "tlf_latent_rows": (c_int32, [_P, _P, _P, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I32,
                                   _I32, _I64, _F, _I32, _P]),
-    "tlf_latent_values": (c_int32, [_P, _P, _I32, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _P]),
-    "tlf_latent_gather": (c_int32, [_P, _P, _I64, _P, _P, _P, _I32, _I32, _I32, _P, _I32, _I32, _I32, _I64, _P]),
-    "tlf_latent_attn_splits": (c_int32, [_I32, _I32, _I32, _I32, _I32]),
-    "tlf_latent_attn_supported": (c_int32, [_I32, _I32, _I32, _I32, _I32]),
-    "tlf_latent_attn": (c_int32, [_P, _P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _P, _P, _I32, _I32, _I32, _I32,
+    "tlf_latent_attn_layout": (c_int32, [_I32, _I32, _I32, _I32, _P]),
+    "tlf_latent_attn_plan": (c_int32, [_P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _P, _P]),
+    "tlf_latent_attn": (c_int32, [_P, _P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _P, _P, _P, _I32, _I32,
                                   _I32, _I32, _I32, _I32, _I32, _I64, _F, _P]),
+    "tlf_latent_values": (c_int32, [_P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _P, _P, _I64, _I32, _I32, _I32, _I32,
+                                    _I32, _I32, _I32, _P]),
+    "tlf_latent_gather": (c_int32, [_P, _P, _I64, _P, _P, _P, _I32, _I32, _I32, _P, _I32, _I32, _I32, _I64, _P]),
+    "tlf_latent_attn_supported": (c_int32, [_I32, _I32, _I32, _I32, _I32]),
     "tlf_latent_prefill_supported": (c_int32, [_I32, _I32, _I32, _I32, _I32]),
     "tlf_latent_prefill": (c_int32, [_P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P, _I64, _I32, _I32, _I32,
                                      _I32, _I32, _I32, _F, _P]),

@@ -48,4 +48,66 @@ __device__ __forceinline__ int64_t latent_row(const LatentCache &c, const int32_
   return page >= 0 && page < c.pages ? page * c.bs + (j - pg * c.bs) : 0;
 }
 
+// ---- jobs of the absorbed kernels: 16 or 32 units (row, head) of one sequence and the key tiles their window covers
+constexpr int kLatentTile = 64;          // keys per tile
+constexpr int kLatentMaxPieces = 128;    // workgroups that share a job, at most
+constexpr int kLatentPlanHead = 4;       // plan: tiles per workgroup, tiles in all, -, -; per workgroup (job, first tile);
+                                         // per job (first workgroup, workgroups).  Piece of (workgroup w, job j): w + j
+
+struct LatentJobs {
+  const int64_t *positions;              // sequence s is the single row s at positions[s] (slots[s] < 0: no keys) ...
+  const int32_t *slots;
+  const int32_t *cu_q, *starts;          // ... or, with cu_q, rows cu_q[s] - first_row .. after starts[s] cached tokens
+  int32_t first_seq, first_row, window;
+  int32_t H, units, hpp, passes, bq, xtiles, jobs;   // heads, units of a job, heads per pass, passes, rows per job
+};
+inline bool latent_jobs(LatentJobs &j, int num_seqs, int max_tokens, int heads) {
+  j.H = heads;
+  j.units = static_cast<int64_t>(max_tokens) * heads > 16 ? 32 : 16;
+  j.hpp = heads < j.units ? heads : j.units;
+  j.passes = (heads + j.hpp - 1) / j.hpp;
+  j.bq = j.units / j.hpp;
+  j.xtiles = (max_tokens + j.bq - 1) / j.bq;
+  const int64_t jobs = static_cast<int64_t>(num_seqs) * j.xtiles * j.passes;
+  j.jobs = static_cast<int32_t>(jobs);
+  return jobs <= (1 << 24);
+}
+// Workgroups of the tile kernel: as many as the chip holds at once.
+inline int latent_workgroups(int lp, int units) { return 256 * (lp <= 128 ? 2 : 1); }
+
+// Loads through the scalar path: the vector path's counter belongs to the copies in flight.
+template <typename T>
+__device__ __forceinline__ T uniform_load(const T *p) {
+  return *(const T __attribute__((address_space(4))) *)(reinterpret_cast<uintptr_t>(p));
+}
+
+struct LatentJob {
+  int seq, q0, start, row0, last_row, head0, heads, w0, tiles;
+};
+// UNIFORM: `job` is the same in all lanes
+template <bool UNIFORM>
+__device__ __forceinline__ LatentJob latent_job(const LatentJobs &a, int job) {
+  auto ld = [](auto *p) __attribute__((always_inline)) { return UNIFORM ? uniform_load(p) : *p; };
+  LatentJob j;
+  const int pass = job % a.passes, rest = job / a.passes, xt = rest % a.xtiles;
+  j.seq = a.first_seq + rest / a.xtiles;
+  int lq = 1;
+  if (a.cu_q) {
+    const int lo = ld(a.cu_q + j.seq);
+    j.q0 = lo - a.first_row;
+    lq = ld(a.cu_q + j.seq + 1) - lo;
+    j.start = ld(a.starts + j.seq);
+  } else {
+    j.q0 = j.seq;
+    j.start = ld(a.slots + j.seq) >= 0 ? static_cast<int>(ld(a.positions + j.seq)) : -1;
+  }
+  j.row0 = xt * a.bq;
+  j.last_row = min(j.row0 + a.bq, lq) - 1;
+  j.head0 = pass * a.hpp;
+  j.heads = min(a.hpp, a.H - j.head0);
+  j.w0 = max(0, j.start + j.row0 - a.window + 1) / kLatentTile * kLatentTile;
+  j.tiles = j.start >= 0 && j.row0 < lq ? (j.start + j.last_row - j.w0) / kLatentTile + 1 : 0;
+  return j;
+}
+
 }  // namespace tlf

@@ -244,60 +244,85 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const LatentRowsArgs a
 // ---------------------------------------------------------------------------------------------------------------
 struct LatentValuesArgs {
   LatentShape s;
-  const float *part, *ml;   // [splits, rows, H, Rp], [splits, rows, H, 2]
+  const float *part, *ml;   // pieces of Rp values, and their maximum and denominator
+  const int32_t *plan;      // of the tile kernel, NULL: one piece per (row, head), in that order
+  LatentJobs jb;
+  const int32_t *row_seq;   // [rows] with jb.cu_q: sequence of a row
   const void *uv;           // [H, Vp, Rp], Vp = vdim rounded up to 16
   void *out;                // [rows, ldo]
   int64_t ldo;
-  int32_t rows, splits, Vp;
+  int32_t rows, Vp, wgs;
 };
 
-// Weight of every split of (row, head) over the common denominator; 0 for a split without keys.
-__device__ __forceinline__ float split_weight(const LatentValuesArgs &a, int64_t rh, int split, int64_t plane, float mx, float inv) {
-  const float *p = a.ml + (split * plane + rh) * 2;
-  return p[1] > 0.f ? exp2f(p[0] - mx) * inv : 0.f;
+// The pieces of (row, head): units first, first + step, ...
+struct Pieces {
+  int64_t first;
+  int32_t step, count;
+};
+__device__ __forceinline__ Pieces latent_pieces(const LatentValuesArgs &a, int row, int h) {
+  if (!a.plan) return Pieces{static_cast<int64_t>(row) * a.s.H + h, 0, 1};
+  const LatentJobs &j = a.jb;
+  int seq = row, r = 0;
+  if (j.cu_q) {
+    seq = a.row_seq[row];
+    r = row + j.first_row - j.cu_q[seq];
+    seq -= j.first_seq;
+  }
+  const int pass = h / j.hpp, job = (seq * j.xtiles + r / j.bq) * j.passes + pass;
+  const int32_t *rec = a.plan + kLatentPlanHead + 2 * (a.wgs + job);
+  const bool ok = rec[0] >= 0 && rec[1] >= 0 && rec[0] + rec[1] <= a.wgs;
+  return Pieces{static_cast<int64_t>(rec[0] + job) * j.units + r % j.bq * j.hpp + h - pass * j.hpp, j.units, ok ? rec[1] : 0};
 }
-__device__ __forceinline__ void split_total(const LatentValuesArgs &a, int64_t rh, int64_t plane, float &mx, float &inv) {
+// Maximum and inverse denominator over the pieces (inverse 0: no keys).
+__device__ __forceinline__ void pieces_total(const LatentValuesArgs &a, const Pieces &p, float &mx, float &inv) {
   mx = -INFINITY;
-  for (int k = 0; k < a.splits; ++k)
-    if (a.ml[(k * plane + rh) * 2 + 1] > 0.f) mx = fmaxf(mx, a.ml[(k * plane + rh) * 2]);
+  for (int k = 0; k < p.count; ++k) {
+    const float2 v = *reinterpret_cast<const float2 *>(a.ml + (p.first + static_cast<int64_t>(k) * p.step) * 2);
+    if (v.y > 0.f) mx = fmaxf(mx, v.x);
+  }
   float den = 0.f;
-  for (int k = 0; k < a.splits; ++k) {
-    const float *p = a.ml + (k * plane + rh) * 2;
-    if (p[1] > 0.f) den = fmaf(p[1], exp2f(p[0] - mx), den);
+  for (int k = 0; k < p.count; ++k) {
+    const float2 v = *reinterpret_cast<const float2 *>(a.ml + (p.first + static_cast<int64_t>(k) * p.step) * 2);
+    if (v.y > 0.f) den = fmaf(v.y, exp2f(v.x - mx), den);
   }
   inv = den > 0.f ? 1.0f / den : 0.f;
+}
+__device__ __forceinline__ float piece_weight(const LatentValuesArgs &a, const Pieces &p, int k, float mx, float inv) {
+  const float2 v = *reinterpret_cast<const float2 *>(a.ml + (p.first + static_cast<int64_t>(k) * p.step) * 2);
+  return v.y > 0.f ? exp2f(v.x - mx) * inv : 0.f;
 }
 
 // bf16: a workgroup takes one head, 16 rows and 64 outputs; the mixed latents of the rows go through LDS once
 __global__ __launch_bounds__(256) void latent_values_kernel(const LatentValuesArgs a) {
   extern __shared__ __attribute__((aligned(16))) unsigned short lat[];   // [16][Rp + 8]
-  __shared__ float wt[16][33];
+  __shared__ float tot[16][2];
+  __shared__ Pieces pcs[16];
   const LatentShape &s = a.s;
   const int h = blockIdx.x, row0 = blockIdx.y * 16, tid = threadIdx.x;
-  const int64_t plane = static_cast<int64_t>(a.rows) * s.H;
   const int stride = s.Rp + 8;
   if (tid < 16) {
-    const int row = row0 + tid;
-    if (row < a.rows) {
-      const int64_t rh = static_cast<int64_t>(row) * s.H + h;
+    Pieces p = Pieces{0, 0, 0};
+    if (row0 + tid < a.rows) {
+      p = latent_pieces(a, row0 + tid, h);
       float mx, inv;
-      split_total(a, rh, plane, mx, inv);
-      for (int k = 0; k < a.splits; ++k) wt[tid][k] = split_weight(a, rh, k, plane, mx, inv);
-    } else {
-      for (int k = 0; k < a.splits; ++k) wt[tid][k] = 0.f;
+      pieces_total(a, p, mx, inv);
+      tot[tid][0] = mx;
+      tot[tid][1] = inv;
     }
+    pcs[tid] = p;
   }
   __syncthreads();
   const int nch = s.Rp / 8;
   for (int item = tid; item < 16 * nch; item += 256) {
     const int r = item / nch, d = (item - r * nch) * 8;
-    const int64_t rh = static_cast<int64_t>(min(row0 + r, a.rows - 1)) * s.H + h;
+    const Pieces p = pcs[r];
+    const float mx = tot[r][0], inv = tot[r][1];
     float o[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < a.splits; ++k) {
-      const float w = wt[r][k];
+    for (int k = 0; k < p.count; ++k) {
+      const float w = piece_weight(a, p, k, mx, inv);
       if (w > 0.f) {
         float f[8];
-        Elem<float>::ld8(a.part + (k * plane + rh) * s.Rp + d, f);
+        Elem<float>::ld8(a.part + (p.first + static_cast<int64_t>(k) * p.step) * s.Rp + d, f);
 #pragma unroll
         for (int e = 0; e < 8; ++e) o[e] = fmaf(w, f[e], o[e]);
       }
@@ -330,14 +355,14 @@ __global__ __launch_bounds__(256) void latent_values_rows_kernel(const LatentVal
   extern __shared__ __attribute__((aligned(16))) float mixed[];   // [Rp]
   const LatentShape &s = a.s;
   const int h = blockIdx.x, row = blockIdx.y;
-  const int64_t plane = static_cast<int64_t>(a.rows) * s.H, rh = static_cast<int64_t>(row) * s.H + h;
+  const Pieces p = latent_pieces(a, row, h);
   float mx, inv;
-  split_total(a, rh, plane, mx, inv);
+  pieces_total(a, p, mx, inv);
   for (int d = threadIdx.x; d < s.Rp; d += 256) {
     float o = 0.f;
-    for (int k = 0; k < a.splits; ++k) {
-      const float w = split_weight(a, rh, k, plane, mx, inv);
-      if (w > 0.f) o = fmaf(w, a.part[(k * plane + rh) * s.Rp + d], o);
+    for (int k = 0; k < p.count; ++k) {
+      const float w = piece_weight(a, p, k, mx, inv);
+      if (w > 0.f) o = fmaf(w, a.part[(p.first + static_cast<int64_t>(k) * p.step) * s.Rp + d], o);
     }
     mixed[d] = Elem<T>::rnd(o);
   }
@@ -447,19 +472,27 @@ extern "C" int tlf_latent_rows(const void *q, const void *cache, const int32_t *
   return launch_status();
 }
 
-extern "C" int tlf_latent_values(const float *part, const float *ml, int32_t splits, const void *uv, void *out,
-                                 int64_t out_stride, int32_t rows, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank,
-                                 int32_t vdim, int32_t dtype, void *stream) {
+extern "C" int tlf_latent_values(const float *part, const float *ml, const int32_t *plan, const int32_t *cu_seqlens_q,
+                                 const int32_t *row_seq, int32_t first_seq, int32_t first_row, int32_t num_seqs,
+                                 int32_t max_tokens, const void *uv, void *out, int64_t out_stride, int32_t rows, int32_t heads,
+                                 int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, int32_t dtype, void *stream) {
   using namespace tlf;
   LatentValuesArgs a{};
-  if (rows < 0 || splits <= 0 || splits > 32 || !latent_shape(a.s, heads, dim, rot_dim, rank, vdim)) return TLF_E_SHAPE;
+  if (rows < 0 || !latent_shape(a.s, heads, dim, rot_dim, rank, vdim)) return TLF_E_SHAPE;
   if (out_stride < static_cast<int64_t>(heads) * vdim) return TLF_E_SHAPE;
   if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
   if (rows == 0) return TLF_OK;
-  if (!part || !ml || !uv || !out) return TLF_E_NULL;
+  if (!part || !ml || !uv || !out || (plan && cu_seqlens_q && !row_seq)) return TLF_E_NULL;
   if (!aligned16(part) || !aligned16(uv)) return TLF_E_ALIGN;
-  a.part = part; a.ml = ml; a.uv = uv; a.out = out; a.ldo = out_stride; a.rows = rows; a.splits = splits;
+  a.part = part; a.ml = ml; a.uv = uv; a.out = out; a.ldo = out_stride; a.rows = rows;
   a.Vp = round_up_to(vdim, 16);
+  if (plan) {
+    if (num_seqs <= 0 || max_tokens <= 0 || first_seq < 0 || (!cu_seqlens_q && rows > num_seqs)) return TLF_E_SHAPE;
+    a.plan = plan; a.row_seq = row_seq;
+    a.jb = LatentJobs{nullptr, nullptr, cu_seqlens_q, nullptr, first_seq, first_row, 1};
+    if (!latent_jobs(a.jb, num_seqs, max_tokens, heads)) return TLF_E_TOO_LARGE;
+    a.wgs = latent_workgroups(a.s.Lp, a.jb.units);
+  }
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (dtype == TLF_DT_BF16) {
     if ((rows + 15) / 16 > 65535) return TLF_E_SHAPE;

@@ -515,6 +515,7 @@ class ModelRunner:
                             block_tables=gv["block_tables"][:bs, :])
             self.plan_decode()
             gv["outputs"][:bs] = self.model(gv["input_ids"][:bs], gv["positions"][:bs])    # warm-up
+            get_context().plans.clear()      # the graph makes its own, from the step's inputs
             launched = lib.tlf_kernel_launches()
             with torch.cuda.graph(graph, pool):
                 self.plan_decode()       # first node of the graph: the attention work split of the step

@@ -71,20 +71,24 @@ class LatentAttention(nn.Module):
                                        ctx.row_seq[:n] if ctx.row_seq is not None else None, self.window, self.scale, s)
             ops.latent_values(part, ml, self.values, out, s)
             return
-        single = ctx.num_single
-        portions = (ctx.num_short if self.expand is not None else ctx.cu_seqlens_q.numel() - 1 - single) if single < n else 0
-        most = ctx.max_short if self.expand is not None else ctx.max_portion
-        for first, rows, seqs, tokens, where in (
-                (0, single, single, 1, dict(positions=positions, slot_mapping=ctx.slot_mapping)),
-                (single, n - single, portions, most, dict(cu_seqlens_q=ctx.cu_seqlens_q, seq_starts=ctx.seq_starts,
-                                                          first_seq=single, first_row=single))):
-            if not rows:
-                continue
-            splits = ops.latent_attention_splits(seqs, tokens, s.heads, self.window, ctx.max_len)
-            part, ml = ops.latent_partials(rows, splits, s, q.device)
-            ops.latent_attention(q[first:first + rows], self.cache, ctx.block_tables, self.window, self.scale, s, part, ml,
-                                 num_seqs=seqs, max_tokens=tokens, **where)
-            ops.latent_values(part, ml, self.values, out[first:first + rows], s)
+        single, short = ctx.num_single, self.expand is not None
+        if single:
+            batch = ops.LatentBatch(single, positions=positions, slot_mapping=ctx.slot_mapping)
+            self._tiles(q[:single], "single", batch, out[:single])
+        if single < n:
+            batch = ops.LatentBatch(ctx.num_short if short else ctx.cu_seqlens_q.numel() - 1 - single,
+                                    ctx.max_short if short else ctx.max_portion, cu_seqlens_q=ctx.cu_seqlens_q,
+                                    seq_starts=ctx.seq_starts, row_seq=ctx.row_seq[single:n], first_seq=single, first_row=single)
+            self._tiles(q[single:], "portions", batch, out[single:])
+
+    def _tiles(self, q, kind: str, batch, out):
+        ctx, s = get_context(), self.shape
+        key = (kind, s.heads, s.lp, self.window)           # layers of these sizes share a step's plan
+        if key not in ctx.plans:
+            ctx.plans[key] = ops.latent_plan(batch, s.heads, s.lp, self.window)
+        plan = ctx.plans[key]
+        part, ml = ops.latent_attention(q, self.cache, ctx.block_tables, self.window, self.scale, s, batch, plan)
+        ops.latent_values(part, ml, self.values, out, s, batch, plan)
 
     def _expanded(self, q, out):
         ctx, w = get_context(), self.window_index

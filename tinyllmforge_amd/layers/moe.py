@@ -53,14 +53,16 @@ class ClippedGLUExperts(nn.Module):
         self.down.data[:, self.width:].zero_()
         self.down.data[..., self.ff:].zero_()
 
+    def tile_rows(self, tokens: int) -> int:
+        """Rows of a tile of the grouped products: rows per expert decide between streaming the weights and reusing them."""
+        if self.router.dtype == torch.float32:
+            return 64
+        return 128 if tokens * self.top >= 48 * self.experts else 32
+
     def forward(self, h: torch.Tensor):
         """``(rows, index)``: the result for token t is the sum of ``rows[index[t]]``."""
         h = pad_columns(h, self.columns)
         ids, weights = ops.moe_route(h, self.router.data, self.experts, self.top)
-        if h.dtype == torch.float32:
-            tile = 64
-        else:       # rows per expert decide between the tile that streams weights and the one that reuses them
-            tile = 128 if h.shape[0] * self.top >= 48 * self.experts else 32
-        rows = ops.moe_group(ids, weights, self.experts, tile)
+        rows = ops.moe_group(ids, weights, self.experts, self.tile_rows(h.shape[0]))
         a = ops.moe_gemm(h, self.gate_up.data, rows, gather=True, clipped_glu=True, limit=self.limit)
         return ops.moe_gemm(a, self.down.data, rows, gather=False), rows.row_of

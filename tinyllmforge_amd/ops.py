@@ -806,55 +806,92 @@ def latent_prefill_supported(shape: LatentShape) -> bool:
     return bool(_lib.load().tlf_latent_prefill_supported(*shape.sizes))
 
 
-def latent_partials(rows, splits, shape: LatentShape, device):
-    return (torch.empty(splits, rows, shape.heads, shape.rp, dtype=torch.float32, device=device),
-            torch.empty(splits, rows, shape.heads, 2, dtype=torch.float32, device=device))
-
-
 def latent_rows(q, cache, block_tables, positions, slot_mapping, row_seq, window, scale, shape: LatentShape):
-    """Absorbed attention of any rows; ``q [N, H, Lp]``.  Returns ``(part, ml)`` of one split."""
+    """Absorbed attention of any rows; ``q [N, H, Lp]``.  Returns ``(part, ml)`` for ``latent_values``."""
     lib = _lib.load()
     _need(q, cache.dtype, "q"); _need(block_tables, torch.int32, "block_tables"); _need(positions, torch.int64, "positions")
     rows = q.shape[0]
     assert q.is_contiguous() and q.shape[1:] == (shape.heads, shape.lp) and block_tables.stride(1) == 1
     assert positions.numel() == rows and slot_mapping.numel() == rows and (row_seq is not None or block_tables.shape[0] >= rows)
-    part, ml = latent_partials(rows, 1, shape, q.device)
+    part = torch.empty(rows, shape.heads, shape.rp, dtype=torch.float32, device=q.device)
+    ml = torch.empty(rows, shape.heads, 2, dtype=torch.float32, device=q.device)
     step = 32768                                     # rows per launch (grid limit)
     for lo in range(0, rows, step):
         n = min(step, rows - lo)
         assert row_seq is not None or lo == 0
         check(lib.tlf_latent_rows(q[lo:].data_ptr(), cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0),
                                   positions[lo:].data_ptr(), slot_mapping[lo:].data_ptr(),
-                                  row_seq[lo:].data_ptr() if row_seq is not None else None, part[0, lo:].data_ptr(),
-                                  ml[0, lo:].data_ptr(), n, *shape.sizes, cache.shape[1], window, cache.shape[0],
+                                  row_seq[lo:].data_ptr() if row_seq is not None else None, part[lo:].data_ptr(),
+                                  ml[lo:].data_ptr(), n, *shape.sizes, cache.shape[1], window, cache.shape[0],
                                   float(scale), _dt(q), _stream()), "tlf_latent_rows")
     return part, ml
 
 
-def latent_attention(q, cache, block_tables, window, scale, shape: LatentShape, part, ml, positions=None, slot_mapping=None,
-                     cu_seqlens_q=None, seq_starts=None, first_seq=0, first_row=0, num_seqs=0, max_tokens=1):
-    """Absorbed attention on the matrix cores: ``num_seqs`` single rows (``positions``, ``slot_mapping``) or portions."""
+class LatentBatch:
+    """Sequences that attend in the latent space in one call: ``num_seqs`` single rows (``positions``, ``slot_mapping``), or
+    portions of at most ``max_tokens`` rows (``cu_seqlens_q``, ``seq_starts``, ``row_seq`` of their rows, the step's row of
+    the first one)."""
+    __slots__ = ("positions", "slot_mapping", "cu_seqlens_q", "seq_starts", "row_seq", "first_seq", "first_row", "num_seqs",
+                 "max_tokens")
+
+    def __init__(self, num_seqs, max_tokens=1, positions=None, slot_mapping=None, cu_seqlens_q=None, seq_starts=None,
+                 row_seq=None, first_seq=0, first_row=0):
+        self.num_seqs, self.max_tokens, self.positions, self.slot_mapping = num_seqs, max_tokens, positions, slot_mapping
+        self.cu_seqlens_q, self.seq_starts, self.row_seq = cu_seqlens_q, seq_starts, row_seq
+        self.first_seq, self.first_row = first_seq, first_row
+
+    @property
+    def where(self):
+        return (_opt(self.positions), _opt(self.slot_mapping), _opt(self.cu_seqlens_q), _opt(self.seq_starts), self.first_seq,
+                self.first_row, self.num_seqs, self.max_tokens)
+
+    def layout(self, heads, row_size):
+        """int32 values of a plan, pieces, units of a piece."""
+        import ctypes
+        out = (ctypes.c_int32 * 3)()
+        check(_lib.load().tlf_latent_attn_layout(self.num_seqs, self.max_tokens, heads, row_size, ctypes.addressof(out)),
+              "tlf_latent_attn_layout")
+        return tuple(out)
+
+
+def latent_plan(batch: LatentBatch, heads, row_size, window):
+    """How a batch's keys are cut into pieces for the workgroups: once per step and window, for all layers of these sizes."""
+    device = (batch.positions if batch.cu_seqlens_q is None else batch.cu_seqlens_q).device
+    plan = torch.empty(batch.layout(heads, row_size)[0], dtype=torch.int32, device=device)
+    check(_lib.load().tlf_latent_attn_plan(*batch.where, heads, row_size, window, plan.data_ptr(), _stream()), "tlf_latent_attn_plan")
+    return plan
+
+
+def latent_attention(q, cache, block_tables, window, scale, shape: LatentShape, batch: LatentBatch, plan):
+    """Absorbed attention on the matrix cores; ``q`` holds the batch's rows.  Returns ``(part, ml)`` for ``latent_values``."""
     lib = _lib.load()
-    _need(q, BF16, "q"); _need(block_tables, torch.int32, "block_tables")
+    _need(q, BF16, "q"); _need(block_tables, torch.int32, "block_tables"); _need(plan, torch.int32, "plan")
     assert q.is_contiguous() and q.shape[1:] == (shape.heads, shape.lp) and block_tables.stride(1) == 1
-    assert block_tables.shape[0] >= first_seq + num_seqs and cache.is_contiguous() and cache.dtype == BF16
-    check(lib.tlf_latent_attn(q.data_ptr(), cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), _opt(positions),
-                              _opt(slot_mapping), _opt(cu_seqlens_q), _opt(seq_starts), first_seq, first_row, num_seqs, max_tokens,
-                              part.data_ptr(), ml.data_ptr(), part.shape[0], part.shape[1], *shape.sizes, cache.shape[1],
-                              window, cache.shape[0], float(scale), _stream()), "tlf_latent_attn")
+    assert block_tables.shape[0] >= batch.first_seq + batch.num_seqs and cache.is_contiguous() and cache.dtype == BF16
+    if batch.cu_seqlens_q is None:
+        assert q.shape[0] == batch.num_seqs <= min(batch.positions.numel(), batch.slot_mapping.numel())
+    need, pieces, units = batch.layout(shape.heads, shape.lp)
+    assert plan.numel() >= need
+    part = torch.empty(pieces, units, shape.rp, dtype=torch.float32, device=q.device)
+    ml = torch.empty(pieces, units, 2, dtype=torch.float32, device=q.device)
+    check(lib.tlf_latent_attn(q.data_ptr(), cache.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), *batch.where,
+                              plan.data_ptr(), part.data_ptr(), ml.data_ptr(), *shape.sizes, cache.shape[1], window,
+                              cache.shape[0], float(scale), _stream()), "tlf_latent_attn")
+    return part, ml
 
 
-def latent_attention_splits(num_seqs, max_tokens, heads, window, max_len) -> int:
-    return _lib.load().tlf_latent_attn_splits(num_seqs, max_tokens, heads, window, max_len)
-
-
-def latent_values(part, ml, uv, out, shape: LatentShape):
-    """``out [N, >= H * vdim]`` from the splits' mixed latents; ``uv [H, vdim rounded up to 16, Rp]``."""
+def latent_values(part, ml, uv, out, shape: LatentShape, batch: LatentBatch | None = None, plan=None):
+    """``out [N, >= H * vdim]`` from the pieces' mixed latents; ``uv [H, vdim rounded up to 16, Rp]``."""
     lib = _lib.load()
-    splits, rows = part.shape[:2]
-    assert out.shape[0] == rows and out.stride(1) == 1 and out.dtype == uv.dtype and part.is_contiguous() and uv.is_contiguous()
-    check(lib.tlf_latent_values(part.data_ptr(), ml.data_ptr(), splits, uv.data_ptr(), out.data_ptr(), out.stride(0), rows,
-                                *shape.sizes, _dt(uv), _stream()), "tlf_latent_values")
+    rows = out.shape[0]
+    assert out.stride(1) == 1 and out.dtype == uv.dtype and part.is_contiguous() and uv.is_contiguous()
+    assert plan is not None or part.shape[0] == rows
+    where = (None, None, 0, 0, 0, 0)
+    if plan is not None:
+        where = (_opt(batch.cu_seqlens_q), _opt(batch.row_seq), batch.first_seq, batch.first_row, batch.num_seqs, batch.max_tokens)
+        assert batch.row_seq is None or batch.row_seq.numel() >= rows
+    check(lib.tlf_latent_values(part.data_ptr(), ml.data_ptr(), _opt(plan), *where, uv.data_ptr(), out.data_ptr(),
+                                out.stride(0), rows, *shape.sizes, _dt(uv), _stream()), "tlf_latent_values")
 
 
 def latent_gather(cache, block_tables, cu_seqlens_q, seq_starts, kv_offsets, kv_rows, first_seq, num_seqs, max_rows, window):
