@@ -937,12 +937,12 @@ def bench_gigopel_kernels(sizes=None):
         gu, dn = bf(2 * ff, w), bf(w, ff)
         for n in (B, 512, N):
             x = bf(n, w)
-            ids, wt = P.moe_route(x, moe.router.data, ne, top)
-            add(f"router, {n} tokens", size, lambda i: P.moe_route(x, moe.router.data, ne, top), ne * w * 2 + n * w * 2, "hbm")
+            sums = P.moe_logits(x, moe.router.data)
+            add(f"router, {n} tokens", size, lambda i: P.moe_logits(x, moe.router.data), ne * w * 2 + n * w * 2, "hbm")
             tile = moe.tile_rows(n)
-            add(f"rows by expert, {n} tokens", size, lambda i: P.moe_group(ids, wt, ne, tile), n * top * 24, "hbm")
-            g = P.moe_group(ids, wt, ne, tile)
-            active = len(set(ids.flatten().tolist()))
+            add(f"rows by expert, {n} tokens", size, lambda i: P.moe_group(sums, ne, top, tile), n * (ne * 4 + top * 20), "hbm")
+            g = P.moe_group(sums, ne, top, tile)
+            active = len(set(g.ids.flatten().tolist()))
             a = P.moe_gemm(x, moe.gate_up.data, g, True, True, 7.0)
             ad = bf(n, ff)
             big = n == N

@@ -658,22 +658,25 @@ int tlf_latent_prefill(const void *q, const void *expanded, int64_t expanded_str
 
 /* Mixture of experts.  Rows (token, k) are put in expert order; nothing on the host depends on the routing.
  *
- * tlf_moe_route: z = router h (router [experts rounded up to 16, K], K a multiple of 64; fp32 sums), ids[token, k] the `top`
- *   largest (ties: the smaller index) and weights[token, k] = sigmoid(z).  experts <= 512.
- * tlf_moe_group: row_of[token * top + k] = the entry's row in expert order, src[row] its token, row_weight[row] its weight;
+ * tlf_gemm_f32_sums: y = x . w^T with bf16 factors as fp32 sums [*splits, M, N] to be added up (*splits in host memory);
+ *   for the router's logits, N = experts rounded up to 16.
+ * tlf_moe_group: from the logits' sums, ids[token, k] the `top` largest (ties: the smaller index) and weights[token, k] =
+ *   sigmoid; row_of[token * top + k] = the entry's row in expert order, src[row] its token, row_weight[row] its weight;
  *   tiles (int32 x 4: expert, first row, rows, 0) cut the rows into at most tile_rows of one expert each, *num_tiles <=
- *   max_tiles of them; max_tiles >= n * top / tile_rows + min(experts, n * top).
+ *   max_tiles of them; max_tiles >= n * top / tile_rows + min(experts, n * top).  experts <= 512.
  * tlf_moe_gemm: y[row] = W[expert] x[x_rows ? x_rows[row] : row]; w [experts, N, K].  clipped_glu: channels are interleaved
  *   as for the SiLU-and-mul products (8 gate, then the 8 matching up); with f = row_scale[row] (NULL: 1), g = min(f gate,
  *   limit), u = clamp(f up, +-limit): y [rows, N / 2] = g sigmoid(1.702 g) (u + 1).  bf16: tile_rows 32 or 128, K a multiple
  *   of 64; fp32: tile_rows 64.  x_count bounds the x rows.
  * tlf_xielu: with a = softplus(pq[0]), b = 1/2 + softplus(pq[1]), out = a z^2 + z / 2 for z > 0, b (e^z - 1 - z) + z / 2
  *   otherwise, z = columns col .. col + cols - 1 of x (or of partial sums); columns cols .. padded_cols - 1 become 0. */
-int tlf_moe_route(const void *h, int64_t h_stride, const void *router, int32_t *ids, float *weights, int32_t n,
-                  int32_t experts, int32_t K, int32_t top, int32_t dtype, void *stream);
-int tlf_moe_group(const int32_t *ids, const float *weights, int32_t *row_of, int32_t *src, float *row_weight, int32_t
-                  *tiles, int32_t *num_tiles, int32_t max_tiles, int32_t n, int32_t top, int32_t experts, int32_t
-                  tile_rows, void *stream);
+size_t tlf_gemm_f32_sums_bytes(int32_t M, int32_t N, int32_t K);
+int tlf_gemm_f32_sums(const void *x, int64_t x_stride, const void *w, float *sums, size_t sums_bytes, int32_t M,
+                      int32_t N, int32_t K, int32_t *splits, void *stream);
+size_t tlf_moe_group_workspace_bytes(int32_t n, int32_t top, int32_t experts);
+int tlf_moe_group(const float *sums, int32_t splits, int32_t *ids, float *weights, int32_t *row_of, int32_t *src,
+                  float *row_weight, int32_t *tiles, int32_t *num_tiles, int32_t max_tiles, int32_t n, int32_t top,
+                  int32_t experts, int32_t tile_rows, void *workspace, size_t workspace_bytes, void *stream);
 int tlf_moe_gemm(const void *x, int64_t x_stride, int32_t x_count, const void *w, void *y, const int32_t *tiles,
                  const int32_t *num_tiles, int32_t max_tiles, int32_t tile_rows, const int32_t *x_rows, const float
                  *row_scale, int32_t rows, int32_t N, int32_t K, int32_t clipped_glu, float limit, int32_t dtype,

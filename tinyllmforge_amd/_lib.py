@@ -106,8 +106,10 @@ SIGNATURES = {
     "tlf_latent_prefill_supported": (c_int32, [_I32, _I32, _I32, _I32, _I32]),
     "tlf_latent_prefill": (c_int32, [_P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P, _I64, _I32, _I32, _I32,
                                      _I32, _I32, _I32, _F, _P]),
-    "tlf_moe_route": (c_int32, [_P, _I64, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P]),
-    "tlf_moe_group": (c_int32, [_P, _P, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P]),
+    "tlf_gemm_f32_sums_bytes": (_SZ, [_I32, _I32, _I32]),
+    "tlf_gemm_f32_sums": (c_int32, [_P, _I64, _P, _P, _SZ, _I32, _I32, _I32, _P, _P]),
+    "tlf_moe_group_workspace_bytes": (_SZ, [_I32, _I32, _I32]),
+    "tlf_moe_group": (c_int32, [_P, _I32, _P, _P, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P, _SZ, _P]),
     "tlf_moe_gemm": (c_int32, [_P, _I64, _I32, _P, _P, _P, _P, _I32, _I32, _P, _P, _I32, _I32, _I32, _I32, _F, _I32,
                                _P]),
     "tlf_xielu": (c_int32, [_P, _I64, _P, _I32, _P, _I32, _P, _P, _I64, _I32, _I32, _I32, _I32, _P]),

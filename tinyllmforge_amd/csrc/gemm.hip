@@ -1615,6 +1615,25 @@ int launch_grouped(GemmParams p, int bm, hipStream_t stream) {
   return launch_status();
 }
 
+// bf16 factors, fp32 result [splits, M, N] (the epilogue of a split plan, whatever the number of splits).  For narrow N:
+// 64 x 64 tiles with wave sets that split K, and a split across workgroups until about 256 of them exist.
+struct F32SumsPlan {
+  int kg, splits, k_per_split;
+};
+inline F32SumsPlan f32_sums_plan(int M, int N, int K) {
+  const int ktiles = K / kBK, tiles = ((N + 63) / 64) * ((M + 63) / 64);
+  F32SumsPlan g;
+  g.kg = ktiles % 4 == 0 ? 4 : ktiles % 2 == 0 ? 2 : 1;
+  int splits = 256 / tiles;
+  if (splits > ktiles / g.kg) splits = ktiles / g.kg;
+  if (splits > 16) splits = 16;
+  if (splits < 1) splits = 1;
+  const int per = ((ktiles + splits - 1) / splits + g.kg - 1) / g.kg * g.kg;
+  g.k_per_split = per * kBK;
+  g.splits = (ktiles + per - 1) / per;
+  return g;
+}
+
 inline size_t align256(size_t n) { return (n + 255) & ~static_cast<size_t>(255); }
 
 // Row-major int8 [N, K] -> tile order (see the head of this file).  One thread moves one 16-byte
@@ -1762,6 +1781,45 @@ extern "C" int tlf_gemm_deferred(const void *x, int64_t x_stride, const void *w,
   hipStream_t s = static_cast<hipStream_t>(stream);
   return scale ? launch_gemm<true>(x, x_stride, w, scale, y, M, N, K, workspace, workspace_bytes, s, nullptr, 0, nullptr, nullptr, splits)
                : launch_gemm<false>(x, x_stride, w, nullptr, y, M, N, K, workspace, workspace_bytes, s, nullptr, 0, nullptr, nullptr, splits);
+}
+
+extern "C" size_t tlf_gemm_f32_sums_bytes(int32_t M, int32_t N, int32_t K) {
+  if (M <= 0 || N <= 0 || K <= 0 || K % kBK) return 0;
+  return static_cast<size_t>(f32_sums_plan(M, N, K).splits) * M * N * 4;
+}
+
+extern "C" int tlf_gemm_f32_sums(const void *x, int64_t x_stride, const void *w, float *sums, size_t sums_bytes, int32_t M,
+                                 int32_t N, int32_t K, int32_t *splits, void *stream) {
+  if (!splits) return TLF_E_NULL;
+  *splits = 1;
+  if (M == 0) return TLF_OK;
+  const int rc = check_gemm_args(x, x_stride, w, sums, M, N, K);
+  if (rc != TLF_OK) return rc;
+  const F32SumsPlan g = f32_sums_plan(M, N, K);
+  if (sums_bytes < static_cast<size_t>(g.splits) * M * N * 4) return TLF_E_WORKSPACE;
+  GemmParams p{};
+  p.x = static_cast<const unsigned char *>(x);
+  p.ldx_bytes = x_stride * 2;
+  p.w = static_cast<const unsigned char *>(w);
+  p.partial = sums;
+  p.M = M; p.N = N; p.K = K;
+  p.k_per_split = g.k_per_split;
+  p.splits = 2;                        // the epilogue that writes fp32
+  p.m_tiles = (M + 63) / 64;
+  p.n_tiles = (N + 63) / 64;
+  p.xcd_rows = 1;
+  p.group_n = 1;
+  p.map_full = p.m_tiles / 8 * 8;
+  p.map_rem = p.m_tiles - p.map_full;
+  p.map_main = p.map_full * p.n_tiles;
+  const dim3 grid(p.map_main + p.map_rem * p.n_tiles, g.splits);
+  if (p.map_rem == 0) p.map_rem = 1;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (g.kg == 4) TLF_LAUNCH((gemm_dlds_kernel<64, 64, 2, 2, false, 2, 4, 4>), grid, dim3(1024), 0, s, p);
+  else if (g.kg == 2) TLF_LAUNCH((gemm_dlds_kernel<64, 64, 2, 2, false, 2, 4, 2>), grid, dim3(512), 0, s, p);
+  else TLF_LAUNCH((gemm_dlds_kernel<64, 64, 2, 2, false, 2, 4, 1>), grid, dim3(256), 0, s, p);
+  *splits = g.splits;
+  return launch_status();
 }
 
 extern "C" int tlf_gemm_plan(int32_t M, int32_t N, int32_t K, int32_t w8, int32_t *plan8) {

@@ -57,34 +57,38 @@ __device__ __forceinline__ void turn8(const LatentPrepArgs &a, const float *cs, 
   }
 }
 
-// blockIdx.y == 0: the latents of 4 tokens, a wave each; otherwise 256 8-value pieces of a token's queries
-template <typename T, bool PART>
+// blockIdx.y == 0: the latents of TOK tokens, a wave each; otherwise 256 8-value pieces of those tokens' queries, all loads
+// in flight before the first is used
+template <typename T, bool PART, int TOK>
 __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a) {
   const LatentShape &s = a.s;
+  const int64_t tok0 = static_cast<int64_t>(blockIdx.x) * TOK;
   if (blockIdx.y == 0) {
-    const int64_t tok = static_cast<int64_t>(blockIdx.x) * 4 + (threadIdx.x >> 6);
+    const int64_t tok = tok0 + (threadIdx.x >> 6);
     const int lane = threadIdx.x & 63;
-    if (tok >= a.n) return;   // whole waves leave together
-    const int64_t slot = a.slots[tok];
-    if (slot < 0 || slot >= a.num_slots) return;
-    const int64_t pos = a.positions[tok];
+    if ((threadIdx.x >> 6) >= TOK || tok >= a.n) return;   // whole waves leave together
+    const int64_t slot = a.slots[tok], pos = a.positions[tok];
     const float *cs = pos >= 0 && pos < a.max_pos ? a.cos_sin + pos * s.rot : nullptr;
-    T *row = static_cast<T *>(a.cache) + slot * s.Lp;
     constexpr int kKeep = 3;   // pieces of 8 a lane holds: rank <= 1536
-    float f[kKeep][8];
+    const T *w = static_cast<const T *>(a.norm);
+    float f[kKeep][8], t[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     float ss = 0.f;
 #pragma unroll
     for (int k = 0; k < kKeep; ++k) {
       const int d = (lane + k * 64) * 8;
-      if (d < s.rank) {
-        prep_ld8<T, PART>(a, tok, a.off, d, s.rank, f[k]);
+      if (d < s.rank) prep_ld8<T, PART>(a, tok, a.off, d, s.rank, f[k]);
+    }
+    if (lane * 8 < s.rot) prep_ld8<T, PART>(a, tok, a.off + s.rank, lane * 8, s.rot, t);
+    if (slot < 0 || slot >= a.num_slots) return;
+    T *row = static_cast<T *>(a.cache) + slot * s.Lp;
+#pragma unroll
+    for (int k = 0; k < kKeep; ++k)
+      if ((lane + k * 64) * 8 < s.rank) {
 #pragma unroll
         for (int e = 0; e < 8; ++e) ss = fmaf(f[k][e], f[k][e], ss);
       }
-    }
     ss = wave_sum(ss);
     const float inv = 1.0f / sqrtf(ss / static_cast<float>(s.rank) + a.eps);
-    const T *w = static_cast<const T *>(a.norm);
 #pragma unroll
     for (int k = 0; k < kKeep; ++k) {
       const int d = (lane + k * 64) * 8;
@@ -95,11 +99,12 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a
       }
     }
     for (int d = lane * 8; d < s.Lp - s.Ra; d += 512) {
-      float t[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-      if (d < s.rot) {
-        prep_ld8<T, PART>(a, tok, a.off + s.rank, d, s.rot, t);
-        turn8(a, cs, d, t);
+      if (d >= 512) {           // rot > 512
+#pragma unroll
+        for (int e = 0; e < 8; ++e) t[e] = 0.f;
+        if (d < s.rot) prep_ld8<T, PART>(a, tok, a.off + s.rank, d, s.rot, t);
       }
+      if (d < s.rot) turn8(a, cs, d, t);
       Elem<T>::st8(row + s.Ra + d, t);
     }
     return;
@@ -109,19 +114,23 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a
   if (item >= s.H * nch) return;
   const int h = item / nch, d = (item - h * nch) * 8;
   const int col = h * (s.dim + s.rot);
+  const bool own = d < s.Da, turned = !own && d < s.Da + s.rot;
+  float f[TOK][8];
+  int64_t pos[TOK];
 #pragma unroll
-  for (int k = 0; k < 4; ++k) {
-    const int64_t tok = static_cast<int64_t>(blockIdx.x) * 4 + k;
-    if (tok >= a.n) return;
-    float f[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    if (d < s.Da) {
-      prep_ld8<T, PART>(a, tok, col, d, s.dim, f);
-    } else if (d < s.Da + s.rot) {
-      const int64_t pos = a.positions[tok];
-      prep_ld8<T, PART>(a, tok, col + s.dim, d - s.Da, s.rot, f);
-      turn8(a, pos >= 0 && pos < a.max_pos ? a.cos_sin + pos * s.rot : nullptr, d - s.Da, f);
-    }
-    Elem<T>::st8(static_cast<T *>(a.q_out) + (tok * s.H + h) * s.Dq + d, f);
+  for (int k = 0; k < TOK; ++k) {
+    const int64_t tok = min(tok0 + k, static_cast<int64_t>(a.n) - 1);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[k][e] = 0.f;
+    if (own) prep_ld8<T, PART>(a, tok, col, d, s.dim, f[k]);
+    else if (turned) prep_ld8<T, PART>(a, tok, col + s.dim, d - s.Da, s.rot, f[k]);
+    pos[k] = turned ? a.positions[tok] : 0;
+  }
+#pragma unroll
+  for (int k = 0; k < TOK; ++k) {
+    if (tok0 + k >= a.n) return;
+    if (turned) turn8(a, pos[k] >= 0 && pos[k] < a.max_pos ? a.cos_sin + pos[k] * s.rot : nullptr, d - s.Da, f[k]);
+    Elem<T>::st8(static_cast<T *>(a.q_out) + ((tok0 + k) * s.H + h) * s.Dq + d, f[k]);
   }
 }
 
@@ -295,36 +304,49 @@ __device__ __forceinline__ float piece_weight(const LatentValuesArgs &a, const P
 // bf16: a workgroup takes one head, 16 rows and 64 outputs; the mixed latents of the rows go through LDS once
 __global__ __launch_bounds__(256) void latent_values_kernel(const LatentValuesArgs a) {
   extern __shared__ __attribute__((aligned(16))) unsigned short lat[];   // [16][Rp + 8]
-  __shared__ float tot[16][2];
+  __shared__ float wt[16][kLatentMaxPieces + 1];
   __shared__ Pieces pcs[16];
   const LatentShape &s = a.s;
   const int h = blockIdx.x, row0 = blockIdx.y * 16, tid = threadIdx.x;
   const int stride = s.Rp + 8;
-  if (tid < 16) {
-    Pieces p = Pieces{0, 0, 0};
-    if (row0 + tid < a.rows) {
-      p = latent_pieces(a, row0 + tid, h);
-      float mx, inv;
-      pieces_total(a, p, mx, inv);
-      tot[tid][0] = mx;
-      tot[tid][1] = inv;
+  {
+    // 16 lanes per row, a piece each at a time
+    const int r = tid >> 4, j = tid & 15;
+    const Pieces p = row0 + r < a.rows ? latent_pieces(a, row0 + r, h) : Pieces{0, 0, 0};
+    if (j == 0) pcs[r] = p;
+    float mx = -INFINITY, den = 0.f;
+    for (int k0 = 0; k0 < p.count; k0 += 16) {
+      float2 v = make_float2(-INFINITY, 0.f);
+      if (k0 + j < p.count) v = *reinterpret_cast<const float2 *>(a.ml + (p.first + static_cast<int64_t>(k0 + j) * p.step) * 2);
+      const float m1 = v.y > 0.f ? v.x : -INFINITY;
+      float mn = m1;
+#pragma unroll
+      for (int o = 1; o < 16; o <<= 1) mn = fmaxf(mn, __shfl_xor(mn, o, 64));
+      mn = fmaxf(mn, mx);
+      den = den * (mx == mn ? 1.f : exp2f(mx - mn)) + group_sum<16>(v.y > 0.f ? v.y * exp2f(m1 - mn) : 0.f);
+      mx = mn;
+      if (k0 + j < p.count) wt[r][k0 + j] = m1;
     }
-    pcs[tid] = p;
+    const float inv = den > 0.f ? 1.0f / den : 0.f;
+    for (int k = j; k < p.count; k += 16) wt[r][k] = wt[r][k] == -INFINITY ? 0.f : exp2f(wt[r][k] - mx) * inv;
   }
   __syncthreads();
   const int nch = s.Rp / 8;
   for (int item = tid; item < 16 * nch; item += 256) {
     const int r = item / nch, d = (item - r * nch) * 8;
     const Pieces p = pcs[r];
-    const float mx = tot[r][0], inv = tot[r][1];
     float o[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < p.count; ++k) {
-      const float w = piece_weight(a, p, k, mx, inv);
-      if (w > 0.f) {
-        float f[8];
-        Elem<float>::ld8(a.part + (p.first + static_cast<int64_t>(k) * p.step) * s.Rp + d, f);
+    const float *src = a.part + p.first * s.Rp + d;
+    const int64_t step = static_cast<int64_t>(p.step) * s.Rp;
+    for (int k0 = 0; k0 < p.count; k0 += 4) {
+      float f[4][8];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) o[e] = fmaf(w, f[e], o[e]);
+      for (int k = 0; k < 4; ++k) Elem<float>::ld8(src + min(k0 + k, p.count - 1) * step, f[k]);
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const float w = k0 + k < p.count ? wt[r][k0 + k] : 0.f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o[e] = fmaf(w, f[k][e], o[e]);
       }
     }
     *reinterpret_cast<uint4 *>(lat + r * stride + d) = pack8(o);
@@ -413,11 +435,18 @@ extern "C" int tlf_latent_prep(const void *proj, int64_t proj_stride, const floa
   a.max_pos = max_pos; a.slots = slot_mapping; a.num_slots = num_slots; a.q_out = q_out; a.cache = cache; a.n = n; a.eps = eps;
   a.vec = dim % 8 == 0 && rot_dim % 8 == 0 && rank % 8 == 0 && latent_col % 8 == 0 && proj_stride % 8 == 0 &&
           (splits > 1 || aligned16(proj));
-  const dim3 grid((n + 3) / 4, 1 + (heads * (a.s.Dq / 8) + 255) / 256);
+  const int tok = splits <= 1 && n > 1024 ? 4 : 1;
+  const dim3 grid((n + tok - 1) / tok, 1 + (heads * (a.s.Dq / 8) + 255) / 256);
   hipStream_t s = static_cast<hipStream_t>(stream);
-  if (splits > 1) TLF_LAUNCH((latent_prep_kernel<unsigned short, true>), grid, dim3(256), 0, s, a);
-  else if (dtype == TLF_DT_BF16) TLF_LAUNCH((latent_prep_kernel<unsigned short, false>), grid, dim3(256), 0, s, a);
-  else TLF_LAUNCH((latent_prep_kernel<float, false>), grid, dim3(256), 0, s, a);
+#define TLF_PREP(T, PART)                                                                        \
+  do {                                                                                           \
+    if (tok == 4) TLF_LAUNCH((latent_prep_kernel<T, PART, 4>), grid, dim3(256), 0, s, a);        \
+    else TLF_LAUNCH((latent_prep_kernel<T, PART, 1>), grid, dim3(256), 0, s, a);                 \
+  } while (0)
+  if (splits > 1) TLF_PREP(unsigned short, true);
+  else if (dtype == TLF_DT_BF16) TLF_PREP(unsigned short, false);
+  else TLF_PREP(float, false);
+#undef TLF_PREP
   return launch_status();
 }
 

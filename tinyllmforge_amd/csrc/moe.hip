@@ -1,8 +1,9 @@
 // Mixture of experts: router, grouping of the rows by expert, the grouped products, and the xIELU activation of dense
 // layers.
 //
-//   router     z = W_router h (bf16 or fp32 factors, fp32 sums), the `top` largest of each row and their sigmoids
-//   group      rows (token, k) in expert order, an index each way, tiles of `tile_rows` rows of one expert
+//   router     z = W_router h (tlf_gemm_f32_sums or the fp32 product)
+//   group      the `top` largest logits of each row and their sigmoids; rows (token, k) in expert order, an index each way,
+//              tiles of `tile_rows` rows of one expert
 //   products   gemm_dlds_kernel<GROUPED> (gemm.hip) in bf16; a plain fp32 kernel here
 // No host value depends on the routing: grids are sized for the worst case and tiles past the list's end leave at once,
 // so a captured graph replays with any routing.
@@ -15,124 +16,79 @@ int launch_grouped(GemmParams p, int bm, hipStream_t stream);
 
 constexpr int kMaxExperts = 512;
 
-struct RouterArgs {
-  const void *h;          // [n, ldh]
-  const void *w;          // [E16, K], E rounded up to 16
-  int64_t ldh;
-  int32_t *ids;           // [n, top]
-  float *weights;         // [n, top]
-  int32_t n, E, E16, K, top;
-};
-
-// One wave picks the `top` largest of logits z[0 .. E): key order is value, then the smaller index.
-__device__ __forceinline__ void pick_top(const RouterArgs &a, const float *z, int64_t tok) {
-  const int lane = threadIdx.x & 63;
-  float v[kMaxExperts / 64];
-  unsigned long long key[kMaxExperts / 64];
-#pragma unroll
-  for (int i = 0; i < kMaxExperts / 64; ++i) {
-    const int e = i * 64 + lane;
-    v[i] = e < a.E ? z[e] : 0.f;
-    unsigned int b = __float_as_uint(v[i] + 0.0f);
-    b = (b & 0x80000000u) ? ~b : (b | 0x80000000u);
-    key[i] = e < a.E ? (static_cast<unsigned long long>(b) << 32) | (0xffffffffu - static_cast<unsigned>(e)) : 0ull;
-  }
-  for (int k = 0; k < a.top; ++k) {
-    unsigned long long best = 0;
-#pragma unroll
-    for (int i = 0; i < kMaxExperts / 64; ++i) best = key[i] > best ? key[i] : best;
-    best = wave_max_u64(best);
-    const int e = static_cast<int>(0xffffffffu - static_cast<unsigned>(best & 0xffffffffu));
-#pragma unroll
-    for (int i = 0; i < kMaxExperts / 64; ++i)
-      if (key[i] == best) {
-        a.ids[tok * a.top + k] = e;
-        a.weights[tok * a.top + k] = sigmoid_f32(v[i]);
-        key[i] = 0;
-      }
-  }
-}
-
-// bf16: 16 tokens per workgroup, eight waves split K, experts 64 at a time
-__global__ __launch_bounds__(512) void router_kernel(const RouterArgs a) {
-  extern __shared__ __attribute__((aligned(16))) float logits[];    // [16][E16 + 4]
-  __shared__ __attribute__((aligned(16))) float red[8][16][68];
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, n = lane & 15, g = lane >> 4;
-  const int tok0 = blockIdx.x * 16, ldz = a.E16 + 4;
-  const unsigned short *hp = static_cast<const unsigned short *>(a.h) + min(tok0 + n, a.n - 1) * a.ldh + g * 8;
-  const int steps = a.K / 32, lo = steps * wave / 8, hi = steps * (wave + 1) / 8;
-  for (int e0 = 0; e0 < a.E16; e0 += 64) {
-    const int tiles = min(4, (a.E16 - e0) / 16);
-    const unsigned short *wp[4];
-    floatx4 acc[4];
-#pragma unroll
-    for (int t = 0; t < 4; ++t) {
-      wp[t] = static_cast<const unsigned short *>(a.w) + static_cast<int64_t>(e0 + min(t, tiles - 1) * 16 + n) * a.K + g * 8;
-      acc[t] = floatx4{0.f, 0.f, 0.f, 0.f};
-    }
-#pragma unroll 2
-    for (int k = lo; k < hi; ++k) {
-      Pack16 x, w[4];
-      x.u = *reinterpret_cast<const uint4 *>(hp + k * 32);
-#pragma unroll
-      for (int t = 0; t < 4; ++t) w[t].u = *reinterpret_cast<const uint4 *>(wp[t] + k * 32);
-#pragma unroll
-      for (int t = 0; t < 4; ++t) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[t].v, x.v, acc[t], 0, 0, 0);
-    }
-#pragma unroll
-    for (int t = 0; t < 4; ++t)
-      *reinterpret_cast<float4 *>(&red[wave][n][t * 16 + g * 4]) = make_float4(acc[t][0], acc[t][1], acc[t][2], acc[t][3]);
-    __syncthreads();
-    for (int i = tid; i < 16 * tiles * 16; i += 512) {
-      const int r = i / (tiles * 16), e = i - r * (tiles * 16);
-      float s = 0.f;
-#pragma unroll
-      for (int w = 0; w < 8; ++w) s += red[w][r][e];
-      logits[r * ldz + e0 + e] = s;
-    }
-    __syncthreads();
-  }
-  for (int r = wave; r < 16 && tok0 + r < a.n; r += 8) pick_top(a, logits + r * ldz, tok0 + r);
-}
-
-// fp32: a workgroup per token, a wave per expert
-__global__ __launch_bounds__(256) void router_f32_kernel(const RouterArgs a) {
-  __shared__ float logits[kMaxExperts];
-  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int64_t tok = blockIdx.x;
-  const float *h = static_cast<const float *>(a.h) + tok * a.ldh;
-  for (int e = wave; e < a.E; e += 4) {
-    const float *w = static_cast<const float *>(a.w) + static_cast<int64_t>(e) * a.K;
-    float s = 0.f;
-    for (int k = lane; k < a.K; k += 64) s = fmaf(h[k], w[k], s);
-    s = wave_sum(s);
-    if (lane == 0) logits[e] = s;
-  }
-  __syncthreads();
-  if (wave == 0) pick_top(a, logits, tok);
-}
-
-// ---------------------------------------------------------------------------------------------------------------
 struct GroupArgs {
-  const int32_t *ids;       // [entries]
-  const float *weights;     // [entries]
+  const float *sums;        // [splits, n, E16] partial router logits
+  int64_t plane;            // n * E16
+  int32_t *ids;             // [entries] expert of entry (token, k)
+  float *weights;           // [entries] its score
   int32_t *row_of;          // [entries] row of an entry in expert order
   int32_t *src;             // [entries] token of a row
   float *row_weight;        // [entries] weight of a row
   int4 *tiles;
   int32_t *num_tiles;
-  int32_t entries, E, top, tile_rows;
+  int32_t *hist;            // [blocks, E]
+  int32_t n, splits, E, E16, top, entries, tile_rows, blocks;
 };
 
-// One workgroup: counts, prefix sums, tile list, placement.  The order of rows inside an expert is arbitrary (it does not
-// enter any value).
-__global__ __launch_bounds__(1024) void moe_group_kernel(const GroupArgs a) {
-  __shared__ int count[kMaxExperts], start[kMaxExperts], cursor[kMaxExperts], tstart[kMaxExperts];
+__device__ __forceinline__ float wave_max(float v) {
+  v = fmaxf(v, dpp_move<0xB1>(v));    // quad_perm [1, 0, 3, 2]
+  v = fmaxf(v, dpp_move<0x4E>(v));    // quad_perm [2, 3, 0, 1]
+  v = fmaxf(v, dpp_move<0x141>(v));   // row_half_mirror
+  v = fmaxf(v, dpp_move<0x140>(v));   // row_mirror
+  return max_lanes_16_32_48(v);
+}
+
+// One wave picks the `top` largest logits of a token: by value, then the smaller index.  logit(e): expert e's.
+template <typename F>
+__device__ __forceinline__ void pick_top(const GroupArgs &a, F logit, int32_t *ids, float *weights) {
+  const int lane = threadIdx.x & 63;
+  constexpr int kEach = kMaxExperts / 64;
+  float v[kEach];
+#pragma unroll
+  for (int i = 0; i < kEach; ++i) {
+    v[i] = -INFINITY;
+    if (i * 64 < a.E) {            // uniform
+      const int e = i * 64 + lane;
+      const float z = logit(min(e, a.E - 1));
+      if (e < a.E) v[i] = z > -3.0e38f ? z : -3.0e38f;     // every pick finds an expert, whatever the input
+    }
+  }
+  for (int k = 0; k < a.top; ++k) {
+    float m = v[0];
+#pragma unroll
+    for (int i = 1; i < kEach; ++i) m = fmaxf(m, v[i]);
+    m = wave_max(m);
+    bool found = false;
+#pragma unroll
+    for (int i = 0; i < kEach; ++i) {
+      if (found || i * 64 >= a.E) continue;          // uniform
+      const unsigned long long who = __ballot(v[i] == m);
+      if (who == 0) continue;
+      found = true;
+      if (lane == __ffsll(who) - 1) {
+        ids[k] = i * 64 + lane;
+        weights[k] = sigmoid_f32(m);
+        v[i] = -INFINITY;
+      }
+    }
+  }
+}
+
+__global__ __launch_bounds__(256) void moe_pick_kernel(const GroupArgs a) {
+  const int64_t tok = blockIdx.x * (blockDim.x / 64) + (threadIdx.x >> 6);
+  if (tok >= a.n) return;
+  const float *z = a.sums + tok * a.E16;
+  pick_top(a, [&](int e) __attribute__((always_inline)) {
+    float v = 0.f;
+#pragma unroll 16
+    for (int k = 0; k < a.splits; ++k) v += z[k * a.plane + e];
+    return v;
+  }, a.ids + tok * a.top, a.weights + tok * a.top);
+}
+
+// From the experts' row counts: first row and first tile of each, the tile list.  The first wave scans, all threads write.
+__device__ __forceinline__ void expert_tiles(const GroupArgs &a, const int *count, int *start, int *tstart) {
   const int tid = threadIdx.x;
-  for (int e = tid; e < a.E; e += 1024) count[e] = 0;
-  __syncthreads();
-  for (int i = tid; i < a.entries; i += 1024) atomicAdd(&count[a.ids[i]], 1);
-  __syncthreads();
   if (tid < 64) {
     constexpr int kEach = kMaxExperts / 64;
     int rows = 0, tiles = 0;
@@ -154,7 +110,7 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const GroupArgs a) {
     for (int k = 0; k < kEach; ++k) {
       const int e = tid * kEach + k;
       if (e < a.E) {
-        start[e] = cursor[e] = r;
+        start[e] = r;
         tstart[e] = t;
         r += count[e];
         t += (count[e] + a.tile_rows - 1) / a.tile_rows;
@@ -162,15 +118,90 @@ __global__ __launch_bounds__(1024) void moe_group_kernel(const GroupArgs a) {
     }
   }
   __syncthreads();
-  for (int e = tid; e < a.E; e += 1024)
+  for (int e = tid; e < a.E; e += blockDim.x)
     for (int k = 0, left = count[e]; left > 0; ++k, left -= a.tile_rows)
       a.tiles[tstart[e] + k] = make_int4(e, start[e] + k * a.tile_rows, min(left, a.tile_rows), 0);
-  for (int i = tid; i < a.entries; i += 1024) {
-    const int r = atomicAdd(&cursor[a.ids[i]], 1);
-    a.row_of[i] = r;
-    a.src[r] = i / a.top;
-    a.row_weight[r] = a.weights[i];
+}
+
+// The order of rows inside an expert is arbitrary (it enters no value).
+__device__ __forceinline__ void place(const GroupArgs &a, int entry, int expert, float weight, int *cursor) {
+  const int r = atomicAdd(&cursor[expert], 1);
+  a.row_of[entry] = r;
+  a.src[r] = entry / a.top;
+  a.row_weight[r] = weight;
+}
+
+// Few entries: grouped by one workgroup.
+constexpr int kSmallEntries = 4096;
+__global__ __launch_bounds__(1024) void moe_small_kernel(const GroupArgs a) {
+  __shared__ int count[kMaxExperts], start[kMaxExperts], tstart[kMaxExperts];
+  const int tid = threadIdx.x;
+  int id[kSmallEntries / 1024];
+  float weight[kSmallEntries / 1024];
+#pragma unroll
+  for (int k = 0; k < kSmallEntries / 1024; ++k) {
+    const int i = tid + k * 1024;
+    if (i < a.entries) {
+      id[k] = a.ids[i];
+      weight[k] = a.weights[i];
+    }
   }
+  for (int e = tid; e < a.E; e += 1024) count[e] = 0;
+  __syncthreads();
+#pragma unroll
+  for (int k = 0; k < kSmallEntries / 1024; ++k)
+    if (tid + k * 1024 < a.entries) atomicAdd(&count[id[k]], 1);
+  __syncthreads();
+  expert_tiles(a, count, start, tstart);
+  __syncthreads();
+#pragma unroll
+  for (int k = 0; k < kSmallEntries / 1024; ++k)
+    if (tid + k * 1024 < a.entries) place(a, tid + k * 1024, id[k], weight[k], start);
+}
+
+// Many tokens: counts per block of entries, a scan over blocks and experts, placement.
+constexpr int kBlockEntries = 1024;
+__global__ __launch_bounds__(1024) void moe_count_kernel(const GroupArgs a) {
+  __shared__ int count[kMaxExperts];
+  for (int e = threadIdx.x; e < a.E; e += 1024) count[e] = 0;
+  __syncthreads();
+  const int i = blockIdx.x * kBlockEntries + threadIdx.x;
+  if (i < a.entries) atomicAdd(&count[a.ids[i]], 1);
+  __syncthreads();
+  for (int e = threadIdx.x; e < a.E; e += 1024) a.hist[blockIdx.x * a.E + e] = count[e];
+}
+__global__ __launch_bounds__(kMaxExperts) void moe_scan_kernel(const GroupArgs a) {
+  __shared__ int count[kMaxExperts], start[kMaxExperts], tstart[kMaxExperts];
+  const int e = threadIdx.x;
+  int sum = 0;
+  if (e < a.E) {
+#pragma unroll 8
+    for (int b = 0; b < a.blocks; ++b) sum += a.hist[b * a.E + e];
+    count[e] = sum;
+  }
+  __syncthreads();
+  expert_tiles(a, count, start, tstart);
+  if (e < a.E) {
+    int at = start[e];
+    for (int b0 = 0; b0 < a.blocks; b0 += 8) {
+      int c[8];
+#pragma unroll
+      for (int k = 0; k < 8; ++k) c[k] = a.hist[min(b0 + k, a.blocks - 1) * a.E + e];
+#pragma unroll
+      for (int k = 0; k < 8; ++k)
+        if (b0 + k < a.blocks) {
+          a.hist[(b0 + k) * a.E + e] = at;
+          at += c[k];
+        }
+    }
+  }
+}
+__global__ __launch_bounds__(1024) void moe_place_kernel(const GroupArgs a) {
+  __shared__ int cursor[kMaxExperts];
+  for (int e = threadIdx.x; e < a.E; e += 1024) cursor[e] = a.hist[blockIdx.x * a.E + e];
+  __syncthreads();
+  const int i = blockIdx.x * kBlockEntries + threadIdx.x;
+  if (i < a.entries) place(a, i, a.ids[i], a.weights[i], cursor);
 }
 
 // ---------------------------------------------------------------------------------------------------------------
@@ -238,8 +269,19 @@ struct XieluArgs {
   int32_t rows, cols, padded;   // columns cols .. padded - 1 of `out` become zeros
 };
 __device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+// e^z - 1 - z without cancellation: five terms of the series near zero (relative error below 2^-24 for |z| < 1/16).
+__device__ __forceinline__ float exp_rest(float z) {
+  if (z > -0.0625f) {
+    float r = fmaf(z, 1.0f / 720.0f, 1.0f / 120.0f);
+    r = fmaf(z, r, 1.0f / 24.0f);
+    r = fmaf(z, r, 1.0f / 6.0f);
+    r = fmaf(z, r, 0.5f);
+    return z * z * r;
+  }
+  return __builtin_amdgcn_exp2f(z * 1.4426950408889634f) - 1.0f - z;
+}
 __device__ __forceinline__ float xielu_f32(float z, float a, float b) {
-  return z > 0.f ? fmaf(a * z, z, 0.5f * z) : fmaf(b, expm1f(z) - z, 0.5f * z);
+  return fmaf(z > 0.f ? a * z * z : b * exp_rest(fminf(z, 0.f)), 1.0f, 0.5f * z);
 }
 template <typename T, int VEC, bool PART>
 __global__ __launch_bounds__(256) void xielu_kernel(const XieluArgs a) {
@@ -268,36 +310,40 @@ __global__ __launch_bounds__(256) void xielu_kernel(const XieluArgs a) {
 
 }  // namespace tlf
 
-extern "C" int tlf_moe_route(const void *h, int64_t h_stride, const void *router, int32_t *ids, float *weights, int32_t n,
-                             int32_t experts, int32_t K, int32_t top, int32_t dtype, void *stream) {
-  using namespace tlf;
-  if (n < 0 || experts <= 0 || experts > kMaxExperts || top <= 0 || top > experts || K <= 0 || K % 64 || h_stride < K) return TLF_E_SHAPE;
-  if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
-  if (n == 0) return TLF_OK;
-  if (!h || !router || !ids || !weights) return TLF_E_NULL;
-  if (!aligned16(h) || !aligned16(router) || h_stride % 8) return TLF_E_ALIGN;
-  const RouterArgs a{h, router, h_stride, ids, weights, n, experts, (experts + 15) / 16 * 16, K, top};
-  hipStream_t s = static_cast<hipStream_t>(stream);
-  if (dtype == TLF_DT_BF16)
-    TLF_LAUNCH(router_kernel, dim3((n + 15) / 16), dim3(512), 16 * (a.E16 + 4) * 4, s, a);
-  else
-    TLF_LAUNCH(router_f32_kernel, dim3(n), dim3(256), 0, s, a);
-  return launch_status();
+extern "C" size_t tlf_moe_group_workspace_bytes(int32_t n, int32_t top, int32_t experts) {
+  if (n <= 0 || top <= 0 || experts <= 0) return 0;
+  const int64_t entries = static_cast<int64_t>(n) * top;
+  return static_cast<size_t>((entries + tlf::kBlockEntries - 1) / tlf::kBlockEntries) * experts * 4;
 }
 
-extern "C" int tlf_moe_group(const int32_t *ids, const float *weights, int32_t *row_of, int32_t *src, float *row_weight,
-                             int32_t *tiles, int32_t *num_tiles, int32_t max_tiles, int32_t n, int32_t top, int32_t experts,
-                             int32_t tile_rows, void *stream) {
+extern "C" int tlf_moe_group(const float *sums, int32_t splits, int32_t *ids, float *weights, int32_t *row_of, int32_t *src,
+                             float *row_weight, int32_t *tiles, int32_t *num_tiles, int32_t max_tiles, int32_t n, int32_t top,
+                             int32_t experts, int32_t tile_rows, void *workspace, size_t workspace_bytes, void *stream) {
   using namespace tlf;
-  if (n < 0 || top <= 0 || experts <= 0 || experts > kMaxExperts || tile_rows <= 0) return TLF_E_SHAPE;
+  if (n < 0 || top <= 0 || experts <= 0 || experts > kMaxExperts || top > experts || tile_rows <= 0 || splits <= 0 || splits > 64) return TLF_E_SHAPE;
   const int64_t entries = static_cast<int64_t>(n) * top;
   if (entries > (1 << 28) || max_tiles < entries / tile_rows + (entries < experts ? entries : experts)) return TLF_E_SHAPE;
   if (n == 0) return TLF_OK;
-  if (!ids || !weights || !row_of || !src || !row_weight || !tiles || !num_tiles) return TLF_E_NULL;
+  if (!sums || !ids || !weights || !row_of || !src || !row_weight || !tiles || !num_tiles) return TLF_E_NULL;
   if (!aligned16(tiles)) return TLF_E_ALIGN;
-  const GroupArgs a{ids, weights, row_of, src, row_weight, reinterpret_cast<int4 *>(tiles), num_tiles,
-                    static_cast<int32_t>(entries), experts, top, tile_rows};
-  TLF_LAUNCH(moe_group_kernel, dim3(1), dim3(1024), 0, static_cast<hipStream_t>(stream), a);
+  GroupArgs a{};
+  a.sums = sums; a.ids = ids; a.weights = weights; a.row_of = row_of; a.src = src; a.row_weight = row_weight;
+  a.tiles = reinterpret_cast<int4 *>(tiles); a.num_tiles = num_tiles; a.hist = static_cast<int32_t *>(workspace);
+  a.n = n; a.splits = splits; a.E = experts; a.E16 = (experts + 15) / 16 * 16; a.top = top;
+  a.plane = static_cast<int64_t>(n) * a.E16;
+  a.entries = static_cast<int32_t>(entries); a.tile_rows = tile_rows;
+  a.blocks = static_cast<int32_t>((entries + kBlockEntries - 1) / kBlockEntries);
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (entries > kSmallEntries && (!workspace || workspace_bytes < tlf_moe_group_workspace_bytes(n, top, experts))) return TLF_E_WORKSPACE;
+  const int waves = n <= 1024 ? 1 : 4;
+  TLF_LAUNCH(moe_pick_kernel, dim3((n + waves - 1) / waves), dim3(64 * waves), 0, s, a);
+  if (entries <= kSmallEntries) {
+    TLF_LAUNCH(moe_small_kernel, dim3(1), dim3(1024), 0, s, a);
+    return launch_status();
+  }
+  TLF_LAUNCH(moe_count_kernel, dim3(a.blocks), dim3(1024), 0, s, a);
+  TLF_LAUNCH(moe_scan_kernel, dim3(1), dim3(kMaxExperts), 0, s, a);
+  TLF_LAUNCH(moe_place_kernel, dim3(a.blocks), dim3(1024), 0, s, a);
   return launch_status();
 }
 

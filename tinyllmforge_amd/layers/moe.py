@@ -62,7 +62,6 @@ class ClippedGLUExperts(nn.Module):
     def forward(self, h: torch.Tensor):
         """``(rows, index)``: the result for token t is the sum of ``rows[index[t]]``."""
         h = pad_columns(h, self.columns)
-        ids, weights = ops.moe_route(h, self.router.data, self.experts, self.top)
-        rows = ops.moe_group(ids, weights, self.experts, self.tile_rows(h.shape[0]))
+        rows = ops.moe_group(ops.moe_logits(h, self.router.data), self.experts, self.top, self.tile_rows(h.shape[0]))
         a = ops.moe_gemm(h, self.gate_up.data, rows, gather=True, clipped_glu=True, limit=self.limit)
         return ops.moe_gemm(a, self.down.data, rows, gather=False), rows.row_of

@@ -921,36 +921,45 @@ def latent_prefill(q, expanded, latents, cu_seqlens_q, seq_starts, kv_offsets, f
 
 
 # ------------------------------------------------------------------ mixture of experts
-def moe_route(h, router, experts, top):
-    """The ``top`` experts of every row by router logit and their sigmoids: int32 and fp32 ``[N, top]``."""
+def moe_logits(h, router):
+    """Router logits of every row as fp32 partial sums ``[splits, N, experts rounded up to 16]``."""
+    import ctypes
+    if router.dtype == torch.float32:
+        return f32_linear(h, router)[None]
     lib = _lib.load()
-    _need(h, router.dtype, "h")
-    n, K = h.shape
-    assert h.stride(1) == 1 and router.is_contiguous() and router.shape[1] == K and router.shape[0] >= experts
-    ids = torch.empty(n, top, dtype=torch.int32, device=h.device)
-    weights = torch.empty(n, top, dtype=torch.float32, device=h.device)
-    check(lib.tlf_moe_route(h.data_ptr(), h.stride(0), router.data_ptr(), ids.data_ptr(), weights.data_ptr(), n, experts, K, top,
-                            _dt(h), _stream()), "tlf_moe_route")
-    return ids, weights
+    _need(h, BF16, "h"); _need(router, BF16, "router")
+    (M, K), N = h.shape, router.shape[0]
+    assert h.stride(1) == 1 and router.is_contiguous() and router.shape[1] == K
+    splits = ctypes.c_int32(1)
+    nbytes = lib.tlf_gemm_f32_sums_bytes(M, N, K)
+    sums = torch.empty(nbytes // 4, dtype=torch.float32, device=h.device)
+    check(lib.tlf_gemm_f32_sums(h.data_ptr(), h.stride(0), router.data_ptr(), sums.data_ptr(), nbytes, M, N, K,
+                                ctypes.addressof(splits), _stream()), "tlf_gemm_f32_sums")
+    return sums.view(splits.value, M, N)
 
 
 class ExpertRows:
-    """Rows (token, k) in expert order: ``row_of [N, top]``, ``src`` / ``weight`` per row, tiles of ``tile_rows`` rows."""
-    __slots__ = ("row_of", "src", "weight", "tiles", "num_tiles", "tile_rows")
+    """The chosen experts ``ids`` / ``scores [N, top]`` and the rows (token, k) in expert order: ``row_of [N, top]``, ``src`` /
+    ``weight`` per row, tiles of ``tile_rows`` rows."""
+    __slots__ = ("ids", "scores", "row_of", "src", "weight", "tiles", "num_tiles", "tile_rows")
 
 
-def moe_group(ids, weights, experts, tile_rows) -> ExpertRows:
+def moe_group(logits, experts, top, tile_rows) -> ExpertRows:
+    """``logits``: partial sums as from ``moe_logits``."""
     lib = _lib.load()
-    _need(ids, torch.int32, "ids"); _need(weights, torch.float32, "weights")
-    assert ids.is_contiguous() and weights.is_contiguous() and ids.shape == weights.shape
-    n, top = ids.shape
-    r = ExpertRows()
-    i32 = lambda *s: torch.empty(*s, dtype=torch.int32, device=ids.device)
-    r.row_of, r.src, r.weight = i32(n, top), i32(n * top), torch.empty(n * top, dtype=torch.float32, device=ids.device)
+    _need(logits, torch.float32, "logits")
+    assert logits.is_contiguous() and logits.shape[2] == -(-experts // 16) * 16
+    splits, n = logits.shape[:2]
+    r, dev = ExpertRows(), logits.device
+    i32 = lambda *s: torch.empty(*s, dtype=torch.int32, device=dev)
+    f32 = lambda *s: torch.empty(*s, dtype=torch.float32, device=dev)
+    r.ids, r.scores, r.row_of, r.src, r.weight = i32(n, top), f32(n, top), i32(n, top), i32(n * top), f32(n * top)
     r.tiles, r.num_tiles, r.tile_rows = i32(n * top // tile_rows + min(experts, n * top), 4), i32(1), tile_rows
-    check(lib.tlf_moe_group(ids.data_ptr(), weights.data_ptr(), r.row_of.data_ptr(), r.src.data_ptr(), r.weight.data_ptr(),
-                            r.tiles.data_ptr(), r.num_tiles.data_ptr(), r.tiles.shape[0], n, top, experts, tile_rows,
-                            _stream()), "tlf_moe_group")
+    ws = _workspace(lib.tlf_moe_group_workspace_bytes(n, top, experts), dev, "moe")
+    check(lib.tlf_moe_group(logits.data_ptr(), splits, r.ids.data_ptr(), r.scores.data_ptr(), r.row_of.data_ptr(),
+                            r.src.data_ptr(), r.weight.data_ptr(), r.tiles.data_ptr(), r.num_tiles.data_ptr(),
+                            r.tiles.shape[0], n, top, experts, tile_rows, ws.data_ptr(), ws.numel(), _stream()),
+          "tlf_moe_group")
     return r
 
 
