@@ -666,8 +666,8 @@ int tlf_latent_prefill(const void *q, const void *expanded, int64_t expanded_str
  *   max_tiles of them; max_tiles >= n * top / tile_rows + min(experts, n * top).  experts <= 512.
  * tlf_moe_gemm: y[row] = W[expert] x[x_rows ? x_rows[row] : row]; w [experts, N, K].  clipped_glu: channels are interleaved
  *   as for the SiLU-and-mul products (8 gate, then the 8 matching up); with f = row_scale[row] (NULL: 1), g = min(f gate,
- *   limit), u = clamp(f up, +-limit): y [rows, N / 2] = g sigmoid(1.702 g) (u + 1).  bf16: tile_rows 32 or 128, K a multiple
- *   of 64; fp32: tile_rows 64.  x_count bounds the x rows.
+ *   limit), u = clamp(f up, +-limit): y [rows, N / 2] = g sigmoid(1.702 g) (u + 1).  bf16: tile_rows 32, 64, 128 or 256, K a
+ *   multiple of 64; fp32: tile_rows 64.  x_count bounds the x rows.
  * tlf_xielu: with a = softplus(pq[0]), b = 1/2 + softplus(pq[1]), out = a z^2 + z / 2 for z > 0, b (e^z - 1 - z) + z / 2
  *   otherwise, z = columns col .. col + cols - 1 of x (or of partial sums); columns cols .. padded_cols - 1 become 0. */
 size_t tlf_gemm_f32_sums_bytes(int32_t M, int32_t N, int32_t K);

@@ -298,7 +298,7 @@ def test_entry_points_reject_bad_arguments_on_the_host():
     group = lambda top=2, E=5, tiles=9, splits=1, n=4: lib.tlf_moe_group(a, splits, a, a, a, a, a, a, a, tiles, n, top, E, 32, None, 0, None)
     assert group(top=6) == -2 and group(E=600) == -2 and group(tiles=4) == -2 and group(n=0) == 0 and group(n=4000, tiles=9999) == -4
     gemm = lambda rows=32, N=32, K=64, dt=0, xs=64, count=4: lib.tlf_moe_gemm(a, xs, count, a, a, a, a, 9, rows, a, None, 8, N, K, 0, 0.0, dt, None)
-    assert gemm(rows=64) == -2 and gemm(N=20) == -2 and gemm(xs=32) == -2 and gemm(dt=1, rows=32) == -2 and gemm(count=1 << 30) == -6
+    assert gemm(rows=48) == -2 and gemm(N=20) == -2 and gemm(xs=32) == -2 and gemm(dt=1, rows=32) == -2 and gemm(count=1 << 30) == -6
     assert gemm(K=80, xs=80) == -2
     assert lib.tlf_gemm_f32_sums(a, 64, a, a, 16, 4, 16, 64, ctypes.addressof(out), None) == -4
     res = lambda top=0, extra=None, es=0, ys=64: lib.tlf_residual_rmsnorm(a, ys, None, 1, None, extra, es, None, top, 0.5, a, a, 1.0, a, 2, 64, 1e-6, 0, None)

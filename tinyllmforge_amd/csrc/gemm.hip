@@ -1581,13 +1581,16 @@ int launch_gemm(const void *x, int64_t x_stride, const void *w, const float *sca
   return rc;
 }
 
-// Grouped product (bf16): rows in expert order, tiles of `bm` rows of one expert each.  Few rows per expert: narrow tiles
-// and wave sets that split K, because the weights stream from HBM; many: the 128 x 128 tile.
+// Grouped product (bf16): rows in expert order, tiles of `bm` rows of one expert each.  The host picks bm by the average rows
+// per expert (ClippedGLUExperts.tile_rows): few, and the weights stream from HBM once through wide flat tiles; many, and the
+// largest tile saves copies.  From a sweep of the tile instances over two mixtures, us for gate_up / down, chosen tile first:
+//   2 rows (64 tokens, 32 experts of 768 at width 1024)     256 x 32: 19.3 / 12.1    64 x 32, K split by 4 wave sets: 25.9 / 15.2
+//   8 rows (64 tokens, 64 of 1536 at 4096)                  256 x 32: 287 / 143      the same: 313 / 176
+//   64 rows (512 tokens, 4096)                              256 x 128: 307 / 168     128 x 64: 347 / 186    128 x 128: 345 / 177
+//   2048 rows (16,384 tokens, 4096)                         256 x 256: 3066 / 1704   256 x 128: 3187 / 1879 128 x 128: 3865 / 2298
 int launch_grouped(GemmParams p, int bm, hipStream_t stream) {
   if (p.N % 16 || p.K % kBK || p.m_tiles <= 0) return TLF_E_SHAPE;
-  const int ktiles = p.K / kBK;
-  const int kg = bm == 32 ? (ktiles % 4 == 0 ? 4 : ktiles % 2 == 0 ? 2 : 1) : 1;
-  const int bn = bm == 32 ? 64 : 128;
+  const int bn = bm == 64 ? 128 : 256;
   p.splits = 1;
   p.k_per_split = p.K;
   p.n_tiles = (p.N + bn - 1) / bn;
@@ -1604,13 +1607,11 @@ int launch_grouped(GemmParams p, int bm, hipStream_t stream) {
 #define TLF_GROUPED(BN_, BM_, WN_, WM_, NS_, OCC_, KG_)                                                             \
   TLF_LAUNCH((gemm_dlds_kernel<BN_, BM_, WN_, WM_, false, NS_, OCC_, KG_, true>), grid, dim3(WN_ * WM_ * KG_ * 64), \
              0, stream, p)
-  if (bm == 32) {
-    if (kg == 4) TLF_GROUPED(64, 32, 2, 1, 2, 4, 4);
-    else if (kg == 2) TLF_GROUPED(64, 32, 2, 1, 3, 4, 2);
-    else TLF_GROUPED(64, 32, 2, 1, 4, 4, 1);
-  } else {
-    TLF_GROUPED(128, 128, 2, 2, 3, 2, 1);
-  }
+  if (bm == 32) TLF_GROUPED(256, 32, 4, 1, 3, 2, 1);
+  else if (bm == 64) TLF_GROUPED(128, 64, 4, 1, 2, 3, 1);
+  else if (bm == 128) TLF_GROUPED(256, 128, 2, 2, 3, 1, 1);
+  else if (bm == 256) TLF_GROUPED(256, 256, 4, 2, 2, 2, 1);
+  else return TLF_E_SHAPE;
 #undef TLF_GROUPED
   return launch_status();
 }

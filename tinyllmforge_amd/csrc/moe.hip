@@ -365,7 +365,7 @@ extern "C" int tlf_moe_gemm(const void *x, int64_t x_stride, int32_t x_count, co
     TLF_LAUNCH(grouped_f32_kernel, dim3((N + kGT - 1) / kGT, max_tiles), dim3(256), 0, s, a);
     return launch_status();
   }
-  if (tile_rows != 32 && tile_rows != 128) return TLF_E_SHAPE;
+  if (tile_rows != 32 && tile_rows != 64 && tile_rows != 128 && tile_rows != 256) return TLF_E_SHAPE;
   if (!aligned16(x) || !aligned16(w) || !aligned16(y) || x_stride % 8) return TLF_E_ALIGN;
   if (static_cast<int64_t>(x_count) * x_stride * 2 > 0xffffffffll) return TLF_E_TOO_LARGE;   // x rows are 32-bit byte offsets
   GemmParams p{};

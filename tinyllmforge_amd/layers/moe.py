@@ -57,7 +57,8 @@ class ClippedGLUExperts(nn.Module):
         """Rows of a tile of the grouped products: rows per expert decide between streaming the weights and reusing them."""
         if self.router.dtype == torch.float32:
             return 64
-        return 128 if tokens * self.top >= 48 * self.experts else 32
+        rows = tokens * self.top / self.experts
+        return 32 if rows <= 8 else 64 if rows <= 32 else 128 if rows < 512 else 256
 
     def forward(self, h: torch.Tensor):
         """``(rows, index)``: the result for token t is the sum of ``rows[index[t]]``."""
