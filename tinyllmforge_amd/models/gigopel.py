@@ -12,7 +12,10 @@ from ..layers.latent_attention import LatentAttention
 from ..layers.linear import JoinedLinear, StackedLinear
 from ..layers.moe import ClippedGLUExperts
 from ..layers.residual_norm import ResidualRMSNorm
+from ..utils.side_stream import on_the_side
 from .layered import LayeredForCausalLM
+
+SIDE_BY_SIDE = 256      # up to this many rows the experts run beside the attention, on a stream of their own
 
 
 class GigopelLayer(nn.Module):
@@ -39,11 +42,19 @@ class GigopelLayer(nn.Module):
         proj = self.inp.forward_deferred(h)         # read by the next two kernels, before any other product
         rows = self.out.input_rows(h.shape[0], h.dtype, h.device)
         q = self.attn.prepare(proj, self.inp.offset("dkv"), positions)
+        extra, join = (None, None), None
         if self.act is not None:
             self.act(proj, self.inp.offset("up"), self.inp.parts["up"], rows[:, self.out.offset("down"):])
-        extra = self.experts(h) if self.experts is not None else (None, None)
+        elif self.experts is not None and h.shape[0] <= SIDE_BY_SIDE:
+            with on_the_side(h.device) as join:
+                extra = self.experts(h)
+        elif self.experts is not None:
+            extra = self.experts(h)
         self.attn(q, positions, rows)
-        return following.after_adding(self.out.forward_deferred(rows), x, self.mult, *extra)
+        y = self.out.forward_deferred(rows)
+        if join is not None:
+            join()
+        return following.after_adding(y, x, self.mult, *extra)
 
     def routes(self) -> dict:
         out = {"norm1": ("norm1.weight", None), "mix.q": ("inp.weight", "q"), "mix.dkv": ("inp.weight", "dkv"),
