@@ -284,7 +284,7 @@ def test_entry_points_reject_bad_arguments_on_the_host():
     assert tile(sizes=(3, 20, 6, 600, 13)) == -5                             # cache rows too long for two tiles in LDS
     out = (ctypes.c_int32 * 3)()
     layout = lambda seqs, most, heads, lp: (lib.tlf_latent_attn_layout(seqs, most, heads, lp, ctypes.addressof(out)), list(out))
-    assert layout(5, 1, 3, 576) == (0, [4 + 2 * (256 + 5), 261, 16])
+    assert layout(5, 1, 3, 576) == (0, [4 + 4 * 261 + 2 * 5, 261, 16])
     assert layout(2, 10, 40, 576)[1][1:] == [256 + 2 * 10 * 2, 32]           # two passes over 40 heads, a row a job
     assert layout(2, 10, 3, 100)[0] == -2
     assert lib.tlf_latent_attn_plan(a, None, None, None, 0, 0, 2, 1, 3, 64, 5, a, None) == -1

@@ -238,9 +238,14 @@ def test_attention_of_many_unequal_sequences():
     part, ml = P.latent_attention(q.cuda(), cache.cuda(), bt.cuda(), window, 0.1, s, batch, plan)
     out = torch.full((B, H * V), 7.0, dtype=torch.bfloat16, device="cuda")
     P.latent_values(part, ml, uv.cuda(), out, s, batch, plan)
-    head = plan[:2].tolist()
+    # every tile of every live sequence is in just one piece
     tiles = [0 if slots[b] < 0 else (int(lens[b]) - 1) // 64 - max(0, int(lens[b]) - window) // 64 + 1 for b in range(B)]
-    assert head[1] == sum(tiles) and head[0] == -(-sum(tiles) // 512)
+    per, pieces = plan[:2].tolist()
+    seen = [[] for _ in range(B)]
+    for count, job, tile, start in plan[4:4 + 4 * pieces].view(-1, 4).tolist():
+        assert 0 < count <= per and start == int(lens[job]) - 1
+        seen[job] += range(tile, tile + count)
+    assert seen == [list(range(t)) for t in tiles]
     for b in range(B):
         if slots[b] < 0:
             assert not out[b].any()

@@ -50,9 +50,15 @@ __device__ __forceinline__ int64_t latent_row(const LatentCache &c, const int32_
 
 // ---- jobs of the absorbed kernels: 16 or 32 units (row, head) of one sequence and the key tiles their window covers
 constexpr int kLatentTile = 64;          // keys per tile
-constexpr int kLatentMaxPieces = 128;    // workgroups that share a job, at most
-constexpr int kLatentPlanHead = 4;       // plan: tiles per workgroup, tiles in all, -, -; per workgroup (job, first tile);
-                                         // per job (first workgroup, workgroups).  Piece of (workgroup w, job j): w + j
+constexpr int kLatentMaxPieces = 128;    // pieces of a job, at most
+// Plan: a head (tiles per piece, pieces), a record per piece (its tiles, job, first tile of it, start of the job's sequence:
+// what a workgroup needs before its first copy) and per job (first piece, pieces).
+constexpr int kLatentPlanHead = 4, kLatentRecord = 4;
+// Pieces there may be: about one per workgroup the chip holds, and one more per job.
+__host__ __device__ __forceinline__ int latent_max_pieces(int wgs, int jobs) { return wgs + jobs; }
+__host__ __device__ __forceinline__ int64_t latent_plan_jobs(int wgs, int jobs) {
+  return kLatentPlanHead + static_cast<int64_t>(kLatentRecord) * latent_max_pieces(wgs, jobs);
+}
 
 struct LatentJobs {
   const int64_t *positions;              // sequence s is the single row s at positions[s] (slots[s] < 0: no keys) ...
@@ -84,9 +90,10 @@ __device__ __forceinline__ T uniform_load(const T *p) {
 struct LatentJob {
   int seq, q0, start, row0, last_row, head0, heads, w0, tiles;
 };
-// UNIFORM: `job` is the same in all lanes
+// UNIFORM: `job` is the same in all lanes.  known_start: the start of a single row's sequence if the caller has it (-1: a
+// padding row)
 template <bool UNIFORM>
-__device__ __forceinline__ LatentJob latent_job(const LatentJobs &a, int job) {
+__device__ __forceinline__ LatentJob latent_job(const LatentJobs &a, int job, int known_start = -2) {
   auto ld = [](auto *p) __attribute__((always_inline)) { return UNIFORM ? uniform_load(p) : *p; };
   LatentJob j;
   const int pass = job % a.passes, rest = job / a.passes, xt = rest % a.xtiles;
@@ -99,7 +106,7 @@ __device__ __forceinline__ LatentJob latent_job(const LatentJobs &a, int job) {
     j.start = ld(a.starts + j.seq);
   } else {
     j.q0 = j.seq;
-    j.start = ld(a.slots + j.seq) >= 0 ? static_cast<int>(ld(a.positions + j.seq)) : -1;
+    j.start = known_start != -2 ? known_start : ld(a.slots + j.seq) >= 0 ? static_cast<int>(ld(a.positions + j.seq)) : -1;
   }
   j.row0 = xt * a.bq;
   j.last_row = min(j.row0 + a.bq, lq) - 1;

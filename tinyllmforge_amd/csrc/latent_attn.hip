@@ -278,9 +278,9 @@ __device__ __forceinline__ Pieces latent_pieces(const LatentValuesArgs &a, int r
     seq -= j.first_seq;
   }
   const int pass = h / j.hpp, job = (seq * j.xtiles + r / j.bq) * j.passes + pass;
-  const int32_t *rec = a.plan + kLatentPlanHead + 2 * (a.wgs + job);
-  const bool ok = rec[0] >= 0 && rec[1] >= 0 && rec[0] + rec[1] <= a.wgs;
-  return Pieces{static_cast<int64_t>(rec[0] + job) * j.units + r % j.bq * j.hpp + h - pass * j.hpp, j.units, ok ? rec[1] : 0};
+  const int32_t *rec = a.plan + latent_plan_jobs(a.wgs, j.jobs) + 2 * job;
+  const bool ok = rec[0] >= 0 && rec[1] >= 0 && rec[1] <= kLatentMaxPieces && rec[0] + rec[1] <= latent_max_pieces(a.wgs, j.jobs);
+  return Pieces{static_cast<int64_t>(rec[0]) * j.units + r % j.bq * j.hpp + h - pass * j.hpp, j.units, ok ? rec[1] : 0};
 }
 // Maximum and inverse denominator over the pieces (inverse 0: no keys).
 __device__ __forceinline__ void pieces_total(const LatentValuesArgs &a, const Pieces &p, float &mx, float &inv) {

@@ -1,9 +1,9 @@
 // Absorbed latent attention on the matrix cores, bf16: decoded tokens and short portions (geometry in latent_attn.h).
 //
 // The (row, head) pairs of a sequence are flattened into units; 16 CT units make a job, whose work is the 64-key tiles that
-// its window covers.  All tiles of all jobs form one line that is cut into equal pieces, one per workgroup (a plan made once
-// per step and window), so sequences of unequal length keep all CUs busy alike; a workgroup that meets the end of a job goes
-// on with the next one while its copies stay in flight.
+// its window covers.  Jobs are cut into pieces of about equal length, one per workgroup, by a plan made once per step and
+// window: as short as the workgroups that the chip holds at once allow, so that sequences of unequal length keep all CUs busy
+// alike.
 //
 // All units share the cache rows, so a tile in LDS serves as keys and as values; 4 CT waves split the work by keys in the
 // first product and by latent dimensions in the second, and each row is read from LDS once per product:
@@ -12,8 +12,8 @@
 //   O^T[dim, unit] += C^T . P^T   wave w: dimension tiles w, w + 4 CT, ...; C^T by LDS transpose reads
 // Tiles travel global -> LDS directly into a ring of stages.  64 rows from a multiple of 64 on are contiguous in a page, so
 // a copy instruction moves 1 KiB; LDS rows are unpadded and their 16-byte pieces are swizzled against bank conflicts (the
-// lane that fills a position picks the matching global piece).  A workgroup writes its unnormalised mix of latents per job
-// with the maximum and the denominator; latent_values_kernel (latent_attn.hip) joins the pieces.
+// lane that fills a position picks the matching global piece).  A workgroup writes its unnormalised mix of latents with
+// the maximum and the denominator; latent_values_kernel (latent_attn.hip) joins the pieces.
 #include <algorithm>
 
 #include "gemm_shared.h"
@@ -25,31 +25,51 @@ __device__ __forceinline__ shortx4 latent_read_tr16(const unsigned short *p) {
   return __builtin_amdgcn_ds_read_tr16_b64_v4i16((shortx4 __attribute__((address_space(3))) *)(p));
 }
 
-// One workgroup: tiles per workgroup, where each workgroup begins, which workgroups a job's pieces come from.
+// One workgroup: the length of a piece, the pieces' records, which pieces a job has.
 __global__ __launch_bounds__(1024) void latent_plan_kernel(const LatentJobs jb, int32_t *plan, int32_t wgs) {
-  __shared__ int part[16], most[16];
+  constexpr int kKept = 4096;                 // jobs whose tile counts are kept
+  __shared__ int tiles[kKept], part[16], most[16], busy[16], per_shared;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  int sum = 0, mx = 0;
+  int sum = 0, mx = 0, some = 0;
   for (int j = tid; j < jb.jobs; j += 1024) {
     const int t = latent_job<false>(jb, j).tiles;
+    if (j < kKept) tiles[j] = t;
     sum += t;
     mx = max(mx, t);
+    some += t > 0;
   }
   for (int o = 32; o > 0; o >>= 1) {
     sum += __shfl_xor(sum, o, 64);
+    some += __shfl_xor(some, o, 64);
     mx = max(mx, __shfl_xor(mx, o, 64));
   }
-  if (lane == 0) { part[wave] = sum; most[wave] = mx; }
+  if (lane == 0) { part[wave] = sum; most[wave] = mx; busy[wave] = some; }
   __syncthreads();
-  int total = 0, longest = 0;
-  for (int w = 0; w < 16; ++w) { total += part[w]; longest = max(longest, most[w]); }
-  const int per = max(1, max((total + wgs - 1) / wgs, (longest + kLatentMaxPieces - 2) / (kLatentMaxPieces - 1)));
-  if (tid == 0) { plan[0] = per; plan[1] = total; }
+  int total = 0, longest = 0, live = 0;
+  for (int w = 0; w < 16; ++w) { total += part[w]; longest = max(longest, most[w]); live += busy[w]; }
+  // not shorter than `least`: more pieces than workgroups, or than a job may have; `safe` needs no look at the jobs
+  const int least = max(1, max((total + wgs - 1) / wgs, (longest + kLatentMaxPieces - 1) / kLatentMaxPieces));
+  const int safe = live < wgs ? max(least, (total + wgs - live - 1) / (wgs - live)) : least;
+  if (tid == 0) per_shared = safe;
+  __syncthreads();
+  if (safe > least && jb.jobs <= kKept) {
+    // 16 lengths between the two, a wave each: the shortest whose pieces fit the workgroups
+    const int per = least + (safe - least) * wave / 16;
+    int pieces = 0;
+    for (int j = lane; j < jb.jobs; j += 64) pieces += (tiles[j] + per - 1) / per;
+    for (int o = 32; o > 0; o >>= 1) pieces += __shfl_xor(pieces, o, 64);
+    if (lane == 0 && pieces <= wgs) atomicMin(&per_shared, per);
+    __syncthreads();
+  }
+  const int per = per_shared;
   int before = 0;
   for (int j0 = 0; j0 < jb.jobs; j0 += 1024) {
     const int j = j0 + tid;
-    const int t = j < jb.jobs ? latent_job<false>(jb, j).tiles : 0;
-    int x = t;
+    LatentJob job;
+    job.tiles = 0;
+    if (j < jb.jobs) job = latent_job<false>(jb, j);
+    const int n = (job.tiles + per - 1) / per;
+    int x = n;
     for (int o = 1; o < 64; o <<= 1) {
       const int y = __shfl_up(x, o, 64);
       if (lane >= o) x += y;
@@ -57,23 +77,22 @@ __global__ __launch_bounds__(1024) void latent_plan_kernel(const LatentJobs jb, 
     __syncthreads();
     if (lane == 63) part[wave] = x;
     __syncthreads();
-    int a = before + x - t;
+    int a = before + x - n;
     for (int w = 0; w < 16; ++w) {
       if (w < wave) a += part[w];
       before += part[w];
     }
     if (j < jb.jobs) {
-      const int w0 = a / per, w1 = (a + t - 1) / per;
-      int32_t *rec = plan + kLatentPlanHead + 2 * wgs + 2 * j;
-      rec[0] = w0;
-      rec[1] = t > 0 ? w1 - w0 + 1 : 0;
-      if (t > 0)
-        for (int w = (a + per - 1) / per; w <= w1; ++w) {
-          plan[kLatentPlanHead + 2 * w] = j;
-          plan[kLatentPlanHead + 2 * w + 1] = w * per - a;
-        }
+      int32_t *rec = plan + latent_plan_jobs(wgs, jb.jobs) + 2 * j;
+      rec[0] = a;
+      rec[1] = n;
+      for (int k = 0; k < n; ++k)
+        *reinterpret_cast<int4 *>(plan + kLatentPlanHead + kLatentRecord * (a + k)) =
+            make_int4(min(per, job.tiles - k * per), j, k * per, job.start);
     }
   }
+  if (tid == 0) { plan[0] = per; plan[1] = before; }
+  for (int w = before + tid; w < latent_max_pieces(wgs, jb.jobs); w += 1024) plan[kLatentPlanHead + kLatentRecord * w] = 0;
 }
 
 struct LatentTileArgs {
@@ -85,7 +104,7 @@ struct LatentTileArgs {
   int32_t bs, bs_shift;
   const unsigned short *q;     // [rows, H, Lp]
   const int32_t *plan;
-  float *part, *ml;            // [workgroups + jobs, 16 CT, Rp], [.., 2]
+  float *part, *ml;            // [pieces, 16 CT, Rp], [.., 2]
   float scale_log2;
 };
 
@@ -103,9 +122,11 @@ __global__ __launch_bounds__(256 * CT) void latent_tile_kernel(const LatentTileA
   const int tid = threadIdx.x, lane = tid & 63, n = lane & 15, g = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6), kt = wave & 3, ct = wave >> 2;
   const int w = blockIdx.x;
-  const int per = uniform_load(a.plan), total = uniform_load(a.plan + 1);
-  if (per <= 0 || static_cast<int64_t>(w) * per >= total) return;
-  const int count = min(per, total - w * per);
+  const int32_t *rec = a.plan + kLatentPlanHead + kLatentRecord * w;
+  const int count = uniform_load(rec), job = uniform_load(rec + 1), tile0 = uniform_load(rec + 2), start = uniform_load(rec + 3);
+  if (count <= 0 || job < 0 || job >= a.jb.jobs) return;
+  const LatentJob J = latent_job<true>(a.jb, job, start);
+  if (tile0 < 0 || count > J.tiles - tile0) return;      // not a plan
   // row R: an odd row begins 32 banks in if NC is odd, so 8 positions and the parity tell 16 rows apart, otherwise 16 positions
   auto swz = [](int row) __attribute__((always_inline)) { return NC % 2 ? (row >> 1) & 7 : row & 15; };
 
@@ -117,66 +138,65 @@ __global__ __launch_bounds__(256 * CT) void latent_tile_kernel(const LatentTileA
   }
   const unsigned int lds0 = TLF_DL_LDSADDR(&pool[0][0]) + wave * 1024;
 
-  // copy side: runs NS - 1 tiles ahead, over the ends of jobs
-  int ijob = uniform_load(a.plan + kLatentPlanHead + 2 * w), itile = uniform_load(a.plan + kLatentPlanHead + 2 * w + 1), issued = 0;
-  if (ijob < 0 || ijob >= a.jb.jobs) return;             // not a plan
-  LatentJob ij = latent_job<true>(a.jb, ijob);
-  if (itile < 0 || itile >= ij.tiles) return;
-  auto issue = [&](int stage) __attribute__((always_inline)) {
-    const int j0 = ij.w0 + itile * kLatentTile;
-    const int pg = a.bs_shift >= 0 ? j0 >> a.bs_shift : j0 / a.bs;
-    const int page = uniform_load(a.bt + ij.seq * a.bt_stride + pg);
-    const int64_t row = page >= 0 && page < a.pages ? static_cast<int64_t>(page) * a.bs + (j0 - pg * a.bs) : 0;
+  // copy side: NS - 1 tiles ahead; the page of the tile to come is looked up one tile early
+  const int32_t *bt = a.bt + J.seq * a.bt_stride;
+  auto page_at = [&](int tile) __attribute__((always_inline)) {
+    const int at = J.w0 + (tile0 + min(tile, count - 1)) * kLatentTile;
+    return uniform_load(bt + (a.bs_shift >= 0 ? at >> a.bs_shift : at / a.bs));
+  };
+  int page = page_at(0);
+  auto issue = [&](int tile, int stage) __attribute__((always_inline)) {
+    const int at = J.w0 + (tile0 + tile) * kLatentTile;
+    const int within = a.bs_shift >= 0 ? at & (a.bs - 1) : at % a.bs;
+    const int64_t row = page >= 0 && page < a.pages ? static_cast<int64_t>(page) * a.bs + within : 0;
     const unsigned char *base = reinterpret_cast<const unsigned char *>(a.rows + row * LP);
     const unsigned int lds = lds0 + stage * (kLatentTile * LP * 2);
 #pragma unroll
     for (int i = 0; i < NL; ++i) TLF_DL_COPY(voff[i], base, lds + i * (W * 1024));
-    if (++issued < count && ++itile == ij.tiles) {   // past the end the last tile is copied again: the counts stay the same
-      itile = 0;
-      do ij = latent_job<true>(a.jb, ++ijob); while (ij.tiles == 0 && ijob + 1 < a.jb.jobs);
-    }
+    page = page_at(tile + 1);
   };
-  int job = ijob, t = itile;
-  LatentJob J = ij;
 #pragma unroll
-  for (int i = 0; i < NS - 1; ++i) issue(i);
+  for (int i = 0; i < NS - 1; ++i)
+    if (i < count) issue(i, i);
 
   int upos[CT];
   bf16x8 qf[KS];
   floatx4 acc[MT][CT];
   float m[CT], l;      // l: this wave's keys, this lane's unit of column tile ct
-  auto begin_job = [&]() __attribute__((always_inline)) {
 #pragma unroll
-    for (int k = 0; k < CT; ++k) {
-      const int u = k * 16 + n, r = J.row0 + u / a.jb.hpp;
-      const bool ok = u < a.jb.bq * a.jb.hpp && r <= J.last_row && u % a.jb.hpp < J.heads;
-      upos[k] = J.start + (ok ? r : J.row0);
-      if (k == ct || CT == 1) {
-        const unsigned short *qp = a.q + (static_cast<int64_t>(J.q0 + (ok ? r : J.row0)) * s.H + J.head0 + (ok ? u % a.jb.hpp : 0)) * LP + g * 8;
+  for (int k = 0; k < CT; ++k) {
+    const int u = k * 16 + n, r = J.row0 + u / a.jb.hpp;
+    const bool ok = u < a.jb.bq * a.jb.hpp && r <= J.last_row && u % a.jb.hpp < J.heads;
+    upos[k] = J.start + (ok ? r : J.row0);
+    m[k] = -INFINITY;
+    if (k == ct || CT == 1) {
+      const unsigned short *qp = a.q + (static_cast<int64_t>(J.q0 + (ok ? r : J.row0)) * s.H + J.head0 + (ok ? u % a.jb.hpp : 0)) * LP + g * 8;
 #pragma unroll
-        for (int i = 0; i < KS; ++i) {
-          Pack16 x;
-          x.u = *reinterpret_cast<const uint4 *>(qp + i * 32);
-          qf[i] = x.v;
-        }
+      for (int i = 0; i < KS; ++i) {
+        Pack16 x;
+        x.u = *reinterpret_cast<const uint4 *>(qp + i * 32);
+        qf[i] = x.v;
       }
-      m[k] = -INFINITY;
     }
-    // the loads end here: a wait inside the loop would be one for the copies, too
+  }
+  // the loads end here: a wait inside the loop would be one for the copies, too
 #pragma unroll
-    for (int i = 0; i < KS; ++i) asm volatile("" : "+v"(qf[i]));
-    l = 0.f;
+  for (int i = 0; i < KS; ++i) asm volatile("" : "+v"(qf[i]));
+  l = 0.f;
 #pragma unroll
-    for (int d = 0; d < MT; ++d)
+  for (int d = 0; d < MT; ++d)
 #pragma unroll
-      for (int k = 0; k < CT; ++k) acc[d][k] = floatx4{0.f, 0.f, 0.f, 0.f};
-  };
-  begin_job();
+    for (int k = 0; k < CT; ++k) acc[d][k] = floatx4{0.f, 0.f, 0.f, 0.f};
 
   int cur = 0;
   for (int i = 0; i < count; ++i) {
-    TLF_DL_BARRIER((NS - 2) * NL);            // the tile is there, for all waves; nobody reads the stage before it
-    issue(cur == 0 ? NS - 1 : cur - 1);
+    // the tile is there, for all waves, and nobody reads the stage before it any more
+    if (i + NS - 1 < count) {
+      TLF_DL_BARRIER((NS - 2) * NL);
+      issue(i + NS - 1, cur == 0 ? NS - 1 : cur - 1);
+    } else {
+      TLF_DL_BARRIER(0);
+    }
     const unsigned short *C = pool[cur];
     cur = cur + 1 == NS ? 0 : cur + 1;
     floatx4 sc = floatx4{0.f, 0.f, 0.f, 0.f};
@@ -191,7 +211,7 @@ __global__ __launch_bounds__(256 * CT) void latent_tile_kernel(const LatentTileA
       }
     }
     // lane (n, g): keys key .. key + 3 of unit n
-    const int key = J.w0 + t * kLatentTile + kt * 16 + g * 4;
+    const int key = J.w0 + (tile0 + i) * kLatentTile + kt * 16 + g * 4;
     const int my_pos = ct == 0 ? upos[0] : upos[CT - 1];
     float p[4];
 #pragma unroll
@@ -256,35 +276,25 @@ __global__ __launch_bounds__(256 * CT) void latent_tile_kernel(const LatentTileA
         }
       }
     }
-    ++t;
-    if (t == J.tiles || i + 1 == count) {       // the end of the job or of this workgroup's part of it
-      l = sum_lanes_16_32_48(l);
-      if (g == 0) mpart[ct][kt][n] = l;         // read last before the barrier in front of the second product
-      lds_barrier();
+  }
+  l = sum_lanes_16_32_48(l);
+  if (g == 0) mpart[ct][kt][n] = l;                      // read last before the barrier in front of the second product
+  lds_barrier();
 #pragma unroll
-      for (int k = 0; k < CT; ++k) {
-        const int64_t at = static_cast<int64_t>(w + job) * U + k * 16 + n;
-        if (wave == 0 && g == 0) {
-          a.ml[at * 2] = m[k];
-          a.ml[at * 2 + 1] = mpart[k][0][n] + mpart[k][1][n] + mpart[k][2][n] + mpart[k][3][n];
-        }
+  for (int k = 0; k < CT; ++k) {
+    const int64_t at = static_cast<int64_t>(w) * U + k * 16 + n;
+    if (wave == 0 && g == 0) {
+      a.ml[at * 2] = m[k];
+      a.ml[at * 2 + 1] = mpart[k][0][n] + mpart[k][1][n] + mpart[k][2][n] + mpart[k][3][n];
+    }
 #pragma unroll
-        for (int d = 0; d < MT; ++d) {
-          const int col = (d * W + wave) * 16 + g * 4;
-          if (col < s.Rp)
-            *reinterpret_cast<float4 *>(a.part + at * s.Rp + col) =
-                col < s.Ra ? make_float4(acc[d][k][0], acc[d][k][1], acc[d][k][2], acc[d][k][3]) : make_float4(0.f, 0.f, 0.f, 0.f);
-        }
-      }
-      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");   // stores share the copies' counter
-      if (i + 1 < count) {
-        do J = latent_job<true>(a.jb, ++job); while (J.tiles == 0 && job + 1 < a.jb.jobs);
-        t = 0;
-        begin_job();
-      }
+    for (int d = 0; d < MT; ++d) {
+      const int col = (d * W + wave) * 16 + g * 4;
+      if (col < s.Rp)
+        *reinterpret_cast<float4 *>(a.part + at * s.Rp + col) =
+            col < s.Ra ? make_float4(acc[d][k][0], acc[d][k][1], acc[d][k][2], acc[d][k][3]) : make_float4(0.f, 0.f, 0.f, 0.f);
     }
   }
-  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");       // the clamped copies must land before LDS is released
 }
 
 }  // namespace tlf
@@ -301,8 +311,8 @@ extern "C" int tlf_latent_attn_layout(int32_t num_seqs, int32_t max_tokens, int3
   LatentJobs jb{};
   if (!latent_jobs(jb, num_seqs, max_tokens, heads)) return TLF_E_TOO_LARGE;
   const int wgs = latent_workgroups(row_size, jb.units);
-  layout[0] = kLatentPlanHead + 2 * (wgs + jb.jobs);   // plan, in int32
-  layout[1] = wgs + jb.jobs;                           // pieces
+  layout[0] = static_cast<int32_t>(latent_plan_jobs(wgs, jb.jobs)) + 2 * jb.jobs;   // plan, in int32
+  layout[1] = latent_max_pieces(wgs, jb.jobs);         // pieces
   layout[2] = jb.units;                                // units of a piece
   return TLF_OK;
 }
@@ -315,6 +325,7 @@ extern "C" int tlf_latent_attn_plan(const int64_t *positions, const int32_t *slo
   if (num_seqs < 0 || max_tokens <= 0 || heads <= 0 || first_seq < 0 || window <= 0 || row_size <= 0 || row_size % 64) return TLF_E_SHAPE;
   if (num_seqs == 0) return TLF_OK;
   if (!plan || (cu_seqlens_q ? !seq_starts : (!positions || !slot_mapping))) return TLF_E_NULL;
+  if (!aligned16(plan)) return TLF_E_ALIGN;
   if (!cu_seqlens_q && max_tokens != 1) return TLF_E_SHAPE;
   LatentJobs jb{positions, slot_mapping, cu_seqlens_q, seq_starts, first_seq, first_row, window};
   if (!latent_jobs(jb, num_seqs, max_tokens, heads)) return TLF_E_TOO_LARGE;
@@ -344,7 +355,7 @@ extern "C" int tlf_latent_attn(const void *q, const void *cache, const int32_t *
   a.rows = static_cast<const unsigned short *>(cache); a.bt = block_tables; a.bt_stride = bt_stride; a.pages = num_pages;
   a.bs = c.bs; a.bs_shift = c.bs_shift; a.q = static_cast<const unsigned short *>(q); a.plan = plan; a.part = part; a.ml = ml;
   a.scale_log2 = scale * 1.4426950408889634f;
-  const dim3 grid(latent_workgroups(a.s.Lp, a.jb.units));
+  const dim3 grid(latent_max_pieces(latent_workgroups(a.s.Lp, a.jb.units), a.jb.jobs));
   hipStream_t st = static_cast<hipStream_t>(stream);
 #define TLF_LT(NC, NS)                                                                                              \
   case NC:                                                                                                          \
