@@ -314,7 +314,7 @@ def experts(dt, width, E, top, ff, limit, seed=0):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("n,width,E,top,ff,limit", [(1, 90, 5, 2, 20, 0.7), (7, 64, 1, 1, 1, 1.0), (64, 192, 33, 6, 72, 0.5), (700, 128, 8, 3, 64, 0.6),
                                                     (300, 320, 4, 2, 136, 0.4), (33, 256, 16, 16, 128, 0.8),
-                                                    (2100, 64, 4, 1, 40, 0.6), (129, 592, 8, 1, 264, 0.5)])
+                                                    (2100, 64, 4, 1, 40, 0.6), (129, 592, 8, 1, 264, 0.5), (9, 4096, 3, 1, 16, 0.5)])
 def test_mixture_of_experts(dtype, n, width, E, top, ff, limit):
     dt = DTYPES[dtype]
     m, w = experts(dt, width, E, top, ff, limit)

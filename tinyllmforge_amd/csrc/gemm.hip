@@ -1582,32 +1582,36 @@ int launch_gemm(const void *x, int64_t x_stride, const void *w, const float *sca
 }
 
 // Grouped product (bf16): rows in expert order, tiles of `bm` rows of one expert each.  The host picks bm by the average rows
-// per expert (ClippedGLUExperts.tile_rows): few, and the weights stream from HBM once through wide flat tiles; many, and the
-// largest tile saves copies.  From a sweep of the tile instances over two mixtures, us for gate_up / down, chosen tile first:
-//   2 rows (64 tokens, 32 experts of 768 at width 1024)     256 x 32: 19.3 / 12.1    64 x 32, K split by 4 wave sets: 25.9 / 15.2
-//   8 rows (64 tokens, 64 of 1536 at 4096)                  256 x 32: 287 / 143      the same: 313 / 176
+// per expert (ClippedGLUExperts.tile_rows): few, and the weights stream from HBM once, the column tiles of an expert side by
+// side on an XCD; many, and the largest tile saves copies.  From a sweep of the tile instances over two mixtures, us for
+// gate_up / down, chosen tile first:
+//   2 rows (64 tokens, 32 experts of 768 at width 1024)     128 x 32: 19.2 / 11.8    64 x 32, K split by 4 wave sets: 26.0 / 14.8
+//   8 rows (64 tokens, 64 of 1536 at 4096)                  64 x 32, K split: 266 / 154    128 x 32: 290 / 140 (chosen for K < 4096)
 //   64 rows (512 tokens, 4096)                              256 x 128: 307 / 168     128 x 64: 347 / 186    128 x 128: 345 / 177
 //   2048 rows (16,384 tokens, 4096)                         256 x 256: 3066 / 1704   256 x 128: 3187 / 1879 128 x 128: 3865 / 2298
 int launch_grouped(GemmParams p, int bm, hipStream_t stream) {
   if (p.N % 16 || p.K % kBK || p.m_tiles <= 0) return TLF_E_SHAPE;
-  const int bn = bm == 64 ? 128 : 256;
+  const int ktiles = p.K / kBK;
+  const bool deep = bm == 32 && ktiles >= 64 && ktiles % 4 == 0;
+  const int bn = deep ? 64 : bm <= 64 ? 128 : 256;
   p.splits = 1;
   p.k_per_split = p.K;
   p.n_tiles = (p.N + bn - 1) / bn;
-  p.xcd_rows = 0;
-  const int each = p.n_tiles / 8;
-  p.group_n = p.m_tiles >= 8 && each > 0 ? (each % 4 == 0 ? 4 : each % 3 == 0 ? 3 : each % 2 == 0 ? 2 : 1) : 1;
+  p.xcd_rows = bm == 32;
+  const int owned = p.xcd_rows ? p.m_tiles : p.n_tiles, walked = p.xcd_rows ? p.n_tiles : p.m_tiles, each = owned / 8;
+  p.group_n = !p.xcd_rows && walked >= 8 && each > 0 ? (each % 4 == 0 ? 4 : each % 3 == 0 ? 3 : each % 2 == 0 ? 2 : 1) : 1;
   p.map_full = each * 8;
-  p.map_rem = p.n_tiles - p.map_full;
-  p.map_main = each * 8 * p.m_tiles;
-  const int64_t wgs = p.map_main + static_cast<int64_t>(p.map_rem) * p.m_tiles;
+  p.map_rem = owned - p.map_full;
+  p.map_main = each * 8 * walked;
+  const int64_t wgs = p.map_main + static_cast<int64_t>(p.map_rem) * walked;
   if (p.map_rem == 0) p.map_rem = 1;
   if (wgs > (1 << 30)) return TLF_E_SHAPE;
   const dim3 grid(static_cast<unsigned>(wgs));
 #define TLF_GROUPED(BN_, BM_, WN_, WM_, NS_, OCC_, KG_)                                                             \
   TLF_LAUNCH((gemm_dlds_kernel<BN_, BM_, WN_, WM_, false, NS_, OCC_, KG_, true>), grid, dim3(WN_ * WM_ * KG_ * 64), \
              0, stream, p)
-  if (bm == 32) TLF_GROUPED(256, 32, 4, 1, 3, 2, 1);
+  if (deep) TLF_GROUPED(64, 32, 2, 1, 3, 4, 4);
+  else if (bm == 32) TLF_GROUPED(128, 32, 4, 1, 4, 4, 1);
   else if (bm == 64) TLF_GROUPED(128, 64, 4, 1, 2, 3, 1);
   else if (bm == 128) TLF_GROUPED(256, 128, 2, 2, 3, 1, 1);
   else if (bm == 256) TLF_GROUPED(256, 256, 4, 2, 2, 2, 1);
