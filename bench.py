@@ -852,6 +852,13 @@ def bench_gigopel_kernels(sizes=None):
         add("paged decode attention (Qwen3)", size,
             lambda i: P.paged_decode_attention(case["q"], case["k_cache"], case["v_cache"], case["ctx"], case["bt"], qd ** -0.5, plan=plan),
             case["algo_bytes"], "hbm")
+        # as many bytes as the latent rows of window 1024: what is left when a call is short
+        each = round(sum(min(int(c), 1024) for c in case["ctx"].cpu()) * (r + t) * 2 / B / (hkv * qd * 4))
+        few = torch.full_like(case["ctx"], each)
+        plan = P.paged_decode_plan(few, case["bt"], bs)
+        add(f"paged decode attention (Qwen3), contexts of {each}", size,
+            lambda i: P.paged_decode_attention(case["q"], case["k_cache"], case["v_cache"], few, case["bt"], qd ** -0.5, plan=plan),
+            B * each * hkv * qd * 4 + B * hq * qd * 4, "hbm")
         del case["k_cache"], case["v_cache"]
         cache = bf(2048, bs, s.lp)
         pos, slots = case["ctx"].long() - 1, torch.zeros(B, dtype=torch.int32, device=dev)
@@ -924,7 +931,13 @@ def bench_gigopel_kernels(sizes=None):
             a = torch.empty(n, ff, device=dev, dtype=BF)
             zz = bf(copies, n, 2 * ff)
             add(f"SiLU and mul (Qwen3), {n} tokens", size, lambda i: P.silu_and_mul(zz[i]), n * ff * 6, "hbm", copies)
-            add(f"xIELU, {n} tokens", size, lambda i: P.xielu(z[i], 0, ff, pq, a), n * ff * 4, "hbm", copies)
+            if n == B:       # many rows: the product's own epilogue
+                add(f"xIELU, {n} tokens", size, lambda i: P.xielu(z[i], 0, ff, pq, a), n * ff * 4, "hbm", copies)
+            else:
+                xin, win = bf(n, w), bf(-(-(h * (d + t) + r + t + ff) // 16) * 16, w)
+                add(f"stacked projection + xIELU, {n} tokens", size, lambda i: P.linear_xielu(xin, win, h * (d + t) + r + t, pq, a),
+                    2.0 * n * win.shape[0] * w, "mfma bf16")
+                del xin, win
             del qkv, kc, vc, proj, y, x, e, rr, z, zz, a
         del cache
         # -- experts

@@ -669,7 +669,9 @@ int tlf_latent_prefill(const void *q, const void *expanded, int64_t expanded_str
  *   limit), u = clamp(f up, +-limit): y [rows, N / 2] = g sigmoid(1.702 g) (u + 1).  bf16: tile_rows 32, 64, 128 or 256, K a
  *   multiple of 64; fp32: tile_rows 64.  x_count bounds the x rows.
  * tlf_xielu: with a = softplus(pq[0]), b = 1/2 + softplus(pq[1]), out = a z^2 + z / 2 for z > 0, b (e^z - 1 - z) + z / 2
- *   otherwise, z = columns col .. col + cols - 1 of x (or of partial sums); columns cols .. padded_cols - 1 become 0. */
+ *   otherwise, z = columns col .. col + cols - 1 of x (or of partial sums); columns cols .. padded_cols - 1 become 0.
+ * tlf_bf16_gemm_xielu: y = x . w^T with that activation on the columns from act_col on (a multiple of 8), which go to `out`
+ *   (its columns 0 .. out_cols - 1, as far as N reaches) instead of y; for many rows. */
 size_t tlf_gemm_f32_sums_bytes(int32_t M, int32_t N, int32_t K);
 int tlf_gemm_f32_sums(const void *x, int64_t x_stride, const void *w, float *sums, size_t sums_bytes, int32_t M,
                       int32_t N, int32_t K, int32_t *splits, void *stream);
@@ -681,6 +683,9 @@ int tlf_moe_gemm(const void *x, int64_t x_stride, int32_t x_count, const void *w
                  const int32_t *num_tiles, int32_t max_tiles, int32_t tile_rows, const int32_t *x_rows, const float
                  *row_scale, int32_t rows, int32_t N, int32_t K, int32_t clipped_glu, float limit, int32_t dtype,
                  void *stream);
+int tlf_bf16_gemm_xielu(const void *x, int64_t x_stride, const void *w, void *y, int32_t M, int32_t N, int32_t K,
+                        int32_t act_col, const void *pq, void *out, int64_t out_stride, int32_t out_cols, void
+                        *stream);
 int tlf_xielu(const void *x, int64_t x_stride, const float *partials, int32_t splits, const float *scale, int32_t
               col, const void *pq, void *out, int64_t out_stride, int32_t rows, int32_t cols, int32_t padded_cols,
               int32_t dtype, void *stream);

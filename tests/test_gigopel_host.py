@@ -303,5 +303,7 @@ def test_entry_points_reject_bad_arguments_on_the_host():
     assert lib.tlf_gemm_f32_sums(a, 64, a, a, 16, 4, 16, 64, ctypes.addressof(out), None) == -4
     res = lambda top=0, extra=None, es=0, ys=64: lib.tlf_residual_rmsnorm(a, ys, None, 1, None, extra, es, None, top, 0.5, a, a, 1.0, a, 2, 64, 1e-6, 0, None)
     assert res(top=2) == -1 and res(ys=32) == -2 and res(top=2, extra=a, es=64) == -1
+    fused = lambda col=40, cols=64, ld=64, pq=a: lib.tlf_bf16_gemm_xielu(a, 64, a, a, 600, 112, 64, col, pq, a, ld, cols, None)
+    assert fused(col=44) == -2 and fused(cols=60) == -2 and fused(ld=56) == -2 and fused(pq=None) == -1
     assert lib.tlf_xielu(a, 10, None, 1, None, 4, a, a, 8, 2, 8, 8, 0, None) == -2
     assert lib.tlf_xielu(a, 16, None, 1, None, 4, None, a, 8, 2, 8, 8, 0, None) == -1

@@ -64,6 +64,32 @@ def test_xielu(dtype, cols, padded, col, ld):
     assert not out[:, 64 + cols:].any() and (out[:, :64] == 7).all()
 
 
+@pytest.mark.parametrize("M,parts,width,ff_pad", [(600, (40, 72), 128, 128), (513, (24, 50), 192, 64), (3000, (1000, 3000), 256, 3008), (700, (8, 64), 64, 64)])
+def test_projection_with_an_activated_part(M, parts, width, ff_pad):
+    """Many rows: the stacked product applies the activation itself; as the two kernels do up to the bf16 rounding between."""
+    from tinyllmforge_amd import ops as P
+    from tinyllmforge_amd.layers.activation import XIELU
+    from tinyllmforge_amd.layers.linear import StackedLinear
+    g = torch.Generator().manual_seed(M)
+    torch.set_default_dtype(torch.bfloat16)
+    lin, act = StackedLinear(width, {"a": parts[0], "up": parts[1]}).cuda(), XIELU().cuda()
+    torch.set_default_dtype(torch.float32)
+    w = (torch.randn(sum(parts), width, generator=g) * 2 * width ** -0.5).to(torch.bfloat16)
+    lin.weight.data[:sum(parts), :width] = w.cuda()
+    act.pq.data.copy_(torch.tensor([0.4, -0.8]))
+    x = torch.randn(M, width, generator=g).to(torch.bfloat16)
+    out = torch.full((M, ff_pad + 64), 7.0, dtype=torch.bfloat16, device="cuda")
+    y = lin.forward_activated(x.cuda(), "up", act, out[:, 64:])
+    assert isinstance(y, torch.Tensor)
+    z = x.double() @ w.double().T
+    assert rel(y[:, :parts[0]], z[:, :parts[0]]) < 3e-3
+    assert rel(out[:, 64:64 + parts[1]], O.xielu(z[:, parts[0]:], *act.pq.double().cpu())) < 3e-3
+    assert (out[:, :64] == 7).all()
+    few = torch.zeros(100, ff_pad, dtype=torch.bfloat16, device="cuda")
+    lin.forward_activated(x[:100].cuda(), "up", act, few)                  # too few rows for it: two kernels
+    assert rel(few[:, :parts[1]], O.xielu(z[:100, parts[0]:], *act.pq.double().cpu())) < 6e-3
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("rows,H,N,K", [(1, 3, 64, 32), (5, 2, 48, 96), (130, 4, 576, 192), (67, 1, 16, 64)])
 def test_head_products(dtype, rows, H, N, K):

@@ -112,6 +112,7 @@ SIGNATURES = {
     "tlf_moe_group": (c_int32, [_P, _I32, _P, _P, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P, _SZ, _P]),
     "tlf_moe_gemm": (c_int32, [_P, _I64, _I32, _P, _P, _P, _P, _I32, _I32, _P, _P, _I32, _I32, _I32, _I32, _F, _I32,
                                _P]),
+    "tlf_bf16_gemm_xielu": (c_int32, [_P, _I64, _P, _P, _I32, _I32, _I32, _I32, _P, _P, _I64, _I32, _P]),
     "tlf_xielu": (c_int32, [_P, _I64, _P, _I32, _P, _I32, _P, _P, _I64, _I32, _I32, _I32, _I32, _P]),
     "tlf_probe_read": (c_int32, [_P, _SZ, _P, _P]),
     "tlf_probe_copy": (c_int32, [_P, _P, _SZ, _P]),

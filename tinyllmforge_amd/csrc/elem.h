@@ -95,6 +95,23 @@ inline int partials_check(const void *partials, const float *scale, int32_t spli
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
 
+// xIELU: a z^2 + z / 2 above zero, b (e^z - 1 - z) + z / 2 below; a = softplus(p), b = 1/2 + softplus(q).
+__device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+// e^z - 1 - z without cancellation: five terms of the series near zero (relative error below 2^-24 for |z| < 1/16).
+__device__ __forceinline__ float exp_rest(float z) {
+  if (z > -0.0625f) {
+    float r = fmaf(z, 1.0f / 720.0f, 1.0f / 120.0f);
+    r = fmaf(z, r, 1.0f / 24.0f);
+    r = fmaf(z, r, 1.0f / 6.0f);
+    r = fmaf(z, r, 0.5f);
+    return z * z * r;
+  }
+  return __builtin_amdgcn_exp2f(z * 1.4426950408889634f) - 1.0f - z;
+}
+__device__ __forceinline__ float xielu_f32(float z, float a, float b) {
+  return fmaf(z > 0.f ? a * z * z : b * exp_rest(fminf(z, 0.f)), 1.0f, 0.5f * z);
+}
+
 // Sum over aligned groups of N lanes (4, 8, 16, 32 or 64), on the vector ALU (DPP) up to a row of 16 lanes.
 template <int CTRL>
 __device__ __forceinline__ float dpp_move(float v) {

@@ -168,11 +168,14 @@ namespace tlf {
 // pipeline over its own 1/KG of the K range in its own LDS stages and the sets' accumulators are
 // summed through LDS at the end.  A latency-bound problem (few tiles, long K) then takes 1/KG of
 // the steps without partial sums in global memory.
-// GROUPED: the rows of y are grouped by expert and every expert has a weight of its own; a tile row comes from a list
-// the device made (which expert, which rows), and an x row may come through an index.
-template <int BN, int BM, int WAVES_N, int WAVES_M, bool W8, int NS, int OCC, int KG, bool GROUPED = false>
+// MODE kGrouped: the rows of y are grouped by expert and every expert has a weight of its own; a tile row comes from a list
+// the device made (which expert, which rows), and an x row may come through an index.  kActivated: the last columns go
+// through an activation into a matrix of their own.
+enum GemmMode { kPlain = 0, kGrouped = 1, kActivated = 2 };
+template <int BN, int BM, int WAVES_N, int WAVES_M, bool W8, int NS, int OCC, int KG, int MODE = kPlain>
 __global__ __launch_bounds__(WAVES_N * WAVES_M * KG * 64) __attribute__((amdgpu_waves_per_eu(OCC, 8)))
 void gemm_dlds_kernel(const GemmParams params) {
+  constexpr bool GROUPED = MODE == kGrouped;
   std::conditional_t<GROUPED, GemmParams, const GemmParams &> p = params;
   static_assert(NS >= 2 && NS <= 8, "2 to 8 stages");
   constexpr int NW = WAVES_N * WAVES_M;       // waves of one set
@@ -377,7 +380,10 @@ void gemm_dlds_kernel(const GemmParams params) {
       return;
     }
   }
-  gemm_epilogue<TN, TM, WN, WM, W8>(p, acc, m0, n0, wn, wm, r, kg, split);
+  if constexpr (MODE == kActivated)
+    gemm_epilogue_activated<TN, TM, WN, WM>(p, acc, m0, n0, wn, wm, r, kg);
+  else
+    gemm_epilogue<TN, TM, WN, WM, W8>(p, acc, m0, n0, wn, wm, r, kg, split);
 }
 
 // ---------------------------------------------------------------------------
@@ -1608,7 +1614,7 @@ int launch_grouped(GemmParams p, int bm, hipStream_t stream) {
   if (wgs > (1 << 30)) return TLF_E_SHAPE;
   const dim3 grid(static_cast<unsigned>(wgs));
 #define TLF_GROUPED(BN_, BM_, WN_, WM_, NS_, OCC_, KG_)                                                             \
-  TLF_LAUNCH((gemm_dlds_kernel<BN_, BM_, WN_, WM_, false, NS_, OCC_, KG_, true>), grid, dim3(WN_ * WM_ * KG_ * 64), \
+  TLF_LAUNCH((gemm_dlds_kernel<BN_, BM_, WN_, WM_, false, NS_, OCC_, KG_, kGrouped>), grid, dim3(WN_ * WM_ * KG_ * 64), \
              0, stream, p)
   if (deep) TLF_GROUPED(64, 32, 2, 1, 3, 4, 4);
   else if (bm == 32) TLF_GROUPED(128, 32, 4, 1, 4, 4, 1);
@@ -1786,6 +1792,43 @@ extern "C" int tlf_gemm_deferred(const void *x, int64_t x_stride, const void *w,
   hipStream_t s = static_cast<hipStream_t>(stream);
   return scale ? launch_gemm<true>(x, x_stride, w, scale, y, M, N, K, workspace, workspace_bytes, s, nullptr, 0, nullptr, nullptr, splits)
                : launch_gemm<false>(x, x_stride, w, nullptr, y, M, N, K, workspace, workspace_bytes, s, nullptr, 0, nullptr, nullptr, splits);
+}
+
+extern "C" int tlf_bf16_gemm_xielu(const void *x, int64_t x_stride, const void *w, void *y, int32_t M, int32_t N, int32_t K,
+                                   int32_t act_col, const void *pq, void *out, int64_t out_stride, int32_t out_cols,
+                                   void *stream) {
+  if (M == 0) return TLF_OK;
+  const int rc = check_gemm_args(x, x_stride, w, y, M, N, K);
+  if (rc != TLF_OK) return rc;
+  if (!pq || !out) return TLF_E_NULL;
+  if (act_col < 0 || act_col % 8 || act_col > N || out_cols <= 0 || out_cols % 8 || out_stride < out_cols) return TLF_E_SHAPE;
+  if (!aligned16(out) || out_stride % 8) return TLF_E_ALIGN;
+  GemmParams p{};
+  p.x = static_cast<const unsigned char *>(x);
+  p.ldx_bytes = x_stride * 2;
+  p.w = static_cast<const unsigned char *>(w);
+  p.y = static_cast<unsigned short *>(y);
+  p.M = M; p.N = N; p.K = K;
+  p.k_per_split = K;
+  p.splits = 1;
+  p.a = ActivatedColumns{static_cast<const unsigned short *>(pq), static_cast<unsigned short *>(out), out_stride, act_col, out_cols};
+  // the plans of the plain product at these sizes: 256 x 256 tiles where they fill the CUs, 128 x 128 below
+  const bool large = static_cast<int64_t>((N + 255) / 256) * ((M + 255) / 256) >= 160;
+  const int bt = large ? 256 : 128;
+  p.m_tiles = (M + bt - 1) / bt;
+  p.n_tiles = (N + bt - 1) / bt;
+  p.xcd_rows = p.m_tiles >= 16;
+  const int owned = p.xcd_rows ? p.m_tiles : p.n_tiles, walked = p.xcd_rows ? p.n_tiles : p.m_tiles, each = owned / 8;
+  p.group_n = walked >= 8 && each > 0 ? (each % 4 == 0 ? 4 : each % 3 == 0 ? 3 : each % 2 == 0 ? 2 : 1) : 1;
+  p.map_full = each * 8;
+  p.map_rem = owned - p.map_full;
+  p.map_main = each * 8 * walked;
+  const dim3 grid(p.map_main + p.map_rem * walked);
+  if (p.map_rem == 0) p.map_rem = 1;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (large) TLF_LAUNCH((gemm_dlds_kernel<256, 256, 8, 1, false, 2, 2, 1, kActivated>), grid, dim3(512), 0, s, p);
+  else TLF_LAUNCH((gemm_dlds_kernel<128, 128, 2, 2, false, 3, 2, 1, kActivated>), grid, dim3(256), 0, s, p);
+  return launch_status();
 }
 
 extern "C" size_t tlf_gemm_f32_sums_bytes(int32_t M, int32_t N, int32_t K) {

@@ -2,7 +2,7 @@
 // conversion, the epilogue over MFMA accumulator tiles and the global -> LDS copy instruction.
 #pragma once
 
-#include "common.h"
+#include "elem.h"
 
 namespace tlf {
 
@@ -28,6 +28,14 @@ struct GroupedRows {
   float limit;
 };
 
+// Columns from `col` on go through xIELU into a matrix of their own
+struct ActivatedColumns {
+  const unsigned short *pq;   // the activation's two numbers
+  unsigned short *out;        // [M, ldo]; columns 0 .. cols - 1 are written
+  int64_t ldo;
+  int32_t col, cols;
+};
+
 struct GemmParams {
   const unsigned char *x;
   int64_t ldx_bytes;
@@ -50,6 +58,7 @@ struct GemmParams {
   unsigned long long *amax;
   int32_t amax_parts;  // key columns per token: one per (N-tile, wave along N)
   GroupedRows g;
+  ActivatedColumns a;
 };
 
 // Clipped GLU with a factor on the products: g = min(f gate, limit), u = clamp(f up, +-limit), g sigmoid(1.702 g) (u + 1).
@@ -242,6 +251,42 @@ __device__ __forceinline__ void gemm_epilogue_clipped_glu(const GemmParams &p, f
         *reinterpret_cast<uint4 *>(p.y + static_cast<int64_t>(m) * (p.N / 2) + nfirst / 2 + kg * 8) =
             make_uint4(rx[0], ry[0], rx[1], ry[1]);
     }
+  }
+}
+
+// Plain bf16 rows up to column a.col, activated ones from there on (a.col is a multiple of 8).
+template <int TN, int TM, int WN, int WM>
+__device__ __forceinline__ void gemm_epilogue_activated(const GemmParams &p, floatx16 (&acc)[TN][TM], int m0, int n0,
+                                                        int wn, int wm, int r, int kg) {
+  const float sa = softplus_f32(bf16_bits_to_float(p.a.pq[0])), sb = 0.5f + softplus_f32(bf16_bits_to_float(p.a.pq[1]));
+#pragma unroll
+  for (int j = 0; j < TM; ++j) {
+    const int m = m0 + wm * WM + j * 32 + r;
+#pragma unroll
+    for (int i = 0; i < TN; ++i)
+#pragma unroll
+      for (int h = 0; h < 2; ++h) {
+        const int first = n0 + wn * WN + i * 32 + h * 16;
+        uint2 st[2];
+#pragma unroll
+        for (int q = 0; q < 2; ++q) {
+          float o[4];
+#pragma unroll
+          for (int e = 0; e < 4; ++e) o[e] = acc[i][j][(2 * h + q) * 4 + e];
+          if (first + q * 8 >= p.a.col) {   // wave uniform
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] = xielu_f32(o[e], sa, sb);
+          }
+          st[q] = make_uint2(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]));
+        }
+        auto rx = __builtin_amdgcn_permlane32_swap(st[0].x, st[1].x, false, false);
+        auto ry = __builtin_amdgcn_permlane32_swap(st[0].y, st[1].y, false, false);
+        const int n = first + kg * 8;
+        const uint4 v = make_uint4(rx[0], ry[0], rx[1], ry[1]);
+        if (m >= p.M || n >= p.N) continue;
+        if (n < p.a.col) *reinterpret_cast<uint4 *>(p.y + static_cast<int64_t>(m) * p.N + n) = v;
+        else if (n - p.a.col < p.a.cols) *reinterpret_cast<uint4 *>(p.a.out + m * p.a.ldo + (n - p.a.col)) = v;
+      }
   }
 }
 

@@ -268,21 +268,6 @@ struct XieluArgs {
   int64_t ldo;
   int32_t rows, cols, padded;   // columns cols .. padded - 1 of `out` become zeros
 };
-__device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
-// e^z - 1 - z without cancellation: five terms of the series near zero (relative error below 2^-24 for |z| < 1/16).
-__device__ __forceinline__ float exp_rest(float z) {
-  if (z > -0.0625f) {
-    float r = fmaf(z, 1.0f / 720.0f, 1.0f / 120.0f);
-    r = fmaf(z, r, 1.0f / 24.0f);
-    r = fmaf(z, r, 1.0f / 6.0f);
-    r = fmaf(z, r, 0.5f);
-    return z * z * r;
-  }
-  return __builtin_amdgcn_exp2f(z * 1.4426950408889634f) - 1.0f - z;
-}
-__device__ __forceinline__ float xielu_f32(float z, float a, float b) {
-  return fmaf(z > 0.f ? a * z * z : b * exp_rest(fminf(z, 0.f)), 1.0f, 0.5f * z);
-}
 template <typename T, int VEC, bool PART>
 __global__ __launch_bounds__(256) void xielu_kernel(const XieluArgs a) {
   const int nch = a.padded / VEC;

@@ -249,6 +249,16 @@ class StackedLinear(LinearBase):
             return ops.linear_deferred(x, self.pack_().qpacked, self.qscale)
         return ops.linear_deferred(x, self.weight.data)
 
+    def forward_activated(self, x: torch.Tensor, name: str, act, out: torch.Tensor):
+        """The same with ``act`` (an ``XIELU``) on the last part, ``name``, whose result goes to ``out``: one kernel for many
+        rows, otherwise two."""
+        at = self.offset(name)
+        if x.shape[0] >= 512 and self.weight.dtype == torch.bfloat16 and not self.is_quantized and at % 8 == 0:
+            return ops.linear_xielu(pad_columns(x, _round_up(self.input_size, 64)), self.weight.data, at, act.pq.data, out)
+        y = self.forward_deferred(x)
+        act(y, at, self.parts[name], out)
+        return y
+
 
 class JoinedLinear(LinearBase):
     """One projection of several inputs laid side by side in a row, in the order of ``parts`` (name -> columns): the sum of

@@ -39,13 +39,15 @@ class GigopelLayer(nn.Module):
         self.out = JoinedLinear(joined, cfg.width)
 
     def forward(self, positions, h, x, following: ResidualRMSNorm):
-        proj = self.inp.forward_deferred(h)         # read by the next two kernels, before any other product
+        # the projections are read by the kernels that follow at once, before any other product
         rows = self.out.input_rows(h.shape[0], h.dtype, h.device)
+        if self.act is not None:
+            proj = self.inp.forward_activated(h, "up", self.act, rows[:, self.out.offset("down"):])
+        else:
+            proj = self.inp.forward_deferred(h)
         q = self.attn.prepare(proj, self.inp.offset("dkv"), positions)
         extra, join = (None, None), None
-        if self.act is not None:
-            self.act(proj, self.inp.offset("up"), self.inp.parts["up"], rows[:, self.out.offset("down"):])
-        elif self.experts is not None and h.shape[0] <= SIDE_BY_SIDE:
+        if self.experts is not None and h.shape[0] <= SIDE_BY_SIDE:
             with on_the_side(h.device) as join:
                 extra = self.experts(h)
         elif self.experts is not None:

@@ -987,3 +987,17 @@ def xielu(x, col, cols, pq, out):
     check(lib.tlf_xielu(*_source(x), col, pq.data_ptr(), out.data_ptr(), out.stride(0), out.shape[0], cols, out.shape[1],
                         _dt(out), _stream()), "tlf_xielu")
     return out
+
+
+def linear_xielu(x, w, act_col, pq, out):
+    """``bf16_linear(x, w)`` with xIELU on the columns from ``act_col`` on, which go to ``out`` instead; returns the rest (its
+    columns from ``act_col`` on are not written)."""
+    lib = _lib.load()
+    _need(x, BF16, "x"); _need(w, BF16, "w"); _need(pq, BF16, "pq"); _need(out, BF16, "out")
+    assert x.dim() == 2 and x.stride(1) == 1 and w.is_contiguous() and out.stride(1) == 1 and out.shape[0] == x.shape[0]
+    (M, K), N = x.shape, w.shape[0]
+    assert w.shape[1] == K and pq.numel() == 2
+    y = torch.empty(M, N, dtype=BF16, device=x.device)
+    check(lib.tlf_bf16_gemm_xielu(x.data_ptr(), x.stride(0), w.data_ptr(), y.data_ptr(), M, N, K, act_col, pq.data_ptr(),
+                                  out.data_ptr(), out.stride(0), out.shape[1], _stream()), "tlf_bf16_gemm_xielu")
+    return y
