@@ -640,7 +640,7 @@ def bench_gitopel_kernels():
     import torch
     from tinyllmforge_amd import ops as P
     from tinyllmforge_amd.layers.rotary_embedding import build_cos_sin_cache
-    from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
+    from tinyllmforge_amd.layers.rotary_embedding import rotation_table
     torch.manual_seed(0)
     BF, F32, dev = torch.bfloat16, torch.float32, "cuda"
     rows = []
@@ -704,7 +704,7 @@ def bench_gitopel_kernels():
         add("pooled rows of a prompt", size, lambda i: P.pool_blocks(kv, bt, cu, starts, 0, S, L),
             N * hkv * d * 4 * (1 + 1 / pool), "hbm")
         # -- what stands between the projections and attention
-        tab, tab2 = build_cos_sin_cache(d, 4096, 1e6).to(dev), interleaved_cos_sin(d, 4096, 1e4).to(dev)
+        tab, tab2 = build_cos_sin_cache(d, 4096, 1e6).to(dev), rotation_table(d, 4096, 1e4).to(dev)
         wd = torch.ones(d, dtype=BF, device=dev)
         slots = torch.arange(N, dtype=torch.int32, device=dev)
         pos = torch.arange(L, device=dev).repeat(S)
@@ -817,7 +817,7 @@ def bench_gigopel_kernels(sizes=None):
     from tinyllmforge_amd import ops as P
     from tinyllmforge_amd.layers.latent_attention import LatentAttention
     from tinyllmforge_amd.layers.moe import ClippedGLUExperts
-    from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
+    from tinyllmforge_amd.layers.rotary_embedding import rotation_table
     torch.manual_seed(0)
     BF, dev = torch.bfloat16, "cuda"
     rows = []
@@ -903,13 +903,13 @@ def bench_gigopel_kernels(sizes=None):
                 2.0 * h * (d + t + v) * seen, "mfma bf16")
         del q, out, expanded, latents
         # -- between the products
-        tab = interleaved_cos_sin(t, 4096, 1e4).to(dev)
+        tab = rotation_table(t, 4096, 1e4).to(dev)
         slots = torch.arange(N, dtype=torch.int32, device=dev)
         pos = torch.arange(L, device=dev).repeat(S)
         ld = -(-(h * (d + t) + r + t) // 16) * 16
         nw = torch.ones(r, device=dev, dtype=BF)
         pq = torch.zeros(2, device=dev, dtype=BF)
-        wd, tabq = torch.ones(qd, dtype=BF, device=dev), interleaved_cos_sin(qd, 4096, 1e6).to(dev)
+        wd, tabq = torch.ones(qd, dtype=BF, device=dev), rotation_table(qd, 4096, 1e6).to(dev)
         for n, copies in ((N, 3), (B, 1)):
             qkv = bf(copies, n, (hq + 2 * hkv) * qd)
             kc, vc = bf(2, N // bs, bs, hkv, qd)

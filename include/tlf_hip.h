@@ -660,13 +660,15 @@ int tlf_latent_prefill(const void *q, const void *expanded, int64_t expanded_str
  *
  * tlf_gemm_f32_sums: y = x . w^T with bf16 factors as fp32 sums [*splits, M, N] to be added up (*splits in host memory);
  *   for the router's logits, N = experts rounded up to 16.
- * tlf_moe_group: from the logits' sums, ids[token, k] the `top` largest (ties: the smaller index) and weights[token, k] =
- *   sigmoid; row_of[token * top + k] = the entry's row in expert order, src[row] its token, row_weight[row] its weight;
+ * tlf_moe_group: from the logits' sums (experts + identity of them), with correction NULL ids[token, k] the `top` largest
+ *   (ties: the smaller index) and weights[token, k] = sigmoid; otherwise the `top` largest of softmax + correction (of `dtype`)
+ *   and weights = softmax values, normalised to a sum of 1.  Experts from `experts` on have no rows: row_of = -1; row_of[token * top + k] = the entry's row in expert order, src[row] its token, row_weight[row] its weight;
  *   tiles (int32 x 4: expert, first row, rows, 0) cut the rows into at most tile_rows of one expert each, *num_tiles <=
- *   max_tiles of them; max_tiles >= n * top / tile_rows + min(experts, n * top).  experts <= 512.
- * tlf_moe_gemm: y[row] = W[expert] x[x_rows ? x_rows[row] : row]; w [experts, N, K].  clipped_glu: channels are interleaved
- *   as for the SiLU-and-mul products (8 gate, then the 8 matching up); with f = row_scale[row] (NULL: 1), g = min(f gate,
- *   limit), u = clamp(f up, +-limit): y [rows, N / 2] = g sigmoid(1.702 g) (u + 1).  bf16: tile_rows 32, 64, 128 or 256, K a
+ *   max_tiles of them; max_tiles >= n * top / tile_rows + min(experts, n * top).  experts + identity <= 512.
+ * tlf_moe_gemm: y[row] = W[expert] x[x_rows ? x_rows[row] : row]; w [experts, N, K].  act 1 and 2: channels are interleaved
+ *   as for the SiLU-and-mul products (8 gate, then the 8 matching up), y [rows, N / 2]; act 1, clipped GLU: with f =
+ *   row_scale[row] (NULL: 1), g = min(f gate, limit), u = clamp(f up, +-limit): y = g sigmoid(1.702 g) (u + 1); act 2: y =
+ *   silu(gate) up in fp32.  bf16: tile_rows 32, 64, 128 or 256, K a
  *   multiple of 64; fp32: tile_rows 64.  x_count bounds the x rows.
  * tlf_xielu: with a = softplus(pq[0]), b = 1/2 + softplus(pq[1]), out = a z^2 + z / 2 for z > 0, b (e^z - 1 - z) + z / 2
  *   otherwise, z = columns col .. col + cols - 1 of x (or of partial sums); columns cols .. padded_cols - 1 become 0.
@@ -678,10 +680,11 @@ int tlf_gemm_f32_sums(const void *x, int64_t x_stride, const void *w, float *sum
 size_t tlf_moe_group_workspace_bytes(int32_t n, int32_t top, int32_t experts);
 int tlf_moe_group(const float *sums, int32_t splits, int32_t *ids, float *weights, int32_t *row_of, int32_t *src,
                   float *row_weight, int32_t *tiles, int32_t *num_tiles, int32_t max_tiles, int32_t n, int32_t top,
-                  int32_t experts, int32_t tile_rows, void *workspace, size_t workspace_bytes, void *stream);
+                  int32_t experts, int32_t identity, const void *correction, int32_t dtype, int32_t tile_rows,
+                  void *workspace, size_t workspace_bytes, void *stream);
 int tlf_moe_gemm(const void *x, int64_t x_stride, int32_t x_count, const void *w, void *y, const int32_t *tiles,
                  const int32_t *num_tiles, int32_t max_tiles, int32_t tile_rows, const int32_t *x_rows, const float
-                 *row_scale, int32_t rows, int32_t N, int32_t K, int32_t clipped_glu, float limit, int32_t dtype,
+                 *row_scale, int32_t rows, int32_t N, int32_t K, int32_t act, float limit, int32_t dtype,
                  void *stream);
 int tlf_bf16_gemm_xielu(const void *x, int64_t x_stride, const void *w, void *y, int32_t M, int32_t N, int32_t K,
                         int32_t act_col, const void *pq, void *out, int64_t out_stride, int32_t out_cols, void
@@ -689,6 +692,63 @@ int tlf_bf16_gemm_xielu(const void *x, int64_t x_stride, const void *w, void *y,
 int tlf_xielu(const void *x, int64_t x_stride, const float *partials, int32_t splits, const float *scale, int32_t
               col, const void *pq, void *out, int64_t out_stride, int32_t rows, int32_t cols, int32_t padded_cols,
               int32_t dtype, void *stream);
+
+/* Layer norm around an fp32 residual stream: with t = x[row] after the step, h = ((t - mean) / sqrt(variance + eps) * w_next +
+ * b_next) * out_scale, the variance being the mean of the squared deviations.
+ *
+ * tlf_embed_layernorm: x = table[id].
+ * tlf_residual_layernorm: x += y (NULL and splits <= 1: none; or its partial sums) + the sum over k < top of extra_weights[row,
+ *   k] (NULL: 1) times extra[extra_rows[row, k]], a negative index standing for self[row]. */
+int tlf_embed_layernorm(const int64_t *ids, const void *table, int32_t vocab, float *x, const void *w_next, const void
+                        *b_next, float out_scale, void *h, int32_t rows, int32_t width, float eps, int32_t dtype,
+                        void *stream);
+int tlf_residual_layernorm(const void *y, int64_t y_stride, const float *partials, int32_t splits, const float *scale,
+                           const void *extra, int64_t extra_stride, const int32_t *extra_rows, const float
+                           *extra_weights, int32_t top, const void *self, int64_t self_stride, float *x, const void
+                           *w_next, const void *b_next, float out_scale, void *h, int32_t rows, int32_t width, float
+                           eps, int32_t dtype, void *stream);
+
+/* Causal grouped-query attention with a sink, a score cap and an output gate on paged, head-major caches k_cache [pages,
+ * kv_heads, block, Dp], v_cache [pages, kv_heads, block, Vp] (Dp, Vp: dim and vdim rounded up to 32, pads are zeros).
+ *   score = scale (q . k), cap > 0: cap tanh(score / cap);  out = sigmoid(gate) * sum exp(score) v / (sum exp(score) + exp(sink))
+ * sink [heads] and gate [rows, heads * vdim] may be NULL (no such term).  dim, vdim <= 512, block a multiple of 64.
+ *
+ * tlf_sink_prep: projection rows [q: heads * dim | k: kv_heads * dim | v: kv_heads * vdim | gate: heads * vdim] -> + bias (NULL:
+ *   none; of the channels of q, k and v) -> with conv [taps, channels] y_p = sum_j conv[j] u_(p - taps + 1 + j), zeros before the
+ *   sequence -> q, k / rms over the head * q_norm / k_norm (NULL: 1) -> q times q_mult[pos] (NULL: 1) -> the first rot_dims
+ *   dimensions of q and k turned by cos_sin[pos] (cos of the pairs, then sin), i with i + rot_dims / 2 -> q_out [n, heads, Dp]
+ *   and the cache rows slot_mapping[token] (negative: not stored).  ring [state slots, taps, channels] holds the projected rows
+ *   (without bias) of a sequence's last positions, p in row p mod taps: rows of one-token sequences (row_seq NULL, or
+ *   cu_seqlens_q of row_seq[row]) are written here, those of portions by tlf_conv_tail afterwards.  gate_out [n, heads * vdim]
+ *   (NULL: not copied) gets the gate's columns; with splits > 1 it must be there and row_seq NULL.
+ * tlf_conv_tail: last taps - 1 projected rows of sequences first_seq .. (proj: the step's rows) into the ring.
+ * tlf_sink_attn_rows: row r of q [rows, heads, Dp] attends to positions 0 .. positions[r] of sequence row_seq[r] (NULL: r);
+ *   slot_mapping[r] < 0: a padding row (zeros).  max_len bounds the positions.  bf16 up to 256 dimensions on the matrix cores.
+ * tlf_sink_attn_prefill: portions of sequences first_seq .., rows as in the step; bf16, dim, vdim <= 256. */
+int tlf_sink_prep(const void *proj, int64_t proj_stride, const float *partials, int32_t splits, const float *scale,
+                  const void *bias, const void *conv, int32_t taps, void *ring, const int32_t *state_slots, int64_t
+                  num_state_slots, const int32_t *row_seq, const int32_t *cu_seqlens_q, const void *q_norm, const void
+                  *k_norm, const int64_t *positions, const float *cos_sin, const float *q_mult, int32_t max_pos,
+                  int32_t rot_dims, const int32_t *slot_mapping, void *q_out, void *k_cache, void *v_cache, void
+                  *gate_out, int32_t n, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t
+                  block_size, int64_t num_pages, float eps, int32_t dtype, void *stream);
+int tlf_conv_tail(const void *proj, int64_t proj_stride, void *ring, const int32_t *state_slots, int64_t
+                  num_state_slots, const int32_t *cu_seqlens_q, const int32_t *seq_starts, int32_t first_seq, int32_t
+                  num_seqs, int32_t taps, int32_t channels, int32_t dtype, void *stream);
+size_t tlf_sink_attn_rows_workspace_bytes(int32_t rows, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim,
+                                          int32_t max_len, int32_t dtype);
+int tlf_sink_attn_rows(const void *q, const void *k_cache, const void *v_cache, const int32_t *block_tables, int64_t
+                       bt_stride, const int64_t *positions, const int32_t *slot_mapping, const int32_t *row_seq, const
+                       void *sink, const void *gate, int64_t gate_stride, void *out, int64_t out_stride, int32_t rows,
+                       int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t block_size, int32_t
+                       max_len, int64_t num_pages, float scale, float cap, int32_t dtype, void *workspace, size_t
+                       workspace_bytes, void *stream);
+int tlf_sink_attn_prefill_supported(int32_t dim, int32_t vdim);
+int tlf_sink_attn_prefill(const void *q, const void *k_cache, const void *v_cache, const int32_t *block_tables, int64_t
+                          bt_stride, const int32_t *cu_seqlens_q, const int32_t *seq_starts, int32_t first_seq,
+                          int32_t num_seqs, int32_t max_tokens, const void *sink, const void *gate, int64_t
+                          gate_stride, void *out, int64_t out_stride, int32_t heads, int32_t kv_heads, int32_t dim,
+                          int32_t vdim, int32_t block_size, int64_t num_pages, float scale, float cap, void *stream);
 
 #ifdef __cplusplus
 }

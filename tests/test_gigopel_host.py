@@ -295,7 +295,7 @@ def test_entry_points_reject_bad_arguments_on_the_host():
     assert lib.tlf_latent_gather(a, a, 4, a, a, a, 0, 1, 8, a, 100, 64, 5, 10, None) == -2
     assert lib.tlf_latent_attn_supported(2, 20, 6, 27, 13) == 1 and lib.tlf_latent_attn_supported(2, 20, 64, 600, 13) == 0
     assert lib.tlf_latent_prefill_supported(2, 20, 6, 27, 129) == 0
-    group = lambda top=2, E=5, tiles=9, splits=1, n=4: lib.tlf_moe_group(a, splits, a, a, a, a, a, a, a, tiles, n, top, E, 32, None, 0, None)
+    group = lambda top=2, E=5, tiles=9, splits=1, n=4: lib.tlf_moe_group(a, splits, a, a, a, a, a, a, a, tiles, n, top, E, 0, None, 0, 32, None, 0, None)
     assert group(top=6) == -2 and group(E=600) == -2 and group(tiles=4) == -2 and group(n=0) == 0 and group(n=4000, tiles=9999) == -4
     gemm = lambda rows=32, N=32, K=64, dt=0, xs=64, count=4: lib.tlf_moe_gemm(a, xs, count, a, a, a, a, 9, rows, a, None, 8, N, K, 0, 0.0, dt, None)
     assert gemm(rows=48) == -2 and gemm(N=20) == -2 and gemm(xs=32) == -2 and gemm(dt=1, rows=32) == -2 and gemm(count=1 << 30) == -6

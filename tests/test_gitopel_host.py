@@ -300,8 +300,8 @@ def test_entry_points_reject_bad_arguments_on_the_host():
 
 
 def test_interleaved_table_is_exact_to_fp32():
-    from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
-    t = interleaved_cos_sin(6, 5000, 10000.0)
+    from tinyllmforge_amd.layers.rotary_embedding import rotation_table
+    t = rotation_table(6, 5000, 10000.0)
     for p in (0, 1, 4999):
         for i in range(3):
             a = p * 10000.0 ** (-2 * i / 6)

@@ -108,7 +108,7 @@ class Attention:
     def __init__(self, sizes, window, lens, dt, seed=0, bs=64, scale=None, long_portion=128, uk=None, uv=None):
         from tinyllmforge_amd.engine.sequence import Sequence
         from tinyllmforge_amd.layers.latent_attention import LatentAttention
-        from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
+        from tinyllmforge_amd.layers.rotary_embedding import rotation_table
         Sequence.block_size = bs
         self.H, self.D, self.R, self.V, self.rank = sizes
         self.window, self.lens, self.dt, self.bs, self.long = window, lens, dt, bs, long_portion
@@ -120,7 +120,7 @@ class Attention:
         self.norm = (1 + 0.2 * rnd(self.rank) if uk is None else torch.ones(self.rank)).to(dt)
         torch.set_default_dtype(dt)
         self.layer = LatentAttention(self.H, self.D, self.R, self.rank, self.V, self.scale, window, 0,
-                                     interleaved_cos_sin(self.R, max(lens) + 1, self.base), self.eps, dt).cuda()
+                                     rotation_table(self.R, max(lens) + 1, self.base), self.eps, dt).cuda()
         torch.set_default_dtype(torch.float32)
         for p, v in ((self.layer.uk, self.uk), (self.layer.uv, self.uv), (self.layer.norm.weight, self.norm)):
             p.data.copy_(v)
@@ -361,7 +361,7 @@ def test_mixture_of_experts(dtype, n, width, E, top, ff, limit):
 def test_consumers_add_up_split_projections():
     """A projection left as partial sums gives the bits of the finished one, in every kernel that may read it."""
     from tinyllmforge_amd import ops as P
-    from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
+    from tinyllmforge_amd.layers.rotary_embedding import rotation_table
     g, n, K = torch.Generator().manual_seed(2), 40, 4096
     bf = lambda *s: torch.randn(*s, generator=g).to(torch.bfloat16).cuda()
 
@@ -374,7 +374,7 @@ def test_consumers_add_up_split_projections():
         s = P.LatentShape(H, D, R, rank, V)
         col = H * (D + R)
         N = -(-(col + rank + R + ff) // 16) * 16
-        tab, pos, slots = interleaved_cos_sin(R, 100, 1e4).cuda(), torch.arange(n).cuda(), torch.arange(n, dtype=torch.int32).cuda()
+        tab, pos, slots = rotation_table(R, 100, 1e4).cuda(), torch.arange(n).cuda(), torch.arange(n, dtype=torch.int32).cuda()
         nw, pq = bf(rank), bf(2)
         cache = torch.zeros(2, 1, 64, s.lp, dtype=torch.bfloat16, device="cuda")
         out = torch.zeros(2, n, -(-ff // 64) * 64, dtype=torch.bfloat16, device="cuda")

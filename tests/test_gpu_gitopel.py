@@ -63,7 +63,7 @@ def test_f32_dense_operations(M, N, K):
 @pytest.mark.parametrize("H,G,D,rot", [(6, 2, 40, 24), (8, 8, 128, 128), (3, 1, 32, 0), (2, 1, 256, 64), (4, 2, 18, 18), (3, 3, 33, 20)])
 def test_attention_preparation(dtype, H, G, D, rot):
     from tinyllmforge_amd import ops as P
-    from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
+    from tinyllmforge_amd.layers.rotary_embedding import rotation_table
     dt, g, n, eps = DTYPES[dtype], torch.Generator().manual_seed(1), 21, 1e-4
     width = (H + G) * D + H
     proj = torch.randn(n, -(-width // 16) * 16, generator=g).to(dt)
@@ -72,7 +72,7 @@ def test_attention_preparation(dtype, H, G, D, rot):
     kv = P.PooledKV(3, 64, G, D, 8, 8, dt, "cuda")
     slots = torch.randperm(3 * 64, generator=g)[:n].to(torch.int32)
     slots[4] = -1
-    table = interleaved_cos_sin(rot, 900, 777.0)
+    table = rotation_table(rot, 900, 777.0)
     q, gate = P.attn_prep(proj.cuda(), qb.cuda(), kb.cuda(), pos.cuda(), table.cuda(), rot, slots.cuda(), kv.k, kv.v, H, D, eps)
     qr = (proj[:, :H * D].double() + qb.double()).view(n, H, D)
     kr = (proj[:, H * D:(H + G) * D].double() + kb.double()).view(n, G, D)
@@ -315,7 +315,7 @@ def test_consumers_add_up_split_projections(quantized):
     """A projection left as partial sums gives the bits of the finished one, in every kernel that may read it."""
     from tinyllmforge_amd import ops as P
     from tinyllmforge_amd.layers.linear import quantize_per_channel
-    from tinyllmforge_amd.layers.pooled_attention import interleaved_cos_sin
+    from tinyllmforge_amd.layers.rotary_embedding import rotation_table
     g, n, K = torch.Generator().manual_seed(2), 40, 4096
     bf = lambda *s: torch.randn(*s, generator=g).to(torch.bfloat16).cuda()
 
@@ -337,7 +337,7 @@ def test_consumers_add_up_split_projections(quantized):
     H, G, D = 8, 2, 96
     y, d = both(-(-((H + G) * D + H) // 16) * 16)
     assert d.splits > 1
-    tab, pos, slots = interleaved_cos_sin(64, 100, 1e4).cuda(), torch.arange(n).cuda(), torch.arange(n, dtype=torch.int32).cuda()
+    tab, pos, slots = rotation_table(64, 100, 1e4).cuda(), torch.arange(n).cuda(), torch.arange(n, dtype=torch.int32).cuda()
     kv = [P.PooledKV(1, 64, G, D, 8, 8, torch.bfloat16, "cuda") for _ in range(2)]
     args = lambda c: (None, None, pos, tab, 64, slots, c.k, c.v, H, D, 1e-6)
     q2, g2 = P.attn_prep(d, *args(kv[1]))

@@ -96,6 +96,10 @@ class LayeredConfig:
     def num_hidden_layers(self) -> int:
         return len(self.layers)
 
+    def layer_runs(self) -> list[int]:
+        """Indices of the layers in the order they run."""
+        return list(range(len(self.layers)))
+
     @classmethod
     def from_dict(cls, src: dict, directory: str | None = None):
         import copy
@@ -162,6 +166,46 @@ class GigopelConfig(LayeredConfig):
         self.windows = tuple(sorted({layer["mixer"]["mask"]["size"] for layer in self.layers}))
 
 
+@dataclass
+class ZuzunexConfig(LayeredConfig):
+    """A Zuzunex model: grouped-query attention with sinks and output gates, and SwiGLU feed-forwards or mixtures of experts.
+
+    Keys of ``config.json``: ``vocab``, ``width``, ``logit_scale``, ``norm`` (``eps``), ``loop`` (null, or layers ``start`` ..
+    ``stop - 1`` run ``times`` times in a row) and ``layers``; a layer has ``type``, ``mixer`` and ``mlp``.  Mixers have ``heads``,
+    ``kv_heads``, ``dim``, ``vdim``, ``scale``; 'attention' also ``q_temp`` (``coef``, ``every``) and ``softcap``, 'attention_2'
+    ``conv`` (taps) and ``rot`` (``dims``, ``base``, ``scaling``: null or ``factor``, ``original``, ``fast``, ``slow``).  ``mlp``:
+    null, ``kind`` 'dense' with ``ff``, or ``kind`` 'moe' with ``expert`` (``ff``), ``router`` (``experts``, ``identity``, ``top``)
+    and ``shared`` (``ff``)."""
+    logit_scale: float = 1.0
+    loop: dict | None = None
+
+    # from this many tokens on a portion's rows share the keys of a tile; shorter portions run row by row
+    long_portion = 16
+
+    def check_layers(self):
+        for layer in self.layers:
+            assert layer["type"] in ("attention", "attention_2"), f"unknown mixer {layer['type']!r}"
+            m, mlp = layer["mixer"], layer.get("mlp")
+            assert m["heads"] % m["kv_heads"] == 0
+            rot = m.get("rot")
+            assert not rot or (rot["dims"] % 2 == 0 and rot["dims"] <= m["dim"])
+            if layer["type"] == "attention_2":
+                assert m["conv"] >= 1
+            assert not mlp or mlp["kind"] in ("dense", "moe")
+            if mlp and mlp["kind"] == "moe":
+                r = mlp["router"]
+                assert 1 <= r["top"] <= r["experts"] + (r.get("identity") or 0)
+        if self.loop:
+            assert 0 <= self.loop["start"] <= self.loop["stop"] <= len(self.layers) and self.loop["times"] >= 1
+        self.recurrent = any(layer["type"] == "attention_2" for layer in self.layers)     # a convolution has a state
+
+    def layer_runs(self) -> list[int]:
+        if not self.loop:
+            return super().layer_runs()
+        start, stop = self.loop["start"], self.loop["stop"]
+        return [*range(start), *list(range(start, stop)) * self.loop["times"], *range(stop, len(self.layers))]
+
+
 def tensor_shapes(directory: str) -> dict:
     """name -> shape of every tensor in ``directory/*.safetensors``, from the files' headers."""
     from glob import glob
@@ -173,7 +217,7 @@ def tensor_shapes(directory: str) -> dict:
     return out
 
 
-LAYERED_DESIGNS = {"Gitopel": GitopelConfig, "Gigopel": GigopelConfig}
+LAYERED_DESIGNS = {"Gitopel": GitopelConfig, "Gigopel": GigopelConfig, "Zuzunex": ZuzunexConfig}
 
 
 def architecture_of(src: dict) -> str:

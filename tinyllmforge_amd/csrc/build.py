@@ -35,6 +35,8 @@ EXTRA_FLAGS = {
     "prefill_attn.hip": ["-fno-honor-nans"],
     "decode_attn.hip": ["-fno-honor-nans"],
     "pooled_prefill.hip": ["-fno-honor-nans"],
+    "sink_prefill.hip": ["-fno-honor-nans"],
+    "sink_decode.hip": ["-fno-honor-nans"],
 }
 
 

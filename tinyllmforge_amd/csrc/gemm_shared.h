@@ -26,6 +26,7 @@ struct GroupedRows {
   const float *row_scale;     // factor of every row of the product (clipped-GLU epilogue)
   int64_t w_bytes;            // from one expert's weight to the next
   float limit;
+  int32_t plain;              // SwiGLU instead of the clipped GLU
 };
 
 // Columns from `col` on go through xIELU into a matrix of their own
@@ -224,7 +225,7 @@ __device__ __forceinline__ void gemm_epilogue_sc(const GemmParams &p, floatx16 (
   }
 }
 
-// Clipped GLU over interleaved gate/up channels (8 gate rows, then the 8 matching up rows), factor per row.
+// Clipped GLU, factor per row, or plain SwiGLU over interleaved gate/up channels (8 gate rows, then the 8 matching up rows).
 template <int TN, int TM, int WN, int WM>
 __device__ __forceinline__ void gemm_epilogue_clipped_glu(const GemmParams &p, floatx16 (&acc)[TN][TM], int m0, int n0,
                                                           int wn, int wm, int r, int kg) {
@@ -240,7 +241,9 @@ __device__ __forceinline__ void gemm_epilogue_clipped_glu(const GemmParams &p, f
       for (int q = 0; q < 4; q += 2) {
         float o[4];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) o[e] = clipped_glu(acc[i][j][q * 4 + e], acc[i][j][(q + 1) * 4 + e], factor, p.g.limit);
+        for (int e = 0; e < 4; ++e)
+          o[e] = p.g.plain ? silu_f32(acc[i][j][q * 4 + e]) * acc[i][j][(q + 1) * 4 + e]
+                           : clipped_glu(acc[i][j][q * 4 + e], acc[i][j][(q + 1) * 4 + e], factor, p.g.limit);
         st[q / 2] = make_uint2(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]));
       }
       // lanes r and r + 32 hold 4 channels each of two groups of 8: one exchange makes 8 consecutive channels per lane

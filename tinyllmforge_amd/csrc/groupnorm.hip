@@ -5,7 +5,9 @@
 //   mode add:    x = x + norm(y + y_bias) * w_post;           h = norm(x) * w_next
 //   mode plain:  x = x + mult * (y + sum of extra rows);      h = norm(x) * (w_next + w_offset)
 //
-// (w_offset 1: a weight stored around zero.  The extra rows are a mixture of experts' results, found through an index.)
+// (w_offset 1: a weight stored around zero.  The extra rows are a mixture of experts' results, found through an index, each
+// with a weight of its own where there are weights; a negative index stands for the row of another tensor, the experts' input.)
+// Modes embed and plain also exist with layer norm: h = ((x - mean) / sqrt(variance + eps) * w_next + b_next) * out_scale.
 // The norm after a sublayer, the residual add and the norm in front of the next sublayer share their grouping, so a
 // (row, group) pair is one independent unit: the three steps are one pass over memory.  HBM bound: y and x are read
 // once, x and h written once.  The residual is fp32; y, h and the weights are T (bf16 or fp32); arithmetic is fp32.
@@ -27,7 +29,11 @@ struct GroupNormArgs {
   void *h;              // [rows, width]
   const void *extra;    // [*, extra_stride] or NULL: rows extra_rows[row * top + k], k < top (plain mode)
   const int32_t *extra_rows;
-  int64_t extra_stride;
+  const float *extra_weights;   // [rows, top] or NULL: 1
+  const void *self;             // [rows, self_stride]: what a negative index stands for
+  const void *b_next;           // [width], layer norm
+  float out_scale;              // layer norm
+  int64_t extra_stride, self_stride;
   int32_t top;
   float mult, w_offset;
   int64_t units;        // rows * groups
@@ -64,7 +70,7 @@ __device__ __forceinline__ void stv(T *p, const float (&f)[VEC]) {
 }
 
 // MODE 0: embed, 1: add, 2: add with y as partial sums, 3: plain, 4: plain with y as partial sums
-template <typename T, int VEC, int TPR, int MAXC, int MODE>
+template <typename T, int VEC, int TPR, int MAXC, int MODE, bool LN>
 __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
   __shared__ float part[4];
   const int tid = threadIdx.x, sub = tid % TPR;
@@ -95,19 +101,25 @@ __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
 #pragma unroll
     for (int c = 0; c < MAXC; ++c) {
       const int at = min(sub + c * TPR, nch - 1) * VEC;
-      if constexpr (MODE == 3) ldv<T, VEC>(yr + at, v[c]);
-      else if constexpr (VEC == 8) a.part.ld8(row, col0 + at, v[c]);
+      if constexpr (MODE == 3) {
+        if (a.y) ldv<T, VEC>(yr + at, v[c]);
+        else
+#pragma unroll
+          for (int i = 0; i < VEC; ++i) v[c][i] = 0.f;
+      } else if constexpr (VEC == 8) a.part.ld8(row, col0 + at, v[c]);
       else v[c][0] = a.part.ld(row, col0 + at);
       ldv<float, VEC>(xr + at, xo[c]);
     }
     for (int k = 0; k < a.top; ++k) {
-      const T *er = static_cast<const T *>(a.extra) + a.extra_rows[row * a.top + k] * a.extra_stride + col0;
+      const int64_t at = a.extra_rows[row * a.top + k];
+      const T *er = (at >= 0 ? static_cast<const T *>(a.extra) + at * a.extra_stride : static_cast<const T *>(a.self) + row * a.self_stride) + col0;
+      const float f0 = a.extra_weights ? a.extra_weights[row * a.top + k] : 1.f;
 #pragma unroll
       for (int c = 0; c < MAXC; ++c) {
         float f[VEC];
         ldv<T, VEC>(er + min(sub + c * TPR, nch - 1) * VEC, f);
 #pragma unroll
-        for (int i = 0; i < VEC; ++i) v[c][i] += f[i];
+        for (int i = 0; i < VEC; ++i) v[c][i] = fmaf(f[i], f0, v[c][i]);
       }
     }
 #pragma unroll
@@ -157,11 +169,24 @@ __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
     if (ch < nch) {
       if (active) stv<float, VEC>(xr + ch * VEC, v[c]);
 #pragma unroll
-      for (int i = 0; i < VEC; ++i) ss = fmaf(v[c][i], v[c][i], ss);
+      for (int i = 0; i < VEC; ++i) ss = LN ? ss + v[c][i] : fmaf(v[c][i], v[c][i], ss);
     }
   }
   if (a.w_next == nullptr) return;  // uniform
   ss = unit_sum<TPR>(ss, part);
+  if constexpr (LN) {               // centred first: the variance is the mean of the squared deviations
+    const float mean = ss * inv_cols;
+    ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < MAXC; ++c)
+      if (sub + c * TPR < nch)
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) {
+          v[c][i] -= mean;
+          ss = fmaf(v[c][i], v[c][i], ss);
+        }
+    ss = unit_sum<TPR>(ss, part);
+  }
   const float inv = 1.0f / sqrtf(ss * inv_cols + a.eps);
   const T *wn = static_cast<const T *>(a.w_next) + col0;
   T *hr = static_cast<T *>(a.h) + row * a.width + col0;
@@ -173,15 +198,21 @@ __global__ __launch_bounds__(256) void groupnorm_kernel(const GroupNormArgs a) {
       ldv<T, VEC>(wn + ch * VEC, w);
 #pragma unroll
       for (int i = 0; i < VEC; ++i) w[i] = v[c][i] * inv * (w[i] + a.w_offset);
+      if constexpr (LN) {
+        float b[VEC];
+        ldv<T, VEC>(static_cast<const T *>(a.b_next) + col0 + ch * VEC, b);
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) w[i] = (w[i] + b[i]) * a.out_scale;
+      }
       stv<T, VEC>(hr + ch * VEC, w);
     }
   }
 }
 
-template <typename T, int MODE>
+template <typename T, int MODE, bool LN>
 int launch_groupnorm(const GroupNormArgs &a, bool vec8, hipStream_t stream) {
 #define TLF_GN(VEC, TPR, MAXC)                                                                               \
-  TLF_LAUNCH((groupnorm_kernel<T, VEC, TPR, MAXC, MODE>),                                                   \
+  TLF_LAUNCH((groupnorm_kernel<T, VEC, TPR, MAXC, MODE, LN>),                                                   \
              dim3(static_cast<unsigned>((a.units + (256 / TPR) - 1) / (256 / TPR))), dim3(256), 0, stream, a)
   if (vec8) {
     if (a.cols <= 128) TLF_GN(8, 16, 1);
@@ -201,7 +232,7 @@ int launch_groupnorm(const GroupNormArgs &a, bool vec8, hipStream_t stream) {
 }
 
 // kMode 0: embed, 1: add, 3: plain
-template <int kMode>
+template <int kMode, bool LN = false>
 int groupnorm_entry(GroupNormArgs &a, int32_t rows, int32_t dtype, hipStream_t stream) {
   if (rows < 0 || a.width <= 0 || a.groups <= 0 || a.width % a.groups) return TLF_E_SHAPE;
   if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
@@ -215,11 +246,12 @@ int groupnorm_entry(GroupNormArgs &a, int32_t rows, int32_t dtype, hipStream_t s
     vec8 = vec8 && aligned16(a.table);
   else
     vec8 = vec8 && aligned16(a.y) && aligned16(a.y_bias) && aligned16(a.w_post) && a.y_stride % 8 == 0;
-  if (kMode == 3) vec8 = vec8 && aligned16(a.extra) && a.extra_stride % 8 == 0;
+  if (kMode == 3) vec8 = vec8 && aligned16(a.extra) && a.extra_stride % 8 == 0 && aligned16(a.self) && a.self_stride % 8 == 0;
+  if (LN) vec8 = vec8 && aligned16(a.b_next);
   if constexpr (kMode != 0)
-    if (a.part.splits > 1) return launch_groupnorm<unsigned short, kMode + 1>(a, vec8, stream);
-  return dtype == TLF_DT_BF16 ? launch_groupnorm<unsigned short, kMode>(a, vec8, stream)
-                              : launch_groupnorm<float, kMode>(a, vec8, stream);
+    if (a.part.splits > 1) return launch_groupnorm<unsigned short, kMode + 1, LN>(a, vec8, stream);
+  return dtype == TLF_DT_BF16 ? launch_groupnorm<unsigned short, kMode, LN>(a, vec8, stream)
+                              : launch_groupnorm<float, kMode, LN>(a, vec8, stream);
 }
 
 }  // namespace tlf
@@ -263,4 +295,32 @@ extern "C" int tlf_residual_rmsnorm(const void *y, int64_t y_stride, const float
   a.extra = extra; a.extra_stride = extra_stride; a.extra_rows = extra_rows; a.top = top; a.mult = mult; a.w_offset = w_offset;
   a.width = width; a.groups = 1; a.eps = eps;
   return tlf::groupnorm_entry<3>(a, rows, dtype, static_cast<hipStream_t>(stream));
+}
+
+extern "C" int tlf_embed_layernorm(const int64_t *ids, const void *table, int32_t vocab, float *x, const void *w_next,
+                                   const void *b_next, float out_scale, void *h, int32_t rows, int32_t width, float eps,
+                                   int32_t dtype, void *stream) {
+  tlf::GroupNormArgs a{};
+  if (rows > 0 && (!ids || !table || !w_next || !b_next)) return TLF_E_NULL;
+  if (vocab <= 0) return TLF_E_SHAPE;
+  a.ids = ids; a.table = table; a.vocab = vocab; a.x = x; a.w_next = w_next; a.b_next = b_next; a.out_scale = out_scale; a.h = h;
+  a.width = width; a.groups = 1; a.eps = eps;
+  return tlf::groupnorm_entry<0, true>(a, rows, dtype, static_cast<hipStream_t>(stream));
+}
+
+extern "C" int tlf_residual_layernorm(const void *y, int64_t y_stride, const float *partials, int32_t splits, const float *scale,
+                                      const void *extra, int64_t extra_stride, const int32_t *extra_rows,
+                                      const float *extra_weights, int32_t top, const void *self, int64_t self_stride, float *x,
+                                      const void *w_next, const void *b_next, float out_scale, void *h, int32_t rows,
+                                      int32_t width, float eps, int32_t dtype, void *stream) {
+  tlf::GroupNormArgs a{};
+  if (int rc = tlf::partials_check(partials, scale, splits, dtype)) return rc;
+  if (rows > 0 && (!w_next || !b_next || (top > 0 && (!extra || !extra_rows || !self)))) return TLF_E_NULL;
+  if ((y && y_stride < width) || top < 0 || (top > 0 && (extra_stride < width || self_stride < width))) return TLF_E_SHAPE;
+  a.part = tlf::Partials{partials, scale, rows * y_stride, static_cast<int32_t>(y_stride), splits};
+  a.y = y; a.y_stride = y_stride; a.x = x; a.w_next = w_next; a.b_next = b_next; a.out_scale = out_scale; a.h = h;
+  a.extra = extra; a.extra_stride = extra_stride; a.extra_rows = extra_rows; a.extra_weights = extra_weights; a.top = top;
+  a.self = self; a.self_stride = self_stride; a.mult = 1.f;
+  a.width = width; a.groups = 1; a.eps = eps;
+  return tlf::groupnorm_entry<3, true>(a, rows, dtype, static_cast<hipStream_t>(stream));
 }

@@ -2,8 +2,9 @@
 // layers.
 //
 //   router     z = W_router h (tlf_gemm_f32_sums or the fp32 product)
-//   group      the `top` largest logits of each row and their sigmoids; rows (token, k) in expert order, an index each way,
-//              tiles of `tile_rows` rows of one expert
+//   group      each row's experts and their weights, either the `top` largest logits and their sigmoids, or the `top` largest
+//              of softmax + correction with their softmax values, normalised to a sum of 1; rows (token, k) in expert order, an
+//              index each way, tiles of `tile_rows` rows of one expert.  Experts from E on (identity experts) have no rows
 //   products   gemm_dlds_kernel<GROUPED> (gemm.hip) in bf16; a plain fp32 kernel here
 // No host value depends on the routing: grids are sized for the worst case and tiles past the list's end leave at once,
 // so a captured graph replays with any routing.
@@ -19,6 +20,8 @@ constexpr int kMaxExperts = 512;
 struct GroupArgs {
   const float *sums;        // [splits, n, E16] partial router logits
   int64_t plane;            // n * E16
+  const void *correction;   // [choices] or NULL: sigmoid scores
+  int32_t choices;          // E and the identity experts
   int32_t *ids;             // [entries] expert of entry (token, k)
   float *weights;           // [entries] its score
   int32_t *row_of;          // [entries] row of an entry in expert order
@@ -27,7 +30,7 @@ struct GroupArgs {
   int4 *tiles;
   int32_t *num_tiles;
   int32_t *hist;            // [blocks, E]
-  int32_t n, splits, E, E16, top, entries, tile_rows, blocks;
+  int32_t n, splits, E, E16, top, entries, tile_rows, blocks, f32;
 };
 
 __device__ __forceinline__ float wave_max(float v) {
@@ -38,21 +41,50 @@ __device__ __forceinline__ float wave_max(float v) {
   return max_lanes_16_32_48(v);
 }
 
-// One wave picks the `top` largest logits of a token: by value, then the smaller index.  logit(e): expert e's.
-template <typename F>
+// One wave picks a token's `top` experts: by value, then the smaller index.  logit(e): expert e's.
+//   NORM false: the largest logits; weights are their sigmoids
+//   NORM true: the largest of softmax + correction; weights are their softmax values over the sum of the chosen ones
+template <bool NORM, typename F>
 __device__ __forceinline__ void pick_top(const GroupArgs &a, F logit, int32_t *ids, float *weights) {
   const int lane = threadIdx.x & 63;
   constexpr int kEach = kMaxExperts / 64;
-  float v[kEach];
+  float v[kEach], s[kEach];
+  int pick[kEach];
+  const int all = a.choices;
 #pragma unroll
   for (int i = 0; i < kEach; ++i) {
     v[i] = -INFINITY;
-    if (i * 64 < a.E) {            // uniform
+    s[i] = 0.f;
+    pick[i] = -1;
+    if (i * 64 < all) {            // uniform
       const int e = i * 64 + lane;
-      const float z = logit(min(e, a.E - 1));
-      if (e < a.E) v[i] = z > -3.0e38f ? z : -3.0e38f;     // every pick finds an expert, whatever the input
+      const float z = logit(min(e, all - 1));
+      if (e < all) v[i] = z > -3.0e38f ? z : -3.0e38f;     // every pick finds an expert, whatever the input
     }
   }
+  if constexpr (NORM) {
+    float m = v[0], sum = 0.f;
+#pragma unroll
+    for (int i = 1; i < kEach; ++i) m = fmaxf(m, v[i]);
+    m = wave_max(m);
+#pragma unroll
+    for (int i = 0; i < kEach; ++i) {
+      if (i * 64 >= all) continue;  // uniform
+      s[i] = v[i] > -INFINITY ? expf(v[i] - m) : 0.f;
+      sum += s[i];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int i = 0; i < kEach; ++i) {
+      const int e = i * 64 + lane;
+      s[i] /= sum;
+      if (e < all) {
+        const float c = a.f32 ? static_cast<const float *>(a.correction)[e] : bf16_bits_to_float(static_cast<const unsigned short *>(a.correction)[e]);
+        v[i] = fmaxf(s[i] + c, -3.0e38f);
+      }
+    }
+  }
+  float chosen = 0.f;
   for (int k = 0; k < a.top; ++k) {
     float m = v[0];
 #pragma unroll
@@ -61,24 +93,32 @@ __device__ __forceinline__ void pick_top(const GroupArgs &a, F logit, int32_t *i
     bool found = false;
 #pragma unroll
     for (int i = 0; i < kEach; ++i) {
-      if (found || i * 64 >= a.E) continue;          // uniform
+      if (found || i * 64 >= all) continue;          // uniform
       const unsigned long long who = __ballot(v[i] == m);
       if (who == 0) continue;
       found = true;
+      if (NORM) chosen += __shfl(s[i], __ffsll(who) - 1, 64);
       if (lane == __ffsll(who) - 1) {
         ids[k] = i * 64 + lane;
-        weights[k] = sigmoid_f32(m);
+        if (!NORM) weights[k] = sigmoid_f32(m);
+        pick[i] = k;
         v[i] = -INFINITY;
       }
     }
   }
+  if constexpr (NORM) {
+#pragma unroll
+    for (int i = 0; i < kEach; ++i)
+      if (pick[i] >= 0) weights[pick[i]] = s[i] / (chosen + 1e-20f);
+  }
 }
 
+template <bool NORM>
 __global__ __launch_bounds__(256) void moe_pick_kernel(const GroupArgs a) {
   const int64_t tok = blockIdx.x * (blockDim.x / 64) + (threadIdx.x >> 6);
   if (tok >= a.n) return;
   const float *z = a.sums + tok * a.E16;
-  pick_top(a, [&](int e) __attribute__((always_inline)) {
+  pick_top<NORM>(a, [&](int e) __attribute__((always_inline)) {
     float v = 0.f;
 #pragma unroll 16
     for (int k = 0; k < a.splits; ++k) v += z[k * a.plane + e];
@@ -125,6 +165,10 @@ __device__ __forceinline__ void expert_tiles(const GroupArgs &a, const int *coun
 
 // The order of rows inside an expert is arbitrary (it enters no value).
 __device__ __forceinline__ void place(const GroupArgs &a, int entry, int expert, float weight, int *cursor) {
+  if (expert >= a.E) {          // an identity expert: no row
+    a.row_of[entry] = -1;
+    return;
+  }
   const int r = atomicAdd(&cursor[expert], 1);
   a.row_of[entry] = r;
   a.src[r] = entry / a.top;
@@ -150,7 +194,7 @@ __global__ __launch_bounds__(1024) void moe_small_kernel(const GroupArgs a) {
   __syncthreads();
 #pragma unroll
   for (int k = 0; k < kSmallEntries / 1024; ++k)
-    if (tid + k * 1024 < a.entries) atomicAdd(&count[id[k]], 1);
+    if (tid + k * 1024 < a.entries && id[k] < a.E) atomicAdd(&count[id[k]], 1);
   __syncthreads();
   expert_tiles(a, count, start, tstart);
   __syncthreads();
@@ -166,7 +210,7 @@ __global__ __launch_bounds__(1024) void moe_count_kernel(const GroupArgs a) {
   for (int e = threadIdx.x; e < a.E; e += 1024) count[e] = 0;
   __syncthreads();
   const int i = blockIdx.x * kBlockEntries + threadIdx.x;
-  if (i < a.entries) atomicAdd(&count[a.ids[i]], 1);
+  if (i < a.entries && a.ids[i] < a.E) atomicAdd(&count[a.ids[i]], 1);
   __syncthreads();
   for (int e = threadIdx.x; e < a.E; e += 1024) a.hist[blockIdx.x * a.E + e] = count[e];
 }
@@ -253,7 +297,8 @@ __global__ __launch_bounds__(256) void grouped_f32_kernel(const GroupedF32Args a
       const int64_t row = m0 + m;
       if (a.act == 0) a.y[row * a.N + c] = acc[i][r];
       else if (n < 8)
-        a.y[row * (a.N / 2) + (c >> 4) * 8 + n] = clipped_glu(acc[i][r], up, a.g.row_scale ? a.g.row_scale[row] : 1.0f, a.g.limit);
+        a.y[row * (a.N / 2) + (c >> 4) * 8 + n] = a.act == 2 ? silu_f32(acc[i][r]) * up
+                                                       : clipped_glu(acc[i][r], up, a.g.row_scale ? a.g.row_scale[row] : 1.0f, a.g.limit);
     }
 }
 
@@ -303,9 +348,11 @@ extern "C" size_t tlf_moe_group_workspace_bytes(int32_t n, int32_t top, int32_t 
 
 extern "C" int tlf_moe_group(const float *sums, int32_t splits, int32_t *ids, float *weights, int32_t *row_of, int32_t *src,
                              float *row_weight, int32_t *tiles, int32_t *num_tiles, int32_t max_tiles, int32_t n, int32_t top,
-                             int32_t experts, int32_t tile_rows, void *workspace, size_t workspace_bytes, void *stream) {
+                             int32_t experts, int32_t identity, const void *correction, int32_t dtype, int32_t tile_rows,
+                             void *workspace, size_t workspace_bytes, void *stream) {
   using namespace tlf;
-  if (n < 0 || top <= 0 || experts <= 0 || experts > kMaxExperts || top > experts || tile_rows <= 0 || splits <= 0 || splits > 64) return TLF_E_SHAPE;
+  if (n < 0 || top <= 0 || experts <= 0 || identity < 0 || experts > kMaxExperts - identity || top > experts + identity || tile_rows <= 0 || splits <= 0 || splits > 64) return TLF_E_SHAPE;
+  if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
   const int64_t entries = static_cast<int64_t>(n) * top;
   if (entries > (1 << 28) || max_tiles < entries / tile_rows + (entries < experts ? entries : experts)) return TLF_E_SHAPE;
   if (n == 0) return TLF_OK;
@@ -314,14 +361,16 @@ extern "C" int tlf_moe_group(const float *sums, int32_t splits, int32_t *ids, fl
   GroupArgs a{};
   a.sums = sums; a.ids = ids; a.weights = weights; a.row_of = row_of; a.src = src; a.row_weight = row_weight;
   a.tiles = reinterpret_cast<int4 *>(tiles); a.num_tiles = num_tiles; a.hist = static_cast<int32_t *>(workspace);
-  a.n = n; a.splits = splits; a.E = experts; a.E16 = (experts + 15) / 16 * 16; a.top = top;
+  a.n = n; a.splits = splits; a.E = experts; a.E16 = (experts + identity + 15) / 16 * 16; a.top = top;
+  a.correction = correction; a.choices = experts + identity; a.f32 = dtype == TLF_DT_F32;
   a.plane = static_cast<int64_t>(n) * a.E16;
   a.entries = static_cast<int32_t>(entries); a.tile_rows = tile_rows;
   a.blocks = static_cast<int32_t>((entries + kBlockEntries - 1) / kBlockEntries);
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (entries > kSmallEntries && (!workspace || workspace_bytes < tlf_moe_group_workspace_bytes(n, top, experts))) return TLF_E_WORKSPACE;
   const int waves = n <= 1024 ? 1 : 4;
-  TLF_LAUNCH(moe_pick_kernel, dim3((n + waves - 1) / waves), dim3(64 * waves), 0, s, a);
+  if (correction) TLF_LAUNCH((moe_pick_kernel<true>), dim3((n + waves - 1) / waves), dim3(64 * waves), 0, s, a);
+  else TLF_LAUNCH((moe_pick_kernel<false>), dim3((n + waves - 1) / waves), dim3(64 * waves), 0, s, a);
   if (entries <= kSmallEntries) {
     TLF_LAUNCH(moe_small_kernel, dim3(1), dim3(1024), 0, s, a);
     return launch_status();
@@ -334,19 +383,20 @@ extern "C" int tlf_moe_group(const float *sums, int32_t splits, int32_t *ids, fl
 
 extern "C" int tlf_moe_gemm(const void *x, int64_t x_stride, int32_t x_count, const void *w, void *y, const int32_t *tiles,
                             const int32_t *num_tiles, int32_t max_tiles, int32_t tile_rows, const int32_t *x_rows,
-                            const float *row_scale, int32_t rows, int32_t N, int32_t K, int32_t clipped_glu, float limit,
+                            const float *row_scale, int32_t rows, int32_t N, int32_t K, int32_t act, float limit,
                             int32_t dtype, void *stream) {
   using namespace tlf;
+  if (act < 0 || act > 2) return TLF_E_UNSUPPORTED;
   if (rows < 0 || N <= 0 || K <= 0 || N % 16 || max_tiles <= 0 || max_tiles > 65535 || x_stride < K || x_count < 0) return TLF_E_SHAPE;
   if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
   if (rows == 0) return TLF_OK;
   if (!x || !w || !y || !tiles || !num_tiles) return TLF_E_NULL;
   const GroupedRows g{reinterpret_cast<const int4 *>(tiles), num_tiles, x_rows, row_scale,
-                      static_cast<int64_t>(N) * K * (dtype == TLF_DT_BF16 ? 2 : 4), limit};
+                      static_cast<int64_t>(N) * K * (dtype == TLF_DT_BF16 ? 2 : 4), limit, act == 2};
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (dtype == TLF_DT_F32) {
     if (tile_rows != kGT) return TLF_E_SHAPE;
-    const GroupedF32Args a{static_cast<const float *>(x), static_cast<const float *>(w), static_cast<float *>(y), x_stride, g, N, K, clipped_glu};
+    const GroupedF32Args a{static_cast<const float *>(x), static_cast<const float *>(w), static_cast<float *>(y), x_stride, g, N, K, act};
     TLF_LAUNCH(grouped_f32_kernel, dim3((N + kGT - 1) / kGT, max_tiles), dim3(256), 0, s, a);
     return launch_status();
   }
@@ -360,7 +410,7 @@ extern "C" int tlf_moe_gemm(const void *x, int64_t x_stride, int32_t x_count, co
   p.y = static_cast<unsigned short *>(y);
   p.M = rows; p.N = N; p.K = K;
   p.m_tiles = max_tiles;
-  p.act = clipped_glu ? 3 : 0;
+  p.act = act ? 3 : 0;
   p.g = g;
   return launch_grouped(p, tile_rows, s);
 }

@@ -9,13 +9,6 @@ from .. import ops
 from ..utils.context import get_context
 
 
-def interleaved_cos_sin(dims: int, max_position: int, base: float) -> torch.Tensor:
-    """fp32 ``[max_position, dims]`` = cos || sin of ``p * base^(-2 i / dims)``; angles in double precision, CPU."""
-    f = torch.tensor(base, dtype=torch.float64, device="cpu") ** (-torch.arange(0, dims, 2, dtype=torch.float64, device="cpu") / max(dims, 1))
-    a = torch.arange(max_position, dtype=torch.float64, device="cpu")[:, None] * f
-    return torch.cat((a.cos(), a.sin()), dim=-1).float()
-
-
 class PooledWindowAttention(nn.Module):
     def __init__(self, num_heads: int, num_kv_heads: int, head_dim: int, scale: float, window: int, pool: int,
                  rot_dims: int, rope: torch.Tensor, eps: float, dtype: torch.dtype):

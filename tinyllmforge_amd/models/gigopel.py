@@ -65,10 +65,7 @@ class GigopelLayer(nn.Module):
         if self.act is not None:
             out |= {"mlp.up": ("inp.weight", "up"), "mlp.down": ("out.weight", "down"), "mlp.act": ("act.pq", None)}
         if self.experts is not None:
-            out["mlp.router"] = ("experts.router", "router")
-            for e in range(self.experts.experts):
-                for kind, target in (("gate", "gate_up"), ("up", "gate_up"), ("down", "down")):
-                    out[f"mlp.e{e}.{kind}"] = ("experts." + target, (e, kind))
+            out |= {"mlp." + n: ("experts." + target, part) for n, (target, part) in self.experts.routes().items()}
         return out
 
 

@@ -2,14 +2,16 @@
 
 A layer is a module with ``norm1`` (the norm in front of it), ``forward(positions, h, x, following)`` that updates the fp32
 residual ``x`` in place and returns it normed by ``following``, and ``routes()``: checkpoint names below ``l<i>.`` ->
-(parameter below the layer, part of it or None)."""
+(parameter below the layer, part of it or None).  A layer that runs more than once takes ``run=`` (0, 1, ...) and keeps a cache
+and a state of its own per run."""
 import re
+from functools import partial
 
 import torch
 from torch import nn
 
 from ..layers.linear import GatedUpLinear, JoinedLinear, StackedLinear
-from ..layers.pooled_attention import interleaved_cos_sin
+from ..layers.rotary_embedding import rotation_table
 
 
 def prefixed(prefix: str, routes: dict) -> dict:
@@ -26,17 +28,30 @@ class LayeredForCausalLM(nn.Module):
         self.loaded_tensors: set[str] = set()
         self._rope_tables = {}
 
-    def rope_table(self, rot: dict):
+    def rope_table(self, rot: dict | None):
         """Layers with the same rotation share a table."""
-        key = (rot["dims"], rot["base"])
+        if not rot or not rot["dims"]:
+            return None
+        scaling = rot.get("scaling") or {}
+        key = (rot["dims"], rot["base"], *sorted(scaling.items()))
         if key not in self._rope_tables:
-            self._rope_tables[key] = interleaved_cos_sin(key[0], self.config.max_position_embeddings, key[1]).to(self.embed.device)
+            table = rotation_table(rot["dims"], self.config.max_position_embeddings, rot["base"], **scaling)
+            self._rope_tables[key] = table.to(self.embed.device)
         return self._rope_tables[key]
 
+    def runs(self):
+        """The layers in the order they run, ``(norm in front, call)``."""
+        order, seen = self.config.layer_runs(), {}
+        for i in order:
+            run = seen[i] = seen.get(i, -1) + 1
+            layer = self.layers[i]
+            yield layer.norm1, partial(layer, run=run) if order.count(i) > 1 else layer
+
     def forward(self, input_ids: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
-        norms = [layer.norm1 for layer in self.layers] + [self.norm]
+        runs = list(self.runs())
+        norms = [norm for norm, _ in runs] + [self.norm]
         x, h = norms[0].after_embedding(input_ids, self.embed.data)
-        for layer, following in zip(self.layers, norms[1:]):
+        for (_, layer), following in zip(runs, norms[1:]):
             h = layer(positions, h, x, following)
         return h
 

@@ -755,6 +755,46 @@ def residual_rms_norm(y, x, mult, w_next, w_offset, eps, extra=None, extra_rows=
     return h
 
 
+def embed_layer_norm(ids, table, w_next, b_next, eps, out_scale=1.0):
+    """``x = table[ids]`` in fp32 and ``layer_norm(x) * out_scale`` in the table's dtype."""
+    lib = _lib.load()
+    _need(ids, torch.int64, "ids"); _need(table, w_next.dtype, "table"); _need(b_next, w_next.dtype, "b_next")
+    assert ids.is_contiguous() and table.is_contiguous()
+    rows, (vocab, width) = ids.numel(), table.shape
+    assert w_next.numel() == width and b_next.numel() == width
+    x = torch.empty(rows, width, dtype=torch.float32, device=table.device)
+    h = torch.empty(rows, width, dtype=table.dtype, device=table.device)
+    check(lib.tlf_embed_layernorm(ids.data_ptr(), table.data_ptr(), vocab, x.data_ptr(), w_next.data_ptr(), b_next.data_ptr(),
+                                  float(out_scale), h.data_ptr(), rows, width, float(eps), _dt(table), _stream()),
+          "tlf_embed_layernorm")
+    return x, h
+
+
+def residual_layer_norm(y, x, w_next, b_next, eps, out_scale=1.0, extra=None, extra_rows=None, extra_weights=None, own=None):
+    """In place ``x += y + sum of extra_weights * extra[extra_rows]`` (``x`` fp32 ``[N, W]``, ``y`` may be None, ``extra_rows``
+    int32 ``[N, top]``, a negative one stands for the row of ``own``), then ``layer_norm(x) * out_scale`` in w_next's dtype."""
+    lib = _lib.load()
+    _need(x, torch.float32, "x"); _need(w_next, None, "w_next"); _need(b_next, w_next.dtype, "b_next")
+    rows, width = x.shape
+    assert x.is_contiguous() and w_next.numel() == width and b_next.numel() == width
+    assert y is None or (y.shape[0] == rows and y.shape[1] >= width and y.dtype == w_next.dtype)
+    top, stride, own_stride = 0, 0, 0
+    if extra is not None:
+        _need(extra, w_next.dtype, "extra"); _need(extra_rows, torch.int32, "extra_rows"); _need(own, w_next.dtype, "own")
+        assert extra.stride(1) == 1 and extra_rows.is_contiguous() and extra_rows.shape[0] == rows
+        assert own.shape[0] == rows and own.shape[1] >= width and own.stride(1) == 1
+        if extra_weights is not None:
+            _need(extra_weights, torch.float32, "extra_weights")
+            assert extra_weights.is_contiguous() and extra_weights.shape == extra_rows.shape
+        top, stride, own_stride = extra_rows.shape[1], extra.stride(0), own.stride(0)
+    h = torch.empty(rows, width, dtype=w_next.dtype, device=x.device)
+    check(lib.tlf_residual_layernorm(*(_source(y) if y is not None else (None, 0, None, 1, None)), _opt(extra), stride,
+                                     _opt(extra_rows), _opt(extra_weights), top, _opt(own), own_stride, x.data_ptr(),
+                                     w_next.data_ptr(), b_next.data_ptr(), float(out_scale), h.data_ptr(), rows, width,
+                                     float(eps), _dt(w_next), _stream()), "tlf_residual_layernorm")
+    return h
+
+
 class LatentShape:
     """Sizes of a latent-attention layer and of the padded rows its kernels read (``include/tlf_hip.h``)."""
     __slots__ = ("heads", "dim", "rot", "rank", "vdim", "da", "ta", "ra", "va", "dq", "lp", "rp")
@@ -920,6 +960,129 @@ def latent_prefill(q, expanded, latents, cu_seqlens_q, seq_starts, kv_offsets, f
     return out
 
 
+# ------------------------------------------------------------------ grouped-query attention with a sink
+class SinkKV:
+    """The paged, head-major caches of one layer: ``k [pages, G, block, Dp]``, ``v [pages, G, block, Vp]``."""
+    __slots__ = ("k", "v", "dim", "vdim")
+
+    def __init__(self, pages, block_size, kv_heads, dim, vdim, dtype, device):
+        self.k = torch.zeros(pages, kv_heads, block_size, self.padded(dim), dtype=dtype, device=device)
+        self.v = torch.zeros(pages, kv_heads, block_size, self.padded(vdim), dtype=dtype, device=device)
+        self.dim, self.vdim = dim, vdim
+
+    @staticmethod
+    def padded(dim):
+        return -(-dim // 32) * 32
+
+    @staticmethod
+    def page_bytes(block_size, kv_heads, dim, vdim, itemsize):
+        return block_size * kv_heads * (SinkKV.padded(dim) + SinkKV.padded(vdim)) * itemsize
+
+
+def sink_prep(proj, kv: SinkKV, heads, positions, slot_mapping, eps, bias=None, conv=None, ring=None, state_slots=None,
+              row_seq=None, cu_seqlens_q=None, q_norm=None, k_norm=None, cos_sin=None, rot_dims=0, q_mult=None):
+    """Projection rows ``[q | k | v | gate]`` -> ``(q [N, H, Dp], gate rows [N, >= H * vdim])``; keys and values go to the
+    caches.  See ``tlf_sink_prep``; ``proj`` may be ``Deferred`` when every row is a sequence of its own."""
+    lib = _lib.load()
+    dt = kv.k.dtype
+    assert proj.dtype == dt
+    _need(positions, torch.int64, "positions"); _need(slot_mapping, torch.int32, "slot_mapping")
+    n = proj.shape[0]
+    pages, G, bs, dp = kv.k.shape
+    channels = (heads + G) * kv.dim + G * kv.vdim
+    assert positions.numel() == n and slot_mapping.numel() == n and proj.shape[1] >= channels + heads * kv.vdim
+    for t, count in ((bias, channels), (q_norm, kv.dim), (k_norm, kv.dim)):
+        assert t is None or (t.dtype == dt and t.numel() == count and t.is_contiguous())
+    taps = 0
+    if conv is not None:
+        taps = conv.shape[0]
+        assert conv.dtype == ring.dtype == dt and conv.is_contiguous() and ring.is_contiguous()
+        assert conv.shape == (taps, channels) and ring.shape[1:] == (taps, channels)
+        _need(state_slots, torch.int32, "state_slots")
+        assert row_seq is not None or state_slots.numel() >= n
+    if row_seq is not None:
+        _need(row_seq, torch.int32, "row_seq"); _need(cu_seqlens_q, torch.int32, "cu_seqlens_q")
+        assert row_seq.numel() == n
+    tables = [t for t in (cos_sin, q_mult) if t is not None]
+    for t in tables:
+        _need(t, torch.float32, "table")
+        assert t.is_contiguous() and t.shape[0] == tables[0].shape[0]
+    assert rot_dims == 0 or cos_sin.shape[1] == rot_dims
+    q = torch.empty(n, heads, dp, dtype=dt, device=kv.k.device)
+    gate = out = None
+    if isinstance(proj, Deferred):
+        gate = out = torch.empty(n, heads * kv.vdim, dtype=dt, device=kv.k.device)
+    else:
+        gate = proj[:, channels:]
+    check(lib.tlf_sink_prep(*_source(proj), _opt(bias), _opt(conv), taps, _opt(ring), _opt(state_slots),
+                            ring.shape[0] if ring is not None else 0, _opt(row_seq), _opt(cu_seqlens_q), _opt(q_norm),
+                            _opt(k_norm), positions.data_ptr(), _opt(cos_sin), _opt(q_mult),
+                            tables[0].shape[0] if tables else 1 << 30, rot_dims, slot_mapping.data_ptr(), q.data_ptr(),
+                            kv.k.data_ptr(), kv.v.data_ptr(), _opt(out), n, heads, G, kv.dim, kv.vdim, bs, pages, float(eps),
+                            _dt(kv.k), _stream()), "tlf_sink_prep")
+    return q, gate
+
+
+def conv_tail(proj, ring, state_slots, cu_seqlens_q, seq_starts, first_seq, num_seqs):
+    """The last projected rows of the portions of sequences ``first_seq ..`` into ``ring [slots, taps, channels]``."""
+    _need(proj, ring.dtype, "proj"); _need(state_slots, torch.int32, "state_slots")
+    slots, taps, channels = ring.shape
+    assert proj.stride(1) == 1 and proj.shape[1] >= channels and ring.is_contiguous()
+    assert state_slots.numel() >= first_seq + num_seqs and cu_seqlens_q.numel() > first_seq + num_seqs
+    check(_lib.load().tlf_conv_tail(proj.data_ptr(), proj.stride(0), ring.data_ptr(), state_slots.data_ptr(), slots,
+                                    cu_seqlens_q.data_ptr(), seq_starts.data_ptr(), first_seq, num_seqs, taps, channels,
+                                    _dt(ring), _stream()), "tlf_conv_tail")
+
+
+def sink_attention_rows(q, kv: SinkKV, block_tables, positions, slot_mapping, sink, gate, scale, cap, max_len, out, row_seq=None):
+    """Row by row: ``q [N, H, Dp]`` -> ``out [N, H * vdim]``; ``row_seq`` None: row r is sequence r."""
+    lib = _lib.load()
+    _need(q, kv.k.dtype, "q"); _need(block_tables, torch.int32, "block_tables"); _need(positions, torch.int64, "positions")
+    n, heads, dp = q.shape
+    pages, G, bs, _ = kv.k.shape
+    assert q.is_contiguous() and dp == kv.k.shape[3] and out.stride(1) == 1 and out.shape[0] == n and out.dtype == q.dtype
+    assert gate is None or (gate.dtype == q.dtype and gate.shape[0] == n and gate.stride(1) == 1)
+    assert sink is None or (sink.dtype == q.dtype and sink.numel() == heads)
+    assert positions.numel() == n and slot_mapping.numel() == n and block_tables.stride(1) == 1
+    assert row_seq.numel() == n if row_seq is not None else block_tables.shape[0] >= n
+    max_len = min(max_len, block_tables.shape[1] * bs)
+    step = 32768                                     # rows per launch (grid limit)
+    for lo in range(0, n, step):
+        m = min(step, n - lo)
+        assert row_seq is not None or lo == 0
+        nbytes = lib.tlf_sink_attn_rows_workspace_bytes(m, heads, G, kv.dim, kv.vdim, max_len, _dt(q))
+        ws = _workspace(nbytes, q.device, "sink_rows")
+        check(lib.tlf_sink_attn_rows(
+            q[lo:].data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), block_tables.data_ptr(), block_tables.stride(0),
+            positions[lo:].data_ptr(), slot_mapping[lo:].data_ptr(), row_seq[lo:].data_ptr() if row_seq is not None else None,
+            _opt(sink), gate[lo:].data_ptr() if gate is not None else None, gate.stride(0) if gate is not None else 0,
+            out[lo:].data_ptr(), out.stride(0), m, heads, G, kv.dim, kv.vdim, bs, max_len, pages, float(scale), float(cap or 0),
+            _dt(q), ws.data_ptr(), ws.numel(), _stream()), "tlf_sink_attn_rows")
+    return out
+
+
+def sink_prefill_supported(dim, vdim) -> bool:
+    return bool(_lib.load().tlf_sink_attn_prefill_supported(dim, vdim))
+
+
+def sink_attention_prefill(q, kv: SinkKV, block_tables, cu_seqlens_q, seq_starts, first_seq, num_seqs, max_tokens, sink, gate,
+                           scale, cap, out):
+    """Portions of sequences ``first_seq ..`` on the matrix cores (bf16); rows indexed as in the step."""
+    _need(q, BF16, "q"); _need(block_tables, torch.int32, "block_tables")
+    n, heads, dp = q.shape
+    pages, G, bs, _ = kv.k.shape
+    assert q.is_contiguous() and dp == kv.k.shape[3] and kv.k.dtype == BF16 and out.stride(1) == 1 and out.shape[0] == n
+    assert gate is None or (gate.dtype == BF16 and gate.shape[0] == n and gate.stride(1) == 1)
+    assert sink is None or (sink.dtype == BF16 and sink.numel() == heads)
+    assert block_tables.stride(1) == 1 and block_tables.shape[0] >= first_seq + num_seqs
+    check(_lib.load().tlf_sink_attn_prefill(
+        q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), cu_seqlens_q.data_ptr(),
+        seq_starts.data_ptr(), first_seq, num_seqs, max_tokens, _opt(sink), _opt(gate), gate.stride(0) if gate is not None else 0,
+        out.data_ptr(), out.stride(0), heads, G, kv.dim, kv.vdim, bs, pages, float(scale), float(cap or 0), _stream()),
+        "tlf_sink_attn_prefill")
+    return out
+
+
 # ------------------------------------------------------------------ mixture of experts
 def moe_logits(h, router):
     """Router logits of every row as fp32 partial sums ``[splits, N, experts rounded up to 16]``."""
@@ -944,11 +1107,14 @@ class ExpertRows:
     __slots__ = ("ids", "scores", "row_of", "src", "weight", "tiles", "num_tiles", "tile_rows")
 
 
-def moe_group(logits, experts, top, tile_rows) -> ExpertRows:
-    """``logits``: partial sums as from ``moe_logits``."""
+def moe_group(logits, experts, top, tile_rows, correction=None, identity=0) -> ExpertRows:
+    """``logits``: partial sums as from ``moe_logits``.  Without ``correction`` sigmoid scores of the largest logits; with it
+    the largest of softmax + correction, weighted by their normalised softmax values.  The last ``identity`` of the router's
+    outputs have no rows (``row_of`` -1)."""
     lib = _lib.load()
     _need(logits, torch.float32, "logits")
-    assert logits.is_contiguous() and logits.shape[2] == -(-experts // 16) * 16
+    assert logits.is_contiguous() and logits.shape[2] == -(-(experts + identity) // 16) * 16
+    assert correction is None or (correction.is_cuda and correction.numel() == experts + identity)
     splits, n = logits.shape[:2]
     r, dev = ExpertRows(), logits.device
     i32 = lambda *s: torch.empty(*s, dtype=torch.int32, device=dev)
@@ -958,24 +1124,28 @@ def moe_group(logits, experts, top, tile_rows) -> ExpertRows:
     ws = _workspace(lib.tlf_moe_group_workspace_bytes(n, top, experts), dev, "moe")
     check(lib.tlf_moe_group(logits.data_ptr(), splits, r.ids.data_ptr(), r.scores.data_ptr(), r.row_of.data_ptr(),
                             r.src.data_ptr(), r.weight.data_ptr(), r.tiles.data_ptr(), r.num_tiles.data_ptr(),
-                            r.tiles.shape[0], n, top, experts, tile_rows, ws.data_ptr(), ws.numel(), _stream()),
+                            r.tiles.shape[0], n, top, experts, identity, _opt(correction),
+                            _dt(correction) if correction is not None else DT_BF16, tile_rows, ws.data_ptr(), ws.numel(),
+                            _stream()),
           "tlf_moe_group")
     return r
 
 
-def moe_gemm(x, w, rows: ExpertRows, gather: bool, clipped_glu: bool = False, limit: float = 0.0):
+def moe_gemm(x, w, rows: ExpertRows, gather: bool, clipped_glu: bool = False, limit: float = 0.0, swiglu: bool = False):
     """One product per expert, ``w [E, Nout, K]``.  ``gather``: x rows are tokens (otherwise rows in expert order);
-    ``clipped_glu``: interleaved gate / up channels, activated, the row's weight on both products."""
+    ``clipped_glu``: interleaved gate / up channels, activated, the row's weight on both products; ``swiglu``: interleaved
+    channels, ``silu(gate) * up``."""
     lib = _lib.load()
     _need(x, w.dtype, "x")
     assert x.stride(1) == 1 and w.is_contiguous() and w.shape[2] == x.shape[1]
     n, N = rows.src.numel(), w.shape[1]
     assert gather or x.shape[0] == n
-    y = torch.empty(n, N // 2 if clipped_glu else N, dtype=x.dtype, device=x.device)
+    assert not (clipped_glu and swiglu)
+    y = torch.empty(n, N // 2 if clipped_glu or swiglu else N, dtype=x.dtype, device=x.device)
     check(lib.tlf_moe_gemm(x.data_ptr(), x.stride(0), x.shape[0], w.data_ptr(), y.data_ptr(), rows.tiles.data_ptr(),
                            rows.num_tiles.data_ptr(), rows.tiles.shape[0], rows.tile_rows,
                            rows.src.data_ptr() if gather else None, rows.weight.data_ptr() if clipped_glu else None, n, N,
-                           w.shape[2], int(clipped_glu), float(limit), _dt(x), _stream()), "tlf_moe_gemm")
+                           w.shape[2], 1 if clipped_glu else 2 if swiglu else 0, float(limit), _dt(x), _stream()), "tlf_moe_gemm")
     return y
 
 
