@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the per-token hot path on one MI355X.
 
-    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload e2e|decode_attn|gemm|gitopel|gigopel|...|all]
+    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload e2e|decode_attn|gemm|gitopel|gigopel|zuzunex|...|all]
 
 Prints ONE JSON line.
 
@@ -53,7 +53,7 @@ def parse():
                     help="engine steps that steps/ms_per_step describe (0 = all); value is always the whole job")
     ap.add_argument("--warmup", type=int, default=1, help="warm-up generate() calls before the timed run")
     ap.add_argument("--workload", default="e2e",
-                    choices=["e2e", "decode_attn", "gemm", "prefill_attn", "elementwise", "clock", "c5", "gitopel", "gigopel", "all"])
+                    choices=["e2e", "decode_attn", "gemm", "prefill_attn", "elementwise", "clock", "c5", "gitopel", "gigopel", "zuzunex", "all"])
     ap.add_argument("--attn-steps", type=int, default=200, help="timed launches of the decode-attention microbench")
     ap.add_argument("--num-seqs", type=int, default=256)
     ap.add_argument("--no-cpu-baseline", action="store_true")
@@ -970,6 +970,155 @@ def bench_gigopel_kernels(sizes=None):
     return rows
 
 
+# ----------------------------------------------------------------------------- Zuzunex beside Qwen3 at equal size
+# experts, identity experts, top, expert ff (also the shared expert's); the rest as GITOPEL_SIZES
+ZUZUNEX_EXPERTS = {"1024-wide": (32, 2, 4, 768), "4096-wide": (64, 4, 8, 1536)}
+
+
+def zuzunex_shape(size, layers=8, vocab=32768, moe=True):
+    """Alternating attention and attention_2; the first layer dense, the others mixtures of experts (``moe=False``: all dense)."""
+    w, hq, hkv, d, ff, *_ = GITOPEL_SIZES[size]
+    ne, ident, top, eff = ZUZUNEX_EXPERTS[size]
+    heads = dict(heads=hq, kv_heads=hkv, dim=d, vdim=d, scale=d ** -0.5)
+    mixers = [("attention", dict(heads, softcap=30.0, q_temp=dict(coef=0.1, every=1024))),
+              ("attention_2", dict(heads, conv=3, rot=dict(base=1e6, dims=d, scaling=dict(factor=4.0, original=1024, fast=32.0, slow=1.0))))]
+    dense = dict(kind="dense", ff=ff)
+    sparse = dict(kind="moe", expert=dict(ff=eff), router=dict(experts=ne, identity=ident, top=top), shared=dict(ff=eff))
+    return dict(architecture="Zuzunex", vocab=vocab, width=w, norm=dict(eps=1e-6), logit_scale=0.5, loop=None,
+                layers=[dict(type=mixers[i % 2][0], mixer=mixers[i % 2][1], mlp=sparse if moe and i else dense) for i in range(layers)])
+
+
+def bench_zuzunex_kernels(sizes=None):
+    """Kernels of the Zuzunex layers beside the like kernel of Qwen3 at the same sizes: algorithmic bytes or flops over the
+    graph-timed launch, as a fraction of the HBM or matrix peak."""
+    import torch
+    from tinyllmforge_amd import ops as P
+    from tinyllmforge_amd.layers.moe import SwiGLUExperts
+    from tinyllmforge_amd.layers.rotary_embedding import rotation_table
+    from tinyllmforge_amd.layers.sink_attention import query_temperatures
+    torch.manual_seed(0)
+    BF, dev = torch.bfloat16, "cuda"
+    rows = []
+
+    def add(name, size, fn, amount, bound, copies=1, launches=10):
+        def cycle():
+            for i in range(copies):
+                fn(i)
+        sec = time_graph(cycle, launches=max(1, launches // copies), replays=10) * 1e-3 / copies
+        peak = {"hbm": HBM_PEAK_GBPS * 1e9, "mfma bf16": MFMA_BF16_PEAK_TFLOPS * 1e12}[bound]
+        rows.append(dict(kernel=name, size=size, us=round(sec * 1e6, 2), bound=bound,
+                         rate=round(amount / sec / (1e9 if bound == "hbm" else 1e12), 1), frac=round(amount / sec / peak, 4)))
+        print(rows[-1], file=sys.stderr, flush=True)
+        torch.cuda.empty_cache()
+
+    bf = lambda *s: torch.randn(*s, device=dev).to(BF)
+    for size in sizes or ZUZUNEX_EXPERTS:
+        w, h, g, d, ff, *_ = GITOPEL_SIZES[size]
+        ne, ident, top, eff = ZUZUNEX_EXPERTS[size]
+        sink, scale = bf(h), d ** -0.5
+        # -- decode: 64 sequences, contexts U[512, 4096], pages of 256
+        B, bs = 64, 256
+        case = make_decode_case(batch=B, hq=h, hkv=g, dh=d)
+        plan = P.paged_decode_plan(case["ctx"], case["bt"], bs)
+        add("paged decode attention (Qwen3)", size,
+            lambda i: P.paged_decode_attention(case["q"], case["k_cache"], case["v_cache"], case["ctx"], case["bt"], scale, plan=plan),
+            case["algo_bytes"], "hbm")
+        del case["k_cache"], case["v_cache"]
+        kv = P.SinkKV(2048, bs, g, d, d, BF, dev)
+        kv.k.normal_()
+        kv.v.normal_()
+        pos, slots = case["ctx"].long() - 1, torch.zeros(B, dtype=torch.int32, device=dev)
+        q, gate, out = bf(B, h, d), bf(B, h * d), torch.empty(B, h * d, device=dev, dtype=BF)
+        for name, cap in (("attention_2", None), ("attention, capped", 30.0)):
+            add(f"{name}: decode attention, gated", size,
+                lambda i: P.sink_attention_rows(q, kv, case["bt"], pos, slots, sink, gate, scale, cap, 4096, out),
+                case["algo_bytes"] + B * h * d * 2, "hbm")
+        del kv, case
+        # -- prompts: 8 x 2048 tokens
+        S, L = 8, 2048
+        N = S * L
+        qq, kk, vv = bf(N, h, d), bf(N, g, d), bf(N, g, d)
+        cu = torch.arange(0, N + 1, L, dtype=torch.int32, device=dev)
+        flops = 4.0 * h * d * S * L * L / 2
+        add("prompt attention (Qwen3)", size, lambda i: P.varlen_prefill_attention(qq, kk, vv, cu, cu, L, scale), flops, "mfma bf16")
+        del kk, vv
+        kv = P.SinkKV(N // bs, bs, g, d, d, BF, dev)
+        kv.k.normal_()
+        kv.v.normal_()
+        bt = torch.arange(N // bs, dtype=torch.int32, device=dev).view(S, -1)
+        starts = torch.zeros(S, dtype=torch.int32, device=dev)
+        gate, out = bf(N, h * d), torch.empty(N, h * d, device=dev, dtype=BF)
+        for name, cap in (("attention_2", None), ("attention, capped", 30.0)):
+            add(f"{name}: prompt attention, gated", size,
+                lambda i: P.sink_attention_prefill(qq, kv, bt, cu, starts, 0, S, L, sink, gate, scale, cap, out), flops, "mfma bf16")
+        del qq, gate, out, kv
+        # -- between the products
+        chan = (h + 2 * g) * d
+        tab, temps = rotation_table(d, 4096, 1e6), query_temperatures(0.1, 1024, 4096).to(dev)
+        tab = tab.to(dev)
+        slots = torch.arange(N, dtype=torch.int32, device=dev)
+        pos = torch.arange(L, device=dev).repeat(S)
+        nw, bias, conv, ring = torch.ones(d, device=dev, dtype=BF), bf(chan), bf(3, chan), torch.zeros(B, 3, chan, device=dev, dtype=BF)
+        for n, copies in ((N, 3), (B, 1)):
+            qkv = bf(copies, n, chan)
+            kc, vc = bf(2, N // bs, bs, g, d)
+            add(f"q/k norm + RoPE + store (Qwen3), {n} tokens", size,
+                lambda i: P.qknorm_rope_store(qkv[i], nw, nw, 1e-6, pos[:n], tab, h, g, d, kc, vc, slots[:n]),
+                n * (chan * 4 + d * 4), "hbm", copies)
+            del qkv, kc, vc
+            kv = P.SinkKV(N // bs, bs, g, d, d, BF, dev)
+            proj = bf(copies, n, chan + h * d)
+            seqs = dict(row_seq=torch.arange(N, device=dev, dtype=torch.int32) // L, cu_seqlens_q=cu) if n == N else {}
+            states = torch.arange(S if n == N else B, device=dev, dtype=torch.int32)
+            add(f"attention: preparation, {n} tokens", size,
+                lambda i: P.sink_prep(proj[i], kv, h, pos[:n], slots[:n], 1e-6, q_mult=temps), n * chan * 4, "hbm", copies)
+            add(f"attention_2: preparation with convolution, {n} tokens", size,
+                lambda i: P.sink_prep(proj[i], kv, h, pos[:n], slots[:n], 1e-6, bias, conv, ring, states, seqs.get("row_seq"),
+                                      seqs.get("cu_seqlens_q"), nw, nw, tab, d), n * (chan * (4 if n == N else 10) + d * 4), "hbm", copies)
+            if n == N:
+                add(f"convolution state, {S} portions", size, lambda i: P.conv_tail(proj[i], ring, states, cu, starts, 0, S), S * 2 * chan * 4, "hbm", copies)
+            del proj, kv
+            y, x, e, rr = bf(copies, n, w), torch.randn(copies, n, w, device=dev), bf(copies, n * top, w), bf(copies, n, w)
+            ww, wb = torch.ones(w, device=dev, dtype=BF), torch.zeros(w, device=dev, dtype=BF)
+            idx = torch.randperm(n * top, device=dev).to(torch.int32).view(n, top)
+            f = torch.rand(n, top, device=dev)
+            add(f"add + RMSNorm (Qwen3), {n} tokens", size, lambda i: P.add_rms_norm(y[i], rr[i], ww, 1e-6), n * w * 8, "hbm", copies)
+            add(f"add + layer norm, {n} tokens", size, lambda i: P.residual_layer_norm(y[i], x[i], ww, wb, 1e-6), n * w * 12, "hbm", copies)
+            add(f"add + {top} weighted expert rows + layer norm, {n} tokens", size,
+                lambda i: P.residual_layer_norm(y[i], x[i], ww, wb, 1e-6, 1.0, e[i], idx, f, rr[i]), n * w * (12 + 2 * top), "hbm", copies)
+            del y, x, e, rr
+        # -- experts
+        torch.set_default_dtype(BF)
+        with torch.device(dev):
+            moe = SwiGLUExperts(w, ne, top, eff, ident)
+        torch.set_default_dtype(torch.float32)
+        for p_ in moe.parameters():
+            p_.data.normal_(0, 0.02)
+        gu, dn = bf(2 * ff, w), bf(w, ff)
+        for n in (B, 512, N):
+            x = bf(n, w)
+            sums = P.moe_logits(x, moe.router.data)
+            tile = moe.tile_rows(n)
+            add(f"router, {n} tokens", size, lambda i: P.moe_logits(x, moe.router.data), (ne + ident) * w * 2 + n * w * 2, "hbm")
+            add(f"choice + rows by expert, {n} tokens", size, lambda i: P.moe_group(sums, ne, top, tile, moe.correction.data, ident),
+                n * ((ne + ident) * 4 + top * 20), "hbm")
+            r = P.moe_group(sums, ne, top, tile, moe.correction.data, ident)
+            ids = r.ids.flatten().tolist()
+            active, entries = len({i for i in ids if i < ne}), sum(i < ne for i in ids)
+            a = P.moe_gemm(x, moe.gate_up.data, r, True, swiglu=True)
+            ad = bf(n, ff)
+            big = n == N
+            amount = lambda parts: (2.0 * entries * parts * eff * w, "mfma bf16") if big else (active * parts * eff * w * 2, "hbm")
+            like = lambda parts: (2.0 * n * parts * ff * w, "mfma bf16") if big else (parts * ff * w * 2, "hbm")
+            add(f"gate_up + SiLU-and-mul (Qwen3), {n} tokens", size, lambda i: P.bf16_linear_silu_mul(x, gu), *like(2))
+            add(f"experts' gate_up + SwiGLU, {n} tokens", size, lambda i: P.moe_gemm(x, moe.gate_up.data, r, True, swiglu=True), *amount(2))
+            add(f"down (Qwen3), {n} tokens", size, lambda i: P.bf16_linear(ad, dn), *like(1))
+            add(f"experts' down, {n} tokens", size, lambda i: P.moe_gemm(a, moe.down.data, r, False), *amount(1))
+            del x, a, ad, r
+        del moe, gu, dn
+    return rows
+
+
 # ----------------------------------------------------------------------------- config 4 (end to end)
 def e2e_workload(num_seqs=256):
     """The reference's bench.py recipe (pure-python ``random``: platform independent)."""
@@ -1135,6 +1284,20 @@ def main():
             "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
             "config": {"workload": "Gigopel layers (latent attention, window 1024; one dense layer, seven of experts) and Qwen3 "
                                    "layers of equal width and active feed-forward, random weights, bf16"},
+            "extra": {"throughput": through, "kernels": rows}}))
+        return
+    if args.workload == "zuzunex":   # likewise
+        rows = bench_zuzunex_kernels()
+        through = [throughput({"zuzunex": zuzunex_shape(size), "zuzunex dense": zuzunex_shape(size, moe=False),
+                               "qwen3": qwen3_shape(size)}, size) for size in ZUZUNEX_EXPERTS]
+        big = through[-1]
+        print(json.dumps({
+            "metric": "output tok/s (Zuzunex, 8 layers of 4096, 64 sequences, decode)", "value": big["zuzunex"]["decode_tok_s"],
+            "unit": "tok/s", "n_gpus": 1, "steps": big["output_tokens"], "warmup": 1,
+            "ms_per_step": big["zuzunex"]["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak",
+            "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+            "config": {"workload": "Zuzunex layers (alternating attention and attention_2; one dense layer, seven of experts "
+                                   "with a shared one) and Qwen3 layers of equal width, random weights, bf16"},
             "extra": {"throughput": through, "kernels": rows}}))
         return
     extra = {}

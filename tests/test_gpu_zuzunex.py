@@ -51,7 +51,7 @@ def test_residual_layer_norm(dtype, rows, width, top):
     assert rel(he, 0.5 * O.layer_norm(table[ids].double(), w.double(), b.double(), 1e-3)) < tol
 
 
-@pytest.mark.parametrize("rows,N,K", [(1, 1024, 2048), (33, 192, 4096), (64, 1024, 4096)])
+@pytest.mark.parametrize("rows,N,K", [(48, 1024, 4096), (33, 192, 4096), (64, 1024, 4096)])
 def test_norm_adds_up_a_split_projection(rows, N, K):
     """Where the projection is split over K the norm sums the partials itself: the same bits as from finished rows."""
     from tinyllmforge_amd import ops as P
@@ -63,6 +63,30 @@ def test_norm_adds_up_a_split_projection(rows, N, K):
     y = P.linear_deferred(a, w)
     h2 = P.residual_layer_norm(y, x2, nw, nb, 1e-5)
     assert y.splits > 1 and torch.equal(x1, x2) and torch.equal(h1, h2)
+
+
+@pytest.mark.parametrize("rows,taps,D,V", [(40, 3, 64, 48), (64, 4, 128, 128), (33, 0, 192, 64), (64, 6, 32, 32)])
+def test_preparation_adds_up_a_split_projection(rows, taps, D, V):
+    """Decoded rows whose projection is split over K: the preparation sums the partials, the same bits as from finished rows."""
+    from tinyllmforge_amd import ops as P
+    H, G, K, g = 4, 2, 4096, torch.Generator().manual_seed(rows)
+    b = lambda *s: torch.randn(*s, generator=g).bfloat16().cuda()
+    chan = (H + G) * D + G * V
+    a, w = b(rows, K), b(chan + H * V, K) * K ** -0.5
+    pos = torch.randint(0, 90, (rows,), generator=g).cuda()
+    slots = torch.randperm(64 * 4, generator=g)[:rows].to(torch.int32).cuda()
+    states = torch.randperm(rows + 2, generator=g)[:rows].to(torch.int32).cuda()
+    slots[3], states[3] = -1, -1                                 # a padding row
+    temps, nw, bias, conv, ring = torch.rand(100, generator=g).cuda(), b(D), b(chan), b(taps, chan), b(rows + 2, taps, chan)
+    cos = torch.rand(100, 16, generator=g).cuda()
+    res = []
+    for proj in (P.bf16_linear(a, w), P.linear_deferred(a, w)):
+        kv, r = P.SinkKV(4, 64, G, D, V, torch.bfloat16, "cuda"), ring.clone()
+        args = (bias, conv, r, states) if taps else (bias,)
+        q, gate = P.sink_prep(proj, kv, H, pos, slots, 1e-5, *args, q_norm=nw, k_norm=nw, cos_sin=cos, rot_dims=16, q_mult=temps)
+        res.append((q, gate.contiguous(), kv.k, kv.v, r))
+    assert proj.splits > 1 and all(torch.equal(x, y) for x, y in zip(*res))
+    assert not torch.equal(res[0][4], ring) or not taps
 
 
 class Attention:
