@@ -1031,7 +1031,7 @@ def bench_zuzunex_kernels(sizes=None):
         q, gate, out = bf(B, h, d), bf(B, h * d), torch.empty(B, h * d, device=dev, dtype=BF)
         for name, cap in (("attention_2", None), ("attention, capped", 30.0)):
             add(f"{name}: decode attention, gated", size,
-                lambda i: P.sink_attention_rows(q, kv, case["bt"], pos, slots, sink, gate, scale, cap, 4096, out),
+                lambda i: P.sink_attention_rows(q, kv, case["bt"], pos, slots, sink, gate, cap, 4096, out),
                 case["algo_bytes"] + B * h * d * 2, "hbm")
         del kv, case
         # -- prompts: 8 x 2048 tokens
@@ -1050,7 +1050,7 @@ def bench_zuzunex_kernels(sizes=None):
         gate, out = bf(N, h * d), torch.empty(N, h * d, device=dev, dtype=BF)
         for name, cap in (("attention_2", None), ("attention, capped", 30.0)):
             add(f"{name}: prompt attention, gated", size,
-                lambda i: P.sink_attention_prefill(qq, kv, bt, cu, starts, 0, S, L, sink, gate, scale, cap, out), flops, "mfma bf16")
+                lambda i: P.sink_attention_prefill(qq, kv, bt, cu, starts, 0, S, L, sink, gate, cap, out), flops, "mfma bf16")
         del qq, gate, out, kv
         # -- between the products
         chan = (h + 2 * g) * d
@@ -1071,9 +1071,9 @@ def bench_zuzunex_kernels(sizes=None):
             seqs = dict(row_seq=torch.arange(N, device=dev, dtype=torch.int32) // L, cu_seqlens_q=cu) if n == N else {}
             states = torch.arange(S if n == N else B, device=dev, dtype=torch.int32)
             add(f"attention: preparation, {n} tokens", size,
-                lambda i: P.sink_prep(proj[i], kv, h, pos[:n], slots[:n], 1e-6, q_mult=temps), n * chan * 4, "hbm", copies)
+                lambda i: P.sink_prep(proj[i], kv, h, pos[:n], slots[:n], 1e-6, scale, 30.0, q_mult=temps), n * chan * 4, "hbm", copies)
             add(f"attention_2: preparation with convolution, {n} tokens", size,
-                lambda i: P.sink_prep(proj[i], kv, h, pos[:n], slots[:n], 1e-6, bias, conv, ring, states, seqs.get("row_seq"),
+                lambda i: P.sink_prep(proj[i], kv, h, pos[:n], slots[:n], 1e-6, scale, None, bias, conv, ring, states, seqs.get("row_seq"),
                                       seqs.get("cu_seqlens_q"), nw, nw, tab, d), n * (chan * (4 if n == N else 10) + d * 4), "hbm", copies)
             if n == N:
                 add(f"convolution state, {S} portions", size, lambda i: P.conv_tail(proj[i], ring, states, cu, starts, 0, S), S * 2 * chan * 4, "hbm", copies)

@@ -716,7 +716,8 @@ int tlf_residual_layernorm(const void *y, int64_t y_stride, const float *partial
  * tlf_sink_prep: projection rows [q: heads * dim | k: kv_heads * dim | v: kv_heads * vdim | gate: heads * vdim] -> + bias (NULL:
  *   none; of the channels of q, k and v) -> with conv [taps, channels] y_p = sum_j conv[j] u_(p - taps + 1 + j), zeros before the
  *   sequence -> q, k / rms over the head * q_norm / k_norm (NULL: 1) -> q times q_mult[pos] (NULL: 1) -> the first rot_dims
- *   dimensions of q and k turned by cos_sin[pos] (cos of the pairs, then sin), i with i + rot_dims / 2 -> q_out [n, heads, Dp]
+ *   dimensions of q and k turned by cos_sin[pos] (cos of the pairs, then sin), i with i + rot_dims / 2 -> q times score_scale
+ *   log2(e), with a cap also times 2 / cap (what the kernels below expect in q) -> q_out [n, heads, Dp]
  *   and the cache rows slot_mapping[token] (negative: not stored).  ring [state slots, taps, channels] holds the projected rows
  *   (without bias) of a sequence's last positions, p in row p mod taps: rows of one-token sequences (row_seq NULL, or
  *   cu_seqlens_q of row_seq[row]) are written here, those of portions by tlf_conv_tail afterwards.  gate_out [n, heads * vdim]
@@ -731,7 +732,8 @@ int tlf_sink_prep(const void *proj, int64_t proj_stride, const float *partials, 
                   *k_norm, const int64_t *positions, const float *cos_sin, const float *q_mult, int32_t max_pos,
                   int32_t rot_dims, const int32_t *slot_mapping, void *q_out, void *k_cache, void *v_cache, void
                   *gate_out, int32_t n, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t
-                  block_size, int64_t num_pages, float eps, int32_t dtype, void *stream);
+                  block_size, int64_t num_pages, float eps, float score_scale, float cap, int32_t dtype, void
+                  *stream);
 int tlf_conv_tail(const void *proj, int64_t proj_stride, void *ring, const int32_t *state_slots, int64_t
                   num_state_slots, const int32_t *cu_seqlens_q, const int32_t *seq_starts, int32_t first_seq, int32_t
                   num_seqs, int32_t taps, int32_t channels, int32_t dtype, void *stream);
@@ -741,14 +743,13 @@ int tlf_sink_attn_rows(const void *q, const void *k_cache, const void *v_cache, 
                        bt_stride, const int64_t *positions, const int32_t *slot_mapping, const int32_t *row_seq, const
                        void *sink, const void *gate, int64_t gate_stride, void *out, int64_t out_stride, int32_t rows,
                        int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t block_size, int32_t
-                       max_len, int64_t num_pages, float scale, float cap, int32_t dtype, void *workspace, size_t
-                       workspace_bytes, void *stream);
+                       max_len, int64_t num_pages, float cap, int32_t dtype, void *workspace, size_t workspace_bytes, void *stream);
 int tlf_sink_attn_prefill_supported(int32_t dim, int32_t vdim);
 int tlf_sink_attn_prefill(const void *q, const void *k_cache, const void *v_cache, const int32_t *block_tables, int64_t
                           bt_stride, const int32_t *cu_seqlens_q, const int32_t *seq_starts, int32_t first_seq,
                           int32_t num_seqs, int32_t max_tokens, const void *sink, const void *gate, int64_t
                           gate_stride, void *out, int64_t out_stride, int32_t heads, int32_t kv_heads, int32_t dim,
-                          int32_t vdim, int32_t block_size, int64_t num_pages, float scale, float cap, void *stream);
+                          int32_t vdim, int32_t block_size, int64_t num_pages, float cap, void *stream);
 
 #ifdef __cplusplus
 }

@@ -83,7 +83,7 @@ def test_preparation_adds_up_a_split_projection(rows, taps, D, V):
     for proj in (P.bf16_linear(a, w), P.linear_deferred(a, w)):
         kv, r = P.SinkKV(4, 64, G, D, V, torch.bfloat16, "cuda"), ring.clone()
         args = (bias, conv, r, states) if taps else (bias,)
-        q, gate = P.sink_prep(proj, kv, H, pos, slots, 1e-5, *args, q_norm=nw, k_norm=nw, cos_sin=cos, rot_dims=16, q_mult=temps)
+        q, gate = P.sink_prep(proj, kv, H, pos, slots, 1e-5, 0.2, None, *args, q_norm=nw, k_norm=nw, cos_sin=cos, rot_dims=16, q_mult=temps)
         res.append((q, gate.contiguous(), kv.k, kv.v, r))
     assert proj.splits > 1 and all(torch.equal(x, y) for x, y in zip(*res))
     assert not torch.equal(res[0][4], ring) or not taps
@@ -303,11 +303,12 @@ def test_rows_of_many_unequal_sequences(dtype):
             at += int(need[i])
         q = torch.zeros(B, H, 64)
         q[..., :D] = torch.randn(B, H, D, generator=g)
+        q = q * 0.4 * 1.4426950408889634                         # the scale and the base of the exponential are in q
         q, gate, sink = q.to(dt), torch.randn(B, H * V, generator=g).to(dt), torch.randn(H, generator=g).to(dt)
         slots = torch.zeros(B, dtype=torch.int32)
         slots[B // 2] = -1 if B > 1 else 0
         out = torch.full((B, H * V + 8), 7.0, dtype=dt, device="cuda")
-        P.sink_attention_rows(q.cuda(), kv, bt.cuda(), (lens - 1).cuda(), slots.cuda(), sink.cuda(), gate.cuda(), 0.4, None, 10 ** 6,
+        P.sink_attention_rows(q.cuda(), kv, bt.cuda(), (lens - 1).cuda(), slots.cuda(), sink.cuda(), gate.cuda(), None, 10 ** 6,
                               out[:, :H * V])
         assert (out[:, H * V:] == 7).all()
         k, v = kv.k.double().cpu(), kv.v.double().cpu()
@@ -318,7 +319,7 @@ def test_rows_of_many_unequal_sequences(dtype):
                 continue
             ki = k[bt[i, :need[i]].long()].transpose(1, 2).reshape(-1, G, 64)[:n, :, :D]
             vi = v[bt[i, :need[i]].long()].transpose(1, 2).reshape(-1, G, 32)[:n, :, :V]
-            s = torch.einsum("gpd,ngd->gpn", q[i, :, :D].double().view(G, H // G, D), ki) * 0.4
+            s = torch.einsum("gpd,ngd->gpn", q[i, :, :D].double().view(G, H // G, D), ki) / 1.4426950408889634
             e = torch.exp(s)
             o = torch.einsum("gpn,ngv->gpv", e / (e.sum(-1) + torch.exp(sink.double()).view(G, -1))[..., None], vi)
             want = o.reshape(-1) * O.sigmoid(gate[i].double())

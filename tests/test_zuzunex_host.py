@@ -346,7 +346,7 @@ def test_entry_points_reject_bad_arguments_on_the_host():
     lib, a = _lib.load(), 4096
     shape = (3, 1, 20, 13)                 # heads, kv heads, dim, value dim: 60 + 20 + 13 + 39 columns
     prep = lambda sizes=shape, ld=136, q=a, n=2, sp=1, p=None, conv=None, taps=0, ring=None, rot=12, bs=64, gate=None, seq=None, dt=0: lib.tlf_sink_prep(
-        a, ld, p, sp, None, a, conv, taps, ring, a, 4, seq, None, a, a, a, a, None, 10, rot, a, q, a, a, gate, n, *sizes, bs, 5, 1e-6, dt, None)
+        a, ld, p, sp, None, a, conv, taps, ring, a, 4, seq, None, a, a, a, a, None, 10, rot, a, q, a, a, gate, n, *sizes, bs, 5, 1e-6, 0.1, 0.0, dt, None)
     assert prep(q=None) == -1 and prep(ld=130) == -2 and prep(n=0) == 0 and prep(rot=22) == -2 and prep(rot=3) == -2
     assert prep(bs=100) == -2 and prep(sizes=(3, 2, 20, 13)) == -2 and prep(sizes=(3, 1, 600, 13), ld=9999) == -2
     assert prep(conv=a, taps=3) == -1 and prep(conv=a, taps=99, ring=a) == -2 and prep(conv=a, taps=3, ring=a, seq=a) == -1
@@ -354,12 +354,12 @@ def test_entry_points_reject_bad_arguments_on_the_host():
     tail = lambda taps=3, ld=136, ring=a, n=1: lib.tlf_conv_tail(a, ld, ring, a, 4, a, a, 0, n, taps, 93, 0, None)
     assert tail(ld=80) == -2 and tail(ring=None) == -1 and tail(n=0) == 0 and tail(taps=1) == 0 and tail(taps=0) == -2
     rows = lambda sizes=shape, cap=0.0, ldo=39, ldg=39, bt=4, most=200, out=a, ws=None, dt=0, n=2: lib.tlf_sink_attn_rows(
-        a, a, a, a, bt, a, a, None, a, a, ldg, out, ldo, n, *sizes, 64, most, 10, 0.1, cap, dt, ws, 0, None)
+        a, a, a, a, bt, a, a, None, a, a, ldg, out, ldo, n, *sizes, 64, most, 10, cap, dt, ws, 0, None)
     assert rows(cap=-1.0) == -2 and rows(ldo=38) == -2 and rows(ldg=30) == -2 and rows(bt=3) == -2 and rows(out=None) == -1
     assert rows() == -4 and rows(dt=3) == -5 and rows(n=0) == 0 and rows(n=70000) == -2
     size = lambda *v: lib.tlf_sink_attn_rows_workspace_bytes(*v)
     assert size(2, *shape, 128, 0) == 0 and size(2, *shape, 200, 0) == 2 * 2 * 3 * (32 + 2) * 4 and size(0, *shape, 200, 0) == 0
-    pre = lambda sizes=shape, ldo=39, out=a, n=1: lib.tlf_sink_attn_prefill(a, a, a, a, 4, a, a, 0, n, 8, a, a, 39, out, ldo, *sizes, 64, 10, 0.1, 0.0, None)
+    pre = lambda sizes=shape, ldo=39, out=a, n=1: lib.tlf_sink_attn_prefill(a, a, a, a, 4, a, a, 0, n, 8, a, a, 39, out, ldo, *sizes, 64, 10, 0.0, None)
     assert pre(ldo=38) == -2 and pre(out=None) == -1 and pre(n=0) == 0 and pre(sizes=(3, 1, 270, 13)) == -5
     assert lib.tlf_sink_attn_prefill_supported(256, 256) == 1 and lib.tlf_sink_attn_prefill_supported(64, 257) == 0
     group = lambda top=2, E=5, ident=1, dt=0: lib.tlf_moe_group(a, 1, a, a, a, a, a, a, a, 99, 4, top, E, ident, a, dt, 32, None, 0, None)

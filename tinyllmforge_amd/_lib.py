@@ -119,14 +119,15 @@ SIGNATURES = {
     "tlf_residual_layernorm": (c_int32, [_P, _I64, _P, _I32, _P, _P, _I64, _P, _P, _I32, _P, _I64, _P, _P, _P, _F, _P,
                                          _I32, _I32, _F, _I32, _P]),
     "tlf_sink_prep": (c_int32, [_P, _I64, _P, _I32, _P, _P, _P, _I32, _P, _P, _I64, _P, _P, _P, _P, _P, _P, _P, _I32,
-                                _I32, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I64, _F, _I32, _P]),
+                                _I32, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I64, _F, _F, _F, _I32,
+                                _P]),
     "tlf_conv_tail": (c_int32, [_P, _I64, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _I32, _I32, _P]),
     "tlf_sink_attn_rows_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32, _I32, _I32, _I32]),
     "tlf_sink_attn_rows": (c_int32, [_P, _P, _P, _P, _I64, _P, _P, _P, _P, _P, _I64, _P, _I64, _I32, _I32, _I32, _I32,
-                                     _I32, _I32, _I32, _I64, _F, _F, _I32, _P, _SZ, _P]),
+                                     _I32, _I32, _I32, _I64, _F, _I32, _P, _SZ, _P]),
     "tlf_sink_attn_prefill_supported": (c_int32, [_I32, _I32]),
     "tlf_sink_attn_prefill": (c_int32, [_P, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _P, _P, _I64, _P, _I64, _I32,
-                                        _I32, _I32, _I32, _I32, _I64, _F, _F, _P]),
+                                        _I32, _I32, _I32, _I32, _I64, _F, _P]),
     "tlf_probe_read": (c_int32, [_P, _SZ, _P, _P]),
     "tlf_probe_copy": (c_int32, [_P, _P, _SZ, _P]),
     "tlf_probe_mfma": (c_int32, [_P, c_int32, c_int32, _P]),

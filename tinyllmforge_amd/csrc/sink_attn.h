@@ -30,18 +30,32 @@ __device__ __forceinline__ int64_t sink_row(const SinkCache &c, int page, int pg
   return (p * c.G + kvh) * c.bs + (j - pg * c.bs);
 }
 
-// Scores in units of log 2.  With a cap: cap log2(e) tanh(s / cap) from one exponential and one reciprocal.
-struct SinkScore {
-  float scale_log2;       // scale * log2(e)
-  float cap_log2, turn;   // cap * log2(e), 2 scale log2(e) / cap; cap_log2 0: no cap
-};
-inline SinkScore sink_score(float scale, float cap) {
-  return SinkScore{scale * kSinkLog2e, cap > 0.f ? cap * kSinkLog2e : 0.f, cap > 0.f ? 2.f * scale * kSinkLog2e / cap : 0.f};
-}
+// Queries are stored with the score's constants in them: q . k is the score times log2(e), or with a cap 2 log2(e) / cap times
+// the score, so that cap log2(e) tanh(score / cap) takes one exponential and one reciprocal.
+inline float sink_query_scale(float scale, float cap) { return scale * kSinkLog2e * (cap > 0.f ? 2.f / cap : 1.f); }
+// The capped score (or the score) in units of log 2.
 template <bool CAP>
-__device__ __forceinline__ float sink_score_log2(float dot, const SinkScore &s) {
-  if (!CAP) return dot * s.scale_log2;
-  return fmaf(-2.f * s.cap_log2, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(dot * s.turn)), s.cap_log2);
+__device__ __forceinline__ float sink_score_log2(float dot, float cap_log2) {
+  if (!CAP) return dot;
+  return fmaf(-2.f * cap_log2, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(dot)), cap_log2);
+}
+
+// acc *= back unless back is 1 in every lane.  Branch and multiplies are one block, so that the accumulators stay in their
+// registers: behind a C++ branch the scaled values land in new ones, and the path that skips the rescale copies them all.
+__device__ __forceinline__ void sink_rescale(floatx4 &x, floatx4 &y, float back) {
+  const unsigned long long moved = __builtin_amdgcn_ballot_w64(back != 1.0f);
+  float t[8] = {x[0], x[1], x[2], x[3], y[0], y[1], y[2], y[3]};
+  asm volatile(
+      "s_cmp_eq_u64 %[m], 0\n\t"
+      "s_cbranch_scc1 .Ltlf_sink_keep%=\n\t"
+      "v_mul_f32_e32 %0, %[a], %0\n\tv_mul_f32_e32 %1, %[a], %1\n\tv_mul_f32_e32 %2, %[a], %2\n\tv_mul_f32_e32 %3, %[a], %3\n\t"
+      "v_mul_f32_e32 %4, %[a], %4\n\tv_mul_f32_e32 %5, %[a], %5\n\tv_mul_f32_e32 %6, %[a], %6\n\tv_mul_f32_e32 %7, %[a], %7\n"
+      ".Ltlf_sink_keep%=:"
+      : "+v"(t[0]), "+v"(t[1]), "+v"(t[2]), "+v"(t[3]), "+v"(t[4]), "+v"(t[5]), "+v"(t[6]), "+v"(t[7])
+      : [a] "v"(back), [m] "s"(moved)
+      : "scc");
+  x = floatx4{t[0], t[1], t[2], t[3]};
+  y = floatx4{t[4], t[5], t[6], t[7]};
 }
 
 inline int sink_cache_make(SinkCache &c, const void *k, const void *v, const int32_t *bt, int64_t bt_stride, int32_t bs, int32_t G,

@@ -2,7 +2,7 @@
 //
 //   sink_prep_kernel   projection row [q | k | v | gate] -> biases, short causal convolution over time per channel, RMS norm
 //                      per head of q and k, a factor per position on q, rotation of the first rot_dims dimensions in halves
-//                      (i with i + rot_dims / 2), K and V stores, q; the gate where the projection exists as partial sums
+//                      (i with i + rot_dims / 2), K and V stores, q with the score's constants; the gate where the projection exists as partial sums
 //   conv_tail_kernel   the last projected rows of a step's portions into the convolution's state
 //
 // Convolution state: a ring of `taps` projected rows per sequence (bias not yet added), position p in row p mod taps.  A
@@ -32,7 +32,27 @@ struct SinkPrepArgs {
   void *q_out, *gate_out;      // [n, H, Dp]; [n, H * Dv] or NULL
   SinkCache c;
   int32_t n, H, taps, channels, heads;
-  float eps;
+  float eps, q_scale;
+};
+
+// Eight values that came from memory as T: held as they were, exact.
+template <typename T, bool PACK>
+struct Few {
+  float f[8];
+  __device__ __forceinline__ void put(const float (&v)[8]) {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[e] = v[e];
+  }
+  __device__ __forceinline__ float operator[](int e) const { return f[e]; }
+};
+template <>
+struct Few<unsigned short, true> {
+  unsigned int w[4];
+  __device__ __forceinline__ void put(const float (&v)[8]) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) w[e] = (__float_as_uint(v[2 * e]) >> 16) | (__float_as_uint(v[2 * e + 1]) & 0xffff0000u);
+  }
+  __device__ __forceinline__ float operator[](int e) const { return __uint_as_float(e & 1 ? w[e / 2] & 0xffff0000u : w[e / 2] << 16); }
 };
 
 // 16 lanes per (token, head), MAXC chunks of 8 elements per lane.  TAPS: 0 no convolution, -1 any (neighbours read again),
@@ -76,15 +96,14 @@ __global__ __launch_bounds__(256) void sink_prep_kernel(const SinkPrepArgs a) {
   };
 
   if (kind == 3) {
-    for (int k = 0; k < TOK; ++k) {
-      if (tok0 + k >= a.n) return;
+    for (int64_t tok = tok0; tok < min(tok0 + TOK, static_cast<int64_t>(a.n)); ++tok) {
 #pragma unroll
       for (int q = 0; q < MAXC; ++q) {
         const int ch = j + q * 16;
         if (ch * 8 >= dims) continue;
         float f[8];
-        row8(tok0 + k, ch, f);
-        T *o = static_cast<T *>(a.gate_out) + (tok0 + k) * (static_cast<int64_t>(a.H) * c.Dv) + static_cast<int64_t>(head - a.H - 2 * G) * c.Dv + ch * 8;
+        row8(tok, ch, f);
+        T *o = static_cast<T *>(a.gate_out) + tok * (static_cast<int64_t>(a.H) * c.Dv) + static_cast<int64_t>(head - a.H - 2 * G) * c.Dv + ch * 8;
         if constexpr (VEC) Elem<T>::st8(o, f);
         else
           for (int e = 0; e < 8; ++e)
@@ -94,18 +113,28 @@ __global__ __launch_bounds__(256) void sink_prep_kernel(const SinkPrepArgs a) {
     return;
   }
 
-  float bias[MAXC][8], wn[MAXC][8], wc[TAPS > 0 ? TAPS : 1][MAXC][8], hist[kBack][MAXC][8];
+  // the weights stay packed: registers decide how many waves hide the loads
+  Few<T, VEC> bias[MAXC], wn[MAXC], wc[TAPS > 0 ? TAPS : 1][MAXC];
+  float hist[kBack][MAXC][8];
   const T *norm = static_cast<const T *>(kind == 0 ? a.q_norm : kind == 1 ? a.k_norm : nullptr);
 #pragma unroll
   for (int q = 0; q < MAXC; ++q) {
     const int ch = j + q * 16;
+    float f[8];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) bias[q][e] = 0.f, wn[q][e] = 1.f;
-    if (a.bias) at8(static_cast<const T *>(a.bias) + chan, ch, bias[q]);
-    if (norm) at8(norm, ch, wn[q]);
+    for (int e = 0; e < 8; ++e) f[e] = 0.f;
+    if (a.bias) at8(static_cast<const T *>(a.bias) + chan, ch, f);
+    bias[q].put(f);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[e] = 1.f;
+    if (norm) at8(norm, ch, f);
+    wn[q].put(f);
     if constexpr (TAPS > 0) {
 #pragma unroll
-      for (int t = 0; t < TAPS; ++t) at8(static_cast<const T *>(a.conv) + static_cast<int64_t>(t) * a.channels + chan, ch, wc[t][q]);
+      for (int t = 0; t < TAPS; ++t) {
+        at8(static_cast<const T *>(a.conv) + static_cast<int64_t>(t) * a.channels + chan, ch, f);
+        wc[t][q].put(f);
+      }
     }
   }
   // the loads of all tokens are in flight before the first is touched
@@ -118,11 +147,36 @@ __global__ __launch_bounds__(256) void sink_prep_kernel(const SinkPrepArgs a) {
         Elem<T>::raw8(proj + min(tok0 + k, static_cast<int64_t>(a.n) - 1) * a.ld + chan + min((j + q * 16) * 8, dims - 8), raw[k][q]);
   }
 
+  // and of the rows before them, of the same sequence or not
+  typename Elem<T>::Raw8 back_rows[kBack][MAXC];
+  if constexpr (VEC && !PART && TAPS > 0 && TOK > 1) {
+#pragma unroll
+    for (int b = 0; b < kBack; ++b)
+#pragma unroll
+      for (int q = 0; q < MAXC; ++q)
+        Elem<T>::raw8(proj + max(tok0 - 1 - b, static_cast<int64_t>(0)) * a.ld + chan + min((j + q * 16) * 8, dims - 8), back_rows[b][q]);
+  }
+  int64_t poss[TOK], slots[TOK];
+  int32_t firsts[TOK], states[TOK];
+  bool singles[TOK];
+#pragma unroll
+  for (int k = 0; k < TOK; ++k) {
+    const int64_t tok = min(tok0 + k, static_cast<int64_t>(a.n) - 1);
+    poss[k] = a.positions[tok];
+    slots[k] = a.slots[tok];
+    if constexpr (TAPS != 0) {
+      const int seq = a.row_seq ? a.row_seq[tok] : static_cast<int>(tok);
+      firsts[k] = a.row_seq ? a.cu_q[seq] : static_cast<int>(tok);
+      singles[k] = !a.row_seq || a.cu_q[seq + 1] - firsts[k] == 1;
+      states[k] = a.state_slots[seq];
+    }
+  }
+  const int half = a.rot_dims / 2;
 #pragma unroll
   for (int k = 0; k < TOK; ++k) {
     const int64_t tok = tok0 + k;
     if (tok >= a.n) return;
-    const int64_t pos = a.positions[tok], slot = a.slots[tok];
+    const int64_t pos = poss[k], slot = slots[k];
     float x[MAXC][8];
 #pragma unroll
     for (int q = 0; q < MAXC; ++q) {
@@ -138,10 +192,8 @@ __global__ __launch_bounds__(256) void sink_prep_kernel(const SinkPrepArgs a) {
     }
     if constexpr (TAPS != 0) {
       const int taps = TAPS > 0 ? TAPS : a.taps;
-      const int seq = a.row_seq ? a.row_seq[tok] : static_cast<int>(tok);
-      const int64_t first = a.row_seq ? a.cu_q[seq] : tok;
-      const bool single = !a.row_seq || a.cu_q[seq + 1] - first == 1;
-      const int64_t st = a.state_slots[seq];
+      const int64_t first = firsts[k], st = states[k];
+      const bool single = singles[k];
       const bool held = st >= 0 && st < a.num_state_slots && pos >= 0;
       T *ring = static_cast<T *>(a.ring) + (held ? st : 0) * taps * a.channels + chan;
       // projected value `back` tokens earlier, with its bias
@@ -152,8 +204,15 @@ __global__ __launch_bounds__(256) void sink_prep_kernel(const SinkPrepArgs a) {
           for (int e = 0; e < 8; ++e) f[e] = 0.f;
           return;
         }
-        if (tok - back >= first) row8(tok - back, ch, f);
-        else at8(ring + (pos - back) % taps * a.channels, ch, f);
+        if (tok - back >= first) {
+          if (VEC && !PART && TOK > 1 && TAPS > 0 && k == 0) {
+            Elem<T>::cvt8(back_rows[TAPS > 0 ? back - 1 : 0][q], f);
+            if (ch * 8 >= dims) {
+#pragma unroll
+              for (int e = 0; e < 8; ++e) f[e] = 0.f;
+            }
+          } else row8(tok - back, ch, f);
+        } else at8(ring + (pos - back) % taps * a.channels, ch, f);
 #pragma unroll
         for (int e = 0; e < 8; ++e) f[e] += bias[q][e];
       };
@@ -237,8 +296,8 @@ __global__ __launch_bounds__(256) void sink_prep_kernel(const SinkPrepArgs a) {
     for (int q = 0; q < MAXC; ++q)
 #pragma unroll
       for (int e = 0; e < 8; ++e) x[q][e] = x[q][e] * inv * wn[q][e];
-    if (kind == 0 && a.q_mult) {
-      const float m = a.q_mult[pos_ok ? pos : 0];
+    if (kind == 0) {
+      const float m = a.q_mult ? a.q_mult[pos_ok ? pos : 0] * a.q_scale : a.q_scale;
 #pragma unroll
       for (int q = 0; q < MAXC; ++q)
 #pragma unroll
@@ -246,7 +305,6 @@ __global__ __launch_bounds__(256) void sink_prep_kernel(const SinkPrepArgs a) {
     }
     if (a.rot_dims > 0 && pos_ok) {                  // the same for the lanes of a team
       float *xs = turn[threadIdx.x / 16];
-      const int half = a.rot_dims / 2;
       const float *cs = a.cos_sin + pos * a.rot_dims;
       wave_lds_fence();
 #pragma unroll
@@ -262,12 +320,12 @@ __global__ __launch_bounds__(256) void sink_prep_kernel(const SinkPrepArgs a) {
         if (at >= a.rot_dims) continue;
         if (VEC && half % 8 == 0) {
           const bool low = at < half;
-          const float *ps = xs + (low ? at + half : at - half), *co = cs + (low ? at : at - half), *si = co + half;
+          const float *ps = xs + (low ? at + half : at - half), *cp = cs + (low ? at : at - half);
           const float sign = low ? -1.f : 1.f;
           float p[8], cv[8], sv[8];
           Elem<float>::ld8(ps, p);
-          Elem<float>::ld8(co, cv);
-          Elem<float>::ld8(si, sv);
+          Elem<float>::ld8(cp, cv);
+          Elem<float>::ld8(cp + half, sv);
 #pragma unroll
           for (int e = 0; e < 8; ++e) x[q][e] = __fmul_rn(x[q][e], cv[e]) + sign * __fmul_rn(p[e], sv[e]);
         } else {
@@ -356,12 +414,12 @@ extern "C" int tlf_sink_prep(const void *proj, int64_t proj_stride, const float 
                              const void *k_norm, const int64_t *positions, const float *cos_sin, const float *q_mult,
                              int32_t max_pos, int32_t rot_dims, const int32_t *slot_mapping, void *q_out, void *k_cache,
                              void *v_cache, void *gate_out, int32_t n, int32_t heads, int32_t kv_heads, int32_t dim,
-                             int32_t vdim, int32_t block_size, int64_t num_pages, float eps, int32_t dtype, void *stream) {
+                             int32_t vdim, int32_t block_size, int64_t num_pages, float eps, float score_scale, float cap, int32_t dtype, void *stream) {
   using namespace tlf;
   SinkPrepArgs a{};
   if (n < 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads || rot_dims < 0 || rot_dims % 2 || rot_dims > dim) return TLF_E_SHAPE;
   if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
-  if (conv && (taps < 1 || taps > 64)) return TLF_E_SHAPE;
+  if (cap < 0.f || (conv && (taps < 1 || taps > 64))) return TLF_E_SHAPE;
   if (n == 0) return TLF_OK;
   if (int rc = partials_check(partials, scale, splits, dtype)) return rc;
   if (int rc = sink_cache_make(a.c, k_cache, v_cache, nullptr, 0, block_size, kv_heads, dim, vdim, num_pages)) return rc;
@@ -377,7 +435,7 @@ extern "C" int tlf_sink_prep(const void *proj, int64_t proj_stride, const float 
   a.row_seq = row_seq; a.cu_q = cu_seqlens_q; a.q_norm = q_norm; a.k_norm = k_norm; a.positions = positions;
   a.cos_sin = cos_sin; a.q_mult = q_mult; a.max_pos = max_pos; a.rot_dims = rot_dims; a.slots = slot_mapping;
   a.q_out = q_out; a.gate_out = gate_out; a.n = n; a.H = heads; a.taps = conv ? taps : 0;
-  a.channels = static_cast<int32_t>(channels); a.eps = eps;
+  a.channels = static_cast<int32_t>(channels); a.eps = eps; a.q_scale = sink_query_scale(score_scale, cap);
   a.heads = heads + 2 * kv_heads + (gate_out ? heads : 0);
   if ((a.heads + 15) / 16 > 65535) return TLF_E_SHAPE;
   const bool vec = dim % 8 == 0 && vdim % 8 == 0 && proj_stride % 8 == 0 && (splits > 1 || aligned16(proj)) && aligned16(bias) &&

@@ -18,8 +18,7 @@ namespace tlf {
 
 struct SinkRowsArgs {
   SinkCache c;
-  SinkScore score;
-  float scale, cap;          // as given, for the rows kernel
+  float cap_log2;            // cap * log2(e), 0: none
   const void *q;             // [rows, H, Dp]
   const void *sink;          // [H] or NULL
   const void *gate;          // [rows, ldg] or NULL: H * Dv columns
@@ -174,7 +173,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
       // lane (n, g) holds head n, keys j0 + g * 8 + e
       float w[8];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) w[e] = sink_score_log2<CAP>(e < 4 ? s0[e & 3] : s1[e & 3], a.score);
+      for (int e = 0; e < 8; ++e) w[e] = sink_score_log2<CAP>(e < 4 ? s0[e & 3] : s1[e & 3], a.cap_log2);
       if (j0 + 32 > hi) {
 #pragma unroll
         for (int e = 0; e < 8; ++e) w[e] = j0 + g * 8 + e < hi ? w[e] : -INFINITY;
@@ -183,13 +182,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
 #pragma unroll
       for (int e = 1; e < 8; ++e) mt = fmaxf(mt, w[e]);
       mt = max_lanes_16_32_48(mt);
-      if (__any(mt > m + 8.f)) {                        // the maximum is moved only when it has grown by a factor of 256
-        const float mn = fmaxf(m, mt), back = mn == m ? 1.f : __builtin_amdgcn_exp2f(m - mn);
-        m = mn;
-        l *= back;
+      // the maximum is moved only when it has grown by a factor of 256
+      const bool grown = mt > m + 8.f;
+      const float back = grown ? __builtin_amdgcn_exp2f(m - mt) : 1.f;
+      m = grown ? mt : m;
+      l *= back;
 #pragma unroll
-        for (int d = 0; d < 2 * VC; ++d) acc[d] *= back;
-      }
+      for (int d = 0; d < VC; ++d) sink_rescale(acc[2 * d], acc[2 * d + 1], back);
       unsigned int ph[4], pl[4];
 #pragma unroll
       for (int e = 0; e < 8; ++e) w[e] = __builtin_amdgcn_exp2f(w[e] - m);
@@ -271,9 +270,8 @@ __global__ __launch_bounds__(256) void sink_rows_kernel(const SinkRowsArgs a) {
         float s = 0.f;
 #pragma unroll
         for (int e = 0; e < 8; ++e) s = fmaf(qf[g][e], kf[e], s);
-        s = group_sum<LPK>(k_ok ? s : 0.f) * a.scale;
-        if (a.cap > 0.f) s = a.cap * tanhf(s / a.cap);
-        s *= kSinkLog2e;
+        s = group_sum<LPK>(k_ok ? s : 0.f);
+        if (a.cap_log2 > 0.f) s = a.cap_log2 * tanhf(s * (0.5f / kSinkLog2e));
         if (ok) {
           const float mn = fmaxf(m[g], s);
           const float f = __builtin_amdgcn_exp2f(m[g] - mn), w = __builtin_amdgcn_exp2f(s - mn);
@@ -375,7 +373,7 @@ int launch_sink_tiles(const SinkRowsArgs &a, hipStream_t s) {
   const int dc = a.c.Dp / 32, vc = a.c.Vp / 32;
 #define TLF_ST(DC, VC)                                                                                   \
   do {                                                                                                   \
-    if (a.score.cap_log2 > 0.f) TLF_LAUNCH((sink_tile_kernel<DC, VC, true>), grid, dim3(256), 0, s, a);  \
+    if (a.cap_log2 > 0.f) TLF_LAUNCH((sink_tile_kernel<DC, VC, true>), grid, dim3(256), 0, s, a);  \
     else TLF_LAUNCH((sink_tile_kernel<DC, VC, false>), grid, dim3(256), 0, s, a);                        \
   } while (0)
 #define TLF_ST_V(DC)                \
@@ -411,7 +409,7 @@ extern "C" int tlf_sink_attn_rows(const void *q, const void *k_cache, const void
                                   int64_t bt_stride, const int64_t *positions, const int32_t *slot_mapping, const int32_t *row_seq,
                                   const void *sink, const void *gate, int64_t gate_stride, void *out, int64_t out_stride,
                                   int32_t rows, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t block_size,
-                                  int32_t max_len, int64_t num_pages, float scale, float cap, int32_t dtype, void *workspace,
+                                  int32_t max_len, int64_t num_pages, float cap, int32_t dtype, void *workspace,
                                   size_t workspace_bytes, void *stream) {
   using namespace tlf;
   if (rows < 0 || rows > 65535 || heads <= 0 || kv_heads <= 0 || heads % kv_heads || max_len <= 0 || cap < 0.f) return TLF_E_SHAPE;
@@ -424,7 +422,7 @@ extern "C" int tlf_sink_attn_rows(const void *q, const void *k_cache, const void
   if (!q || !block_tables || !positions || !slot_mapping || !out) return TLF_E_NULL;
   if (!aligned16(q)) return TLF_E_ALIGN;
   if (bt_stride < (max_len + block_size - 1) / block_size) return TLF_E_SHAPE;
-  a.score = sink_score(scale, cap); a.scale = scale; a.cap = cap;
+  a.cap_log2 = cap * kSinkLog2e;
   a.q = q; a.sink = sink; a.gate = gate; a.positions = positions; a.slots = slot_mapping; a.row_seq = row_seq; a.out = out;
   a.ldo = out_stride; a.ldg = gate_stride; a.rows = rows; a.H = heads; a.group = heads / kv_heads; a.max_len = max_len;
   const bool tiles = sink_tiles(a.c, dtype);

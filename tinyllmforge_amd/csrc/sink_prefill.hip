@@ -17,7 +17,7 @@ constexpr int kSK = 64;   // keys per tile
 
 struct SinkPrefillArgs {
   SinkCache c;
-  SinkScore score;
+  float cap_log2;                   // cap * log2(e), 0: none
   const unsigned short *q;          // [rows, H, Dp]
   const unsigned short *sink;       // [H] or NULL
   const unsigned short *gate;       // [rows, ldg] or NULL
@@ -33,9 +33,14 @@ __device__ __forceinline__ shortx4 sinkp_read_tr16(const unsigned short *p) {
   return __builtin_amdgcn_ds_read_tr16_b64_v4i16((shortx4 __attribute__((address_space(3))) *)(p));
 }
 
-template <int DC, int VC, int CT, bool CAP>
+// MODE 0: no cap, 1: a cap, 2: a cap small enough to take the largest score it allows as everyone's maximum
+template <int DC, int VC, int CT, int MODE>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) void sink_prefill_kernel(const SinkPrefillArgs p) {
   constexpr int DP = DC * 32, VP = VC * 32, KCH = DC * 4, VCH = VC * 4;
+  #ifndef STAGES
+#define STAGES 1
+#endif
+  constexpr int ST = DC + VC <= 8 ? STAGES : 1;                   // tiles in LDS
   __shared__ __attribute__((aligned(16))) unsigned short Ks[kSK][DP + 8], Vs[kSK][VP + 16];
   // consecutive row tiles of one KV head share keys: they go to the same XCD (workgroup w runs on XCD w % 8); the last row
   // tiles, which see the most keys, come first
@@ -115,7 +120,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   float m[CT], l[CT];
 #pragma unroll
   for (int k = 0; k < CT; ++k) {
-    m[k] = -INFINITY;
+    m[k] = MODE == 2 ? p.cap_log2 : -INFINITY;
     l[k] = 0.f;
 #pragma unroll
     for (int d = 0; d < 2 * VC; ++d) acc[k][d] = floatx4{0.f, 0.f, 0.f, 0.f};
@@ -156,7 +161,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
 #pragma unroll
         for (int k = 0; k < CT; ++k) {
 #pragma unroll
-          for (int j = 0; j < 8; ++j) w[k][hf][j] = sink_score_log2<CAP>(j < 4 ? s0[k][j & 3] : s1[k][j & 3], p.score);
+          for (int j = 0; j < 8; ++j) {
+            const float dot = j < 4 ? s0[k][j & 3] : s1[k][j & 3];
+            if (MODE == 2) w[k][hf][j] = -2.f * p.cap_log2 * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(dot));
+            else w[k][hf][j] = sink_score_log2<MODE == 1>(dot, p.cap_log2);
+          }
           if (need_mask) {
             const int key = k0 + hf * 32 + g * 8;
 #pragma unroll
@@ -164,25 +173,25 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
           }
         }
       }
-      float mt[CT];
-      bool grown = false;
+      if constexpr (MODE == 2) {
+        // nothing to rescale; without this the compiler moves the accumulators back and forth on every tile
 #pragma unroll
-      for (int k = 0; k < CT; ++k) {
-        float x = w[k][0][0];
+        for (int k = 0; k < CT; ++k)
 #pragma unroll
-        for (int j = 1; j < 16; ++j) x = fmaxf(x, w[k][j >> 3][j & 7]);
-        mt[k] = max_lanes_16_32_48(x);
-        grown = grown || mt[k] > m[k] + 8.f;
-      }
-      if (__any(grown)) {
+          for (int d = 0; d < 2 * VC; ++d) asm volatile("" : "+v"(acc[k][d]));
+      } else {
 #pragma unroll
         for (int k = 0; k < CT; ++k) {
-          const float mn = fmaxf(m[k], mt[k]);
-          const float back = mn == m[k] ? 1.f : __builtin_amdgcn_exp2f(m[k] - mn);
-          m[k] = mn;
+          float x = w[k][0][0];
+#pragma unroll
+          for (int j = 1; j < 16; ++j) x = fmaxf(x, w[k][j >> 3][j & 7]);
+          x = max_lanes_16_32_48(x);
+          const bool grown = x > m[k] + 8.f;
+          const float back = grown ? __builtin_amdgcn_exp2f(m[k] - x) : 1.f;
+          m[k] = grown ? x : m[k];
           l[k] *= back;
 #pragma unroll
-          for (int d = 0; d < 2 * VC; ++d) acc[k][d] *= back;
+          for (int d = 0; d < VC; ++d) sink_rescale(acc[k][2 * d], acc[k][2 * d + 1], back);
         }
       }
 #pragma unroll
@@ -190,7 +199,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
         uint4 ph[CT], pl[CT];
 #pragma unroll
         for (int k = 0; k < CT; ++k) {
-          const float ms = m[k] == -INFINITY ? 0.f : m[k];
+          const float ms = MODE == 2 || m[k] == -INFINITY ? 0.f : m[k];
           float e[8];
 #pragma unroll
           for (int j = 0; j < 8; ++j) e[j] = __builtin_amdgcn_exp2f(w[k][hf][j] - ms);
@@ -275,7 +284,7 @@ extern "C" int tlf_sink_attn_prefill(const void *q, const void *k_cache, const v
                                      int64_t bt_stride, const int32_t *cu_seqlens_q, const int32_t *seq_starts, int32_t first_seq,
                                      int32_t num_seqs, int32_t max_tokens, const void *sink, const void *gate, int64_t gate_stride,
                                      void *out, int64_t out_stride, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim,
-                                     int32_t block_size, int64_t num_pages, float scale, float cap, void *stream) {
+                                     int32_t block_size, int64_t num_pages, float cap, void *stream) {
   using namespace tlf;
   if (num_seqs < 0 || max_tokens < 0 || first_seq < 0 || heads <= 0 || kv_heads <= 0 || heads % kv_heads || cap < 0.f) return TLF_E_SHAPE;
   const int64_t cols = static_cast<int64_t>(heads) * vdim;
@@ -287,7 +296,7 @@ extern "C" int tlf_sink_attn_prefill(const void *q, const void *k_cache, const v
   if (!q || !block_tables || !cu_seqlens_q || !seq_starts || !out) return TLF_E_NULL;
   if (!aligned16(q)) return TLF_E_ALIGN;
   const int dc = a.c.Dp / 32, vc = a.c.Vp / 32, ct = dc <= 4 && vc <= 4 ? 2 : 1, units = 64 * ct;
-  a.score = sink_score(scale, cap);
+  a.cap_log2 = cap * kSinkLog2e;
   a.q = static_cast<const unsigned short *>(q); a.sink = static_cast<const unsigned short *>(sink);
   a.gate = static_cast<const unsigned short *>(gate); a.cu_q = cu_seqlens_q; a.starts = seq_starts;
   a.out = static_cast<unsigned short *>(out); a.ldo = out_stride; a.ldg = gate ? gate_stride : 0;
@@ -305,8 +314,9 @@ extern "C" int tlf_sink_attn_prefill(const void *q, const void *k_cache, const v
 #define TLF_SP(DC, VC)                                                                                                        \
   do {                                                                                                                        \
     constexpr int kCT = (DC) <= 4 && (VC) <= 4 ? 2 : 1;                                                                       \
-    if (a.score.cap_log2 > 0.f) TLF_LAUNCH((sink_prefill_kernel<DC, VC, kCT, true>), grid, dim3(256), 0, s, a);               \
-    else TLF_LAUNCH((sink_prefill_kernel<DC, VC, kCT, false>), grid, dim3(256), 0, s, a);                                     \
+    if (cap <= 0.f) TLF_LAUNCH((sink_prefill_kernel<DC, VC, kCT, 0>), grid, dim3(256), 0, s, a);                              \
+    else if (cap <= 32.f) TLF_LAUNCH((sink_prefill_kernel<DC, VC, kCT, 2>), grid, dim3(256), 0, s, a);                        \
+    else TLF_LAUNCH((sink_prefill_kernel<DC, VC, kCT, 1>), grid, dim3(256), 0, s, a);                                         \
   } while (0)
 #define TLF_SP_V(DC)                \
   do {                              \

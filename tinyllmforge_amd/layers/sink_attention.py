@@ -83,7 +83,8 @@ class SinkAttention(nn.Module):
         n, single = proj.shape[0], ctx.num_single
         data = lambda p: p.data if p is not None else None
         weight = lambda m: m.weight.data if m is not None else None
-        q, gate = ops.sink_prep(proj, kv, self.num_heads, positions, ctx.slot_mapping, self.eps, data(self.bias), data(self.conv),
+        q, gate = ops.sink_prep(proj, kv, self.num_heads, positions, ctx.slot_mapping, self.eps, self.scale, self.cap,
+                                data(self.bias), data(self.conv),
                                 ring, ctx.state_slots, ctx.row_seq if single < n else None, ctx.cu_seqlens_q, weight(self.q_norm),
                                 weight(self.k_norm), self.cos_sin, self.rot_dims, self.temperatures)
         if ring is not None and single < n:
@@ -93,11 +94,10 @@ class SinkAttention(nn.Module):
         rows = n if not tiles else ctx.num_short_rows if self.short_rows else single
         if rows:
             ops.sink_attention_rows(q[:rows], kv, ctx.block_tables, positions[:rows], ctx.slot_mapping[:rows], self.sink.data,
-                                    gate[:rows], self.scale, self.cap, ctx.max_len, out[:rows],
+                                    gate[:rows], self.cap, ctx.max_len, out[:rows],
                                     ctx.row_seq[:rows] if single < rows else None)
         if rows < n:
             first = single + (ctx.num_short if self.short_rows else 0)
             ops.sink_attention_prefill(q, kv, ctx.block_tables, ctx.cu_seqlens_q, ctx.seq_starts, first,
-                                       ctx.cu_seqlens_q.numel() - 1 - first, ctx.max_portion, self.sink.data, gate, self.scale,
-                                       self.cap, out)
+                                       ctx.cu_seqlens_q.numel() - 1 - first, ctx.max_portion, self.sink.data, gate, self.cap, out)
         return out

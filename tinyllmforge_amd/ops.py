@@ -979,10 +979,10 @@ class SinkKV:
         return block_size * kv_heads * (SinkKV.padded(dim) + SinkKV.padded(vdim)) * itemsize
 
 
-def sink_prep(proj, kv: SinkKV, heads, positions, slot_mapping, eps, bias=None, conv=None, ring=None, state_slots=None,
+def sink_prep(proj, kv: SinkKV, heads, positions, slot_mapping, eps, scale=1.0, cap=None, bias=None, conv=None, ring=None, state_slots=None,
               row_seq=None, cu_seqlens_q=None, q_norm=None, k_norm=None, cos_sin=None, rot_dims=0, q_mult=None):
     """Projection rows ``[q | k | v | gate]`` -> ``(q [N, H, Dp], gate rows [N, >= H * vdim])``; keys and values go to the
-    caches.  See ``tlf_sink_prep``; ``proj`` may be ``Deferred`` when every row is a sequence of its own."""
+    caches, the score's constants into q.  See ``tlf_sink_prep``; ``proj`` may be ``Deferred`` when every row is a sequence of its own."""
     lib = _lib.load()
     dt = kv.k.dtype
     assert proj.dtype == dt
@@ -1019,7 +1019,7 @@ def sink_prep(proj, kv: SinkKV, heads, positions, slot_mapping, eps, bias=None, 
                             _opt(k_norm), positions.data_ptr(), _opt(cos_sin), _opt(q_mult),
                             tables[0].shape[0] if tables else 1 << 30, rot_dims, slot_mapping.data_ptr(), q.data_ptr(),
                             kv.k.data_ptr(), kv.v.data_ptr(), _opt(out), n, heads, G, kv.dim, kv.vdim, bs, pages, float(eps),
-                            _dt(kv.k), _stream()), "tlf_sink_prep")
+                            float(scale), float(cap or 0), _dt(kv.k), _stream()), "tlf_sink_prep")
     return q, gate
 
 
@@ -1034,8 +1034,8 @@ def conv_tail(proj, ring, state_slots, cu_seqlens_q, seq_starts, first_seq, num_
                                     _dt(ring), _stream()), "tlf_conv_tail")
 
 
-def sink_attention_rows(q, kv: SinkKV, block_tables, positions, slot_mapping, sink, gate, scale, cap, max_len, out, row_seq=None):
-    """Row by row: ``q [N, H, Dp]`` -> ``out [N, H * vdim]``; ``row_seq`` None: row r is sequence r."""
+def sink_attention_rows(q, kv: SinkKV, block_tables, positions, slot_mapping, sink, gate, cap, max_len, out, row_seq=None):
+    """Row by row: ``q [N, H, Dp]`` as from ``sink_prep`` -> ``out [N, H * vdim]``; ``row_seq`` None: row r is sequence r."""
     lib = _lib.load()
     _need(q, kv.k.dtype, "q"); _need(block_tables, torch.int32, "block_tables"); _need(positions, torch.int64, "positions")
     n, heads, dp = q.shape
@@ -1056,7 +1056,7 @@ def sink_attention_rows(q, kv: SinkKV, block_tables, positions, slot_mapping, si
             q[lo:].data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), block_tables.data_ptr(), block_tables.stride(0),
             positions[lo:].data_ptr(), slot_mapping[lo:].data_ptr(), row_seq[lo:].data_ptr() if row_seq is not None else None,
             _opt(sink), gate[lo:].data_ptr() if gate is not None else None, gate.stride(0) if gate is not None else 0,
-            out[lo:].data_ptr(), out.stride(0), m, heads, G, kv.dim, kv.vdim, bs, max_len, pages, float(scale), float(cap or 0),
+            out[lo:].data_ptr(), out.stride(0), m, heads, G, kv.dim, kv.vdim, bs, max_len, pages, float(cap or 0),
             _dt(q), ws.data_ptr(), ws.numel(), _stream()), "tlf_sink_attn_rows")
     return out
 
@@ -1066,7 +1066,7 @@ def sink_prefill_supported(dim, vdim) -> bool:
 
 
 def sink_attention_prefill(q, kv: SinkKV, block_tables, cu_seqlens_q, seq_starts, first_seq, num_seqs, max_tokens, sink, gate,
-                           scale, cap, out):
+                           cap, out):
     """Portions of sequences ``first_seq ..`` on the matrix cores (bf16); rows indexed as in the step."""
     _need(q, BF16, "q"); _need(block_tables, torch.int32, "block_tables")
     n, heads, dp = q.shape
@@ -1078,7 +1078,7 @@ def sink_attention_prefill(q, kv: SinkKV, block_tables, cu_seqlens_q, seq_starts
     check(_lib.load().tlf_sink_attn_prefill(
         q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), cu_seqlens_q.data_ptr(),
         seq_starts.data_ptr(), first_seq, num_seqs, max_tokens, _opt(sink), _opt(gate), gate.stride(0) if gate is not None else 0,
-        out.data_ptr(), out.stride(0), heads, G, kv.dim, kv.vdim, bs, pages, float(scale), float(cap or 0), _stream()),
+        out.data_ptr(), out.stride(0), heads, G, kv.dim, kv.vdim, bs, pages, float(cap or 0), _stream()),
         "tlf_sink_attn_prefill")
     return out
 
