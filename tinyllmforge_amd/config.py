@@ -189,15 +189,14 @@ class ZuzunexConfig(LayeredConfig):
             assert m["heads"] % m["kv_heads"] == 0
             rot = m.get("rot")
             assert not rot or (rot["dims"] % 2 == 0 and rot["dims"] <= m["dim"])
-            if layer["type"] == "attention_2":
-                assert m["conv"] >= 1
             assert not mlp or mlp["kind"] in ("dense", "moe")
             if mlp and mlp["kind"] == "moe":
                 r = mlp["router"]
                 assert 1 <= r["top"] <= r["experts"] + (r.get("identity") or 0)
         if self.loop:
             assert 0 <= self.loop["start"] <= self.loop["stop"] <= len(self.layers) and self.loop["times"] >= 1
-        self.recurrent = any(layer["type"] == "attention_2" for layer in self.layers)     # a convolution has a state
+        # a convolution has a state
+        self.recurrent = any(layer["type"] == "attention_2" and layer["mixer"].get("conv") for layer in self.layers)
 
     def layer_runs(self) -> list[int]:
         if not self.loop:

@@ -29,18 +29,23 @@ struct SinkRowsArgs {
   int64_t ldo, ldg;
   float *part_o;             // [splits, rows, H, Vp]
   float *part_ml;            // [splits, rows, H, 2]: maximum (log 2 units), sum
-  int32_t rows, H, group, per_pass, passes, splits, max_len;
+  int32_t rows, H, group, per_pass, passes, splits, least, max_len;
 };
 
 __device__ __forceinline__ shortx4 sink_read_tr16(const unsigned short *p) {
   return __builtin_amdgcn_ds_read_tr16_b64_v4i16((shortx4 __attribute__((address_space(3))) *)(p));
 }
 
-// Keys [lo, hi) of a split of a row with `total` keys, in multiples of 64.
-__device__ __forceinline__ void sink_split(int total, int splits, int split, int &lo, int &hi) {
-  const int per = max(((total + splits - 1) / splits + 63) & ~63, 128);
+// A row's keys are cut into pieces of equal length, a multiple of 64 and at least `least`, so short rows use few of the splits.
+// Split `split` has keys [lo, hi); returns how many splits the row uses, 0 for a padding row.
+__device__ __forceinline__ int sink_split(const SinkRowsArgs &a, int64_t row, int split, int &lo, int &hi) {
+  const int64_t i = a.positions[row];
+  lo = hi = 0;
+  if (a.slots[row] < 0 || i < 0 || i >= a.max_len) return 0;
+  const int total = static_cast<int>(i) + 1, per = max(((total + a.splits - 1) / a.splits + 63) & ~63, a.least);
   lo = min(total, split * per);
   hi = min(total, lo + per);
+  return (total + per - 1) / per;
 }
 // Row r's output element: mix / denominator, the sink in the denominator, the gate on top.
 template <typename T>
@@ -55,7 +60,7 @@ __device__ __forceinline__ float sink_finish(const SinkRowsArgs &a, int64_t row,
 // Four waves' (m, l, O) in LDS -> one; written as the row's result or as a partial one.  O[wave][head][dim], rows of `ldw`.
 template <typename T>
 __device__ __forceinline__ void sink_join_waves(const SinkRowsArgs &a, const float *ow, int ldw, int heads_w, const float (*ml)[16][2],
-                                                int64_t row, int split, int h0, int nh, bool live) {
+                                                int64_t row, int split, int h0, int nh, int used) {
   const int Vp = a.c.Vp;
   for (int t = threadIdx.x; t < nh * Vp; t += 256) {
     const int g = t / Vp, d = t - g * Vp;
@@ -71,13 +76,13 @@ __device__ __forceinline__ void sink_join_waves(const SinkRowsArgs &a, const flo
         if (f > 0.f) o += f * ow[(w * heads_w + g) * ldw + d];
       }
     }
-    if (a.splits > 1) {
+    if (used > 1) {
       const int64_t at = (static_cast<int64_t>(split) * a.rows + row) * a.H + head;
       if (l > 0.f) a.part_o[at * Vp + d] = o;
       if (d == 0) a.part_ml[at * 2] = m, a.part_ml[at * 2 + 1] = l;
     } else if (d < a.c.Dv) {
       Elem<T>::st(static_cast<T *>(a.out) + row * a.ldo + static_cast<int64_t>(head) * a.c.Dv + d,
-                  live ? sink_finish<T>(a, row, head, d, o, m, l) : 0.f);
+                  used ? sink_finish<T>(a, row, head, d, o, m, l) : 0.f);
     }
   }
 }
@@ -90,15 +95,14 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
   __shared__ __attribute__((aligned(16))) unsigned char lds[kBytes];
   __shared__ float ml[4][16][2];
   const SinkCache &c = a.c;
-  const int64_t row = blockIdx.z;
-  const int split = blockIdx.x, kvh = blockIdx.y / a.passes, pass = blockIdx.y % a.passes;
+  const int64_t row = blockIdx.y;
+  const int split = blockIdx.z, kvh = blockIdx.x / a.passes, pass = blockIdx.x % a.passes;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, n = lane & 15, g = lane >> 4;
   const int seq = a.row_seq ? a.row_seq[row] : static_cast<int>(row);
-  const int i = static_cast<int>(a.positions[row]);
-  const bool live = a.slots[row] >= 0 && i >= 0 && i < a.max_len;    // workgroup uniform
+  int lo, hi;
+  const int used = sink_split(a, row, split, lo, hi);
+  if (split >= max(used, 1)) return;                    // workgroup uniform; split 0 of a padding row writes its zeros
   const int h0 = kvh * a.group + pass * a.per_pass, nh = min(a.per_pass, a.group - pass * a.per_pass);
-  int lo = 0, hi = 0;
-  if (live) sink_split(i + 1, a.splits, split, lo, hi);
   unsigned short(*Vs)[LV] = reinterpret_cast<unsigned short(*)[LV]>(lds) + wave * 32;
 
   bf16x8 qf[DC];
@@ -219,7 +223,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2))) void s
     *reinterpret_cast<float4 *>(&ow[(wave * 16 + n) * LO + d * 16 + g * 4]) = make_float4(acc[d][0], acc[d][1], acc[d][2], acc[d][3]);
   if (g == 0) ml[wave][n][0] = m, ml[wave][n][1] = l;
   __syncthreads();
-  sink_join_waves<unsigned short>(a, ow, LO, 16, ml, row, split, h0, nh, live);
+  sink_join_waves<unsigned short>(a, ow, LO, 16, ml, row, split, h0, nh, used);
 }
 
 // LPK lanes per key; every group of LPK lanes keeps its own running maximum, sum and mix for GH heads.
@@ -229,17 +233,16 @@ __global__ __launch_bounds__(256) void sink_rows_kernel(const SinkRowsArgs a) {
   __shared__ __attribute__((aligned(16))) float red[4][GH][LPK * 8];
   __shared__ float ml[4][16][2];
   const SinkCache &c = a.c;
-  const int64_t row = blockIdx.z;
-  const int split = blockIdx.x, kvh = blockIdx.y / a.passes, pass = blockIdx.y % a.passes;
+  const int64_t row = blockIdx.y;
+  const int split = blockIdx.z, kvh = blockIdx.x / a.passes, pass = blockIdx.x % a.passes;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, sub = lane / LPK, dl = lane % LPK;
   const int seq = a.row_seq ? a.row_seq[row] : static_cast<int>(row);
-  const int i = static_cast<int>(a.positions[row]);
-  const bool live = a.slots[row] >= 0 && i >= 0 && i < a.max_len;
+  int lo, hi;
+  const int used = sink_split(a, row, split, lo, hi);
+  if (split >= max(used, 1)) return;                    // workgroup uniform; split 0 of a padding row writes its zeros
   const int h0 = kvh * a.group + pass * a.per_pass, nh = min(a.per_pass, a.group - pass * a.per_pass);
   const bool k_ok = dl * 8 < c.Dp, v_ok = dl * 8 < c.Vp;
   const int kcol = k_ok ? dl * 8 : 0, vcol = v_ok ? dl * 8 : 0;
-  int lo = 0, hi = 0;
-  if (live) sink_split(i + 1, a.splits, split, lo, hi);
   float qf[GH][8], o[GH][8], m[GH], l[GH];
 #pragma unroll
   for (int g = 0; g < GH; ++g) {
@@ -303,7 +306,7 @@ __global__ __launch_bounds__(256) void sink_rows_kernel(const SinkRowsArgs a) {
     if (lane == 0) ml[wave][g][0] = top, ml[wave][g][1] = l[g];
   }
   __syncthreads();
-  sink_join_waves<T>(a, &red[0][0][0], LPK * 8, GH, ml, row, split, h0, nh, live);
+  sink_join_waves<T>(a, &red[0][0][0], LPK * 8, GH, ml, row, split, h0, nh, used);
 }
 
 // The splits of a row joined: 4 value dimensions per thread.
@@ -317,24 +320,40 @@ __global__ __launch_bounds__(256) void sink_merge_kernel(const SinkRowsArgs a) {
   if (d >= Dv) return;
   const int64_t plane = static_cast<int64_t>(a.rows) * a.H;
   T *out = static_cast<T *>(a.out) + row * a.ldo + static_cast<int64_t>(head) * Dv + d;
-  const bool live = a.slots[row] >= 0 && a.positions[row] >= 0 && a.positions[row] < a.max_len;
+  int lo, hi;
+  const int used = sink_split(a, row, 0, lo, hi);
+  if (used <= 1) return;                                // finished by its one workgroup
   float m = -INFINITY, l = 0.f, o[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int s = 0; s < a.splits; ++s) m = fmaxf(m, a.part_ml[(s * plane + rh) * 2]);
-#pragma unroll 4
-  for (int s = 0; s < a.splits; ++s) {
-    const float2 ml = *reinterpret_cast<const float2 *>(a.part_ml + (s * plane + rh) * 2);
-    if (ml.y > 0.f) {
-      const float f = __builtin_amdgcn_exp2f(ml.x - m);
-      const float4 p = *reinterpret_cast<const float4 *>(a.part_o + (s * plane + rh) * a.c.Vp + d);
-      l = fmaf(f, ml.y, l);
-      o[0] = fmaf(f, p.x, o[0]); o[1] = fmaf(f, p.y, o[1]);
-      o[2] = fmaf(f, p.z, o[2]); o[3] = fmaf(f, p.w, o[3]);
+  for (int s0 = 0; s0 < used; s0 += 8) {               // eight splits' loads in flight
+    float2 ml[8];
+    float4 p[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int64_t at = min(s0 + i, used - 1) * plane + rh;
+      ml[i] = *reinterpret_cast<const float2 *>(a.part_ml + at * 2);
+      p[i] = *reinterpret_cast<const float4 *>(a.part_o + at * a.c.Vp + d);
+    }
+    float top = m;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) top = fmaxf(top, ml[i].x);
+    const float back = __builtin_amdgcn_exp2f(m - top);
+    m = top;
+    l *= back;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) o[e] *= back;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      if (s0 + i < used && ml[i].y > 0.f) {
+        const float f = __builtin_amdgcn_exp2f(ml[i].x - m);
+        l = fmaf(f, ml[i].y, l);
+        o[0] = fmaf(f, p[i].x, o[0]); o[1] = fmaf(f, p[i].y, o[1]);
+        o[2] = fmaf(f, p[i].z, o[2]); o[3] = fmaf(f, p[i].w, o[3]);
+      }
     }
   }
 #pragma unroll
   for (int e = 0; e < 4; ++e)
-    if (d + e < Dv) Elem<T>::st(out + e, live ? sink_finish<T>(a, row, head, d + e, o[e], m, l) : 0.f);
+    if (d + e < Dv) Elem<T>::st(out + e, sink_finish<T>(a, row, head, d + e, o[e], m, l));
 }
 
 int sink_splits(int64_t groups, int64_t max_keys) {
@@ -350,7 +369,7 @@ size_t sink_rows_bytes(int64_t splits, int64_t rows, int64_t H, int64_t Vp) { re
 
 template <typename T>
 int launch_sink_rows(const SinkRowsArgs &a, hipStream_t s) {
-  const dim3 grid(a.splits, a.c.G * a.passes, a.rows);
+  const dim3 grid(a.c.G * a.passes, a.rows, a.splits);      // splits outermost: the unused ones come last, on all XCDs alike
   const int most = a.c.Dp > a.c.Vp ? a.c.Dp : a.c.Vp;
 #define TLF_SR(LPK, GH) TLF_LAUNCH((sink_rows_kernel<T, LPK, GH>), grid, dim3(256), 0, s, a)
 #define TLF_SR_GH(LPK)                    \
@@ -369,7 +388,7 @@ int launch_sink_rows(const SinkRowsArgs &a, hipStream_t s) {
   return launch_status();
 }
 int launch_sink_tiles(const SinkRowsArgs &a, hipStream_t s) {
-  const dim3 grid(a.splits, a.c.G * a.passes, a.rows);
+  const dim3 grid(a.c.G * a.passes, a.rows, a.splits);      // splits outermost: the unused ones come last, on all XCDs alike
   const int dc = a.c.Dp / 32, vc = a.c.Vp / 32;
 #define TLF_ST(DC, VC)                                                                                   \
   do {                                                                                                   \
@@ -430,6 +449,7 @@ extern "C" int tlf_sink_attn_rows(const void *q, const void *k_cache, const void
   a.passes = (a.group + a.per_pass - 1) / a.per_pass;
   if (static_cast<int64_t>(kv_heads) * a.passes > 65535) return TLF_E_SHAPE;
   a.splits = sink_splits(static_cast<int64_t>(rows) * kv_heads * a.passes, max_len);
+  a.least = static_cast<int64_t>(rows) * kv_heads * a.passes >= 256 ? 512 : 128;      // short pieces only where workgroups are few
   if (a.splits > 1) {
     if (!workspace || workspace_bytes < sink_rows_bytes(a.splits, rows, heads, a.c.Vp)) return TLF_E_WORKSPACE;
     if (!aligned16(workspace)) return TLF_E_ALIGN;

@@ -23,7 +23,7 @@ class ZuzunexAttention(nn.Module):
         m, second = layer["mixer"], layer["type"] == "attention_2"
         rot = m.get("rot")
         self.attn = SinkAttention(m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["scale"], cfg.norm["eps"], cfg.torch_dtype,
-                                  cap=m.get("softcap"), bias=second, taps=m["conv"] if second else 0, weighted_norm=second,
+                                  cap=m.get("softcap"), bias=second, taps=(m.get("conv") or 0) if second else 0, weighted_norm=second,
                                   rot_dims=rot["dims"] if rot else 0, rope=rope, temperatures=temperatures, runs=runs)
         self.qkvg = StackedLinear(cfg.width, self.attn.parts)
         self.o = StackedLinear(self.attn.parts["g"], {"o": cfg.width})
