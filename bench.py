@@ -980,11 +980,11 @@ def zuzunex_shape(size, layers=8, vocab=32768, moe=True):
     w, hq, hkv, d, ff, *_ = GITOPEL_SIZES[size]
     ne, ident, top, eff = ZUZUNEX_EXPERTS[size]
     heads = dict(heads=hq, kv_heads=hkv, dim=d, vdim=d, scale=d ** -0.5)
-    mixers = [("attention", dict(heads, softcap=30.0, q_temp=dict(coef=0.1, every=1024))),
-              ("attention_2", dict(heads, conv=3, rot=dict(base=1e6, dims=d, scaling=dict(factor=4.0, original=1024, fast=32.0, slow=1.0))))]
+    mixers = [("attention", dict(heads, softcap=20.0, q_temp=dict(coef=0.1, every=1024))),
+              ("attention_2", dict(heads, conv=4, rot=dict(base=1e6, dims=d, scaling=dict(factor=8.0, original=4096, fast=16.0, slow=2.0))))]
     dense = dict(kind="dense", ff=ff)
     sparse = dict(kind="moe", expert=dict(ff=eff), router=dict(experts=ne, identity=ident, top=top), shared=dict(ff=eff))
-    return dict(architecture="Zuzunex", vocab=vocab, width=w, norm=dict(eps=1e-6), logit_scale=0.5, loop=None,
+    return dict(architecture="Zuzunex", vocab=vocab, width=w, norm=dict(eps=1e-6), logit_scale=0.8, loop=None,
                 layers=[dict(type=mixers[i % 2][0], mixer=mixers[i % 2][1], mlp=sparse if moe and i else dense) for i in range(layers)])
 
 
@@ -1029,7 +1029,7 @@ def bench_zuzunex_kernels(sizes=None):
         kv.v.normal_()
         pos, slots = case["ctx"].long() - 1, torch.zeros(B, dtype=torch.int32, device=dev)
         q, gate, out = bf(B, h, d), bf(B, h * d), torch.empty(B, h * d, device=dev, dtype=BF)
-        for name, cap in (("attention_2", None), ("attention, capped", 30.0)):
+        for name, cap in (("attention_2", None), ("attention, capped", 20.0)):
             add(f"{name}: decode attention, gated", size,
                 lambda i: P.sink_attention_rows(q, kv, case["bt"], pos, slots, sink, gate, cap, 4096, out),
                 case["algo_bytes"] + B * h * d * 2, "hbm")
@@ -1048,7 +1048,7 @@ def bench_zuzunex_kernels(sizes=None):
         bt = torch.arange(N // bs, dtype=torch.int32, device=dev).view(S, -1)
         starts = torch.zeros(S, dtype=torch.int32, device=dev)
         gate, out = bf(N, h * d), torch.empty(N, h * d, device=dev, dtype=BF)
-        for name, cap in (("attention_2", None), ("attention, capped", 30.0)):
+        for name, cap in (("attention_2", None), ("attention, capped", 20.0)):
             add(f"{name}: prompt attention, gated", size,
                 lambda i: P.sink_attention_prefill(qq, kv, bt, cu, starts, 0, S, L, sink, gate, cap, out), flops, "mfma bf16")
         del qq, gate, out, kv
@@ -1058,7 +1058,7 @@ def bench_zuzunex_kernels(sizes=None):
         tab = tab.to(dev)
         slots = torch.arange(N, dtype=torch.int32, device=dev)
         pos = torch.arange(L, device=dev).repeat(S)
-        nw, bias, conv, ring = torch.ones(d, device=dev, dtype=BF), bf(chan), bf(3, chan), torch.zeros(B, 3, chan, device=dev, dtype=BF)
+        nw, bias, conv, ring = torch.ones(d, device=dev, dtype=BF), bf(chan), bf(4, chan), torch.zeros(B, 4, chan, device=dev, dtype=BF)
         for n, copies in ((N, 3), (B, 1)):
             qkv = bf(copies, n, chan)
             kc, vc = bf(2, N // bs, bs, g, d)
@@ -1071,12 +1071,12 @@ def bench_zuzunex_kernels(sizes=None):
             seqs = dict(row_seq=torch.arange(N, device=dev, dtype=torch.int32) // L, cu_seqlens_q=cu) if n == N else {}
             states = torch.arange(S if n == N else B, device=dev, dtype=torch.int32)
             add(f"attention: preparation, {n} tokens", size,
-                lambda i: P.sink_prep(proj[i], kv, h, pos[:n], slots[:n], 1e-6, scale, 30.0, q_mult=temps), n * chan * 4, "hbm", copies)
+                lambda i: P.sink_prep(proj[i], kv, h, pos[:n], slots[:n], 1e-6, scale, 20.0, q_mult=temps), n * chan * 4, "hbm", copies)
             add(f"attention_2: preparation with convolution, {n} tokens", size,
                 lambda i: P.sink_prep(proj[i], kv, h, pos[:n], slots[:n], 1e-6, scale, None, bias, conv, ring, states, seqs.get("row_seq"),
-                                      seqs.get("cu_seqlens_q"), nw, nw, tab, d), n * (chan * (4 if n == N else 10) + d * 4), "hbm", copies)
+                                      seqs.get("cu_seqlens_q"), nw, nw, tab, d), n * (chan * (4 if n == N else 12) + d * 4), "hbm", copies)
             if n == N:
-                add(f"convolution state, {S} portions", size, lambda i: P.conv_tail(proj[i], ring, states, cu, starts, 0, S), S * 2 * chan * 4, "hbm", copies)
+                add(f"convolution state, {S} portions", size, lambda i: P.conv_tail(proj[i], ring, states, cu, starts, 0, S), S * 3 * chan * 4, "hbm", copies)
             del proj, kv
             y, x, e, rr = bf(copies, n, w), torch.randn(copies, n, w, device=dev), bf(copies, n * top, w), bf(copies, n, w)
             ww, wb = torch.ones(w, device=dev, dtype=BF), torch.zeros(w, device=dev, dtype=BF)
