@@ -601,7 +601,10 @@ int tlf_residual_rmsnorm(const void *y, int64_t y_stride, const float *partials,
  *
  * tlf_latent_prep: projection rows [q: heads * (dim + rot_dim), own part first in a head | ... | latent at latent_col: rank |
  *   rot_dim] -> q_out [n, heads, Dq] with the rotated part turned pairwise (2 i, 2 i + 1) by cos_sin[pos] (cos of the pairs,
- *   then sin), latent / rms * norm_weight and the turned key into the cache row slot_mapping[token] (negative: not stored).
+ *   then sin; with `halves` pairs (i, i + rot_dim / 2)), latent / rms * norm_weight and the turned key into the cache row
+ *   slot_mapping[token] (negative: not stored).  q_out or cache NULL: without the queries or the latents (latent_col then counts
+ *   from the row's first column, queries may lie in another tensor).  cq_norm: the cq_rank columns from cq_col on, / rms * cq_norm,
+ *   to cq_out [n, cq_stride] (zeros behind).  gate_out [n, heads] (with cache): sigmoid of the columns from gate_col on.
  * tlf_head_gemm: y[row, head] = W[head] x[row, head], W [heads, N, K]; N a multiple of 16, K of 32.  In rows below n_main
  *   only the first k_main columns hold weights (n_main 0: all).
  * tlf_latent_rows: absorbed attention, any rows in either dtype: q [rows, heads, Lp] = [Uk_h^T q_own | q_rot | 0]; writes
@@ -615,15 +618,16 @@ int tlf_residual_rmsnorm(const void *y, int64_t y_stride, const float *partials,
  *   2].  tlf_latent_attn_layout gives (host memory) layout[3] = int32 values of a plan, pieces, units.
  * tlf_latent_values: out[row, head] = Uv_h (sum of the pieces / denominator); uv [heads, vdim rounded up to 16, Rp]; plan
  *   NULL: part as from tlf_latent_rows, otherwise the plan and its arguments (with cu_seqlens_q, row_seq[r] is the sequence
- *   of row r of `out`).  Rows without keys give 0.
+ *   of row r of `out`).  gate [rows, heads] (NULL: none) multiplies a head's result.  Rows without keys give 0.
  * tlf_latent_gather: for the expanded form: cache rows of the keys that sequence first_seq + s sees in this step (from
  *   position max(0, start - window + 1) on) as rows kv_offsets[s] .. kv_offsets[s + 1] - 1 of `out`; max_rows bounds them.
  * tlf_latent_prefill: portions from expanded keys and values (rows [heads * Da | heads * Va], Va = vdim rounded up to 8) and
- *   the gathered rows; bf16, Dq <= 256, vdim <= 128 (tlf_latent_prefill_supported). */
+ *   the gathered rows; gate as above, by the step's rows; bf16, Dq <= 256, vdim <= 128 (tlf_latent_prefill_supported). */
 int tlf_latent_prep(const void *proj, int64_t proj_stride, const float *partials, int32_t splits, const float *scale,
                     int32_t latent_col, const void *norm_weight, const int64_t *positions, const float *cos_sin,
-                    int32_t max_pos, const int32_t *slot_mapping, int64_t num_slots, void *q_out, void *cache,
-                    int32_t n, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, float eps,
+                    int32_t max_pos, int32_t halves, const int32_t *slot_mapping, int64_t num_slots, void *q_out, void *cache,
+                    int32_t cq_col, int32_t cq_rank, const void *cq_norm, void *cq_out, int32_t cq_stride,
+                    int32_t gate_col, float *gate_out, int32_t n, int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, float eps,
                     int32_t dtype, void *stream);
 int tlf_head_gemm(const void *x, const void *w, void *y, int32_t rows, int32_t heads, int32_t N, int32_t K, int32_t
                   n_main, int32_t k_main, int32_t dtype, void *stream);
@@ -642,7 +646,7 @@ int tlf_latent_attn(const void *q, const void *cache, const int32_t *block_table
                     int32_t block_size, int32_t window, int64_t num_pages, float scale, void *stream);
 int tlf_latent_values(const float *part, const float *ml, const int32_t *plan, const int32_t *cu_seqlens_q, const
                       int32_t *row_seq, int32_t first_seq, int32_t first_row, int32_t num_seqs, int32_t max_tokens,
-                      const void *uv, void *out, int64_t out_stride, int32_t rows, int32_t heads, int32_t dim,
+                      const void *uv, const float *gate, void *out, int64_t out_stride, int32_t rows, int32_t heads, int32_t dim,
                       int32_t rot_dim, int32_t rank, int32_t vdim, int32_t dtype, void *stream);
 int tlf_latent_attn_supported(int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim);
 int tlf_latent_gather(const void *cache, const int32_t *block_tables, int64_t bt_stride, const int32_t *cu_seqlens_q,
@@ -652,7 +656,7 @@ int tlf_latent_gather(const void *cache, const int32_t *block_tables, int64_t bt
 int tlf_latent_prefill_supported(int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim);
 int tlf_latent_prefill(const void *q, const void *expanded, int64_t expanded_stride, const void *latents, const
                        int32_t *cu_seqlens_q, const int32_t *seq_starts, const int32_t *kv_offsets, int32_t
-                       first_seq, int32_t num_seqs, int32_t max_tokens, void *out, int64_t out_stride, int32_t heads,
+                       first_seq, int32_t num_seqs, int32_t max_tokens, const float *gate, void *out, int64_t out_stride, int32_t heads,
                        int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, int32_t window, float scale, void
                        *stream);
 
@@ -750,6 +754,84 @@ int tlf_sink_attn_prefill(const void *q, const void *k_cache, const void *v_cach
                           int32_t num_seqs, int32_t max_tokens, const void *sink, const void *gate, int64_t
                           gate_stride, void *out, int64_t out_stride, int32_t heads, int32_t kv_heads, int32_t dim,
                           int32_t vdim, int32_t block_size, int64_t num_pages, float cap, void *stream);
+
+/* Norm behind the sum, with what follows it:
+ *   x_out = rms_norm(alpha * x + layer_scale * y) * w   (tlf_post_rmsnorm; y or its partial sums as above)
+ *   x_out = embed_scale * table[id]                      (tlf_embed_shift; an id outside [0, vocab) embeds as zeros)
+ *   h = x_out, or with w_next (no mix) rms_norm(x_out) * w_next, or with mix  v + (v_before - v) * mix  for v = x_out's row and v_before
+ *       the row of the token before (zeros at position 0)
+ * x, x_out fp32 [rows, width]; h, table, weights: dtype; h may be NULL without mix and w_next.  ring fp32 [num_slots, 2, width] holds the
+ * rows before, position p in row p mod 2: a sequence's first row of the step reads it, single rows write it (portions:
+ * tlf_conv_tail with taps 2 on x_out).  row_seq NULL: row r is the one row of sequence r; otherwise rows cu_seqlens_q[s] .. belong to
+ * sequence s and x_out must not be x.  A state slot outside [0, num_slots) reads zeros and is not written.  width <= 16384.
+ * tlf_rows_rmsnorm: rows of x in `groups` equal parts, each / its rms, * w, to out [rows, out_stride] (zeros from cols on). */
+int tlf_post_rmsnorm(const void *y, int64_t y_stride, const float *partials, int32_t splits, const float *scale, const void
+                     *layer_scale, float alpha, const float *x, const void *w, float eps, float *x_out, const void *mix,
+                     float *ring, int64_t num_slots, const int32_t *state_slots, const int32_t *row_seq, const int32_t
+                     *cu_seqlens_q, const int64_t *positions, const void *w_next, void *h, int32_t rows, int32_t width,
+                     int32_t dtype, void *stream);
+int tlf_embed_shift(const int64_t *ids, const void *table, int32_t vocab, float embed_scale, float *x_out, const void *mix,
+                    float *ring, int64_t num_slots, const int32_t *state_slots, const int32_t *row_seq, const int32_t
+                    *cu_seqlens_q, const int64_t *positions, void *h, int32_t rows, int32_t width, int32_t dtype, void
+                    *stream);
+int tlf_rows_rmsnorm(const void *x, int64_t x_stride, const void *w, void *out, int64_t out_stride, int32_t rows, int32_t
+                     cols, int32_t groups, float eps, int32_t dtype, void *stream);
+
+/* Causal grouped-query attention whose heads mix their weights after the softmax, on the caches of the sink attention:
+ *   w_h = softmax(score_scale temp_h (q_h . k));  out_h = sum_j (sum_g talk[h, g] w_g(j)) v(j) of head h's KV head
+ *
+ * tlf_talk_prep: projection rows [q: heads * dim | k: kv_heads * dim | v: kv_heads * vdim] -> q and k / rms over all of q, all of k
+ *   * q_norm, k_norm -> the first rot_dims dimensions of every head turned pairwise (2 i, 2 i + 1) by cos_sin[pos] (cos of the pairs,
+ *   then sin) -> q times temp[head] (NULL: 1) score_scale log2(e) -> q_out [n, heads, Dp] and the cache rows
+ *   slot_mapping[token] (negative: not stored).  heads * Dp <= 32768.
+ * tlf_talk_attn_rows: row r of q attends to positions 0 .. positions[r] of sequence row_seq[r] (NULL: r); slot_mapping[r] < 0: a
+ *   padding row (zeros).  max_len bounds the positions.  talk [heads, heads].  heads <= 1024; bf16 up to 128 heads and 256
+ *   dimensions on the matrix cores.  The workspace holds the scores (4 bytes per row, head and key).
+ * tlf_talk_attn_prefill: portions of sequences first_seq .., rows as in the step; bf16, heads <= 32, dim, vdim <= 128 and a limit
+ *   on kv_heads * vdim (tlf_talk_attn_prefill_supported). */
+int tlf_talk_prep(const void *proj, int64_t proj_stride, const float *partials, int32_t splits, const float *scale, const void
+                  *q_norm, const void *k_norm, const void *temp, const int64_t *positions, const float *cos_sin, int32_t
+                  max_pos, int32_t rot_dims, const int32_t *slot_mapping, void *q_out, void *k_cache, void *v_cache,
+                  int32_t n, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim, int32_t block_size, int64_t
+                  num_pages, float eps, float score_scale, int32_t dtype, void *stream);
+size_t tlf_talk_attn_rows_workspace_bytes(int32_t rows, int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim,
+                                          int32_t max_len, int32_t dtype);
+int tlf_talk_attn_rows(const void *q, const void *k_cache, const void *v_cache, const int32_t *block_tables, int64_t
+                       bt_stride, const int64_t *positions, const int32_t *slot_mapping, const int32_t *row_seq, const
+                       void *talk, void *out, int64_t out_stride, int32_t rows, int32_t heads, int32_t kv_heads, int32_t
+                       dim, int32_t vdim, int32_t block_size, int32_t max_len, int64_t num_pages, int32_t dtype, void
+                       *workspace, size_t workspace_bytes, void *stream);
+int tlf_talk_attn_prefill_supported(int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim);
+int tlf_talk_attn_prefill(const void *q, const void *k_cache, const void *v_cache, const int32_t *block_tables, int64_t
+                          bt_stride, const int32_t *cu_seqlens_q, const int32_t *seq_starts, int32_t first_seq, int32_t
+                          num_seqs, int32_t max_tokens, const void *talk, void *out, int64_t out_stride, int32_t heads,
+                          int32_t kv_heads, int32_t dim, int32_t vdim, int32_t block_size, int64_t num_pages, void
+                          *stream);
+
+/* State-space layer with a scalar decay per head (Mamba-2).  Projection rows [z: inner | x: inner | B: groups * state_dim | C: groups *
+ * state_dim | dt: heads], inner = heads * vdim; head h uses group h / (heads / groups).
+ *   [x | B | C] = silu(conv_bias + sum_j conv[j] u_(p - taps + 1 + j)), zeros before the sequence;  dt = softplus(dt + dt_bias)
+ *   S = exp(-exp(A_log) dt) S + dt B x^T;  out = (S^T C + D x) * silu(z)          state fp32 [slots, heads, state_dim, vdim]
+ * conv [taps, channels of x, B, C]; ring [slots, taps, channels]: projected rows of a sequence's last positions, p in row p mod taps.
+ * Position 0 starts from a zero state.  state_dim, vdim <= 512.
+ *
+ * tlf_ssd_decode: one token per row, ring and state updated; a slot outside [0, num_slots) is a padding row (out = 0).
+ * tlf_ssd_portions: sequences first_seq .. + num_seqs - 1 of at most max_tokens rows, whose rows are the last `rows` of the step,
+ *   from first_row on (positions, row_seq, cu_seqlens_q, proj, out: of the whole step).  The ring is read, not written
+ *   (tlf_conv_tail).  bf16 with state_dim <= 256 on the matrix cores, otherwise token by token. */
+int tlf_ssd_decode(const void *proj, int64_t proj_stride, const float *partials, int32_t splits, const float *scale, const
+                   void *conv, const void *conv_bias, int32_t taps, const void *dt_bias, const void *A_log, const void *D,
+                   void *ring, float *state, const int32_t *state_slots, int32_t num_slots, const int64_t *positions, void
+                   *out, int64_t out_stride, int32_t rows, int32_t heads, int32_t vdim, int32_t state_dim, int32_t groups,
+                   int32_t dtype, void *stream);
+size_t tlf_ssd_portions_workspace_bytes(int32_t rows, int32_t num_seqs, int32_t max_tokens, int32_t heads, int32_t vdim,
+                                        int32_t state_dim, int32_t groups, int32_t dtype);
+int tlf_ssd_portions(const void *proj, int64_t proj_stride, const void *conv, const void *conv_bias, int32_t taps, const void
+                     *dt_bias, const void *A_log, const void *D, void *ring, float *state, const int32_t *state_slots,
+                     int32_t num_slots, const int64_t *positions, const int32_t *row_seq, const int32_t *cu_seqlens_q,
+                     const int32_t *seq_starts, int32_t first_seq, int32_t num_seqs, int32_t first_row, int32_t max_tokens,
+                     void *out, int64_t out_stride, int32_t rows, int32_t heads, int32_t vdim, int32_t state_dim, int32_t
+                     groups, int32_t dtype, void *workspace, size_t workspace_bytes, void *stream);
 
 #ifdef __cplusplus
 }

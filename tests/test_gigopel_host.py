@@ -271,9 +271,9 @@ def test_entry_points_reject_bad_arguments_on_the_host():
     shape = (3, 20, 6, 27, 13)             # heads, dim, rotated dim, latent, value dim
     s = ops.LatentShape(*shape)
     assert (s.da, s.ta, s.ra, s.va, s.dq, s.lp, s.rp) == (24, 8, 32, 16, 32, 64, 32)
-    prep = lambda sizes=shape, ld=120, col=78, q=a, n=2, sp=1, p=None: lib.tlf_latent_prep(
-        a, ld, p, sp, None, col, a, a, a, 10, a, 64, q, a, n, *sizes, 1e-6, 0, None)
-    assert prep(q=None) == -1 and prep(ld=100) == -2 and prep(col=70) == -2 and prep(n=0) == 0 and prep(sp=3) == -1
+    prep = lambda sizes=shape, ld=120, col=78, q=a, n=2, sp=1, p=None, c=a: lib.tlf_latent_prep(
+        a, ld, p, sp, None, col, a, a, a, 10, 0, a, 64, q, c, 0, 0, None, None, 0, 0, None, n, *sizes, 1e-6, 0, None)
+    assert prep(q=None, c=None) == -1 and prep(ld=100) == -2 and prep(col=70) == -2 and prep(n=0) == 0 and prep(sp=3) == -1
     assert prep(sizes=(3, 20, 5, 27, 13)) == -2 and prep(sizes=(3, 20, 6, 2000, 13)) == -2 and prep(sizes=(0, 20, 6, 27, 13)) == -2
     assert lib.tlf_head_gemm(a, a, a, 2, 3, 20, 32, 0, 0, 0, None) == -2 and lib.tlf_head_gemm(a, a, None, 2, 3, 32, 32, 0, 0, 0, None) == -1
     rows = lambda bs=64, win=5, ml=a, dt=0: lib.tlf_latent_rows(a, a, a, 4, a, a, None, a, ml, 2, *shape, bs, win, 10, 0.1, dt, None)
@@ -288,9 +288,9 @@ def test_entry_points_reject_bad_arguments_on_the_host():
     assert layout(2, 10, 40, 576)[1][1:] == [256 + 2 * 10 * 2, 32]           # two passes over 40 heads, a row a job
     assert layout(2, 10, 3, 100)[0] == -2
     assert lib.tlf_latent_attn_plan(a, None, None, None, 0, 0, 2, 1, 3, 64, 5, a, None) == -1
-    values = lambda ld=39, plan=None, uv=a, cu=None: lib.tlf_latent_values(a, a, plan, cu, None, 0, 0, 2, 1, uv, a, ld, 2, *shape, 0, None)
+    values = lambda ld=39, plan=None, uv=a, cu=None: lib.tlf_latent_values(a, a, plan, cu, None, 0, 0, 2, 1, uv, None, a, ld, 2, *shape, 0, None)
     assert values(ld=38) == -2 and values(uv=None) == -1 and values(plan=a, cu=a) == -1
-    pre = lambda sizes=shape, lde=120, win=5: lib.tlf_latent_prefill(a, a, lde, a, a, a, a, 0, 1, 8, None, 39, *sizes, win, 0.1, None)
+    pre = lambda sizes=shape, lde=120, win=5: lib.tlf_latent_prefill(a, a, lde, a, a, a, a, 0, 1, 8, None, None, 39, *sizes, win, 0.1, None)
     assert pre() == -1 and pre(lde=112) == -2 and pre(sizes=(3, 300, 6, 27, 13)) == -5 and pre(win=0) == -2
     assert lib.tlf_latent_gather(a, a, 4, a, a, a, 0, 1, 8, a, 100, 64, 5, 10, None) == -2
     assert lib.tlf_latent_attn_supported(2, 20, 6, 27, 13) == 1 and lib.tlf_latent_attn_supported(2, 20, 64, 600, 13) == 0

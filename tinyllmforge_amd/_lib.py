@@ -90,8 +90,8 @@ SIGNATURES = {
                                    _I32, _I32, _I32, _I32, _F, _F, _F, _I32, _P, _SZ, _P]),
     "tlf_residual_rmsnorm": (c_int32, [_P, _I64, _P, _I32, _P, _P, _I64, _P, _I32, _F, _P, _P, _F, _P, _I32, _I32,
                                        _F, _I32, _P]),
-    "tlf_latent_prep": (c_int32, [_P, _I64, _P, _I32, _P, _I32, _P, _P, _P, _I32, _P, _I64, _P, _P, _I32, _I32, _I32,
-                                  _I32, _I32, _I32, _F, _I32, _P]),
+    "tlf_latent_prep": (c_int32, [_P, _I64, _P, _I32, _P, _I32, _P, _P, _P, _I32, _I32, _P, _I64, _P, _P, _I32, _I32, _P, _P, _I32,
+                                  _I32, _P, _I32, _I32, _I32, _I32, _I32, _I32, _F, _I32, _P]),
     "tlf_head_gemm": (c_int32, [_P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _P]),
     "tlf_latent_rows": (c_int32, [_P, _P, _P, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I32,
                                   _I32, _I64, _F, _I32, _P]),
@@ -99,12 +99,12 @@ SIGNATURES = {
     "tlf_latent_attn_plan": (c_int32, [_P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _P, _P]),
     "tlf_latent_attn": (c_int32, [_P, _P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _P, _P, _P, _I32, _I32,
                                   _I32, _I32, _I32, _I32, _I32, _I64, _F, _P]),
-    "tlf_latent_values": (c_int32, [_P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _P, _P, _I64, _I32, _I32, _I32, _I32,
+    "tlf_latent_values": (c_int32, [_P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _P, _P, _P, _I64, _I32, _I32, _I32, _I32,
                                     _I32, _I32, _I32, _P]),
     "tlf_latent_gather": (c_int32, [_P, _P, _I64, _P, _P, _P, _I32, _I32, _I32, _P, _I32, _I32, _I32, _I64, _P]),
     "tlf_latent_attn_supported": (c_int32, [_I32, _I32, _I32, _I32, _I32]),
     "tlf_latent_prefill_supported": (c_int32, [_I32, _I32, _I32, _I32, _I32]),
-    "tlf_latent_prefill": (c_int32, [_P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P, _I64, _I32, _I32, _I32,
+    "tlf_latent_prefill": (c_int32, [_P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P, _P, _I64, _I32, _I32, _I32,
                                      _I32, _I32, _I32, _F, _P]),
     "tlf_gemm_f32_sums_bytes": (_SZ, [_I32, _I32, _I32]),
     "tlf_gemm_f32_sums": (c_int32, [_P, _I64, _P, _P, _SZ, _I32, _I32, _I32, _P, _P]),
@@ -128,6 +128,23 @@ SIGNATURES = {
     "tlf_sink_attn_prefill_supported": (c_int32, [_I32, _I32]),
     "tlf_sink_attn_prefill": (c_int32, [_P, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _P, _P, _I64, _P, _I64, _I32,
                                         _I32, _I32, _I32, _I32, _I64, _F, _P]),
+    "tlf_post_rmsnorm": (c_int32, [_P, _I64, _P, _I32, _P, _P, _F, _P, _P, _F, _P, _P, _P, _I64, _P, _P, _P, _P, _P,
+                                   _P, _I32, _I32, _I32, _P]),
+    "tlf_embed_shift": (c_int32, [_P, _P, _I32, _F, _P, _P, _P, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _P]),
+    "tlf_rows_rmsnorm": (c_int32, [_P, _I64, _P, _P, _I64, _I32, _I32, _I32, _F, _I32, _P]),
+    "tlf_talk_prep": (c_int32, [_P, _I64, _P, _I32, _P, _P, _P, _P, _P, _P, _I32, _I32, _P, _P, _P, _P, _I32, _I32,
+                                _I32, _I32, _I32, _I32, _I64, _F, _F, _I32, _P]),
+    "tlf_talk_attn_rows_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32, _I32, _I32, _I32]),
+    "tlf_talk_attn_rows": (c_int32, [_P, _P, _P, _P, _I64, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32,
+                                     _I32, _I32, _I64, _I32, _P, _SZ, _P]),
+    "tlf_talk_attn_prefill_supported": (c_int32, [_I32, _I32, _I32, _I32]),
+    "tlf_talk_attn_prefill": (c_int32, [_P, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _P, _P, _I64, _I32, _I32,
+                                        _I32, _I32, _I32, _I64, _P]),
+    "tlf_ssd_decode": (c_int32, [_P, _I64, _P, _I32, _P, _P, _P, _I32, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _I64,
+                                 _I32, _I32, _I32, _I32, _I32, _I32, _P]),
+    "tlf_ssd_portions_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32, _I32, _I32, _I32, _I32]),
+    "tlf_ssd_portions": (c_int32, [_P, _I64, _P, _P, _I32, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _P, _P, _I32, _I32,
+                                   _I32, _I32, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32, _P, _SZ, _P]),
     "tlf_probe_read": (c_int32, [_P, _SZ, _P, _P]),
     "tlf_probe_copy": (c_int32, [_P, _P, _SZ, _P]),
     "tlf_probe_mfma": (c_int32, [_P, c_int32, c_int32, _P]),

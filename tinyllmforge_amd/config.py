@@ -205,6 +205,48 @@ class ZuzunexConfig(LayeredConfig):
         return [*range(start), *list(range(start, stop)) * self.loop["times"], *range(stop, len(self.layers))]
 
 
+NO_WINDOW = 1 << 30      # an attention window that every position is inside of
+
+
+@dataclass
+class TibenexConfig(LayeredConfig):
+    """A Tibenex model: post-norm layers of latent attention, of attention whose heads mix their weights or of a state-space
+    recurrence, each with an optional dense feed-forward, and a token shift in front of every mixer.
+
+    Keys of ``config.json``: ``vocab``, ``width``, ``embedding`` (``scale``), ``postln_alpha``, ``norm`` (``eps``) and ``layers``; a
+    layer has ``type``, ``mixer`` and ``mlp`` (null, or ``kind`` 'dense' with ``ff``).  ``mixer`` of 'latent_attention': ``heads``,
+    ``dim``, ``rot_dim``, ``vdim``, ``q_rank``, ``kv_rank``, ``scale``, ``rot`` (``dims``, ``base``, ``scaling``: null or ``factor``,
+    ``original``, ``fast``, ``slow``); of 'attention': ``heads``, ``kv_heads``, ``dim``, ``vdim``, ``scale``, ``rot``; of 'mamba2':
+    ``heads``, ``vdim``, ``state``, ``groups``, ``conv`` (taps), ``norm_groups``."""
+    embedding: dict | None = None
+    postln_alpha: float = 1.0
+
+    recurrent = True         # every layer keeps the row before
+
+    # portions from about this many tokens on expand the keys and values of latent attention, and share the keys of a tile
+    # in the others; shorter ones run row by row
+    long_portion = 128
+
+    @property
+    def embedding_scale(self) -> float:
+        return float((self.embedding or {}).get("scale", 1.0))
+
+    def check_layers(self):
+        for layer in self.layers:
+            m, kind, mlp = layer["mixer"], layer["type"], layer.get("mlp")
+            if kind == "latent_attention":
+                assert m["rot"]["dims"] == m["rot_dim"] and m["rot_dim"] % 2 == 0 and m["q_rank"] >= 1
+            elif kind == "attention":
+                assert m["heads"] % m["kv_heads"] == 0
+                assert not m.get("rot") or (m["rot"]["dims"] % 2 == 0 and m["rot"]["dims"] <= m["dim"])
+            else:
+                assert kind == "mamba2", f"unknown mixer {kind!r}"
+                assert m["heads"] % m["groups"] == 0 and m["conv"] >= 1 and m["heads"] * m["vdim"] % m["norm_groups"] == 0
+            assert not mlp or mlp["kind"] == "dense"
+        if any(layer["type"] == "latent_attention" for layer in self.layers):
+            self.windows = (NO_WINDOW,)
+
+
 def tensor_shapes(directory: str) -> dict:
     """name -> shape of every tensor in ``directory/*.safetensors``, from the files' headers."""
     from glob import glob
@@ -216,7 +258,7 @@ def tensor_shapes(directory: str) -> dict:
     return out
 
 
-LAYERED_DESIGNS = {"Gitopel": GitopelConfig, "Gigopel": GigopelConfig, "Zuzunex": ZuzunexConfig}
+LAYERED_DESIGNS = {"Gitopel": GitopelConfig, "Gigopel": GigopelConfig, "Zuzunex": ZuzunexConfig, "Tibenex": TibenexConfig}
 
 
 def architecture_of(src: dict) -> str:

@@ -37,6 +37,8 @@ EXTRA_FLAGS = {
     "pooled_prefill.hip": ["-fno-honor-nans"],
     "sink_prefill.hip": ["-fno-honor-nans"],
     "sink_decode.hip": ["-fno-honor-nans"],
+    "talk_prefill.hip": ["-fno-honor-nans"],
+    "talk_decode.hip": ["-fno-honor-nans"],
 }
 
 

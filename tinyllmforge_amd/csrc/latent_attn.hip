@@ -1,7 +1,7 @@
 // Latent attention (geometry in latent_attn.h): everything but the two matrix-core attention kernels.
 //
 //   latent_prep_kernel    projection row [q | latent | rotated key] -> rotated queries, normed latent and rotated key into
-//                         the paged cache
+//                         the paged cache; where queries come through a latent of their own, that one normed; output gates
 //   head_gemm_kernel      y[row, h] = W[h] x[row, h] for every head (the queries' way into the latent space)
 //   latent_rows_kernel    one workgroup per (query row, head): 32-bit mode, and sizes the matrix-core kernel does not take
 //   latent_values_kernel  sum of the key splits, softmax denominator, Uv_h
@@ -26,6 +26,12 @@ struct LatentPrepArgs {
   void *cache;              // [slots, Lp]
   int32_t n, vec;           // vec: parts of a projection row may be read 8 elements at a time
   float eps;
+  int32_t halves;           // rotation: pairs (i, i + rot / 2) instead of (2 i, 2 i + 1)
+  int32_t latents;          // blockIdx.y == 0 prepares latents (and gates); then query latents, then queries
+  const void *cq_norm;      // [cq_rank] or NULL
+  void *cq_out;             // [n, cq_ld], zeros from cq_rank on
+  int32_t cq_col, cq_rank, cq_ld, gate_col;
+  float *gate_out;          // [n, H] or NULL: sigmoid
 };
 
 template <typename T, bool PART>
@@ -57,16 +63,80 @@ __device__ __forceinline__ void turn8(const LatentPrepArgs &a, const float *cs, 
   }
 }
 
-// blockIdx.y == 0: the latents of TOK tokens, a wave each; otherwise 256 8-value pieces of those tokens' queries, all loads
-// in flight before the first is used
+// Piece d .. d + 7 of the rotated part that begins at column `col`, partners rot / 2 away.
+template <typename T, bool PART>
+__device__ __forceinline__ void turn8_halves(const LatentPrepArgs &a, const float *cs, int64_t tok, int col, int d, float (&f)[8]) {
+  if (cs == nullptr) return;
+  const int half = a.s.rot / 2;
+  float p[8];
+  if (a.vec && half % 8 == 0) {
+    prep_ld8<T, PART>(a, tok, col, d < half ? d + half : d - half, a.s.rot, p);
+  } else {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int i = d + e;
+      p[e] = i < a.s.rot ? prep_ld<T, PART>(a, tok, col + (i < half ? i + half : i - half)) : 0.f;
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const int i = d + e;
+    if (i < half) f[e] = __fmul_rn(f[e], cs[i]) - __fmul_rn(p[e], cs[half + i]);
+    else if (i < a.s.rot) f[e] = __fmul_rn(f[e], cs[i - half]) + __fmul_rn(p[e], cs[i]);
+  }
+}
+
+// blockIdx.y == 0 with `latents`: the latents of TOK tokens, a wave each; then, with cq_norm, their query latents; then 256
+// 8-value pieces of those tokens' queries, all loads in flight before the first is used
 template <typename T, bool PART, int TOK>
 __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a) {
   const LatentShape &s = a.s;
   const int64_t tok0 = static_cast<int64_t>(blockIdx.x) * TOK;
-  if (blockIdx.y == 0) {
+  if (a.cq_norm && static_cast<int>(blockIdx.y) == a.latents) {
     const int64_t tok = tok0 + (threadIdx.x >> 6);
     const int lane = threadIdx.x & 63;
     if ((threadIdx.x >> 6) >= TOK || tok >= a.n) return;   // whole waves leave together
+    const T *w = static_cast<const T *>(a.cq_norm);
+    T *row = static_cast<T *>(a.cq_out) + tok * a.cq_ld;
+    constexpr int kKeep = 2;                               // pieces of 8 a lane holds, longer rows are read twice
+    float f[kKeep][8], ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < kKeep; ++k) {
+      const int d = (lane + k * 64) * 8;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) f[k][e] = 0.f;
+      if (d < a.cq_rank) prep_ld8<T, PART>(a, tok, a.cq_col, d, a.cq_rank, f[k]);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss = fmaf(f[k][e], f[k][e], ss);
+    }
+    for (int d = (lane + kKeep * 64) * 8; d < a.cq_rank; d += 512) {
+      float t[8];
+      prep_ld8<T, PART>(a, tok, a.cq_col, d, a.cq_rank, t);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss = fmaf(t[e], t[e], ss);
+    }
+    ss = wave_sum(ss);
+    const float inv = 1.0f / sqrtf(ss / static_cast<float>(a.cq_rank) + a.eps);
+    for (int d = lane * 8, k = 0; d < a.cq_ld; d += 512, ++k) {
+      float t[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+      if (d < a.cq_rank) {
+        if (k >= kKeep) prep_ld8<T, PART>(a, tok, a.cq_col, d, a.cq_rank, t);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          if (k < kKeep) t[e] = k == 0 ? f[0][e] : f[1][e];
+          t[e] = d + e < a.cq_rank ? t[e] * inv * Elem<T>::ld(w + d + e) : 0.f;
+        }
+      }
+      Elem<T>::st8(row + d, t);
+    }
+    return;
+  }
+  if (a.latents && blockIdx.y == 0) {
+    const int64_t tok = tok0 + (threadIdx.x >> 6);
+    const int lane = threadIdx.x & 63;
+    if ((threadIdx.x >> 6) >= TOK || tok >= a.n) return;   // whole waves leave together
+    if (a.gate_out)
+      for (int h = lane; h < s.H; h += 64) a.gate_out[tok * s.H + h] = sigmoid_f32(prep_ld<T, PART>(a, tok, a.gate_col + h));
     const int64_t slot = a.slots[tok], pos = a.positions[tok];
     const float *cs = pos >= 0 && pos < a.max_pos ? a.cos_sin + pos * s.rot : nullptr;
     constexpr int kKeep = 3;   // pieces of 8 a lane holds: rank <= 1536
@@ -104,13 +174,16 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a
         for (int e = 0; e < 8; ++e) t[e] = 0.f;
         if (d < s.rot) prep_ld8<T, PART>(a, tok, a.off + s.rank, d, s.rot, t);
       }
-      if (d < s.rot) turn8(a, cs, d, t);
+      if (d < s.rot) {
+        if (a.halves) turn8_halves<T, PART>(a, cs, tok, a.off + s.rank, d, t);
+        else turn8(a, cs, d, t);
+      }
       Elem<T>::st8(row + s.Ra + d, t);
     }
     return;
   }
   const int nch = s.Dq / 8;
-  const int item = (blockIdx.y - 1) * 256 + threadIdx.x;
+  const int item = (blockIdx.y - a.latents - (a.cq_norm ? 1 : 0)) * 256 + threadIdx.x;
   if (item >= s.H * nch) return;
   const int h = item / nch, d = (item - h * nch) * 8;
   const int col = h * (s.dim + s.rot);
@@ -129,7 +202,11 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a
 #pragma unroll
   for (int k = 0; k < TOK; ++k) {
     if (tok0 + k >= a.n) return;
-    if (turned) turn8(a, pos[k] >= 0 && pos[k] < a.max_pos ? a.cos_sin + pos[k] * s.rot : nullptr, d - s.Da, f[k]);
+    if (turned) {
+      const float *cs = pos[k] >= 0 && pos[k] < a.max_pos ? a.cos_sin + pos[k] * s.rot : nullptr;
+      if (a.halves) turn8_halves<T, PART>(a, cs, tok0 + k, col + s.dim, d - s.Da, f[k]);
+      else turn8(a, cs, d - s.Da, f[k]);
+    }
     Elem<T>::st8(static_cast<T *>(a.q_out) + ((tok0 + k) * s.H + h) * s.Dq + d, f[k]);
   }
 }
@@ -258,6 +335,7 @@ struct LatentValuesArgs {
   LatentJobs jb;
   const int32_t *row_seq;   // [rows] with jb.cu_q: sequence of a row
   const void *uv;           // [H, Vp, Rp], Vp = vdim rounded up to 16
+  const float *gate;        // [rows, H] or NULL
   void *out;                // [rows, ldo]
   int64_t ldo;
   int32_t rows, Vp, wgs;
@@ -366,6 +444,7 @@ __global__ __launch_bounds__(256) void latent_values_kernel(const LatentValuesAr
   }
   const int row = row0 + n;
   if (row >= a.rows) return;
+  if (a.gate) acc *= a.gate[static_cast<int64_t>(row) * s.H + h];
   unsigned short *o = static_cast<unsigned short *>(a.out) + row * a.ldo + static_cast<int64_t>(h) * s.vdim + v0 + g * 4;
 #pragma unroll
   for (int e = 0; e < 4; ++e)
@@ -393,6 +472,7 @@ __global__ __launch_bounds__(256) void latent_values_rows_kernel(const LatentVal
     const T *w = static_cast<const T *>(a.uv) + (static_cast<int64_t>(h) * a.Vp + v) * s.Rp;
     float o = 0.f;
     for (int r = 0; r < s.rank; ++r) o = fmaf(mixed[r], Elem<T>::ld(w + r), o);
+    if (a.gate) o *= a.gate[static_cast<int64_t>(row) * s.H + h];
     Elem<T>::st(static_cast<T *>(a.out) + row * a.ldo + static_cast<int64_t>(h) * s.vdim + v, o);
   }
 }
@@ -418,25 +498,33 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(const LatentCache c,
 
 extern "C" int tlf_latent_prep(const void *proj, int64_t proj_stride, const float *partials, int32_t splits,
                                const float *scale, int32_t latent_col, const void *norm_weight, const int64_t *positions,
-                               const float *cos_sin, int32_t max_pos, const int32_t *slot_mapping, int64_t num_slots,
-                               void *q_out, void *cache, int32_t n, int32_t heads, int32_t dim, int32_t rot_dim,
-                               int32_t rank, int32_t vdim, float eps, int32_t dtype, void *stream) {
+                               const float *cos_sin, int32_t max_pos, int32_t halves, const int32_t *slot_mapping,
+                               int64_t num_slots, void *q_out, void *cache, int32_t cq_col, int32_t cq_rank, const void *cq_norm,
+                               void *cq_out, int32_t cq_stride, int32_t gate_col, float *gate_out, int32_t n, int32_t heads,
+                               int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, float eps, int32_t dtype, void *stream) {
   using namespace tlf;
   LatentPrepArgs a{};
   if (n < 0 || !latent_shape(a.s, heads, dim, rot_dim, rank, vdim)) return TLF_E_SHAPE;
-  if (latent_col < heads * (dim + rot_dim) || proj_stride < latent_col + rank + rot_dim) return TLF_E_SHAPE;
+  if (!q_out && !cache) return TLF_E_NULL;
+  if (q_out && proj_stride < heads * (dim + rot_dim)) return TLF_E_SHAPE;
+  if (cache && (latent_col < (q_out ? heads * (dim + rot_dim) : 0) || proj_stride < latent_col + rank + rot_dim)) return TLF_E_SHAPE;
+  if (cq_norm && (cq_rank <= 0 || cq_col < 0 || proj_stride < cq_col + cq_rank || cq_stride < cq_rank || cq_stride % 8)) return TLF_E_SHAPE;
+  if (gate_out && (!cache || gate_col < 0 || proj_stride < gate_col + heads)) return TLF_E_SHAPE;
   if (dtype != TLF_DT_BF16 && dtype != TLF_DT_F32) return TLF_E_UNSUPPORTED;
   if (n == 0) return TLF_OK;
   if (int rc = partials_check(partials, scale, splits, dtype)) return rc;
-  if ((!proj && splits <= 1) || !norm_weight || !positions || (rot_dim && !cos_sin) || !slot_mapping || !q_out || !cache) return TLF_E_NULL;
-  if (!aligned16(q_out) || !aligned16(cache)) return TLF_E_ALIGN;
+  if ((!proj && splits <= 1) || !positions || (rot_dim && !cos_sin) || (cache && (!slot_mapping || !norm_weight)) || (cq_norm && !cq_out)) return TLF_E_NULL;
+  if (!aligned16(q_out) || !aligned16(cache) || !aligned16(cq_out)) return TLF_E_ALIGN;
   a.proj = proj; a.ld = proj_stride; a.off = latent_col; a.norm = norm_weight; a.positions = positions; a.cos_sin = cos_sin;
   a.part = Partials{partials, scale, n * proj_stride, static_cast<int32_t>(proj_stride), splits};
   a.max_pos = max_pos; a.slots = slot_mapping; a.num_slots = num_slots; a.q_out = q_out; a.cache = cache; a.n = n; a.eps = eps;
-  a.vec = dim % 8 == 0 && rot_dim % 8 == 0 && rank % 8 == 0 && latent_col % 8 == 0 && proj_stride % 8 == 0 &&
-          (splits > 1 || aligned16(proj));
+  a.halves = halves; a.latents = cache ? 1 : 0;
+  a.cq_norm = cq_norm; a.cq_out = cq_out; a.cq_col = cq_col; a.cq_rank = cq_rank; a.cq_ld = cq_stride;
+  a.gate_col = gate_col; a.gate_out = gate_out;
+  a.vec = dim % 8 == 0 && rot_dim % 8 == 0 && proj_stride % 8 == 0 && (splits > 1 || aligned16(proj)) &&
+          (!cache || (rank % 8 == 0 && latent_col % 8 == 0)) && (!cq_norm || (cq_rank % 8 == 0 && cq_col % 8 == 0));
   const int tok = splits <= 1 && n > 1024 ? 4 : 1;
-  const dim3 grid((n + tok - 1) / tok, 1 + (heads * (a.s.Dq / 8) + 255) / 256);
+  const dim3 grid((n + tok - 1) / tok, a.latents + (cq_norm ? 1 : 0) + (q_out ? (heads * (a.s.Dq / 8) + 255) / 256 : 0));
   hipStream_t s = static_cast<hipStream_t>(stream);
 #define TLF_PREP(T, PART)                                                                        \
   do {                                                                                           \
@@ -503,7 +591,7 @@ extern "C" int tlf_latent_rows(const void *q, const void *cache, const int32_t *
 
 extern "C" int tlf_latent_values(const float *part, const float *ml, const int32_t *plan, const int32_t *cu_seqlens_q,
                                  const int32_t *row_seq, int32_t first_seq, int32_t first_row, int32_t num_seqs,
-                                 int32_t max_tokens, const void *uv, void *out, int64_t out_stride, int32_t rows, int32_t heads,
+                                 int32_t max_tokens, const void *uv, const float *gate, void *out, int64_t out_stride, int32_t rows, int32_t heads,
                                  int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, int32_t dtype, void *stream) {
   using namespace tlf;
   LatentValuesArgs a{};
@@ -513,7 +601,7 @@ extern "C" int tlf_latent_values(const float *part, const float *ml, const int32
   if (rows == 0) return TLF_OK;
   if (!part || !ml || !uv || !out || (plan && cu_seqlens_q && !row_seq)) return TLF_E_NULL;
   if (!aligned16(part) || !aligned16(uv)) return TLF_E_ALIGN;
-  a.part = part; a.ml = ml; a.uv = uv; a.out = out; a.ldo = out_stride; a.rows = rows;
+  a.part = part; a.ml = ml; a.uv = uv; a.gate = gate; a.out = out; a.ldo = out_stride; a.rows = rows;
   a.Vp = round_up_to(vdim, 16);
   if (plan) {
     if (num_seqs <= 0 || max_tokens <= 0 || first_seq < 0 || (!cu_seqlens_q && rows > num_seqs)) return TLF_E_SHAPE;

@@ -22,6 +22,7 @@ struct LatentPrefillArgs {
   const unsigned short *expanded;   // [kv rows, lde]: H * Da, then H * Va
   const unsigned short *latents;    // [kv rows, Lp]
   const int32_t *cu_q, *starts, *kv_off;
+  const float *gate;                // [rows, H] or NULL
   unsigned short *out;              // [rows, ldo]
   int64_t lde, ldo;
   int32_t first_seq, window, xtiles, total, per_xcd;
@@ -216,7 +217,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) voi
   for (int k = 0; k < CT; ++k) {
     const float den = sum_lanes_16_32_48(l[k]);
     if (!uok[k]) continue;
-    const float inv = 1.0f / den;                            // a row sees itself: den > 0
+    float inv = 1.0f / den;                                  // a row sees itself: den > 0
+    if (p.gate) inv *= p.gate[static_cast<int64_t>(q0 + upos[k] - start) * s.H + h];
     unsigned short *o = p.out + static_cast<int64_t>(q0 + upos[k] - start) * p.ldo + static_cast<int64_t>(h) * s.vdim;
 #pragma unroll
     for (int d = 0; d < 2 * VC; ++d) {
@@ -245,7 +247,7 @@ extern "C" int tlf_latent_prefill_supported(int32_t heads, int32_t dim, int32_t 
 
 extern "C" int tlf_latent_prefill(const void *q, const void *expanded, int64_t expanded_stride, const void *latents,
                                   const int32_t *cu_seqlens_q, const int32_t *seq_starts, const int32_t *kv_offsets,
-                                  int32_t first_seq, int32_t num_seqs, int32_t max_tokens, void *out, int64_t out_stride,
+                                  int32_t first_seq, int32_t num_seqs, int32_t max_tokens, const float *gate, void *out, int64_t out_stride,
                                   int32_t heads, int32_t dim, int32_t rot_dim, int32_t rank, int32_t vdim, int32_t window,
                                   float scale, void *stream) {
   using namespace tlf;
@@ -259,7 +261,7 @@ extern "C" int tlf_latent_prefill(const void *q, const void *expanded, int64_t e
   a.q = static_cast<const unsigned short *>(q); a.expanded = static_cast<const unsigned short *>(expanded);
   a.latents = static_cast<const unsigned short *>(latents); a.cu_q = cu_seqlens_q; a.starts = seq_starts; a.kv_off = kv_offsets;
   a.out = static_cast<unsigned short *>(out); a.lde = expanded_stride; a.ldo = out_stride; a.first_seq = first_seq;
-  a.window = window; a.scale_log2 = scale * 1.4426950408889634f;
+  a.gate = gate; a.window = window; a.scale_log2 = scale * 1.4426950408889634f;
   a.xtiles = (max_tokens + kPQ - 1) / kPQ;
   const int64_t total = static_cast<int64_t>(a.xtiles) * heads * num_seqs;
   if (total > (1 << 30)) return TLF_E_SHAPE;

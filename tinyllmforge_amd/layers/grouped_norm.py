@@ -11,7 +11,7 @@ class GroupedRMSNorm(nn.Module):
         self.groups, self.eps = groups, eps
         self.weight = nn.Parameter(torch.ones(size))
 
-    def after_embedding(self, ids: torch.Tensor, table: torch.Tensor):
+    def after_embedding(self, ids: torch.Tensor, table: torch.Tensor, positions=None):
         """``(x, self(x))`` with ``x`` the fp32 embedding rows."""
         return ops.embed_group_rms_norm(ids, table, self.weight.data, self.groups, self.eps)
 

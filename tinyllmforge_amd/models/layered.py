@@ -1,7 +1,8 @@
 """What designs with a list of unlike layers share: rotation tables, the forward loop, checkpoint names, packing.
 
-A layer is a module with ``norm1`` (the norm in front of it), ``forward(positions, h, x, following)`` that updates the fp32
-residual ``x`` in place and returns it normed by ``following``, and ``routes()``: checkpoint names below ``l<i>.`` ->
+A layer is a module with what turns the stream into its input (the attribute that ``front`` names: the norm in front of it, or a
+token shift), ``forward(positions, h, x, following)`` that updates the fp32 stream ``x`` in place and returns it as ``following``
+makes it the next input, and ``routes()``: checkpoint names below ``l<i>.`` ->
 (parameter below the layer, part of it or None).  A layer that runs more than once takes ``run=`` (0, 1, ...) and keeps a cache
 and a state of its own per run."""
 import re
@@ -19,6 +20,7 @@ def prefixed(prefix: str, routes: dict) -> dict:
 
 
 class LayeredForCausalLM(nn.Module):
+    front = "norm1"
     fixed_tensors = {"embed": ("embed", None), "final.norm": ("norm.weight", None)}
 
     def __init__(self, config):
@@ -40,18 +42,18 @@ class LayeredForCausalLM(nn.Module):
         return self._rope_tables[key]
 
     def runs(self):
-        """The layers in the order they run, ``(norm in front, call)``."""
+        """The layers in the order they run, ``(what makes its input, call)``."""
         order, seen = self.config.layer_runs(), {}
         for i in order:
             run = seen[i] = seen.get(i, -1) + 1
             layer = self.layers[i]
-            yield layer.norm1, partial(layer, run=run) if order.count(i) > 1 else layer
+            yield getattr(layer, self.front), partial(layer, run=run) if order.count(i) > 1 else layer
 
     def forward(self, input_ids: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
         runs = list(self.runs())
-        norms = [norm for norm, _ in runs] + [self.norm]
-        x, h = norms[0].after_embedding(input_ids, self.embed.data)
-        for (_, layer), following in zip(runs, norms[1:]):
+        fronts = [front for front, _ in runs] + [self.norm]
+        x, h = fronts[0].after_embedding(input_ids, self.embed.data, positions)
+        for (_, layer), following in zip(runs, fronts[1:]):
             h = layer(positions, h, x, following)
         return h
 

@@ -812,18 +812,50 @@ class LatentShape:
 
 def latent_prep(proj, latent_col, norm_weight, positions, cos_sin, slot_mapping, cache, shape: LatentShape, eps):
     """Rotated queries ``[N, H, Dq]``; the normed latent and the rotated key part go to ``cache [pages, bs, Lp]``."""
-    lib = _lib.load()
-    assert proj.dtype == cache.dtype == norm_weight.dtype and cache.is_contiguous() and cache.shape[2] == shape.lp
-    _need(positions, torch.int64, "positions"); _need(slot_mapping, torch.int32, "slot_mapping")
-    n = proj.shape[0]
-    assert positions.numel() == n and slot_mapping.numel() == n and norm_weight.numel() == shape.rank
-    assert cos_sin is None or cos_sin.shape[1] == shape.rot
-    q = torch.empty(n, shape.heads, shape.dq, dtype=proj.dtype, device=proj.device)
-    check(lib.tlf_latent_prep(*_source(proj), latent_col, norm_weight.data_ptr(), positions.data_ptr(), _opt(cos_sin),
-                              cos_sin.shape[0] if cos_sin is not None else 0, slot_mapping.data_ptr(),
-                              cache.shape[0] * cache.shape[1], q.data_ptr(), cache.data_ptr(), n, *shape.sizes, float(eps),
-                              _dt(proj), _stream()), "tlf_latent_prep")
+    q = _latent_queries(proj, shape)
+    _latent_prep(proj, positions, cos_sin, shape, eps, False, q=q, cache=cache, latent_col=latent_col, norm=norm_weight, slot_mapping=slot_mapping)
     return q
+
+
+def latent_prep_queries(proj, positions, cos_sin, shape: LatentShape, halves: bool):
+    """Rotated queries ``[N, H, Dq]`` from rows of their own."""
+    q = _latent_queries(proj, shape)
+    _latent_prep(proj, positions, cos_sin, shape, 1.0, halves, q=q)
+    return q
+
+
+def latent_prep_down(proj, latent_col, norm_weight, positions, cos_sin, slot_mapping, cache, shape: LatentShape, eps, halves: bool,
+                     cq_col=0, cq_norm=None, gate_col=None):
+    """The latent and the rotated key into the cache; ``(normed query latent or None, gates fp32 [N, H] or None)``: the columns
+    from ``cq_col`` on (padded with zeros to a multiple of 64) and sigmoids of those from ``gate_col`` on."""
+    n, dev = proj.shape[0], cache.device
+    cq = torch.empty(n, -(-cq_norm.numel() // 64) * 64, dtype=cache.dtype, device=dev) if cq_norm is not None else None
+    gate = torch.empty(n, shape.heads, dtype=torch.float32, device=dev) if gate_col is not None else None
+    _latent_prep(proj, positions, cos_sin, shape, eps, halves, cache=cache, latent_col=latent_col, norm=norm_weight,
+                 slot_mapping=slot_mapping, cq_col=cq_col, cq_norm=cq_norm, cq=cq, gate_col=gate_col or 0, gate=gate)
+    return cq, gate
+
+
+def _latent_queries(proj, shape):
+    return torch.empty(proj.shape[0], shape.heads, shape.dq, dtype=proj.dtype, device=proj.device)
+
+
+def _latent_prep(proj, positions, cos_sin, shape, eps, halves, q=None, cache=None, latent_col=0, norm=None, slot_mapping=None,
+                 cq_col=0, cq_norm=None, cq=None, gate_col=0, gate=None):
+    lib = _lib.load()
+    n = proj.shape[0]
+    _need(positions, torch.int64, "positions")
+    assert positions.numel() == n and (cos_sin is None or cos_sin.shape[1] == shape.rot)
+    if cache is not None:
+        _need(slot_mapping, torch.int32, "slot_mapping")
+        assert proj.dtype == cache.dtype == norm.dtype and cache.is_contiguous() and cache.shape[2] == shape.lp
+        assert slot_mapping.numel() == n and norm.numel() == shape.rank
+    assert cq_norm is None or cq_norm.dtype == proj.dtype
+    check(lib.tlf_latent_prep(*_source(proj), latent_col, _opt(norm), positions.data_ptr(), _opt(cos_sin),
+                              cos_sin.shape[0] if cos_sin is not None else 0, int(halves), _opt(slot_mapping),
+                              cache.shape[0] * cache.shape[1] if cache is not None else 0, _opt(q), _opt(cache), cq_col,
+                              cq_norm.numel() if cq_norm is not None else 0, _opt(cq_norm), _opt(cq), cq.shape[1] if cq is not None else 0,
+                              gate_col, _opt(gate), n, *shape.sizes, float(eps), _dt(proj), _stream()), "tlf_latent_prep")
 
 
 def head_gemm(x, w, n_main=0, k_main=0):
@@ -920,17 +952,24 @@ def latent_attention(q, cache, block_tables, window, scale, shape: LatentShape, 
     return part, ml
 
 
-def latent_values(part, ml, uv, out, shape: LatentShape, batch: LatentBatch | None = None, plan=None):
-    """``out [N, >= H * vdim]`` from the pieces' mixed latents; ``uv [H, vdim rounded up to 16, Rp]``."""
+def _check_gate(gate, rows, shape):
+    if gate is not None:
+        _need(gate, torch.float32, "gate")
+        assert gate.is_contiguous() and gate.shape == (rows, shape.heads)
+
+
+def latent_values(part, ml, uv, out, shape: LatentShape, batch: LatentBatch | None = None, plan=None, gate=None):
+    """``out [N, >= H * vdim]`` from the pieces' mixed latents; ``uv [H, vdim rounded up to 16, Rp]``, ``gate`` fp32 ``[N, H]``."""
     lib = _lib.load()
     rows = out.shape[0]
     assert out.stride(1) == 1 and out.dtype == uv.dtype and part.is_contiguous() and uv.is_contiguous()
     assert plan is not None or part.shape[0] == rows
+    _check_gate(gate, rows, shape)
     where = (None, None, 0, 0, 0, 0)
     if plan is not None:
         where = (_opt(batch.cu_seqlens_q), _opt(batch.row_seq), batch.first_seq, batch.first_row, batch.num_seqs, batch.max_tokens)
         assert batch.row_seq is None or batch.row_seq.numel() >= rows
-    check(lib.tlf_latent_values(part.data_ptr(), ml.data_ptr(), _opt(plan), *where, uv.data_ptr(), out.data_ptr(),
+    check(lib.tlf_latent_values(part.data_ptr(), ml.data_ptr(), _opt(plan), *where, uv.data_ptr(), _opt(gate), out.data_ptr(),
                                 out.stride(0), rows, *shape.sizes, _dt(uv), _stream()), "tlf_latent_values")
 
 
@@ -947,16 +986,17 @@ def latent_gather(cache, block_tables, cu_seqlens_q, seq_starts, kv_offsets, kv_
 
 
 def latent_prefill(q, expanded, latents, cu_seqlens_q, seq_starts, kv_offsets, first_seq, num_seqs, max_tokens, window, scale,
-                   shape: LatentShape, out):
-    """Portions from expanded keys and values; ``q`` and ``out`` are indexed by the step's rows."""
+                   shape: LatentShape, out, gate=None):
+    """Portions from expanded keys and values; ``q``, ``out`` and ``gate`` are indexed by the step's rows."""
     lib = _lib.load()
+    _check_gate(gate, q.shape[0], shape)
     _need(q, BF16, "q"); _need(expanded, BF16, "expanded"); _need(latents, BF16, "latents")
     assert q.is_contiguous() and q.shape[1:] == (shape.heads, shape.dq) and out.stride(1) == 1
     assert expanded.stride(1) == 1 and latents.is_contiguous() and latents.shape[1] == shape.lp
     check(lib.tlf_latent_prefill(q.data_ptr(), expanded.data_ptr(), expanded.stride(0), latents.data_ptr(),
                                  cu_seqlens_q.data_ptr(), seq_starts.data_ptr(), kv_offsets.data_ptr(), first_seq, num_seqs,
-                                 max_tokens, out.data_ptr(), out.stride(0), *shape.sizes, window, float(scale), _stream()),
-          "tlf_latent_prefill")
+                                 max_tokens, _opt(gate), out.data_ptr(), out.stride(0), *shape.sizes, window, float(scale),
+                                 _stream()), "tlf_latent_prefill")
     return out
 
 
@@ -1080,6 +1120,180 @@ def sink_attention_prefill(q, kv: SinkKV, block_tables, cu_seqlens_q, seq_starts
         seq_starts.data_ptr(), first_seq, num_seqs, max_tokens, _opt(sink), _opt(gate), gate.stride(0) if gate is not None else 0,
         out.data_ptr(), out.stride(0), heads, G, kv.dim, kv.vdim, bs, pages, float(cap or 0), _stream()),
         "tlf_sink_attn_prefill")
+    return out
+
+
+# ------------------------------------------------------------------ post-norm and token shift
+class ShiftArguments:
+    """Token shift: ``mix [W]``, the rows before (``ring`` fp32 ``[slots, 2, W]``), and where a step's rows belong (``row_seq`` None:
+    row r is the one row of sequence r)."""
+    __slots__ = ("mix", "ring", "state_slots", "positions", "row_seq", "cu_seqlens_q")
+
+    def __init__(self, mix, ring, state_slots, positions, row_seq=None, cu_seqlens_q=None):
+        self.mix, self.ring, self.state_slots, self.positions = mix, ring, state_slots, positions
+        self.row_seq, self.cu_seqlens_q = row_seq, cu_seqlens_q
+
+    def pointers(self, rows, width, dtype):
+        _need(self.ring, torch.float32, "ring"); _need(self.state_slots, torch.int32, "state_slots")
+        _need(self.positions, torch.int64, "positions")
+        assert self.mix.numel() == width and self.mix.dtype == dtype and self.ring.is_contiguous() and self.ring.shape[1:] == (2, width)
+        assert self.positions.numel() == rows and (self.row_seq is not None or self.state_slots.numel() >= rows)
+        assert self.row_seq is None or (self.row_seq.numel() == rows and self.cu_seqlens_q.dtype == torch.int32)
+        return (self.mix.data_ptr(), self.ring.data_ptr(), self.ring.shape[0], self.state_slots.data_ptr(), _opt(self.row_seq),
+                _opt(self.cu_seqlens_q), self.positions.data_ptr())
+
+
+def post_rms_norm(y, x, alpha, layer_scale, w, eps, shift: ShiftArguments | None = None, w_next=None):
+    """``x' = rms_norm(alpha x + layer_scale * y) * w`` (``x`` fp32 ``[N, W]``; in place unless portions are shifted) and in w's
+    dtype its rows, shifted rows or ``rms_norm(x') * w_next``.  Returns ``(x', rows)``."""
+    lib = _lib.load()
+    _need(x, torch.float32, "x"); _need(w, y.dtype, "w"); _need(layer_scale, y.dtype, "layer_scale")
+    rows, width = x.shape
+    assert y.shape[0] == rows and y.shape[1] >= width and x.is_contiguous() and w.numel() == layer_scale.numel() == width
+    assert w_next is None or (w_next.numel() == width and w_next.dtype == w.dtype)
+    out = torch.empty_like(x) if shift is not None and shift.row_seq is not None else x
+    plain = shift is None and w_next is None and w.dtype == torch.float32          # the rows are x' itself
+    h = out if plain else torch.empty(rows, width, dtype=w.dtype, device=x.device)
+    where = shift.pointers(rows, width, w.dtype) if shift is not None else (None, None, 0, None, None, None, None)
+    check(lib.tlf_post_rmsnorm(*_source(y), layer_scale.data_ptr(), float(alpha), x.data_ptr(), w.data_ptr(), float(eps), out.data_ptr(),
+                               *where, _opt(w_next), None if plain else h.data_ptr(), rows, width, _dt(w), _stream()), "tlf_post_rmsnorm")
+    return out, h
+
+
+def embed_shift(ids, table, embed_scale, shift: ShiftArguments):
+    """``x = embed_scale * table[ids]`` in fp32 and its shifted rows in the table's dtype."""
+    lib = _lib.load()
+    _need(ids, torch.int64, "ids"); _need(table, None, "table")
+    assert ids.is_contiguous() and table.is_contiguous()
+    rows, (vocab, width) = ids.numel(), table.shape
+    x = torch.empty(rows, width, dtype=torch.float32, device=table.device)
+    h = torch.empty(rows, width, dtype=table.dtype, device=table.device)
+    check(lib.tlf_embed_shift(ids.data_ptr(), table.data_ptr(), vocab, float(embed_scale), x.data_ptr(),
+                              *shift.pointers(rows, width, table.dtype), h.data_ptr(), rows, width, _dt(table), _stream()), "tlf_embed_shift")
+    return x, h
+
+
+def rows_rms_norm(x, w, groups, eps, pad=1):
+    """Rows of ``x [N, C]`` in ``groups`` equal parts, each divided by its root mean square, times ``w``; zero columns up to a multiple
+    of ``pad``."""
+    _need(x, w.dtype, "x")
+    (rows, cols), dt = x.shape, x.dtype
+    assert x.stride(1) == 1 and w.numel() == cols
+    out = torch.empty(rows, -(-cols // pad) * pad, dtype=dt, device=x.device)
+    check(_lib.load().tlf_rows_rmsnorm(x.data_ptr(), x.stride(0), w.data_ptr(), out.data_ptr(), out.stride(0), rows, cols, groups, float(eps),
+                                       _dt(x), _stream()), "tlf_rows_rmsnorm")
+    return out
+
+
+# ------------------------------------------------------------------ attention whose heads mix their weights
+def talk_prep(proj, kv: SinkKV, heads, positions, slot_mapping, q_norm, k_norm, temp, cos_sin, rot_dims, eps, scale):
+    """Projection rows ``[q | k | v]`` -> ``q [N, H, Dp]`` with the score's constants; keys and values go to the caches."""
+    lib = _lib.load()
+    dt, n = kv.k.dtype, proj.shape[0]
+    _need(positions, torch.int64, "positions"); _need(slot_mapping, torch.int32, "slot_mapping")
+    pages, G, bs, dp = kv.k.shape
+    assert proj.dtype == q_norm.dtype == k_norm.dtype == dt and (temp is None or (temp.dtype == dt and temp.numel() == heads))
+    assert positions.numel() == n and slot_mapping.numel() == n and proj.shape[1] >= (heads + G) * kv.dim + G * kv.vdim
+    assert q_norm.numel() == heads * kv.dim and k_norm.numel() == G * kv.dim
+    assert rot_dims == 0 or (cos_sin.dtype == torch.float32 and cos_sin.is_contiguous() and cos_sin.shape[1] == rot_dims)
+    q = torch.empty(n, heads, dp, dtype=dt, device=kv.k.device)
+    check(lib.tlf_talk_prep(*_source(proj), q_norm.data_ptr(), k_norm.data_ptr(), _opt(temp), positions.data_ptr(), _opt(cos_sin),
+                            cos_sin.shape[0] if cos_sin is not None else 0, rot_dims, slot_mapping.data_ptr(), q.data_ptr(),
+                            kv.k.data_ptr(), kv.v.data_ptr(), n, heads, G, kv.dim, kv.vdim, bs, pages, float(eps), float(scale), _dt(kv.k),
+                            _stream()), "tlf_talk_prep")
+    return q
+
+
+def talk_attention_rows(q, kv: SinkKV, block_tables, positions, slot_mapping, talk, max_len, out, row_seq=None):
+    """Row by row: ``q [N, H, Dp]`` as from ``talk_prep`` -> ``out [N, H * vdim]``; ``row_seq`` None: row r is sequence r."""
+    lib = _lib.load()
+    _need(q, kv.k.dtype, "q"); _need(talk, q.dtype, "talk"); _need(block_tables, torch.int32, "block_tables")
+    _need(positions, torch.int64, "positions")
+    n, heads, dp = q.shape
+    pages, G, bs, _ = kv.k.shape
+    assert q.is_contiguous() and dp == kv.k.shape[3] and out.stride(1) == 1 and out.shape[0] == n and out.dtype == q.dtype
+    assert talk.is_contiguous() and talk.shape == (heads, heads) and block_tables.stride(1) == 1
+    assert positions.numel() == n and slot_mapping.numel() == n
+    assert row_seq.numel() == n if row_seq is not None else block_tables.shape[0] >= n
+    max_len = min(max_len, block_tables.shape[1] * bs)
+    step = max(1, min(32768, (1 << 28) // (heads * -(-max_len // 64) * 64)))     # rows per launch: grid limit, a gigabyte of scores
+    for lo in range(0, n, step):
+        m = min(step, n - lo)
+        tables = block_tables if row_seq is not None else block_tables[lo:]
+        nbytes = lib.tlf_talk_attn_rows_workspace_bytes(m, heads, G, kv.dim, kv.vdim, max_len, _dt(q))
+        ws = _workspace(nbytes, q.device, "talk_rows")
+        check(lib.tlf_talk_attn_rows(
+            q[lo:].data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), tables.data_ptr(), tables.stride(0), positions[lo:].data_ptr(),
+            slot_mapping[lo:].data_ptr(), row_seq[lo:].data_ptr() if row_seq is not None else None, talk.data_ptr(), out[lo:].data_ptr(),
+            out.stride(0), m, heads, G, kv.dim, kv.vdim, bs, max_len, pages, _dt(q), ws.data_ptr(), ws.numel(), _stream()),
+            "tlf_talk_attn_rows")
+    return out
+
+
+def talk_prefill_supported(heads, kv_heads, dim, vdim) -> bool:
+    return bool(_lib.load().tlf_talk_attn_prefill_supported(heads, kv_heads, dim, vdim))
+
+
+def talk_attention_prefill(q, kv: SinkKV, block_tables, cu_seqlens_q, seq_starts, first_seq, num_seqs, max_tokens, talk, out):
+    """Portions of sequences ``first_seq ..`` on the matrix cores (bf16); rows indexed as in the step."""
+    _need(q, BF16, "q"); _need(talk, BF16, "talk"); _need(block_tables, torch.int32, "block_tables")
+    n, heads, dp = q.shape
+    pages, G, bs, _ = kv.k.shape
+    assert q.is_contiguous() and dp == kv.k.shape[3] and kv.k.dtype == BF16 and out.stride(1) == 1 and out.shape[0] == n
+    assert talk.is_contiguous() and talk.shape == (heads, heads)
+    assert block_tables.stride(1) == 1 and block_tables.shape[0] >= first_seq + num_seqs
+    check(_lib.load().tlf_talk_attn_prefill(
+        q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), cu_seqlens_q.data_ptr(),
+        seq_starts.data_ptr(), first_seq, num_seqs, max_tokens, talk.data_ptr(), out.data_ptr(), out.stride(0), heads, G, kv.dim, kv.vdim,
+        bs, pages, _stream()), "tlf_talk_attn_prefill")
+    return out
+
+
+# ------------------------------------------------------------------ state-space layer
+class SsdWeights:
+    """``conv [taps, channels]``, ``conv_bias [channels]``, ``dt_bias``, ``A_log``, ``D [heads]``, all of one dtype."""
+    __slots__ = ("conv", "conv_bias", "dt_bias", "A_log", "D")
+
+    def __init__(self, conv, conv_bias, dt_bias, A_log, D):
+        self.conv, self.conv_bias, self.dt_bias, self.A_log, self.D = conv, conv_bias, dt_bias, A_log, D
+
+    def pointers(self, proj, ring, state, state_slots, groups):
+        """Checked; the arguments from ``conv`` to ``num_slots`` and the sizes."""
+        slots, heads, N, P = state.shape
+        taps, channels = self.conv.shape
+        _need(state, torch.float32, "state"); _need(state_slots, torch.int32, "state_slots")
+        for t in (self.conv, self.conv_bias, self.dt_bias, self.A_log, self.D, ring):
+            assert t.dtype == proj.dtype and t.is_contiguous()
+        assert channels == heads * P + 2 * groups * N == self.conv_bias.numel() and self.dt_bias.numel() == self.A_log.numel() == self.D.numel() == heads
+        assert state.is_contiguous() and ring.shape == (slots, taps, channels) and proj.shape[1] >= heads * P + channels + heads
+        return ((self.conv.data_ptr(), self.conv_bias.data_ptr(), taps, self.dt_bias.data_ptr(), self.A_log.data_ptr(), self.D.data_ptr(),
+                 ring.data_ptr(), state.data_ptr(), state_slots.data_ptr(), slots), (heads, P, N, groups))
+
+
+def ssd_decode(proj, weights: SsdWeights, ring, state, state_slots, positions, groups, out):
+    """One token per row of ``proj [N, z | x | B | C | dt]``; ``ring`` and ``state`` updated in place; ``out`` gated, not normed."""
+    lib = _lib.load()
+    rows = proj.shape[0]
+    args, sizes = weights.pointers(proj, ring, state, state_slots, groups)
+    assert out.stride(1) == 1 and out.shape[0] == rows and state_slots.numel() >= rows and positions.numel() == rows
+    check(lib.tlf_ssd_decode(*_source(proj), *args, positions.data_ptr(), out.data_ptr(), out.stride(0), rows, *sizes, _dt(proj), _stream()),
+          "tlf_ssd_decode")
+    return out
+
+
+def ssd_portions(proj, weights: SsdWeights, ring, state, state_slots, positions, row_seq, cu_seqlens_q, seq_starts, first_seq, num_seqs,
+                 first_row, max_tokens, groups, out):
+    """Portions of sequences ``first_seq ..``, whose rows begin at ``first_row`` of the step's; the ring is only read."""
+    lib = _lib.load()
+    rows = proj.shape[0] - first_row
+    args, sizes = weights.pointers(proj, ring, state, state_slots, groups)
+    _need(row_seq, torch.int32, "row_seq"); _need(cu_seqlens_q, torch.int32, "cu_seqlens_q")
+    assert proj.stride(1) == 1 and out.stride(1) == 1 and out.shape[0] == proj.shape[0] == positions.numel() == row_seq.numel()
+    assert state_slots.numel() >= first_seq + num_seqs and cu_seqlens_q.numel() > first_seq + num_seqs
+    ws = _workspace(lib.tlf_ssd_portions_workspace_bytes(rows, num_seqs, max_tokens, *sizes, _dt(proj)), proj.device, "ssd")
+    check(lib.tlf_ssd_portions(proj.data_ptr(), proj.stride(0), *args, positions.data_ptr(), row_seq.data_ptr(), cu_seqlens_q.data_ptr(),
+                               seq_starts.data_ptr(), first_seq, num_seqs, first_row, max_tokens, out.data_ptr(), out.stride(0), rows, *sizes,
+                               _dt(proj), ws.data_ptr(), ws.numel(), _stream()), "tlf_ssd_portions")
     return out
 
 
