@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the per-token hot path on one MI355X.
 
-    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload e2e|decode_attn|gemm|gitopel|gigopel|zuzunex|...|all]
+    python bench.py [--gpus 1] [--steps K] [--warmup W] [--workload e2e|decode_attn|gemm|gitopel|gigopel|zuzunex|tibenex|...|all]
 
 Prints ONE JSON line.
 
@@ -53,7 +53,7 @@ def parse():
                     help="engine steps that steps/ms_per_step describe (0 = all); value is always the whole job")
     ap.add_argument("--warmup", type=int, default=1, help="warm-up generate() calls before the timed run")
     ap.add_argument("--workload", default="e2e",
-                    choices=["e2e", "decode_attn", "gemm", "prefill_attn", "elementwise", "clock", "c5", "gitopel", "gigopel", "zuzunex", "all"])
+                    choices=["e2e", "decode_attn", "gemm", "prefill_attn", "elementwise", "clock", "c5", "gitopel", "gigopel", "zuzunex", "tibenex", "all"])
     ap.add_argument("--attn-steps", type=int, default=200, help="timed launches of the decode-attention microbench")
     ap.add_argument("--num-seqs", type=int, default=256)
     ap.add_argument("--no-cpu-baseline", action="store_true")
@@ -1119,6 +1119,194 @@ def bench_zuzunex_kernels(sizes=None):
     return rows
 
 
+# ----------------------------------------------------------------------------- Tibenex beside the nearest kernels at equal size
+# state-space heads, their value size, state, groups; the rest as GITOPEL_SIZES and GIGOPEL_SIZES
+TIBENEX_STATES = {"1024-wide": (32, 64, 128, 1), "4096-wide": (128, 64, 128, 8)}
+
+
+def tibenex_shape(size, layers=8, vocab=32768, kinds=("attention", "mamba2", "mamba2", "latent_attention")):
+    """The three mixers in turn, all layers with a dense feed-forward."""
+    w, hq, hkv, d, ff, *_ = GITOPEL_SIZES[size]
+    _, lh, ld, t, lv, r, *_ = GIGOPEL_SIZES[size]
+    sh, sp, sn, sg = TIBENEX_STATES[size]
+    mixers = {"attention": dict(heads=hq, kv_heads=hkv, dim=d, vdim=d, scale=d ** -0.5, rot=dict(base=1e6, dims=d)),
+              "latent_attention": dict(heads=lh, dim=ld, rot_dim=t, vdim=lv, kv_rank=r, q_rank=w // 2, scale=(ld + t) ** -0.5,
+                                       rot=dict(base=1e4, dims=t, scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0))),
+              "mamba2": dict(heads=sh, vdim=sp, state=sn, groups=sg, conv=4, norm_groups=sg)}
+    return dict(architecture="Tibenex", vocab=vocab, width=w, norm=dict(eps=1e-6), embedding=dict(scale=1.0), postln_alpha=2.0,
+                layers=[dict(type=kinds[i % len(kinds)], mixer=mixers[kinds[i % len(kinds)]], mlp=dict(kind="dense", ff=ff)) for i in range(layers)])
+
+
+def bench_tibenex_kernels(sizes=None):
+    """Kernels of the Tibenex layers beside the like kernel of the nearest model at the same sizes: algorithmic bytes or flops over
+    the graph-timed launch, as a fraction of the HBM or matrix peak."""
+    import torch
+    from tinyllmforge_amd import ops as P
+    from tinyllmforge_amd.layers.latent_attention import LatentAttention
+    from tinyllmforge_amd.layers.rotary_embedding import rotation_table
+    torch.manual_seed(0)
+    BF, I32, dev = torch.bfloat16, torch.int32, "cuda"
+    rows = []
+
+    def add(name, size, fn, amount, bound, copies=1, launches=10):
+        def cycle():
+            for i in range(copies):
+                fn(i)
+        sec = time_graph(cycle, launches=max(1, launches // copies), replays=10) * 1e-3 / copies
+        peak = {"hbm": HBM_PEAK_GBPS * 1e9, "mfma bf16": MFMA_BF16_PEAK_TFLOPS * 1e12, "mfma f32": MFMA_F32_PEAK_TFLOPS * 1e12}[bound]
+        rows.append(dict(kernel=name, size=size, us=round(sec * 1e6, 2), bound=bound,
+                         rate=round(amount / sec / (1e9 if bound == "hbm" else 1e12), 1), frac=round(amount / sec / peak, 4)))
+        print(rows[-1], file=sys.stderr, flush=True)
+        torch.cuda.empty_cache()
+
+    bf = lambda *s: torch.randn(*s, device=dev).to(BF)
+    ar = lambda n: torch.arange(n, dtype=I32, device=dev)
+    for size in sizes or TIBENEX_STATES:
+        w, h, g, d, ff, gh, gk, gv = GITOPEL_SIZES[size]
+        _, lh, ld, t, lv, r, *_ = GIGOPEL_SIZES[size]
+        sh, sp, sn, sg = TIBENEX_STATES[size]
+        B, bs, S, L = 64, 256, 8, 2048
+        N, scale = S * L, d ** -0.5
+        cu, starts = torch.arange(0, N + 1, L, dtype=I32, device=dev), torch.zeros(S, dtype=I32, device=dev)
+        seqs = dict(row_seq=ar(N) // L, cu_seqlens_q=cu)
+        where = {N: torch.arange(L, device=dev).repeat(S), B: torch.full((B,), 5, device=dev)}
+        # -- attention that mixes its heads: 64 sequences, contexts U[512, 4096], pages of 256; prompts 8 x 2048
+        case = make_decode_case(batch=B, hq=h, hkv=g, dh=d)
+        kv = P.SinkKV(2048, bs, g, d, d, BF, dev)
+        kv.k.normal_()
+        kv.v.normal_()
+        pos, slots = case["ctx"].long() - 1, torch.zeros(B, dtype=I32, device=dev)
+        q, out, talk = bf(B, h, d) * 0.1, torch.empty(B, h * d, device=dev, dtype=BF), bf(h, h)
+        add("decode attention with sink (Zuzunex)", size,
+            lambda i: P.sink_attention_rows(q, kv, case["bt"], pos, slots, None, None, None, 4096, out), case["algo_bytes"], "hbm")
+        add("attention: decode, heads mixed", size, lambda i: P.talk_attention_rows(q, kv, case["bt"], pos, slots, talk, 4096, out),
+            case["algo_bytes"], "hbm")
+        del kv
+        kv = P.SinkKV(N // bs, bs, g, d, d, BF, dev)
+        kv.k.normal_()
+        kv.v.normal_()
+        bt = ar(N // bs).view(S, -1)
+        q, out = bf(N, h, d) * 0.1, torch.empty(N, h * d, device=dev, dtype=BF)
+        pairs = S * L * L / 2
+        add("prompt attention with sink (Zuzunex)", size,
+            lambda i: P.sink_attention_prefill(q, kv, bt, cu, starts, 0, S, L, None, None, None, out), 4.0 * h * d * pairs, "mfma bf16")
+        add("attention: prompt, heads mixed", size, lambda i: P.talk_attention_prefill(q, kv, bt, cu, starts, 0, S, L, talk, out),
+            (4.0 * h * d + 2.0 * h * h) * pairs, "mfma bf16")
+        del q, out, kv
+        tab, slots = rotation_table(d, 4096, 1e6).to(dev), ar(N)
+        chan = (h + 2 * g) * d
+        qn, kn, dn, temp = torch.ones(h * d, device=dev, dtype=BF), torch.ones(g * d, device=dev, dtype=BF), torch.ones(d, device=dev, dtype=BF), bf(h)
+        for n, copies in ((N, 3), (B, 1)):
+            kv = P.SinkKV(N // bs, bs, g, d, d, BF, dev)
+            proj = bf(copies, n, chan + h * d)
+            add(f"preparation (Zuzunex), {n} tokens", size,
+                lambda i: P.sink_prep(proj[i], kv, h, where[n], slots[:n], 1e-6, scale, None, q_norm=dn, k_norm=dn, cos_sin=tab, rot_dims=d),
+                n * (chan * 4 + d * 4), "hbm", copies)
+            proj = proj[..., :chan].contiguous()
+            add(f"attention: preparation, {n} tokens", size,
+                lambda i: P.talk_prep(proj[i], kv, h, where[n], slots[:n], qn, kn, temp, tab, d, 1e-6, scale), n * (chan * 4 + d * 4), "hbm", copies)
+            del proj, kv
+        # -- latent attention: causal, gated, queries through a latent of their own
+        torch.set_default_dtype(BF)
+        with torch.device(dev):
+            layer = LatentAttention(lh, ld, t, r, lv, (ld + t) ** -0.5, 1 << 30, 0, None, 1e-6, BF, halves=True)
+        torch.set_default_dtype(torch.float32)
+        layer.uk.data.normal_(0, r ** -0.5)
+        layer.uv.data.normal_(0, r ** -0.5)
+        layer.pack_()
+        s = layer.shape
+        cache = bf(2048, bs, s.lp)
+        pos, slots1 = case["ctx"].long() - 1, torch.zeros(B, dtype=I32, device=dev)
+        q = bf(B, lh, s.lp)
+        batch = P.LatentBatch(B, positions=pos, slot_mapping=slots1)
+        for name, window in (("latent decode attention, windowed (Gigopel)", 4096), ("latent decode attention, causal", 1 << 30)):
+            plan = P.latent_plan(batch, lh, s.lp, window)
+            add(name, size, lambda i: P.latent_attention(q, cache, case["bt"], window, layer.scale, s, batch, plan),
+                sum(int(c) for c in case["ctx"].cpu()) * (r + t) * 2 + B * lh * (r + t) * 2 + B * lh * r * 4, "hbm")
+        part, ml = P.latent_attention(q, cache, case["bt"], 1 << 30, layer.scale, s, batch, plan)
+        out, gate = torch.zeros(B, lh * lv, device=dev, dtype=BF), torch.rand(B, lh, device=dev)
+        for name, gt in (("pieces joined + values (Gigopel), 64 tokens", None), ("pieces joined + values, gated, 64 tokens", gate)):
+            add(name, size, lambda i: P.latent_values(part, ml, layer.values, out, s, batch, plan, gt),
+                lh * lv * r * 2 + B * lh * r * 4 + B * lh * lv * 2, "hbm")
+        del part, ml, plan, case, cache
+        cache = bf(N // bs, bs, s.lp)
+        q, out, gate = bf(N, lh, s.dq), torch.empty(N, lh * lv, device=dev, dtype=BF), torch.rand(N, lh, device=dev)
+        latents = P.latent_gather(cache, bt, cu, starts, cu, N, 0, S, L, 1 << 30)
+        expanded = P.linear(latents[:, :layer.expand.shape[1]], layer.expand)
+        for name, window, gt in (("latent prompt attention, windowed (Gigopel)", 2048, None), ("latent prompt attention, causal, gated", 1 << 30, gate)):
+            add(name, size, lambda i: P.latent_prefill(q, expanded, latents, cu, starts, cu, 0, S, L, window, layer.scale, s, out, gt),
+                2.0 * lh * (ld + t + lv) * pairs, "mfma bf16")
+        del q, out, expanded, latents
+        ltab, lw = rotation_table(t, 4096, 1e4).to(dev), torch.ones(r, device=dev, dtype=BF)
+        qr = w // 2
+        cw = torch.ones(qr, device=dev, dtype=BF)
+        for n, copies in ((N, 3), (B, 1)):
+            row = lh * (ld + t) + r + t
+            proj = bf(copies, n, -(-row // 16) * 16)
+            add(f"latent preparation (Gigopel), {n} tokens", size,
+                lambda i: P.latent_prep(proj[i], lh * (ld + t), lw, where[n], ltab, slots[:n], cache, s, 1e-6), n * (row * 4 + t * 4), "hbm", copies)
+            add(f"query preparation, {n} tokens", size, lambda i: P.latent_prep_queries(proj[i], where[n], ltab, s, True),
+                n * (lh * (ld + t) * 4 + t * 4), "hbm", copies)
+            proj = bf(copies, n, -(-(qr + r + t + lh) // 16) * 16)
+            add(f"latents, query latent and gates, {n} tokens", size,
+                lambda i: P.latent_prep_down(proj[i], qr, lw, where[n], ltab, slots[:n], cache, s, 1e-6, True, 0, cw, qr + r + t),
+                n * ((qr + r + t) * 4 + lh * 6 + t * 4), "hbm", copies)
+            del proj
+        del cache, layer
+        # -- norms
+        for n, copies in ((N, 3), (B, 1)):
+            y, x, ww = bf(copies, n, w), torch.randn(copies, n, w, device=dev), torch.ones(w, device=dev, dtype=BF)
+            add(f"add + norm (Gigopel), {n} tokens", size, lambda i: P.residual_rms_norm(y[i], x[i], 0.5, ww, 1.0, 1e-6), n * w * 12, "hbm", copies)
+            add(f"scaled add + norm, {n} tokens", size, lambda i: P.post_rms_norm(y[i], x[i], 2.0, ww, ww, 1e-6), n * w * 12, "hbm", copies)
+            shift = P.ShiftArguments(ww, torch.zeros(B, 2, w, device=dev), ar(B), where[n], **(seqs if n == N else {}))
+            add(f"scaled add + norm + token shift, {n} tokens", size, lambda i: P.post_rms_norm(y[i], x[i], 2.0, ww, ww, 1e-6, shift),
+                n * w * (12 if n == N else 20), "hbm", copies)
+            if n == N:
+                add(f"last rows of {S} portions", size, lambda i: P.conv_tail(x[i], shift.ring, shift.state_slots, cu, starts, 0, S), S * w * 8, "hbm", copies)
+            o = bf(copies, n, sh * sp)
+            wide = torch.ones(sh * sp, device=dev, dtype=BF)
+            add(f"norm in parts of {sh * sp // sg}, {n} tokens", size, lambda i: P.rows_rms_norm(o[i], wide, sg, 1e-6), n * sh * sp * 4, "hbm", copies)
+            del y, x, o
+        # -- recurrences
+        rank = 16
+        gld = 2 * gh * (gk + gv) + rank
+        a2, a2b = (torch.randn(gh * gk, rank, device=dev) * 0.1).to(BF), torch.zeros(gh * gk, device=dev, dtype=BF)
+        gw = torch.ones(gv, device=dev, dtype=BF)
+        schan = sh * sp + 2 * sg * sn
+        sld = -(-(sh * sp + schan + sh) // 16) * 16
+        sw = P.SsdWeights(bf(4, schan) * 0.5, bf(schan), bf(sh), bf(sh) * 0.5, bf(sh))
+        for b in (64, 256):
+            sl, ps = ar(b), torch.full((b,), 5, device=dev)
+            state = torch.zeros(b, gh, gk, gv, device=dev)
+            proj, out = bf(b, gld), torch.empty(b, gh * gv, device=dev, dtype=BF)
+            add(f"gated linear attention (Gitopel), {b} decoded tokens", size,
+                lambda i: P.gla_decode(proj, a2, a2b, gw, state, sl, ps, 16.0, 1e-6, out), b * gh * gk * gv * 8, "hbm")
+            state, ring = torch.zeros(b, sh, sn, sp, device=dev), torch.zeros(b, 4, schan, device=dev, dtype=BF)
+            proj, out = bf(b, sld), torch.empty(b, sh * sp, device=dev, dtype=BF)
+            add(f"state space, {b} decoded tokens", size, lambda i: P.ssd_decode(proj, sw, ring, state, sl, ps, sg, out), b * sh * sn * sp * 8, "hbm")
+            del state, ring, proj, out
+        for s_, l_ in ((8, 2048), (1, 8192)):
+            n = s_ * l_
+            sl, st, cus = ar(s_), torch.zeros(s_, dtype=I32, device=dev), torch.arange(0, n + 1, l_, dtype=I32, device=dev)
+            state = torch.zeros(s_, gh, gk, gv, device=dev)
+            proj, out = bf(n, gld), torch.empty(n, gh * gv, device=dev, dtype=BF)
+            chunk_rows = torch.arange(0, n, 16, dtype=I32, device=dev)
+            chunk_lens, cuc = torch.full_like(chunk_rows, 16), torch.arange(0, n // 16 + 1, l_ // 16, dtype=I32, device=dev)
+            add(f"gated linear attention (Gitopel), prompts {s_} x {l_}", size,
+                lambda i: P.gla_portions(proj, a2, a2b, gw, state, sl, st, chunk_rows, chunk_lens, cuc, 0, s_, 16.0, 1e-6, out),
+                n * gh * (4.0 * gk * gv + 2 * 16 * (gk + gv)), "mfma f32")
+            state, ring = torch.zeros(s_, sh, sn, sp, device=dev), torch.zeros(s_, 4, schan, device=dev, dtype=BF)
+            proj, out = bf(n, sld), torch.empty(n, sh * sp, device=dev, dtype=BF)
+            ps, rs = torch.arange(l_, device=dev).repeat(s_), ar(n) // l_
+            # bytes: a projection row read, the result written (the convolved rows in between stay in the chip's caches at best)
+            add(f"state space, prompts {s_} x {l_}", size,
+                lambda i: P.ssd_portions(proj, sw, ring, state, sl, ps, rs, cus, st, 0, s_, 0, l_, sg, out),
+                n * sh * (4.0 * sn * sp + 64.0 * (sn + sp)), "mfma bf16")
+            add(f"convolution state, {s_} portions", size, lambda i: P.conv_tail(proj[:, sh * sp:], ring, sl, cus, st, 0, s_), s_ * 3 * schan * 4, "hbm")
+            del state, ring, proj, out
+    return rows
+
+
 # ----------------------------------------------------------------------------- config 4 (end to end)
 def e2e_workload(num_seqs=256):
     """The reference's bench.py recipe (pure-python ``random``: platform independent)."""
@@ -1298,6 +1486,21 @@ def main():
             "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
             "config": {"workload": "Zuzunex layers (alternating attention and attention_2; one dense layer, seven of experts "
                                    "with a shared one) and Qwen3 layers of equal width, random weights, bf16"},
+            "extra": {"throughput": through, "kernels": rows}}))
+        return
+    if args.workload == "tibenex":   # likewise
+        rows = bench_tibenex_kernels()
+        through = [throughput({"tibenex": tibenex_shape(size), **{f"tibenex, {k} only": tibenex_shape(size, kinds=(k,)) for k in
+                               ("attention", "mamba2", "latent_attention")},
+                               "gitopel": gitopel_shape(size), "qwen3": qwen3_shape(size)}, size) for size in TIBENEX_STATES]
+        big = through[-1]
+        print(json.dumps({
+            "metric": "output tok/s (Tibenex, 8 layers of 4096, 64 sequences, decode)", "value": big["tibenex"]["decode_tok_s"],
+            "unit": "tok/s", "n_gpus": 1, "steps": big["output_tokens"], "warmup": 1,
+            "ms_per_step": big["tibenex"]["decode_ms_per_step"], "higher_is_better": True, "scaling": "weak",
+            "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+            "config": {"workload": "Tibenex layers (attention, two state-space layers and latent attention in turn, dense feed-forwards), "
+                                   "Gitopel and Qwen3 layers of equal width, random weights, bf16"},
             "extra": {"throughput": through, "kernels": rows}}))
         return
     extra = {}

@@ -788,7 +788,7 @@ int tlf_rows_rmsnorm(const void *x, int64_t x_stride, const void *w, void *out, 
  *   padding row (zeros).  max_len bounds the positions.  talk [heads, heads].  heads <= 1024; bf16 up to 128 heads and 256
  *   dimensions on the matrix cores.  The workspace holds the scores (4 bytes per row, head and key).
  * tlf_talk_attn_prefill: portions of sequences first_seq .., rows as in the step; bf16, heads <= 32, dim, vdim <= 128 and a limit
- *   on kv_heads * vdim (tlf_talk_attn_prefill_supported). */
+ *   on kv_heads * vdim (tlf_talk_attn_prefill_supported).  stats: scratch, [rows of the step, heads]. */
 int tlf_talk_prep(const void *proj, int64_t proj_stride, const float *partials, int32_t splits, const float *scale, const void
                   *q_norm, const void *k_norm, const void *temp, const int64_t *positions, const float *cos_sin, int32_t
                   max_pos, int32_t rot_dims, const int32_t *slot_mapping, void *q_out, void *k_cache, void *v_cache,
@@ -804,7 +804,7 @@ int tlf_talk_attn_rows(const void *q, const void *k_cache, const void *v_cache, 
 int tlf_talk_attn_prefill_supported(int32_t heads, int32_t kv_heads, int32_t dim, int32_t vdim);
 int tlf_talk_attn_prefill(const void *q, const void *k_cache, const void *v_cache, const int32_t *block_tables, int64_t
                           bt_stride, const int32_t *cu_seqlens_q, const int32_t *seq_starts, int32_t first_seq, int32_t
-                          num_seqs, int32_t max_tokens, const void *talk, void *out, int64_t out_stride, int32_t heads,
+                          num_seqs, int32_t max_tokens, const void *talk, float *stats, void *out, int64_t out_stride, int32_t heads,
                           int32_t kv_heads, int32_t dim, int32_t vdim, int32_t block_size, int64_t num_pages, void
                           *stream);
 

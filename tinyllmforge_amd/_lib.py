@@ -138,7 +138,7 @@ SIGNATURES = {
     "tlf_talk_attn_rows": (c_int32, [_P, _P, _P, _P, _I64, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32,
                                      _I32, _I32, _I64, _I32, _P, _SZ, _P]),
     "tlf_talk_attn_prefill_supported": (c_int32, [_I32, _I32, _I32, _I32]),
-    "tlf_talk_attn_prefill": (c_int32, [_P, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _P, _P, _I64, _I32, _I32,
+    "tlf_talk_attn_prefill": (c_int32, [_P, _P, _P, _P, _I64, _P, _P, _I32, _I32, _I32, _P, _P, _P, _I64, _I32, _I32,
                                         _I32, _I32, _I32, _I64, _P]),
     "tlf_ssd_decode": (c_int32, [_P, _I64, _P, _I32, _P, _P, _P, _I32, _P, _P, _P, _P, _P, _P, _I32, _P, _P, _I64,
                                  _I32, _I32, _I32, _I32, _I32, _I32, _P]),

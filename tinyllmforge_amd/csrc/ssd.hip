@@ -16,8 +16,8 @@
 //                      chunks of 64 tokens.  With c_t the sum of the log2 decays within the chunk:
 //                        G^T[s, t] = B_s . C_t;  M^T[s, t] = G^T 2^(c_t - c_s) dt_s for s <= t
 //                        Y^T[p, t] = X^T M^T + 2^(c_t) (S^T C^T)
-//                        S = 2^(c_end) S + B^T (dt_s 2^(c_end - c_s) X)
-//                      Every exponent is <= 0.  x, B and C are exact in bf16; M, the scaled x and S enter as bf16 hi + lo pairs (16
+//                        S = 2^(c_end) S + (dt_s 2^(c_end - c_s) B)^T X
+//                      Every exponent is <= 0.  x, B and C are exact in bf16; M, the scaled B and S enter as bf16 hi + lo pairs (16
 //                      significant bits), S itself stays in fp32 accumulators.  The s rows of two 16-row tiles are picked so that
 //                      their accumulators are the next product's operand.  Where (sequences, heads, columns) alone leave CUs idle
 //                      a sequence is cut into segments: a first pass gathers each segment's own contribution from zero,
@@ -59,6 +59,13 @@ __device__ __forceinline__ float ssd_step(const SsdArgs &a, float raw, int h) {
 template <typename T>
 __device__ __forceinline__ float ssd_log2_decay(const SsdArgs &a, float dt, int h) {
   return -expf(Elem<T>::ld(static_cast<const T *>(a.A_log) + h)) * dt * 1.4426950408889634f;
+}
+
+// 32-bit rows: the library's exponential; bf16 rows: the hardware's, far more exact than the rounding that follows.
+template <typename T>
+__device__ __forceinline__ float ssd_silu(float z) {
+  if constexpr (sizeof(T) == 4) return silu_f32(z);
+  return z * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
 }
 
 // The state's N rows are dealt to teams of lanes_v threads, VEC columns each; osum[team][P] gets the teams' parts of S^T C.
@@ -132,7 +139,7 @@ __global__ __launch_bounds__(256) void ssd_decode_kernel(const SsdArgs a, int la
       if (pos >= b) y = fmaf(Elem<T>::ld(static_cast<const T *>(a.conv) + static_cast<int64_t>(a.taps - 1 - b) * a.channels + ch),
                              Elem<T>::ld(ring + (pos - b) % a.taps * a.channels + ch), y);
     y = fmaf(Elem<T>::ld(static_cast<const T *>(a.conv) + static_cast<int64_t>(a.taps - 1) * a.channels + ch), now, y);
-    y = Elem<T>::rnd(silu_f32(y));
+    y = Elem<T>::rnd(ssd_silu<T>(y));
     // the row written is none of those read: heads that share a group do not disturb each other
     if (own || h == grp * share) Elem<T>::st(ring + pos % a.taps * a.channels + ch, now);
     if (own) xs[i] = y;
@@ -151,7 +158,7 @@ __global__ __launch_bounds__(256) void ssd_decode_kernel(const SsdArgs a, int la
   for (int v = tid; v < a.P; v += 256) {
     float y = 0.f;
     for (int t = 0; t < teams; ++t) y += osum[t * a.P + v];
-    Elem<T>::st(out + v, fmaf(D, xs[v], y) * silu_f32(in(h * a.P + v)));
+    Elem<T>::st(out + v, fmaf(D, xs[v], y) * ssd_silu<T>(in(h * a.P + v)));
   }
 }
 
@@ -181,16 +188,42 @@ __global__ __launch_bounds__(256) void ssd_conv_kernel(const SsdArgs a) {
     else f[0] = Elem<T>::ld(p);
   };
   const T *base = static_cast<const T *>(a.proj) + a.inner + ch, *w = static_cast<const T *>(a.conv) + ch;
-  float u[TOK + kBack][VEC], wt[TAPS > 0 ? TAPS : 1][VEC], bias[VEC];
-#pragma unroll
-  for (int i = 0; i < TOK + kBack; ++i) {
-    const int64_t r = a.first_row + r0 - kBack + i;
-    ldv(base + min(max(r, static_cast<int64_t>(0)), static_cast<int64_t>(a.first_row) + a.rows - 1) * a.ld, u[i]);
-  }
+  float bias[VEC];
   ldv(static_cast<const T *>(a.conv_bias) + ch, bias);
+  auto put = [&](int64_t r, float (&y)[VEC]) __attribute__((always_inline)) {
+    T *o = static_cast<T *>(a.xbc) + r * a.channels + ch;
 #pragma unroll
-  for (int t = 0; t < (TAPS > 0 ? TAPS : 0); ++t) ldv(w + static_cast<int64_t>(t) * a.channels, wt[t]);
+    for (int e = 0; e < VEC; ++e) y[e] = ssd_silu<T>(y[e]);
+    if constexpr (VEC == 8) Elem<T>::st8(o, y);
+    else Elem<T>::st(o, y[0]);
+  };
+  if constexpr (TAPS > 0 && VEC == 8) {
+    // one sequence from the first row looked at to the last: all loads in flight, every row read once
+    const int64_t first = a.first_row + r0 - kBack, last = a.first_row + r0 + TOK - 1;
+    if (r0 + TOK <= a.rows && first >= a.first_row && a.row_seq[first] == a.row_seq[last]) {
+      typename Elem<T>::Raw8 u[TOK + kBack], wt[TAPS];
 #pragma unroll
+      for (int i = 0; i < TOK + kBack; ++i) Elem<T>::raw8(base + (first + i) * a.ld, u[i]);
+#pragma unroll
+      for (int t = 0; t < TAPS; ++t) Elem<T>::raw8(w + static_cast<int64_t>(t) * a.channels, wt[t]);
+#pragma unroll
+      for (int k = 0; k < TOK; ++k) {
+        float y[VEC];
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) y[e] = bias[e];
+#pragma unroll
+        for (int t = 0; t < TAPS; ++t) {
+          float f[8], wf[8];
+          Elem<T>::cvt8(u[k + t], f);
+          Elem<T>::cvt8(wt[t], wf);
+#pragma unroll
+          for (int e = 0; e < VEC; ++e) y[e] = fmaf(wf[e], f[e], y[e]);
+        }
+        put(r0 + k, y);
+      }
+      return;
+    }
+  }
   for (int k = 0; k < TOK; ++k) {
     const int64_t r = r0 + k, row = a.first_row + r;
     if (r >= a.rows) return;
@@ -198,31 +231,18 @@ __global__ __launch_bounds__(256) void ssd_conv_kernel(const SsdArgs a) {
     const int64_t begin = a.cu_q[seq], pos = a.positions[row], slot = a.state_slots[seq];
     const bool held = slot >= 0 && slot < a.num_slots;
     const T *ring = static_cast<const T *>(a.ring) + (held ? slot : 0) * a.taps * a.channels + ch;
-    float y[VEC], f[VEC], wb[VEC];
+    float y[VEC];
 #pragma unroll
     for (int e = 0; e < VEC; ++e) y[e] = bias[e];
-    auto tap = [&](int b) __attribute__((always_inline)) {     // b > 0 rows back
-      if (pos < b || (row - b < begin && !held)) return;
-      if (row - b >= begin) ldv(base + (row - b) * a.ld, f);
-      else ldv(ring + (pos - b) % a.taps * a.channels, f);
-      ldv(w + static_cast<int64_t>(a.taps - 1 - b) * a.channels, wb);
+    for (int b = a.taps - 1; b >= 0; --b) {          // rows back
+      if (pos < b || (row - b < begin && !held)) continue;
+      float f[VEC], wf[VEC];
+      ldv(row - b >= begin ? base + (row - b) * a.ld : ring + (pos - b) % a.taps * a.channels, f);
+      ldv(w + static_cast<int64_t>(a.taps - 1 - b) * a.channels, wf);
 #pragma unroll
-      for (int e = 0; e < VEC; ++e) y[e] = fmaf(wb[e], f[e], y[e]);
-    };
-    if (TAPS > 0 && row - kBack >= begin) {
-#pragma unroll
-      for (int b = kBack; b > 0; --b)
-#pragma unroll
-        for (int e = 0; e < VEC; ++e) y[e] = fmaf(wt[TAPS > 0 ? TAPS - 1 - b : 0][e], u[k + kBack - b][e], y[e]);
-    } else {
-      for (int b = a.taps - 1; b > 0; --b) tap(b);
+      for (int e = 0; e < VEC; ++e) y[e] = fmaf(wf[e], f[e], y[e]);
     }
-    ldv(w + static_cast<int64_t>(a.taps - 1) * a.channels, wb);
-    T *o = static_cast<T *>(a.xbc) + r * a.channels + ch;
-#pragma unroll
-    for (int e = 0; e < VEC; ++e) y[e] = silu_f32(fmaf(wb[e], u[k + kBack][e], y[e]));
-    if constexpr (VEC == 8) Elem<T>::st8(o, y);
-    else Elem<T>::st(o, y[0]);
+    put(r, y);
   }
 }
 
@@ -254,7 +274,7 @@ __global__ __launch_bounds__(256) void ssd_scan_kernel(const SsdArgs a, int lane
     for (int v = tid; v < a.P; v += 256) {
       float y = 0.f;
       for (int t = 0; t < teams; ++t) y += osum[t * a.P + v];
-      Elem<T>::st(out + v, fmaf(D, xs[v], y) * silu_f32(Elem<T>::ld(z + v)));
+      Elem<T>::st(out + v, fmaf(D, xs[v], y) * ssd_silu<T>(Elem<T>::ld(z + v)));
     }
   }
 }
@@ -276,19 +296,42 @@ __device__ __forceinline__ void ssd_pair(const float (&w)[8], uint4 &hi, uint4 &
   lo = make_uint4(l[0], l[1], l[2], l[3]);
 }
 
+// Inclusive sum over the wave's 64 lanes, on the vector ALU.
+template <int CTRL, int ROWS>
+__device__ __forceinline__ float ssd_dpp_add(float v) {
+  return v + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, ROWS, 0xf, false));
+}
+__device__ __forceinline__ float ssd_wave_scan(float v) {
+  v = ssd_dpp_add<0x111, 0xf>(v);      // row_shr 1, 2, 4, 8: within rows of 16 lanes
+  v = ssd_dpp_add<0x112, 0xf>(v);
+  v = ssd_dpp_add<0x114, 0xf>(v);
+  v = ssd_dpp_add<0x118, 0xf>(v);
+  v = ssd_dpp_add<0x142, 0xa>(v);      // row_bcast 15 into rows 1 and 3
+  return ssd_dpp_add<0x143, 0xc>(v);   // row_bcast 31 into rows 2 and 3
+}
+
 // NN: N in units of 32, PT: columns of P in units of 16.  MODE 0: the whole portion from the state slot and back, 1: a
 // segment's own contribution from zero, 2: a segment from the state ssd_segments_kernel left for it.
+// Eight waves (four where P has 16 columns only): for Y a wave has 16 tokens and half of the columns, for S some of its 16 x 16 tiles.
+template <int PT>
+constexpr int ssd_waves() { return PT >= 2 ? 8 : 4; }
 template <int NN, int PT, int MODE, bool VEC>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) void ssd_chunk_kernel(const SsdArgs a) {
+__global__ __launch_bounds__(ssd_waves<PT>() * 64) void ssd_chunk_kernel(const SsdArgs a) {
   typedef unsigned short T;
-  constexpr int NP = NN * 32, PS = PT * 16, LN = NP + 8, LX = PS + 8;
-  constexpr int NTW = NN >= 2 ? NN / 2 : 1;          // 16-row tiles of N per wave
-  constexpr int CN = NP / 32, CX = (64 * PS / 8 + 255) / 256;   // 16-byte pieces per thread
-  __shared__ __attribute__((aligned(16))) T Cs[MODE == 1 ? 1 : kSC][LN], Bs[kSC][LN], Xs[kSC][LX], Xh[kSC][LX], Xl[kSC][LX];
+  constexpr int NW = ssd_waves<PT>(), TH = NW * 64;
+  constexpr int NP = NN * 32, PS = PT * 16, LN = NP + 8, LX = PS + 8, NT = 2 * NN;
+  constexpr int PTY = PT * 4 / NW;                   // column tiles of a wave's Y
+  constexpr int NTW = NT >= NW ? NT / NW : 1;        // row tiles of a wave's S, waves that share one, their column tiles
+  constexpr int WPN = NT >= NW ? 1 : NW / NT < PT ? NW / NT : PT, PTU = PT / WPN;
+  constexpr int CN = (kSC * NP / 8 + TH - 1) / TH, CX = (kSC * PS / 8 + TH - 1) / TH;   // 16-byte pieces per thread
+  __shared__ __attribute__((aligned(16))) T Cs[MODE == 1 ? 1 : kSC][LN], Bs[kSC][LN], Xs[kSC][LX];
   __shared__ __attribute__((aligned(16))) T Sh[MODE == 1 ? 1 : NP][LX], Sl[MODE == 1 ? 1 : NP][LX];
-  __shared__ __attribute__((aligned(16))) float cum[kSC], dts[kSC];
-  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, n = lane & 15, g = lane >> 4;
-  const int h = blockIdx.x, slice = blockIdx.y, sq = MODE == 0 ? blockIdx.z : blockIdx.z / a.segs, seg = MODE == 0 ? 0 : blockIdx.z % a.segs;
+  __shared__ __attribute__((aligned(16))) float cum[kSC], dts[kSC], into_end[kSC];
+  const int tid = threadIdx.x, lane = tid & 63, n = lane & 15, g = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  // workgroup w runs on XCD w % 8: neighbouring heads, which share B and C, on one
+  const int h = a.H % 8 == 0 ? blockIdx.x % 8 * (a.H / 8) + blockIdx.x / 8 : blockIdx.x;
+  const int slice = blockIdx.y, sq = MODE == 0 ? blockIdx.z : blockIdx.z / a.segs, seg = MODE == 0 ? 0 : blockIdx.z % a.segs;
   const bool last_seg = MODE == 0 || seg == a.segs - 1;
   if (MODE == 1 && last_seg) return;                 // nobody starts behind the last segment
   const int seq = a.first_seq + sq, grp = h / (a.H / a.G), p0 = slice * PS;
@@ -307,32 +350,33 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) void s
   float *gst = MODE == 0 ? st : a.seg_state + sg * plane;
   const bool from_zero = MODE == 1 || (MODE == 0 && (!slot_ok || a.starts[seq] == 0));
 
-  // S^T tiles: column n of tile j is row (wave NTW + j) 16 + n of the state, rows 4 g + r its columns
-  floatx4 S[NTW][PT];
+  // S^T tiles: column n of tile j is row (nt0 + j) 16 + n of the state, rows 4 g + r of tile i its columns (pt0 + i) 16 + 4 g + r
+  const bool has_state = wave < NT * WPN;            // wave uniform
+  const int nt0 = wave / WPN * NTW, pt0 = wave % WPN * PTU;
+  floatx4 S[NTW][PTU];
 #pragma unroll
   for (int j = 0; j < NTW; ++j)
 #pragma unroll
-    for (int i = 0; i < PT; ++i) {
-      const int d = (wave * NTW + j) * 16 + n, p = p0 + i * 16 + g * 4;
+    for (int i = 0; i < PTU; ++i) {
+      const int d = (nt0 + j) * 16 + n, p = p0 + (pt0 + i) * 16 + g * 4;
       S[j][i] = floatx4{0.f, 0.f, 0.f, 0.f};
-      if (!from_zero && d < a.N) {
+      if (has_state && !from_zero && d < a.N) {
 #pragma unroll
         for (int r = 0; r < 4; ++r)
           if (p + r < a.P) S[j][i][r] = gst[static_cast<int64_t>(d) * a.P + p + r];
       }
     }
   auto put_state = [&]() __attribute__((always_inline)) {
-    if (MODE == 1) return;
+    if (MODE == 1 || !has_state) return;
 #pragma unroll
     for (int j = 0; j < NTW; ++j)
 #pragma unroll
-      for (int i = 0; i < PT; ++i) {
-        const int d = (wave * NTW + j) * 16 + n;
-        if (d >= NP) continue;
+      for (int i = 0; i < PTU; ++i) {
+        const int d = MODE == 1 ? 0 : (nt0 + j) * 16 + n;
         const floatx4 v = S[j][i];
         const unsigned int h0 = pack_bf16x2(v[0], v[1]), h1 = pack_bf16x2(v[2], v[3]);
-        *reinterpret_cast<uint2 *>(&Sh[MODE == 1 ? 0 : d][i * 16 + g * 4]) = make_uint2(h0, h1);
-        *reinterpret_cast<uint2 *>(&Sl[MODE == 1 ? 0 : d][i * 16 + g * 4]) =
+        *reinterpret_cast<uint2 *>(&Sh[d][(pt0 + i) * 16 + g * 4]) = make_uint2(h0, h1);
+        *reinterpret_cast<uint2 *>(&Sl[d][(pt0 + i) * 16 + g * 4]) =
             make_uint2(pack_bf16x2(v[0] - __uint_as_float(h0 << 16), v[1] - __uint_as_float(h0 & 0xffff0000u)),
                        pack_bf16x2(v[2] - __uint_as_float(h1 << 16), v[3] - __uint_as_float(h1 & 0xffff0000u)));
       }
@@ -340,6 +384,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) void s
 
   // a chunk's rows, registers one chunk ahead
   uint4 creg[CN], breg[CN], xreg[CX];
+#pragma unroll
+  for (int i = 0; i < CN; ++i) creg[i] = breg[i] = make_uint4(0, 0, 0, 0);
+#pragma unroll
+  for (int i = 0; i < CX; ++i) xreg[i] = make_uint4(0, 0, 0, 0);
   float dt_now = 0.f, dec_now = 0.f;
   auto piece = [&](const T *row, int d, int len) __attribute__((always_inline)) {     // 8 values from d on, zeros from len on
     Pack16 t;
@@ -353,77 +401,109 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) void s
     }
     return t.u;
   };
+  // byte offsets of this thread's pieces in a full chunk
+  unsigned int boff[CN], xoff[CX];
+#pragma unroll
+  for (int i = 0; i < CN; ++i) {
+    const int item = tid + i * TH, r = min(item / (NP / 8), kSC - 1), d = item % (NP / 8) * 8;
+    boff[i] = static_cast<unsigned int>(r * a.channels + (d < a.N ? d : 0)) * 2;
+  }
+#pragma unroll
+  for (int i = 0; i < CX; ++i) {
+    const int item = tid + i * TH, r = min(item / (PS / 8), kSC - 1), d = item % (PS / 8) * 8;
+    xoff[i] = static_cast<unsigned int>(r * a.channels + (d < a.P - p0 ? d : 0)) * 2;
+  }
   auto load = [&](int c) __attribute__((always_inline)) {
     const int64_t r0 = begin - a.first_row + static_cast<int64_t>(c) * kSC;
     const int len = min(kSC, tokens - c * kSC);
-    const T *xbc = static_cast<const T *>(a.xbc);
-#pragma unroll
-    for (int i = 0; i < CN; ++i) {
-      const int item = tid + i * 256, r = item / (NP / 8), d = item % (NP / 8) * 8;
-      const T *row = xbc + (r0 + min(r, len - 1)) * a.channels + a.inner;
-      breg[i] = piece(row + grp * a.N, d, a.N);
-      if (MODE != 1) creg[i] = piece(row + (a.G + grp) * a.N, d, a.N);
-    }
-#pragma unroll
-    for (int i = 0; i < CX; ++i) {
-      const int item = tid + i * 256, r = item / (PS / 8), d = item % (PS / 8) * 8;
-      if (r < kSC) xreg[i] = piece(xbc + (r0 + min(r, len - 1)) * a.channels + h * a.P + p0, d, a.P - p0);
-    }
+    const T *first = static_cast<const T *>(a.xbc) + r0 * a.channels;               // uniform
+    const T *bp = first + a.inner + grp * a.N, *cp = bp + a.G * a.N, *xp = first + h * a.P + p0;
     const int64_t at = (r0 + min(lane, len - 1)) * a.H + h;
     dt_now = lane < len ? a.dt[at] : 0.f;
     dec_now = lane < len ? a.decay[at] : 0.f;
+    if (VEC && len == kSC) {
+#pragma unroll
+      for (int i = 0; i < CN; ++i) {
+        breg[i] = *reinterpret_cast<const uint4 *>(reinterpret_cast<const char *>(bp) + boff[i]);
+        if (MODE != 1) creg[i] = *reinterpret_cast<const uint4 *>(reinterpret_cast<const char *>(cp) + boff[i]);
+      }
+#pragma unroll
+      for (int i = 0; i < CX; ++i) xreg[i] = *reinterpret_cast<const uint4 *>(reinterpret_cast<const char *>(xp) + xoff[i]);
+      return;
+    }
+#pragma unroll
+    for (int i = 0; i < CN; ++i) {
+      const int item = tid + i * TH, r = min(item / (NP / 8), len - 1), d = item % (NP / 8) * 8;
+      breg[i] = piece(bp + static_cast<int64_t>(r) * a.channels, d, a.N);
+      if (MODE != 1) creg[i] = piece(cp + static_cast<int64_t>(r) * a.channels, d, a.N);
+    }
+#pragma unroll
+    for (int i = 0; i < CX; ++i) {
+      const int item = tid + i * TH, r = min(item / (PS / 8), len - 1), d = item % (PS / 8) * 8;
+      xreg[i] = piece(xp + static_cast<int64_t>(r) * a.channels, d, a.P - p0);
+    }
   };
   float total = 0.f;                                 // log2 decay of the whole segment
   float end_decay = 1.f;                             // 2^(c_end) of the chunk in LDS
   auto store = [&]() __attribute__((always_inline)) {
-    float c = dec_now;                               // every wave has all 64 tokens, a lane each
-#pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-      const float y = __shfl_up(c, o, 64);
-      if (lane >= o) c += y;
-    }
-    const float c_end = __shfl(c, 63, 64), scale = dt_now * __builtin_amdgcn_exp2f(c_end - c);
+    const float c = ssd_wave_scan(dec_now);          // every wave has all 64 tokens, a lane each
+    const float c_end = __int_as_float(__builtin_amdgcn_readlane(__float_as_int(c), 63));
     total += c_end;
     end_decay = __builtin_amdgcn_exp2f(c_end);
-    if (wave == 0) cum[lane] = c, dts[lane] = dt_now;
+    if (wave == 0) {
+      cum[lane] = c;
+      dts[lane] = dt_now;
+      into_end[lane] = dt_now * __builtin_amdgcn_exp2f(c_end - c);
+    }
 #pragma unroll
     for (int i = 0; i < CN; ++i) {
-      const int item = tid + i * 256, r = item / (NP / 8), d = item % (NP / 8) * 8;
-      *reinterpret_cast<uint4 *>(&Bs[r][d]) = breg[i];
-      if (MODE != 1) *reinterpret_cast<uint4 *>(&Cs[MODE == 1 ? 0 : r][d]) = creg[i];
+      const int item = tid + i * TH, r = item / (NP / 8), d = item % (NP / 8) * 8;
+      if (r < kSC) {
+        const bool in = !VEC || d < a.N;             // pads are zeros
+        *reinterpret_cast<uint4 *>(&Bs[r][d]) = in ? breg[i] : make_uint4(0, 0, 0, 0);
+        if (MODE != 1) *reinterpret_cast<uint4 *>(&Cs[MODE == 1 ? 0 : r][d]) = in ? creg[i] : make_uint4(0, 0, 0, 0);
+      }
     }
 #pragma unroll
     for (int i = 0; i < CX; ++i) {
-      const int item = tid + i * 256, r = item / (PS / 8), d = item % (PS / 8) * 8;
-      const float f = __shfl(scale, r & 63, 64);
-      if (r >= kSC) continue;
-      float x[8];
-      unpack8(xreg[i], x);
-#pragma unroll
-      for (int e = 0; e < 8; ++e) x[e] *= f;
-      uint4 hi, lo;
-      ssd_pair(x, hi, lo);
-      if (MODE != 1) *reinterpret_cast<uint4 *>(&Xs[r][d]) = xreg[i];
-      *reinterpret_cast<uint4 *>(&Xh[r][d]) = hi;
-      *reinterpret_cast<uint4 *>(&Xl[r][d]) = lo;
+      const int item = tid + i * TH, r = item / (PS / 8), d = item % (PS / 8) * 8;
+      if (r < kSC) *reinterpret_cast<uint4 *>(&Xs[r][d]) = !VEC || d < a.P - p0 ? xreg[i] : make_uint4(0, 0, 0, 0);
     }
   };
 
   const float D = MODE == 1 ? 0.f : Elem<T>::ld(static_cast<const T *>(a.D) + h);
   const int krow = (n >> 2) * 8 + (n & 3);           // s rows of a 32-row block as two 16-row tiles (+ 4)
   const int vrow = g * 8 + (n >> 2), vcol = (n & 3) * 4;
+  const int tt = wave & 3, py = NW == 8 ? wave / 4 * PTY : 0;        // this wave's tokens and first column tile of Y
   if (c0 < c1) {
     load(c0);
     put_state();
     store();
   }
   for (int c = c0; c < c1; ++c) {
-    lds_barrier();
-    if (c + 1 < c1) load(c + 1);
+    const int t = tt * 16 + n, tok = c * kSC + t;    // this lane's token
+    const int64_t row = begin + min(tok, tokens - 1);
+    uint2 zr[PTY];
     if constexpr (MODE != 1) {
-      const int t = wave * 16 + n;                   // this lane's token
-      const int tok = c * kSC + t;
-      const int64_t row = begin + min(tok, tokens - 1);
+      const T *zp = static_cast<const T *>(a.proj) + row * a.ld + h * a.P + p0;
+#pragma unroll
+      for (int i = 0; i < PTY; ++i) {
+        const int p = (py + i) * 16 + g * 4;
+        zr[i] = make_uint2(0, 0);
+        if (VEC) {
+          if (p0 + p < a.P) zr[i] = *reinterpret_cast<const uint2 *>(zp + p);
+        } else {
+          unsigned int z[4] = {0, 0, 0, 0};
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            if (p0 + p + r < a.P) z[r] = zp[p + r];
+          zr[i] = make_uint2(z[0] | z[1] << 16, z[2] | z[3] << 16);
+        }
+      }
+    }
+    if (c + 1 < c1) load(c + 1);
+    lds_barrier();
+    if constexpr (MODE != 1) {
       bf16x8 cf[NN];
 #pragma unroll
       for (int k = 0; k < NN; ++k) {
@@ -431,11 +511,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) void s
         x.u = *reinterpret_cast<const uint4 *>(&Cs[t][k * 32 + g * 8]);
         cf[k] = x.v;
       }
-      floatx4 y[PT], yi[PT];
+      floatx4 y[PTY], yl[PTY], yi[PTY], yil[PTY];    // sums over the pairs' halves apart: neighbouring products do not wait for each other
 #pragma unroll
-      for (int i = 0; i < PT; ++i) y[i] = yi[i] = floatx4{0.f, 0.f, 0.f, 0.f};
+      for (int i = 0; i < PTY; ++i) y[i] = yl[i] = yi[i] = yil[i] = floatx4{0.f, 0.f, 0.f, 0.f};
       const float ct = cum[t];
-      for (int blk = 0; blk <= wave / 2; ++blk) {    // 32 tokens s; none lies wholly behind the wave's
+#pragma unroll
+      for (int k = 0; k < NN; ++k)
+#pragma unroll
+        for (int i = 0; i < PTY; ++i) {
+          yi[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ssd_tr(&Sh[k * 32 + vrow][(py + i) * 16 + vcol], LX), cf[k], yi[i], 0, 0, 0);
+          yil[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ssd_tr(&Sl[k * 32 + vrow][(py + i) * 16 + vcol], LX), cf[k], yil[i], 0, 0, 0);
+        }
+      for (int blk = 0; blk <= tt / 2; ++blk) {      // 32 tokens s; none lies wholly behind the wave's
         floatx4 g0 = floatx4{0.f, 0.f, 0.f, 0.f}, g1 = g0;
 #pragma unroll
         for (int k = 0; k < NN; ++k) {
@@ -451,50 +538,36 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) void s
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
           const float v = e < 4 ? g0[e & 3] : g1[e & 3];
-          m[e] = blk * 32 + g * 8 + e <= t ? v * d8[e] * __builtin_amdgcn_exp2f(fminf(ct - cs8[e], 0.f)) : 0.f;
+          m[e] = v * d8[e] * __builtin_amdgcn_exp2f(ct - cs8[e]);
+        }
+        if (blk == tt / 2) {                         // the diagonal; an exponent above 0 is dropped here
+          const int last = t - blk * 32 - g * 8;
+#pragma unroll
+          for (int e = 0; e < 8; ++e) m[e] = e <= last ? m[e] : 0.f;
         }
         uint4 mh, ml;
         ssd_pair(m, mh, ml);
 #pragma unroll
-        for (int i = 0; i < PT; ++i) {
-          const bf16x8 xv = ssd_tr(&Xs[blk * 32 + vrow][i * 16 + vcol], LX);
+        for (int i = 0; i < PTY; ++i) {
+          const bf16x8 xv = ssd_tr(&Xs[blk * 32 + vrow][(py + i) * 16 + vcol], LX);
           y[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xv, __builtin_bit_cast(bf16x8, mh), y[i], 0, 0, 0);
-          y[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xv, __builtin_bit_cast(bf16x8, ml), y[i], 0, 0, 0);
+          yl[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xv, __builtin_bit_cast(bf16x8, ml), yl[i], 0, 0, 0);
         }
       }
-#pragma unroll
-      for (int k = 0; k < NN; ++k)
-#pragma unroll
-        for (int i = 0; i < PT; ++i) {
-          yi[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ssd_tr(&Sh[k * 32 + vrow][i * 16 + vcol], LX), cf[k], yi[i], 0, 0, 0);
-          yi[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ssd_tr(&Sl[k * 32 + vrow][i * 16 + vcol], LX), cf[k], yi[i], 0, 0, 0);
-        }
       const float into = __builtin_amdgcn_exp2f(ct);
       if (tok < tokens) {
-        const T *zp = static_cast<const T *>(a.proj) + row * a.ld + h * a.P + p0;
         T *op = static_cast<T *>(a.out) + row * a.ldo + static_cast<int64_t>(h) * a.P + p0;
 #pragma unroll
-        for (int i = 0; i < PT; ++i) {
-          const int p = i * 16 + g * 4;
+        for (int i = 0; i < PTY; ++i) {
+          const int p = (py + i) * 16 + g * 4;
           if (p0 + p >= a.P) continue;
-          float z[4], x[4];
-          const uint2 xr = *reinterpret_cast<const uint2 *>(&Xs[t][p]);
-          x[0] = __uint_as_float(xr.x << 16); x[1] = __uint_as_float(xr.x & 0xffff0000u);
-          x[2] = __uint_as_float(xr.y << 16); x[3] = __uint_as_float(xr.y & 0xffff0000u);
-          if (VEC) {
-            const uint2 zr = *reinterpret_cast<const uint2 *>(zp + p);
-            z[0] = __uint_as_float(zr.x << 16); z[1] = __uint_as_float(zr.x & 0xffff0000u);
-            z[2] = __uint_as_float(zr.y << 16); z[3] = __uint_as_float(zr.y & 0xffff0000u);
-          } else {
-#pragma unroll
-            for (int r = 0; r < 4; ++r) z[r] = p0 + p + r < a.P ? Elem<T>::ld(zp + p + r) : 0.f;
-          }
           float o[4];
+          const uint2 xr = *reinterpret_cast<const uint2 *>(&Xs[t][p]);
+          const float x[4] = {__uint_as_float(xr.x << 16), __uint_as_float(xr.x & 0xffff0000u), __uint_as_float(xr.y << 16), __uint_as_float(xr.y & 0xffff0000u)};
+          const float z[4] = {__uint_as_float(zr[i].x << 16), __uint_as_float(zr[i].x & 0xffff0000u), __uint_as_float(zr[i].y << 16),
+                              __uint_as_float(zr[i].y & 0xffff0000u)};
 #pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const float v = fmaf(D, x[r], fmaf(into, yi[i][r], y[i][r]));
-            o[r] = v * z[r] * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z[r]));
-          }
+          for (int r = 0; r < 4; ++r) o[r] = fmaf(D, x[r], fmaf(into, yi[i][r] + yil[i][r], y[i][r] + yl[i][r])) * ssd_silu<T>(z[r]);
           if (VEC) *reinterpret_cast<uint2 *>(op + p) = make_uint2(pack_bf16x2(o[0], o[1]), pack_bf16x2(o[2], o[3]));
           else
 #pragma unroll
@@ -503,24 +576,33 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) void s
         }
       }
     }
+    if (has_state) {
 #pragma unroll
-    for (int j = 0; j < NTW; ++j)
+      for (int j = 0; j < NTW; ++j)
 #pragma unroll
-      for (int i = 0; i < PT; ++i) S[j][i] *= end_decay;
-    if ((wave * NTW) * 16 < NP) {                    // wave uniform
+        for (int i = 0; i < PTU; ++i) S[j][i] *= end_decay;
 #pragma unroll
       for (int ks = 0; ks < 2; ++ks) {
-        bf16x8 bf[NTW];
+        float f[8];
+        Elem<float>::ld8(&into_end[ks * 32 + g * 8], f);
+        uint4 bh[NTW], bl[NTW];                      // B rows times dt 2^(c_end - c)
 #pragma unroll
-        for (int j = 0; j < NTW; ++j) bf[j] = ssd_tr(&Bs[ks * 32 + vrow][(wave * NTW + j) * 16 + vcol], LN);
+        for (int j = 0; j < NTW; ++j) {
+          float b[8];
+          unpack8(__builtin_bit_cast(uint4, ssd_tr(&Bs[ks * 32 + vrow][(nt0 + j) * 16 + vcol], LN)), b);
 #pragma unroll
-        for (int i = 0; i < PT; ++i) {
-          const bf16x8 xh = ssd_tr(&Xh[ks * 32 + vrow][i * 16 + vcol], LX), xl = ssd_tr(&Xl[ks * 32 + vrow][i * 16 + vcol], LX);
+          for (int e = 0; e < 8; ++e) b[e] *= f[e];
+          ssd_pair(b, bh[j], bl[j]);
+        }
+        bf16x8 xv[PTU];
 #pragma unroll
-          for (int j = 0; j < NTW; ++j) {
-            S[j][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xh, bf[j], S[j][i], 0, 0, 0);
-            S[j][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xl, bf[j], S[j][i], 0, 0, 0);
-          }
+        for (int i = 0; i < PTU; ++i) xv[i] = ssd_tr(&Xs[ks * 32 + vrow][(pt0 + i) * 16 + vcol], LX);
+#pragma unroll
+        for (int j = 0; j < NTW; ++j) {
+#pragma unroll
+          for (int i = 0; i < PTU; ++i) S[j][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xv[i], __builtin_bit_cast(bf16x8, bh[j]), S[j][i], 0, 0, 0);
+#pragma unroll
+          for (int i = 0; i < PTU; ++i) S[j][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xv[i], __builtin_bit_cast(bf16x8, bl[j]), S[j][i], 0, 0, 0);
         }
       }
     }
@@ -535,12 +617,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1))) void s
   } else {
     if (!last_seg || !slot_ok || tokens == 0) return;
   }
+  if (!has_state) return;
   float *dst = MODE == 1 ? gst : st;
 #pragma unroll
   for (int j = 0; j < NTW; ++j)
 #pragma unroll
-    for (int i = 0; i < PT; ++i) {
-      const int d = (wave * NTW + j) * 16 + n, p = p0 + i * 16 + g * 4;
+    for (int i = 0; i < PTU; ++i) {
+      const int d = (nt0 + j) * 16 + n, p = p0 + (pt0 + i) * 16 + g * 4;
       if (d < a.N) {
 #pragma unroll
         for (int r = 0; r < 4; ++r)
@@ -629,9 +712,9 @@ int launch_ssd_conv(const SsdArgs &a, hipStream_t s) {
              dim3((a.rows + (TOK) - 1) / (TOK), (a.channels + 256 * (VEC) - 1) / (256 * (VEC)) + 1), dim3(256), 0, s, a)
   if (vec) {
     switch (a.taps) {
-      case 2: TLF_SC(8, 2, 4); break;
-      case 3: TLF_SC(8, 3, 4); break;
-      case 4: TLF_SC(8, 4, 4); break;
+      case 2: if (a.rows >= 2048) TLF_SC(8, 2, 8); else TLF_SC(8, 2, 2); break;
+      case 3: if (a.rows >= 2048) TLF_SC(8, 3, 8); else TLF_SC(8, 3, 2); break;
+      case 4: if (a.rows >= 2048) TLF_SC(8, 4, 8); else TLF_SC(8, 4, 2); break;
       default: TLF_SC(8, 0, 1); break;
     }
   } else {
@@ -644,13 +727,14 @@ int launch_ssd_conv(const SsdArgs &a, hipStream_t s) {
 template <int NN, int PT, bool VEC>
 void launch_ssd_chunks(const SsdArgs &a, hipStream_t s) {
   const dim3 grid(a.H, a.slices, a.seqs * a.segs);
+  const dim3 block(ssd_waves<PT>() * 64);
   if (a.segs == 1) {
-    TLF_LAUNCH((ssd_chunk_kernel<NN, PT, 0, VEC>), grid, dim3(256), 0, s, a);
+    TLF_LAUNCH((ssd_chunk_kernel<NN, PT, 0, VEC>), grid, block, 0, s, a);
     return;
   }
-  TLF_LAUNCH((ssd_chunk_kernel<NN, PT, 1, VEC>), grid, dim3(256), 0, s, a);
+  TLF_LAUNCH((ssd_chunk_kernel<NN, PT, 1, VEC>), grid, block, 0, s, a);
   TLF_LAUNCH(ssd_segments_kernel, dim3((a.N * a.P + 255) / 256, a.H, a.seqs), dim3(256), 0, s, a);
-  TLF_LAUNCH((ssd_chunk_kernel<NN, PT, 2, VEC>), grid, dim3(256), 0, s, a);
+  TLF_LAUNCH((ssd_chunk_kernel<NN, PT, 2, VEC>), grid, block, 0, s, a);
 }
 
 }  // namespace tlf

@@ -1242,9 +1242,10 @@ def talk_attention_prefill(q, kv: SinkKV, block_tables, cu_seqlens_q, seq_starts
     assert q.is_contiguous() and dp == kv.k.shape[3] and kv.k.dtype == BF16 and out.stride(1) == 1 and out.shape[0] == n
     assert talk.is_contiguous() and talk.shape == (heads, heads)
     assert block_tables.stride(1) == 1 and block_tables.shape[0] >= first_seq + num_seqs
+    stats = torch.empty(n, heads, dtype=torch.float32, device=q.device)
     check(_lib.load().tlf_talk_attn_prefill(
         q.data_ptr(), kv.k.data_ptr(), kv.v.data_ptr(), block_tables.data_ptr(), block_tables.stride(0), cu_seqlens_q.data_ptr(),
-        seq_starts.data_ptr(), first_seq, num_seqs, max_tokens, talk.data_ptr(), out.data_ptr(), out.stride(0), heads, G, kv.dim, kv.vdim,
+        seq_starts.data_ptr(), first_seq, num_seqs, max_tokens, talk.data_ptr(), stats.data_ptr(), out.data_ptr(), out.stride(0), heads, G, kv.dim, kv.vdim,
         bs, pages, _stream()), "tlf_talk_attn_prefill")
     return out
 
