@@ -1153,7 +1153,7 @@ def bench_tibenex_kernels(sizes=None):
             for i in range(copies):
                 fn(i)
         sec = time_graph(cycle, launches=max(1, launches // copies), replays=10) * 1e-3 / copies
-        peak = {"hbm": HBM_PEAK_GBPS * 1e9, "mfma bf16": MFMA_BF16_PEAK_TFLOPS * 1e12, "mfma f32": MFMA_F32_PEAK_TFLOPS * 1e12}[bound]
+        peak = {"hbm": HBM_PEAK_GBPS * 1e9, "mfma bf16": MFMA_BF16_PEAK_TFLOPS * 1e12}[bound]
         rows.append(dict(kernel=name, size=size, us=round(sec * 1e6, 2), bound=bound,
                          rate=round(amount / sec / (1e9 if bound == "hbm" else 1e12), 1), frac=round(amount / sec / peak, 4)))
         print(rows[-1], file=sys.stderr, flush=True)
@@ -1285,7 +1285,7 @@ def bench_tibenex_kernels(sizes=None):
             proj, out = bf(b, sld), torch.empty(b, sh * sp, device=dev, dtype=BF)
             add(f"state space, {b} decoded tokens", size, lambda i: P.ssd_decode(proj, sw, ring, state, sl, ps, sg, out), b * sh * sn * sp * 8, "hbm")
             del state, ring, proj, out
-        for s_, l_ in ((8, 2048), (1, 8192)):
+        for s_, l_ in ((8, 2048), (1, 8192)):                    # bytes: a projection row read, the result written
             n = s_ * l_
             sl, st, cus = ar(s_), torch.zeros(s_, dtype=I32, device=dev), torch.arange(0, n + 1, l_, dtype=I32, device=dev)
             state = torch.zeros(s_, gh, gk, gv, device=dev)
@@ -1294,14 +1294,13 @@ def bench_tibenex_kernels(sizes=None):
             chunk_lens, cuc = torch.full_like(chunk_rows, 16), torch.arange(0, n // 16 + 1, l_ // 16, dtype=I32, device=dev)
             add(f"gated linear attention (Gitopel), prompts {s_} x {l_}", size,
                 lambda i: P.gla_portions(proj, a2, a2b, gw, state, sl, st, chunk_rows, chunk_lens, cuc, 0, s_, 16.0, 1e-6, out),
-                n * gh * (4.0 * gk * gv + 2 * 16 * (gk + gv)), "mfma f32")
+                n * (gld + gh * gv) * 2, "hbm")
             state, ring = torch.zeros(s_, sh, sn, sp, device=dev), torch.zeros(s_, 4, schan, device=dev, dtype=BF)
             proj, out = bf(n, sld), torch.empty(n, sh * sp, device=dev, dtype=BF)
             ps, rs = torch.arange(l_, device=dev).repeat(s_), ar(n) // l_
-            # bytes: a projection row read, the result written (the convolved rows in between stay in the chip's caches at best)
             add(f"state space, prompts {s_} x {l_}", size,
                 lambda i: P.ssd_portions(proj, sw, ring, state, sl, ps, rs, cus, st, 0, s_, 0, l_, sg, out),
-                n * sh * (4.0 * sn * sp + 64.0 * (sn + sp)), "mfma bf16")
+                n * (sld + sh * sp) * 2, "hbm")
             add(f"convolution state, {s_} portions", size, lambda i: P.conv_tail(proj[:, sh * sp:], ring, sl, cus, st, 0, s_), s_ * 3 * schan * 4, "hbm")
             del state, ring, proj, out
     return rows

@@ -218,7 +218,8 @@ def test_talking_heads_of_many_unequal_sequences(dtype):
 
 # ---------------------------------------------------------------------------------------------- state-space recurrence
 # heads, value dim, state, groups, taps: sizes that no tile divides, one of everything, beyond the matrix cores
-SSD = [(6, 10, 13, 3, 3), (1, 1, 1, 1, 1), (4, 64, 64, 1, 4), (8, 64, 128, 2, 4), (2, 128, 256, 2, 5), (12, 24, 40, 12, 2), (3, 200, 96, 1, 4), (2, 300, 280, 1, 2), (5, 16, 300, 5, 3)]
+SSD = [(6, 10, 13, 3, 3), (1, 1, 1, 1, 1), (4, 64, 64, 1, 4), (8, 64, 128, 2, 4), (2, 128, 256, 2, 5), (12, 24, 40, 12, 2), (3, 200, 96, 1, 4), (2, 300, 280, 1, 2), (5, 16, 300, 5, 3),
+       (3, 20, 24, 1, 9)]
 
 
 def ssd_case(sizes, lens, dt, seed, decay=0.0, step=-1.5):

@@ -63,12 +63,10 @@ __device__ __forceinline__ void turn8(const LatentPrepArgs &a, const float *cs, 
   }
 }
 
-// Piece d .. d + 7 of the rotated part that begins at column `col`, partners rot / 2 away.
+// The partners, rot / 2 away, of piece d .. d + 7 of the rotated part that begins at column `col`.
 template <typename T, bool PART>
-__device__ __forceinline__ void turn8_halves(const LatentPrepArgs &a, const float *cs, int64_t tok, int col, int d, float (&f)[8]) {
-  if (cs == nullptr) return;
+__device__ __forceinline__ void partner8(const LatentPrepArgs &a, int64_t tok, int col, int d, float (&p)[8]) {
   const int half = a.s.rot / 2;
-  float p[8];
   if (a.vec && half % 8 == 0) {
     prep_ld8<T, PART>(a, tok, col, d < half ? d + half : d - half, a.s.rot, p);
   } else {
@@ -77,6 +75,18 @@ __device__ __forceinline__ void turn8_halves(const LatentPrepArgs &a, const floa
       const int i = d + e;
       p[e] = i < a.s.rot ? prep_ld<T, PART>(a, tok, col + (i < half ? i + half : i - half)) : 0.f;
     }
+  }
+}
+
+__device__ __forceinline__ void turn8_halves(const LatentPrepArgs &a, const float *cs, int d, const float (&p)[8], float (&f)[8]) {
+  if (cs == nullptr) return;
+  const int half = a.s.rot / 2;
+  if (half % 8 == 0) {                                     // the piece lies on one side
+    const float *c = cs + (d < half ? d : d - half);
+    const float sign = d < half ? -1.f : 1.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[e] = __fmul_rn(f[e], c[e]) + sign * __fmul_rn(p[e], c[half + e]);
+    return;
   }
 #pragma unroll
   for (int e = 0; e < 8; ++e) {
@@ -175,8 +185,13 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a
         if (d < s.rot) prep_ld8<T, PART>(a, tok, a.off + s.rank, d, s.rot, t);
       }
       if (d < s.rot) {
-        if (a.halves) turn8_halves<T, PART>(a, cs, tok, a.off + s.rank, d, t);
-        else turn8(a, cs, d, t);
+        if (a.halves) {
+          float p[8];
+          partner8<T, PART>(a, tok, a.off + s.rank, d, p);
+          turn8_halves(a, cs, d, p, t);
+        } else {
+          turn8(a, cs, d, t);
+        }
       }
       Elem<T>::st8(row + s.Ra + d, t);
     }
@@ -188,13 +203,14 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a
   const int h = item / nch, d = (item - h * nch) * 8;
   const int col = h * (s.dim + s.rot);
   const bool own = d < s.Da, turned = !own && d < s.Da + s.rot;
-  float f[TOK][8];
+  float f[TOK][8], p[TOK][8];
   int64_t pos[TOK];
 #pragma unroll
   for (int k = 0; k < TOK; ++k) {
     const int64_t tok = min(tok0 + k, static_cast<int64_t>(a.n) - 1);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) f[k][e] = 0.f;
+    for (int e = 0; e < 8; ++e) f[k][e] = p[k][e] = 0.f;
+    if (turned && a.halves) partner8<T, PART>(a, tok, col + s.dim, d - s.Da, p[k]);
     if (own) prep_ld8<T, PART>(a, tok, col, d, s.dim, f[k]);
     else if (turned) prep_ld8<T, PART>(a, tok, col + s.dim, d - s.Da, s.rot, f[k]);
     pos[k] = turned ? a.positions[tok] : 0;
@@ -204,7 +220,7 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(const LatentPrepArgs a
     if (tok0 + k >= a.n) return;
     if (turned) {
       const float *cs = pos[k] >= 0 && pos[k] < a.max_pos ? a.cos_sin + pos[k] * s.rot : nullptr;
-      if (a.halves) turn8_halves<T, PART>(a, cs, tok0 + k, col + s.dim, d - s.Da, f[k]);
+      if (a.halves) turn8_halves(a, cs, d - s.Da, p[k], f[k]);
       else turn8(a, cs, d - s.Da, f[k]);
     }
     Elem<T>::st8(static_cast<T *>(a.q_out) + ((tok0 + k) * s.H + h) * s.Dq + d, f[k]);
