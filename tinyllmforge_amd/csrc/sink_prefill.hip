@@ -37,10 +37,6 @@ __device__ __forceinline__ shortx4 sinkp_read_tr16(const unsigned short *p) {
 template <int DC, int VC, int CT, int MODE>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(2, 2))) void sink_prefill_kernel(const SinkPrefillArgs p) {
   constexpr int DP = DC * 32, VP = VC * 32, KCH = DC * 4, VCH = VC * 4;
-  #ifndef STAGES
-#define STAGES 1
-#endif
-  constexpr int ST = DC + VC <= 8 ? STAGES : 1;                   // tiles in LDS
   __shared__ __attribute__((aligned(16))) unsigned short Ks[kSK][DP + 8], Vs[kSK][VP + 16];
   // consecutive row tiles of one KV head share keys: they go to the same XCD (workgroup w runs on XCD w % 8); the last row
   // tiles, which see the most keys, come first

@@ -185,6 +185,7 @@ __global__ __launch_bounds__(WV * RT * 64) void talk_prefill_kernel(const TalkPr
   constexpr int VP = VC * 32, PIECES = VP / 8, RW = RT < 4 / GS ? RT : 4 / GS, HW = 4 / RW, KV = HW > GS ? HW / GS : 1, HK = HW / KV;
   constexpr int PER = 4 / KV;                                        // items of a KV head
   constexpr int TS = KH * 32 + 8;                                    // heads of a talk row in LDS
+  constexpr int kAtOnce = HT == 1 ? 4 : 1;                           // rows of the mix, as registers allow
   extern __shared__ __attribute__((aligned(1024))) unsigned short lds[];
   unsigned short *Vs = lds, *Wh = lds + p.c.G * kTK * VP, *Wl = Wh + TQ * ROW, *Ts = Wl + TQ * ROW;    // Vs [G][32][VP], Ts [16 HT][TS]
   const int id = (blockIdx.x & 7) * p.per_xcd + (blockIdx.x >> 3);   // neighbours in rows share keys: the same XCD
@@ -346,7 +347,7 @@ __global__ __launch_bounds__(WV * RT * 64) void talk_prefill_kernel(const TalkPr
     for (int ht = 0; ht < HT; ++ht)
 #pragma unroll
       for (int k = 0; k < KH; ++k) tf[ht][k] = talk_ld<bf16x8>(tat + (ht * 16 * TS + k * 32) * 2);
-#pragma unroll (HT == 1 ? 4 : 1)
+#pragma unroll kAtOnce
     for (int i = 0; i < TQ / NW; ++i) {                              // a row's W is read and its M written by the same wave
       const unsigned int row_at = i * (NW * ROW * 2);
       floatx4 mx[HT][2];
